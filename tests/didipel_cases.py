@@ -1,0 +1,117 @@
+"""Small random Didipel checkpoints for the tests."""
+import copy
+import json
+
+import torch
+
+BASE = {
+  "architecture": "Didipel", "vocab": 101, "width": 72, "norm": {"eps": 1e-5},
+  "layers": [
+    {"type": "parallel", "mlp": {"kind": "dense", "ff": 96}, "mixer": {
+      "left": {"heads": 6, "kv_heads": 2, "dim": 20, "vdim": 12, "scale": 0.31, "bias_max": 17,
+               "mask": {"size": 11}},
+      "right": {"heads": 4, "kv_heads": 2, "dim": 12, "vdim": 20, "conv": 4},
+      "left_scale": 0.55, "right_scale": 1.3}},
+    {"type": "wkv", "mlp": None, "mixer": {"heads": 3, "dim": 28}},
+    {"type": "parallel", "mlp": {"kind": "dense", "ff": 56}, "mixer": {
+      "left": {"heads": 4, "kv_heads": 4, "dim": 32, "vdim": 40, "scale": 0.2, "bias_max": 40,
+               "mask": {"size": 33}},
+      "right": {"heads": 3, "kv_heads": 3, "dim": 40, "vdim": 16, "conv": 2},
+      "left_scale": 1.0, "right_scale": 0.4}},
+    {"type": "wkv", "mlp": {"kind": "dense", "ff": 64}, "mixer": {"heads": 2, "dim": 64}},
+  ],
+}
+RANKS = {"rel": 8, "a1": 10, "g1": 14, "w1": 6}
+
+
+def small(**changes):
+  cfg = copy.deepcopy(BASE)
+  cfg.update(changes)
+  return cfg
+
+
+def random_weights(cfg, seed=0, rel_rows=RANKS["rel"]):
+  """Weights at sizes where every mechanism moves the logits: decays spread
+  over (0, 1), norms and mixing weights away from their neutral values. All
+  rounded to bfloat16, as a checkpoint holds them."""
+  g = torch.Generator().manual_seed(seed)
+  w = {}
+
+  def normal(name, *shape, std=None):
+    w[name] = torch.randn(*shape, generator=g) * (shape[-1] ** -0.5 if std is None else std)
+
+  def uniform(name, lo, hi, *shape):
+    w[name] = torch.rand(*shape, generator=g) * (hi - lo) + lo
+
+  D = cfg["width"]
+  normal("embed", cfg["vocab"], D, std=1.0)
+  for i, layer in enumerate(cfg["layers"]):
+    p, m = f"l{i}.mix.", layer["mixer"]
+    for n in ("norm1", "norm1b") + (("norm2", "norm2b") if layer["mlp"] else ()):
+      normal(f"l{i}.{n}", D, std=0.3)
+    if layer["type"] == "parallel":
+      a, q = m["left"], p + "left."
+      H, G, d, e = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+      for n, rows in (("q", H * d), ("k", G * d), ("v", G * e), ("g", H)):
+        normal(q + n, rows, D)
+      uniform(q + "q.norm", 0.5, 1.8, H * d)
+      uniform(q + "k.norm", 0.5, 1.8, G * d)
+      normal(q + "rel", rel_rows, H, std=1.0)
+      normal(q + "o", D, H * e)
+      b, q = m["right"], p + "right."
+      H, G, d, e = b["heads"], b["kv_heads"], b["dim"], b["vdim"]
+      for n, rows in (("q", G * d), ("k", G * d), ("v", H * e)):
+        normal(q + n, rows, D)
+        normal(q + n + ".conv", rows, b["conv"], std=0.6)
+      normal(q + "b", H, D)
+      uniform(q + "A_log", -1.0, 1.0, H)
+      uniform(q + "norm", 0.5, 1.5, e)
+      normal(q + "a1", RANKS["a1"], D)
+      normal(q + "a2", H * d, RANKS["a1"])
+      uniform(q + "dt_bias", -6.0, 0.0, H * d)
+      normal(q + "g1", RANKS["g1"], D)
+      normal(q + "g2", H * e, RANKS["g1"])
+      normal(q + "o", D, H * e)
+    else:
+      H, d = m["heads"], m["dim"]
+      for n in "rkvgw":
+        uniform(p + "mu." + n, 0.0, 1.0, D)
+      for n in "rkvg":
+        normal(p + n, H * d, D)
+      normal(p + "w1", RANKS["w1"], D)
+      normal(p + "w2", H * d, RANKS["w1"])
+      uniform(p + "w0", -6.0, 0.0, H * d)
+      normal(p + "u", H, d, std=0.5)
+      uniform(p + "norm", 0.5, 1.5, H * d)
+      normal(p + "o", D, H * d)
+    if layer["mlp"]:
+      ff = layer["mlp"]["ff"]
+      normal(f"l{i}.mlp.gate", ff, D)
+      normal(f"l{i}.mlp.up", ff, D)
+      normal(f"l{i}.mlp.down", D, ff)
+  normal("final.norm", D, std=0.3)
+  normal("head", cfg["vocab"], D)
+  return {n: t.to(torch.bfloat16) for n, t in w.items()}
+
+
+def write_checkpoint(folder, cfg, w):
+  from safetensors.torch import save_file
+  folder.mkdir(parents=True, exist_ok=True)
+  (folder / "config.json").write_text(json.dumps(cfg))
+  save_file({n: t.contiguous() for n, t in w.items()}, str(folder / "model.safetensors"))
+  return folder
+
+
+def load_model(folder, device="cpu", dtype=torch.float32, layers=None):
+  """The framework's own model class and loader on a checkpoint folder;
+  layers: (first, last) of a shard."""
+  from xotorch_amd.models import config_from_hf, model_class_for
+  from xotorch_amd.models.weights import load_shard_weights
+  from xotorch_amd.shard import Shard
+  cfg = config_from_hf(folder / "config.json", "case")
+  first, last = layers or (0, cfg.n_layers - 1)
+  model = model_class_for(cfg)(cfg, Shard("case", first, last, cfg.n_layers)).to(dtype)
+  load_shard_weights(model, folder)
+  model = model.to(device)
+  model.reset_rope()
+  return model.eval()

@@ -286,8 +286,8 @@ def test_registry_consistency():
     assert card.get("layers", 0) > 0, mid
     cfg = builtin_config(mid)
     if cfg is not None:
-      assert cfg["num_hidden_layers"] == card["layers"], \
-        f"{mid}: card layers {card['layers']} != builtin {cfg['num_hidden_layers']}"
+      n = config_from_hf(cfg, mid).n_layers
+      assert n == card["layers"], f"{mid}: card layers {card['layers']} != builtin {n}"
   # every builtin config belongs to a card
   for mid in BUILTIN_CONFIGS:
     assert mid in model_cards or mid in ("dummy",), mid

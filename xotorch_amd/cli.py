@@ -19,13 +19,15 @@ import uuid
 from pathlib import Path
 
 from xotorch_amd.helpers import DEBUG, find_available_port, get_or_create_node_id
-from xotorch_amd.models.registry import build_base_shard, get_supported_models
+from xotorch_amd.models.registry import build_base_shard, get_supported_models, register_local_model
 
 
 def build_parser() -> argparse.ArgumentParser:
   p = argparse.ArgumentParser("xot", description="MI355X-native distributed LLM runtime")
   p.add_argument("command", nargs="?", choices=["run", "eval", "train", "serve"], help="one-shot verb (default: daemon)")
   p.add_argument("model_name", nargs="?", help="model id (see --list-models)")
+  p.add_argument("--model-dir", type=str, default=None,
+                 help="folder with config.json and safetensors, used as the model named model_name")
   p.add_argument("--list-models", action="store_true")
   p.add_argument("--prompt", type=str, default=None,
                  help="run: one-shot prompt; omit for the interactive chat TUI")
@@ -66,14 +68,18 @@ def pick_engine(args) -> str:
 
 async def make_node(args):
   from xotorch_amd.engine.interface import get_inference_engine
-  from xotorch_amd.download.downloader import new_shard_downloader
+  from xotorch_amd.download.downloader import NoopShardDownloader, new_shard_downloader
   from xotorch_amd.orchestration.discovery import ManualDiscovery, UDPDiscovery
   from xotorch_amd.orchestration.node import Node
   from xotorch_amd.orchestration.server import Server
 
   node_id = args.node_id or get_or_create_node_id()
   node_port = args.node_port or find_available_port()
-  downloader = new_shard_downloader("noop" if os.getenv("XOT_OFFLINE") == "1" else "hf")
+  if args.model_dir:
+    register_local_model(args.model_name, args.model_dir)
+    downloader = NoopShardDownloader(Path(args.model_dir))  # nothing to fetch
+  else:
+    downloader = new_shard_downloader("noop" if os.getenv("XOT_OFFLINE") == "1" else "hf")
   engine = get_inference_engine(pick_engine(args), downloader)
   if args.discovery_module == "udp":
     discovery = UDPDiscovery(node_id, node_port, args.listen_port, args.broadcast_port,
@@ -217,6 +223,8 @@ def serve_ring(args):
          "--model", args.model_name or "llama-3-8b",
          "--port", str(args.chatgpt_api_port),
          "--slots", str(args.slots)]
+  if args.model_dir:
+    cmd += ["--model-dir", args.model_dir]
   if args.no_graphs:
     cmd.append("--no-graphs")
   raise SystemExit(subprocess.run(cmd).returncode)
@@ -224,6 +232,8 @@ def serve_ring(args):
 
 def run():
   args = build_parser().parse_args()
+  if args.model_dir and not args.model_name:
+    raise SystemExit("--model-dir needs a model name to go by")
   if args.list_models:
     for mid in get_supported_models():
       print(mid)

@@ -111,3 +111,47 @@ class ShardKVCache:
       if c.kp is not None:
         total += c.kp.numel() * c.kp.element_size() + c.vp.numel() * c.vp.element_size()
     return total
+
+
+class MixerStateCache:
+  """State of the layers of a design whose mixers differ (cfg.layer_specs):
+  per local layer a list with one tuple of tensors per branch of its mixer,
+  each tensor [slots, ...] as the mixer's `state_spec` says. Slots are
+  independent and constant in size; a sequence that starts at position 0
+  ignores what its slot held before."""
+
+  def __init__(self, cfg, shard, slots: int, capacity: int, dtype: torch.dtype = torch.bfloat16,
+               device: str = "cpu"):
+    from xotorch_amd.models.mixers import MIXERS
+    self.batch, self.capacity = slots, capacity
+    self.caches: List[list] = []
+    for lid in range(shard.start_layer, shard.end_layer + 1):
+      spec = cfg.layer_specs[lid]
+      self.caches.append([
+        tuple(torch.zeros(slots, *shape, dtype=dt, device=device) for shape, dt in branch.values())
+        for branch in MIXERS[spec.mixer].state_spec(spec.params, capacity, dtype, device)
+      ])
+
+  def __getitem__(self, i):
+    return self.caches[i]
+
+  def __len__(self):
+    return len(self.caches)
+
+  def _tensors(self):
+    return [t for layer in self.caches for branch in layer for t in branch]
+
+  def reset(self):
+    for t in self._tensors():
+      t.zero_()
+
+  def nbytes(self) -> int:
+    return sum(t.numel() * t.element_size() for t in self._tensors())
+
+
+def make_cache(cfg, shard, batch: int, capacity: int, dtype: torch.dtype = torch.bfloat16, device: str = "cpu"):
+  """The cache or state manager that a model's shard decodes with."""
+  if cfg.layer_specs is not None:
+    return MixerStateCache(cfg, shard, batch, capacity, dtype, device)
+  heads, k_dim, v_dim = cfg.kv_cache_dims()
+  return ShardKVCache(shard.get_layer_count(), batch, heads, capacity, k_dim, dtype, device, v_dim=v_dim)

@@ -56,6 +56,9 @@ class SpeculativeDecoder:
     self.device, self.dtype = device, dtype
     self.gamma = gamma
     self.max_seq = min(max_seq, target_cfg.max_seq_len, draft_cfg.max_seq_len)
+    for cfg in (target_cfg, draft_cfg):
+      if cfg.layer_specs is not None:
+        raise ValueError(f"{cfg.model_id}: speculative decoding rewinds positions, which a recurrent state cannot")
     th, tk, tv = target_cfg.kv_cache_dims()
     dh, dk, dv = draft_cfg.kv_cache_dims()
     self.t_cache = ShardKVCache(target_cfg.n_layers, 1, th, self.max_seq, tk, dtype, device, v_dim=tv)

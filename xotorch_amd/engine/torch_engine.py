@@ -26,9 +26,10 @@ import torch
 
 from xotorch_amd import ops
 from xotorch_amd.engine.interface import InferenceEngine
-from xotorch_amd.engine.kvcache import ShardKVCache
+from xotorch_amd.engine.kvcache import ShardKVCache, make_cache
 from xotorch_amd.engine.state import ShardInferenceState
 from xotorch_amd.engine.tokenizers import DummyTokenizer, resolve_tokenizer
+from xotorch_amd.models import model_class_for
 from xotorch_amd.models.config import ModelConfig, config_from_hf
 from xotorch_amd.models.llama import ShardedModel
 from xotorch_amd.models.registry import builtin_config, get_repo
@@ -104,14 +105,7 @@ class TorchEngine(InferenceEngine):
     if cfg_dict is None:
       raise ValueError(f"no config available for model {shard.model_id}")
     cfg = config_from_hf(cfg_dict, model_id=shard.model_id)
-    if cfg.model_type == "gemma2":
-      from xotorch_amd.models.gemma2 import Gemma2Model
-      model_cls = Gemma2Model
-    elif cfg.model_type in ("deepseek_v3", "deepseek_v2"):
-      from xotorch_amd.models.deepseek_v3 import DeepseekV3Model
-      model_cls = DeepseekV3Model
-    else:
-      model_cls = ShardedModel
+    model_cls = model_class_for(cfg)
     # construct at the target dtype so to_empty materializes it directly
     # (fp32-then-cast would peak at 2x the weight bytes)
     prev_dtype = torch.get_default_dtype()
@@ -147,11 +141,7 @@ class TorchEngine(InferenceEngine):
   def _session(self, request_id: str, batch: int, total_len: int) -> Session:
     sess = self.sessions.get(request_id)
     if sess is None or sess.cache.batch != batch or sess.cache.capacity < total_len:
-      heads, k_dim, v_dim = self.cfg.kv_cache_dims()
-      cache = ShardKVCache(
-        n_layers=self.shard.get_layer_count(), batch=batch, n_kv_heads=heads,
-        capacity=total_len, head_dim=k_dim, dtype=self.dtype, device=self.device, v_dim=v_dim,
-      )
+      cache = make_cache(self.cfg, self.shard, batch, total_len, self.dtype, self.device)
       sess = Session(cache=cache, state=ShardInferenceState(total_len=total_len, batch=batch))
       self.sessions[request_id] = sess
     return sess
@@ -209,7 +199,7 @@ class TorchEngine(InferenceEngine):
       )
     x = x.to(self.device)
     if not is_tokens:
-      x = x.to(self.dtype)
+      x = x.to(getattr(self.model, "hidden_dtype", self.dtype))
     positions = torch.arange(start_pos, start_pos + S, dtype=torch.int32, device=self.device)
     is_decode = S == 1 and start_pos > 0
     try:
@@ -307,7 +297,7 @@ class TorchEngine(InferenceEngine):
       model.train(was_training)
       return loss_val, None
     if not is_tokens:
-      x = x.to(self.dtype).requires_grad_(True)
+      x = x.to(getattr(model, "hidden_dtype", self.dtype)).requires_grad_(True)
     with torch.enable_grad():
       out = self._train_forward(x)
       if loss == "back_gradient":

@@ -10,7 +10,11 @@ from xotorch_amd.models.registry import (  # noqa: F401
 
 
 def model_class_for(cfg: ModelConfig):
-  """Decoder class for a parsed config (ShardedModel / Gemma2 / DeepSeek-MLA)."""
+  """Decoder class for a parsed config (ShardedModel / Gemma2 / DeepSeek-MLA /
+  Didipel)."""
+  if cfg.model_type == "didipel":
+    from xotorch_amd.models.didipel import DidipelModel
+    return DidipelModel
   if cfg.model_type == "gemma2":
     from xotorch_amd.models.gemma2 import Gemma2Model
     return Gemma2Model

@@ -13,7 +13,7 @@ import math
 import os
 from dataclasses import dataclass, field
 from pathlib import Path
-from typing import Optional
+from typing import Dict, List, Optional, Tuple
 
 import torch
 
@@ -38,6 +38,16 @@ class RopeScaling:
   mscale: float = 1.0
   mscale_all_dim: float = 0.0
   truncate: bool = True
+
+
+@dataclass
+class LayerSpec:
+  """One layer of a design whose layers are listed one by one: the kind of
+  its mixer (a key of models.mixers.MIXERS), that mixer's sizes and constants,
+  and the width of its dense feed-forward (0: none)."""
+  mixer: str
+  params: dict
+  ff: int = 0
 
 
 @dataclass
@@ -92,6 +102,8 @@ class ModelConfig:
   n_experts_per_tok: int = 2
   moe_intermediate_dim: int = 0   # per-expert I (qwen3moe); 0 → intermediate_dim
   moe_style: str = "mixtral"      # HF checkpoint key layout: mixtral | qwen3
+  # designs whose layers differ (models/didipel.py); None → n_layers alike
+  layer_specs: Optional[List[LayerSpec]] = None
 
   @property
   def kv_mult(self) -> int:
@@ -99,6 +111,11 @@ class ModelConfig:
 
   def estimate_param_bytes(self) -> int:
     """Rough bf16 parameter footprint — used by the partitioner for sizing."""
+    if self.layer_specs is not None:
+      from xotorch_amd.models.mixers import MIXERS
+      mixers = sum(MIXERS[s.mixer].param_count(self.dim, s.params) for s in self.layer_specs)
+      ff = sum(3 * self.dim * s.ff for s in self.layer_specs)
+      return 2 * (mixers + ff + 4 * self.n_layers * self.dim + 2 * self.vocab_size * self.dim)
     per_layer = (
       self.dim * (self.n_heads + 2 * self.n_kv_heads) * self.head_dim  # qkv
       + self.n_heads * self.head_dim * self.dim  # o
@@ -109,13 +126,37 @@ class ModelConfig:
     return 2 * (self.n_layers * per_layer + embed + self.dim)
 
 
+def checkpoint_shapes(model_dir: Path) -> Dict[str, Tuple[int, ...]]:
+  """Tensor shapes of every safetensors file in a folder, from the headers
+  alone (8-byte little-endian length, then JSON)."""
+  shapes: Dict[str, Tuple[int, ...]] = {}
+  for path in sorted(Path(model_dir).glob("*.safetensors")):
+    with open(path, "rb") as f:
+      header = json.loads(f.read(int.from_bytes(f.read(8), "little")))
+    for name, info in header.items():
+      if name != "__metadata__":
+        shapes[name] = tuple(info["shape"])
+  return shapes
+
+
 def config_from_hf(config_path: Path | str | dict, model_id: str = "unknown") -> ModelConfig:
-  """Parse a HF-style config.json (path or dict) into a ModelConfig."""
+  """Parse a HF-style config.json (path or dict) into a ModelConfig. A config
+  with an "architecture" key belongs to a design with a reader of its own;
+  sizes that it leaves to the checkpoint are read from the tensor shapes of
+  the folder the file lies in."""
+  shapes: Dict[str, Tuple[int, ...]] = {}
   if isinstance(config_path, (str, Path)):
     with open(config_path) as f:
       raw = json.load(f)
+    if "architecture" in raw:
+      shapes = checkpoint_shapes(Path(config_path).parent)
   else:
     raw = dict(config_path)
+  if "architecture" in raw:
+    if raw["architecture"] == "Didipel":
+      from xotorch_amd.models.didipel import didipel_config
+      return didipel_config(raw, model_id, shapes)
+    raise ValueError(f"unknown architecture {raw['architecture']!r}")
 
   n_heads = raw.get("num_attention_heads", 32)
   dim = raw.get("hidden_size", 4096)

@@ -260,6 +260,10 @@ class MLP(nn.Module):
     self.gate_up_proj = XotLinear(cfg.dim, 2 * I, bias=False)
     self.down_proj = XotLinear(I, cfg.dim, bias=False)
 
+  @staticmethod
+  def act(gu):
+    return ops.swiglu_packed(gu)
+
   def forward(self, x):
     gu = self.gate_up_proj(x)
     dp = self.down_proj
@@ -281,7 +285,7 @@ class MLP(nn.Module):
             else:
               wp = dp.weight_packed
               t_fused = _time_us(lambda: hip.skinny_gemm_packed_swiglu(gu, wp, N, dp.bias))
-              t_split = _time_us(lambda: dp(ops.swiglu_packed(gu)))
+              t_split = _time_us(lambda: dp(self.act(gu)))
               use = "fused" if t_fused < t_split * 0.98 else "split"
               _PACKED_WINS[key] = use
               if os.getenv("XOT_DEBUG", "0") != "0":
@@ -290,7 +294,7 @@ class MLP(nn.Module):
           if use == "fused":
             y = hip.skinny_gemm_packed_swiglu(gu, dp.weight_packed, N, dp.bias)
             return y.view(list(x.shape[:-1]) + [N])
-    return self.down_proj(ops.swiglu_packed(gu))
+    return self.down_proj(self.act(gu))
 
 
 class MoEMLP(nn.Module):

@@ -1,0 +1,298 @@
+"""Token mixers beyond plain GQA attention, composable per layer.
+
+A design that lists its layers (ModelConfig.layer_specs) names a mixer for
+each; MIXERS maps that name to a class here. Every constant of a mechanism is
+a parameter of its branch, so another design can use it with its own.
+
+Branches that read projections of the layer's input (`WindowBiasAttention`,
+`GatedDeltaRule`) are combined by `BranchMixer`: ONE fused input GEMM over
+the parts of all branches and ONE output GEMM over their concatenated
+activations (branch weights fold into the activations in fp32), however many
+branches run side by side. `WKVMixer` shifts its input per projection and so
+keeps GEMMs of its own.
+
+State lives outside (engine/kvcache.py): each class says in `state_spec` what
+one slot holds and gets the tensors back in `forward`.
+"""
+from __future__ import annotations
+
+import math
+from typing import Dict, List, Optional, Tuple
+
+import torch
+import torch.nn as nn
+
+from xotorch_amd.models.llama import XotLinear
+from xotorch_amd.ops import mixer_ops as mo
+
+StateSpec = Dict[str, Tuple[tuple, torch.dtype]]  # name -> (shape per slot, dtype)
+
+
+def _up(n: int, to: int) -> int:
+  return -(-n // to) * to
+
+
+def distance_buckets(rows: int, far: int, length: int) -> torch.Tensor:
+  """Bucket of every distance 0..length-1: the first half of `rows` one each,
+  the rest logarithmic up to distance `far`, clamped to the last."""
+  half = rows // 2
+  out = []
+  for n in range(length):
+    if n < half:
+      out.append(n)
+      continue
+    # the nudge keeps exact powers on their own side of the floor
+    steps = math.log(n / half) / math.log(far / half) * (rows - half)
+    out.append(min(rows - 1, half + math.floor(steps + 1e-9)))
+  return torch.tensor(out, dtype=torch.int32)
+
+
+class WindowBiasAttention(nn.Module):
+  """GQA attention over a sliding window: RMS norm over the whole q and k
+  projections, no rotation, a learned bias per distance bucket, a sink of
+  score zero in the softmax, one sigmoid output gate per head."""
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__()
+    self.H, self.G, self.dim, self.vdim = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    if self.H % self.G:
+      raise ValueError(f"{self.H} query heads do not divide into {self.G} key/value heads")
+    self.scale, self.window, self.far, self.eps = float(p["scale"]), int(p["mask"]["size"]), p["bias_max"], eps
+    if self.window < 1:
+      raise ValueError(f"window of {self.window} tokens")
+    self.parts = [("q", self.H * self.dim), ("k", self.G * self.dim), ("v", self.G * self.vdim), ("g", self.H)]
+    self.width = self.H * self.vdim
+    self.q_norm = nn.Parameter(torch.ones(self.H * self.dim))
+    self.k_norm = nn.Parameter(torch.ones(self.G * self.dim))
+    self.rel = nn.Parameter(torch.zeros(p["buckets"], self.H))
+    self.init_ranges = {"q_norm": (0.8, 1.2), "k_norm": (0.8, 1.2), "rel": (-0.5, 0.5)}
+    self.register_buffer("bucket", torch.empty(0, dtype=torch.int32), persistent=False)
+    self.reset_tables()
+
+  def reset_tables(self, device=None):
+    # the last bucket starts at distance `far` at the latest, so the table
+    # ends there and longer distances read its last entry
+    length = min(self.window, max(int(math.ceil(self.far)), self.rel.shape[0] // 2) + 1)
+    self.bucket = distance_buckets(self.rel.shape[0], self.far, length).to(device or self.bucket.device)
+
+  @staticmethod
+  def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> StateSpec:
+    G, d, e = p["kv_heads"], p["dim"], p["vdim"]
+    ring = min(p["mask"]["size"], capacity)  # only a window of keys is ever read
+    if mo.packed_kv(dtype, device):
+      ring = _up(ring, 32)
+      # MFMA fragment order, dims padded with zeros: 16-token x 32-dim key
+      # tiles, 32-token x 16-dim value tiles
+      return {"k": ((G, ring // 16, _up(d, 32) // 32, 64, 8), dtype),
+              "v": ((G, _up(e, 16) // 16, ring // 32, 64, 8), dtype)}
+    return {"k": ((G, ring, d), dtype), "v": ((G, ring, e), dtype)}
+
+  @staticmethod
+  def param_count(dim: int, p: dict) -> int:
+    H, G, d, e = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    return dim * (H * d + G * d + G * e + H + H * e) + H * d + G * d + p["buckets"] * H
+
+  def forward(self, h, proj, at, state, rows, **out):
+    return mo.window_attn(proj, [at[n] for n, _ in self.parts], self.H, self.G, self.dim, self.vdim,
+                          self.q_norm, self.k_norm, self.bucket, self.rel, self.scale, self.eps, self.window,
+                          state, rows, **out)
+
+
+class GatedDeltaRule(nn.Module):
+  """Gated delta rule: short causal convolutions on q, k, v, unit q and k, a
+  decay per head and key channel and an output gate through low-rank pairs,
+  fp32 state [heads, vdim, dim]."""
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__()
+    self.H, self.G, self.dim, self.vdim = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    if self.H % self.G:
+      raise ValueError(f"{self.H} heads do not divide into {self.G} key heads")
+    self.eps = eps
+    H, G, d, e, taps = self.H, self.G, self.dim, self.vdim, p["conv"]
+    self.ranks = (p["decay_rank"], p["gate_rank"])
+    self.parts = [("q", G * d), ("k", G * d), ("v", H * e), ("a1", self.ranks[0]), ("g1", self.ranks[1]), ("b", H)]
+    self.width = H * e
+    self.q_conv = nn.Parameter(torch.zeros(G * d, taps))
+    self.k_conv = nn.Parameter(torch.zeros(G * d, taps))
+    self.v_conv = nn.Parameter(torch.zeros(H * e, taps))
+    self.decay_up = XotLinear(self.ranks[0], H * d, bias=False)
+    self.gate_up = XotLinear(self.ranks[1], H * e, bias=False)
+    self.a_log = nn.Parameter(torch.zeros(H))
+    self.dt_bias = nn.Parameter(torch.zeros(H * d))
+    self.norm = nn.Parameter(torch.ones(e))
+    conv = (-0.5, 0.5)
+    self.init_ranges = {"q_conv": conv, "k_conv": conv, "v_conv": conv, "a_log": (0.0, 1.0),
+                        "dt_bias": (-5.0, -2.0), "norm": (0.8, 1.2)}
+
+  @staticmethod
+  def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> StateSpec:
+    H, G, d, e = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    return {"s": ((H, e, mo.row_pad(d)), torch.float32),
+            # the convolutions' last inputs, position p in row p % taps
+            "conv": ((p["conv"], 2 * G * d + H * e), dtype)}
+
+  @staticmethod
+  def param_count(dim: int, p: dict) -> int:
+    H, G, d, e = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    ra, rg = p["decay_rank"], p["gate_rank"]
+    channels = 2 * G * d + H * e
+    return dim * (channels + ra + rg + H + H * e) + channels * p["conv"] + H * d * (ra + 1) + H * e * rg + H + e
+
+  def forward(self, h, proj, at, state, rows, **out):
+    pre_decay = self.decay_up(proj[..., at["a1"]:at["a1"] + self.ranks[0]])
+    pre_gate = self.gate_up(proj[..., at["g1"]:at["g1"] + self.ranks[1]])
+    return mo.delta_rule(proj, [at[n] for n in ("q", "k", "v", "b")], self.H, self.G, self.dim, self.vdim,
+                         (self.q_conv, self.k_conv, self.v_conv), pre_decay, pre_gate, self.a_log, self.dt_bias,
+                         self.norm, self.eps, state, rows, **out)
+
+
+class BranchMixer(nn.Module):
+  """Branches side by side on one input: weight_0 * branch_0 + ... through a
+  fused input projection and a fused output projection."""
+
+  def __init__(self, dim: int, branches: List[Tuple[str, nn.Module, float]]):
+    super().__init__()
+    self.names = [n for n, _, _ in branches]
+    self.weights = [float(s) for _, _, s in branches]
+    self.branches = nn.ModuleDict({n: b for n, b, _ in branches})
+    # parts start at multiples of 8 (vector loads), the whole at a multiple of
+    # 128 rows (the packed decode GEMM's tile); the gaps are zero weights
+    self.at: Dict[str, Dict[str, int]] = {}
+    n = 0
+    for name, branch, _ in branches:
+      self.at[name] = {}
+      for part, rows in branch.parts:
+        self.at[name][part] = n
+        n = _up(n + rows, 8)
+    self.in_proj = XotLinear(dim, _up(n, 128), bias=False)
+    self.out_at, k = {}, 0
+    for name, branch, _ in branches:
+      self.out_at[name] = k
+      k = _up(k + branch.width, 8)
+    self.out_width = _up(k, 64)
+    self.gapless = self.out_width == sum(b.width for _, b, _ in branches)
+    self.o_proj = XotLinear(self.out_width, dim, bias=False)
+
+  def forward(self, h, state, rows):
+    proj = self.in_proj(h)
+    if proj.is_cuda and not (torch.is_grad_enabled() and proj.requires_grad):
+      # zero columns between branches must hold numbers, not leftovers
+      new = torch.empty if self.gapless else torch.zeros
+      act = new(*proj.shape[:-1], self.out_width, dtype=proj.dtype, device=proj.device)
+      for i, name in enumerate(self.names):
+        self.branches[name](h, proj, self.at[name], state[i], rows,
+                            out=act, out_at=self.out_at[name], out_scale=self.weights[i])
+    else:
+      pieces, n = [], 0
+      for i, name in enumerate(self.names):
+        o = self.branches[name](h, proj, self.at[name], state[i] if state is not None else None, rows,
+                                out_scale=self.weights[i])
+        pieces += [o.new_zeros(*o.shape[:-1], self.out_at[name] - n), o]
+        n = self.out_at[name] + o.shape[-1]
+      pieces.append(proj.new_zeros(*proj.shape[:-1], self.out_width - n))
+      act = torch.cat(pieces, dim=-1)
+    return self.o_proj(act)
+
+
+class ParallelMixer(BranchMixer):
+  """Window attention (left) and a gated delta rule (right) on one input."""
+
+  BRANCHES = (("left", WindowBiasAttention), ("right", GatedDeltaRule))
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__(dim, [(n, c(dim, p[n], eps), p[n + "_scale"]) for n, c in self.BRANCHES])
+
+  @classmethod
+  def state_spec(cls, p: dict, capacity: int, dtype: torch.dtype, device) -> List[StateSpec]:
+    return [c.state_spec(p[n], capacity, dtype, device) for n, c in cls.BRANCHES]
+
+  @classmethod
+  def param_count(cls, dim: int, p: dict) -> int:
+    return sum(c.param_count(dim, p[n]) for n, c in cls.BRANCHES)
+
+  @classmethod
+  def fill_sizes(cls, p: dict, shapes: Dict[str, tuple], prefix: str):
+    """Sizes that only the checkpoint's tensors give."""
+    for n, part, key, name, axis in (("left", "rel", "buckets", "bias rows", 0),
+                                     ("right", "a1", "decay_rank", "decay rank", 0),
+                                     ("right", "g1", "gate_rank", "gate rank", 0)):
+      _fill(p[n], key, shapes, f"{prefix}{n}.{part}", axis, name)
+
+  def key_map(self, src: str, dst: str) -> Dict[str, str]:
+    """Checkpoint tensor -> parameter of this module (models/weights.py)."""
+    m = {}
+    for name in self.names:
+      for part, _ in self.branches[name].parts:
+        m[f"{src}{name}.{part}"] = f"{dst}in_proj.weight@{self.at[name][part]}"
+      m[f"{src}{name}.o"] = f"{dst}o_proj.weight@0,{self.out_at[name]}"
+    left, right = (f"{dst}branches.{n}." for n in ("left", "right"))
+    for theirs, ours in (("q.norm", "q_norm"), ("k.norm", "k_norm"), ("rel", "rel")):
+      m[f"{src}left.{theirs}"] = left + ours
+    for theirs, ours in (("q.conv", "q_conv"), ("k.conv", "k_conv"), ("v.conv", "v_conv"), ("A_log", "a_log"),
+                         ("dt_bias", "dt_bias"), ("norm", "norm"), ("a2", "decay_up.weight"), ("g2", "gate_up.weight")):
+      m[f"{src}right.{theirs}"] = right + ours
+    return m
+
+
+class WKVMixer(nn.Module):
+  """RWKV-style time mixing: every projection reads its own blend of the
+  current and the previous token, a decayed fp32 outer-product memory with a
+  bonus for the current token, an RMS norm per head and a silu gate."""
+
+  MIX = ("r", "k", "v", "g", "w")
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__()
+    self.H, self.dim, self.eps = p["heads"], p["dim"], eps
+    n = self.H * self.dim
+    self.mu = nn.Parameter(torch.zeros(len(self.MIX), dim))
+    for name in ("r", "k", "v", "g"):
+      setattr(self, f"{name}_proj", XotLinear(dim, n, bias=False))
+    self.decay_down = XotLinear(dim, p["decay_rank"], bias=False)
+    self.decay_up = XotLinear(p["decay_rank"], n, bias=False)
+    self.w0 = nn.Parameter(torch.zeros(n))
+    self.u = nn.Parameter(torch.zeros(self.H, self.dim))
+    self.norm = nn.Parameter(torch.ones(n))
+    self.o_proj = XotLinear(n, dim, bias=False)
+    self.init_ranges = {"mu": (0.0, 1.0), "w0": (-6.0, -1.0), "u": (-0.5, 0.5), "norm": (0.8, 1.2)}
+
+  @staticmethod
+  def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> List[StateSpec]:
+    H, d = p["heads"], p["dim"]
+    return [{"s": ((H, d, mo.row_pad(d)), torch.float32), "shift": ((2, p["width"]), dtype)}]
+
+  @staticmethod
+  def param_count(dim: int, p: dict) -> int:
+    n, r = p["heads"] * p["dim"], p["decay_rank"]
+    return 5 * dim * n + r * (dim + n) + 5 * dim + 3 * n
+
+  @staticmethod
+  def fill_sizes(p: dict, shapes: Dict[str, tuple], prefix: str):
+    _fill(p, "decay_rank", shapes, f"{prefix}w1", 0, "decay rank")
+
+  def key_map(self, src: str, dst: str) -> Dict[str, str]:
+    m = {f"{src}mu.{n}": f"{dst}mu@{i}" for i, n in enumerate(self.MIX)}
+    for n in ("r", "k", "v", "g", "o"):
+      m[f"{src}{n}"] = f"{dst}{n}_proj.weight"
+    m[f"{src}w1"], m[f"{src}w2"] = f"{dst}decay_down.weight", f"{dst}decay_up.weight"
+    m[f"{src}w0"], m[f"{src}u"], m[f"{src}norm"] = f"{dst}w0", f"{dst}u", f"{dst}norm"
+    return m
+
+  def forward(self, h, state, rows):
+    S, shift = state[0] if state is not None else (None, None)
+    r, k, v, g, w = mo.token_shift(h, self.mu, shift, rows)
+    pre = self.decay_up(mo.tanh(self.decay_down(w)))
+    o = mo.wkv(self.r_proj(r), self.k_proj(k), self.v_proj(v), self.g_proj(g), pre,
+               self.w0, self.u, self.norm, self.H, self.dim, self.eps, S, rows)
+    return self.o_proj(o)
+
+
+def _fill(p: dict, key: str, shapes: Dict[str, tuple], tensor: str, axis: int, what: str):
+  if tensor in shapes:
+    p[key] = shapes[tensor][axis]
+  elif key not in p:
+    raise ValueError(f"no tensor {tensor} and no '{key}' in the configuration: {what} unknown")
+
+
+MIXERS = {"parallel": ParallelMixer, "wkv": WKVMixer}

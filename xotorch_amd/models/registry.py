@@ -120,6 +120,29 @@ def _mixtral_cfg(dim, n_layers, n_heads, n_kv, inter, n_experts=8, top_k=2):
   }
 
 
+def _didipel_cfg(width, order, ff, vocab, left, right, wkv, left_scale=1.0, right_scale=1.0, eps=1e-6):
+  """order: one letter a layer, p(arallel) or w(kv). Sizes that a checkpoint's
+  tensors give (bias rows, low ranks) are spelled out here."""
+  parallel = {"left": left, "right": right, "left_scale": left_scale, "right_scale": right_scale}
+  kinds = {"p": ("parallel", parallel), "w": ("wkv", wkv)}
+  return {
+    "architecture": "Didipel", "vocab": vocab, "width": width, "norm": {"eps": eps},
+    "layers": [{"type": kinds[c][0], "mixer": kinds[c][1], "mlp": {"kind": "dense", "ff": ff}} for c in order],
+  }
+
+
+def _didipel_sized(width, order, ff, vocab, dim=128, kv_heads=4, window=1024, rank=128):
+  """Real-model proportions: both branches and the wkv heads span the width."""
+  heads = width // dim
+  return _didipel_cfg(
+    width, order, ff, vocab,
+    left={"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+          "bias_max": 1024, "buckets": 32, "mask": {"size": window}},
+    right={"heads": heads, "kv_heads": heads, "dim": dim, "vdim": dim, "conv": 4,
+           "decay_rank": rank, "gate_rank": rank},
+    wkv={"heads": heads, "dim": dim, "decay_rank": rank}, left_scale=0.7, right_scale=0.7)
+
+
 BUILTIN_CONFIGS: Dict[str, dict] = {
   # llama 3.x family
   "llama-3.2-1b": _llama_cfg(2048, 16, 32, 8, 8192, tie=True, llama3_scaling=True, head_dim=64),
@@ -193,6 +216,16 @@ BUILTIN_CONFIGS: Dict[str, dict] = {
   "phi-4-mini": _llama_cfg(3072, 32, 24, 8, 8192, vocab=200064, theta=10000.0, max_pos=131072, tie=True),
   "phi-4-mini-instruct": _llama_cfg(3072, 32, 24, 8, 8192, vocab=200064, theta=10000.0, max_pos=131072, tie=True),
   # tiny test model
+  # didipel (no published checkpoints: sizes like a 1B and a 7B model, and a
+  # tiny one whose sizes all differ)
+  "didipel-1b": _didipel_sized(2048, "pppwppp" * 2 + "pw", 5632, 32000),
+  "didipel-7b": _didipel_sized(4096, "pppwppp" * 3 + "pwp", 11008, 32000, kv_heads=8),
+  "didipel-dummy": _didipel_cfg(
+    96, "pwp", 160, 256,
+    left={"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 16, "scale": 0.2, "bias_max": 20, "buckets": 8,
+          "mask": {"size": 12}},
+    right={"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "conv": 4, "decay_rank": 8, "gate_rank": 12},
+    wkv={"heads": 3, "dim": 32, "decay_rank": 8}, left_scale=0.8, right_scale=0.6),
   "dummy": _llama_cfg(64, 4, 4, 2, 128, vocab=256, theta=10000.0, max_pos=256, tie=True),
 }
 # DeepSeek-Coder-V2-Lite shares the V2-Lite architecture exactly
@@ -256,6 +289,9 @@ model_cards: Dict[str, dict] = {
   # llava needs PIL for the image path (not present in this environment);
   # the reference's vision handling is also vestigial
   "llava-1.5-7b-hf": {"layers": 32, "repo": {}},
+  "didipel-1b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "didipel-7b": {"layers": 24, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "didipel-dummy": {"layers": 3, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "dummy": {"layers": 4, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy", "DummyEngine": "dummy"}},
 }
 
@@ -306,6 +342,9 @@ pretty_names = {
   "deepseek-v3": "DeepSeek V3",
   "llava-1.5-7b-hf": "LLaVa 1.5 7B (unsupported arch)",
   "phi-4-mini": "Phi-4 Mini",
+  "didipel-1b": "Didipel 1B (random weights)",
+  "didipel-7b": "Didipel 7B (random weights)",
+  "didipel-dummy": "Didipel dummy (test)",
   "dummy": "Dummy (test)",
 }
 
@@ -347,6 +386,16 @@ def get_supported_models(supported_engine_lists: Optional[List[List[str]]] = Non
     if all(any(e in repos for e in engines) for engines in supported_engine_lists):
       out.append(model_id)
   return out
+
+
+def register_local_model(model_id: str, model_dir) -> None:
+  """Make a checkpoint folder (config.json + safetensors) available under
+  `model_id`, as if it had a card; the folder's config gives the layers."""
+  from pathlib import Path
+  from xotorch_amd.models.config import config_from_hf
+  n_layers = config_from_hf(Path(model_dir) / "config.json", model_id).n_layers
+  local = str(model_dir)
+  model_cards[model_id] = {"layers": n_layers, "repo": {"TorchEngine": local, "HIPEngine": local}}
 
 
 def builtin_config(model_id: str) -> Optional[dict]:

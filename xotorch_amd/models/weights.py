@@ -16,6 +16,7 @@ import torch
 
 from xotorch_amd.models.config import ModelConfig
 from xotorch_amd.models.llama import ShardedModel, hf_key_map as _hf_key_map_llama
+from xotorch_amd.shard import Shard
 
 
 def hf_key_map(shard, cfg):
@@ -27,8 +28,10 @@ def hf_key_map(shard, cfg):
   if mtype in ("deepseek_v3", "deepseek_v2"):
     from xotorch_amd.models.deepseek_v3 import hf_key_map_deepseek
     return hf_key_map_deepseek(shard, cfg)
+  if mtype == "didipel":
+    from xotorch_amd.models.didipel import key_map_didipel
+    return key_map_didipel(shard, cfg)
   return _hf_key_map_llama(shard, cfg)
-from xotorch_amd.shard import Shard
 
 
 def shard_file_set(model_dir: Path, shard: Shard, cfg: ModelConfig) -> Optional[Dict[str, list]]:
@@ -60,23 +63,17 @@ def load_shard_weights(model: ShardedModel, model_dir: Path, device: str = "cpu"
   files = shard_file_set(model_dir, shard, cfg)
   if files is None:
     raise FileNotFoundError(f"no safetensors found under {model_dir}")
-  state: Dict[str, torch.Tensor] = {}
-  packed: Dict[str, Dict[int, torch.Tensor]] = {}
+  tensors: Dict[str, torch.Tensor] = {}
   for fn, keys in files.items():
     with safe_open(str(model_dir / fn), framework="pt", device=device) as f:
       names = set(f.keys())
       for hf_key in keys:
-        if hf_key not in names:
-          continue
-        our = mapping[hf_key]
-        if "#" in our:
-          base, part = our.split("#")
-          packed.setdefault(base, {})[int(part)] = f.get_tensor(hf_key)
-        else:
-          state[our] = f.get_tensor(hf_key)
-  # fused qkv_proj / gate_up_proj: concatenate the HF fragments along dim 0
-  for base, parts in packed.items():
-    state[base] = torch.cat([parts[i] for i in sorted(parts)], dim=0)
+        if hf_key in names:
+          tensors[hf_key] = f.get_tensor(hf_key)
+  placed_missing = [k for k, our in mapping.items() if "@" in our and k not in tensors]
+  if placed_missing:
+    raise RuntimeError(f"missing weights for shard {shard}: {placed_missing[:8]}")
+  state = remap_hf_state(tensors, mapping, {n: p.shape for n, p in model.named_parameters()})
   missing, unexpected = model.load_state_dict(state, strict=False)
   # tied-embedding models ship no lm_head tensor; rope buffers are computed
   real_missing = [m for m in missing if not m.startswith("rope_")]
@@ -91,10 +88,14 @@ def load_shard_weights(model: ShardedModel, model_dir: Path, device: str = "cpu"
   return len(state)
 
 
-def remap_hf_state(sd: Dict[str, torch.Tensor], mapping: Dict[str, str]) -> Dict[str, torch.Tensor]:
-  """Apply an hf_key_map to an in-memory HF state dict: rename keys and
-  concatenate `key#N` fused parts along dim 0 in N order (same semantics as
-  load_shard_weights' safetensors path; used by tests and converters)."""
+def remap_hf_state(sd: Dict[str, torch.Tensor], mapping: Dict[str, str],
+                   shapes: Optional[Dict[str, tuple]] = None) -> Dict[str, torch.Tensor]:
+  """Apply an hf_key_map to an in-memory HF state dict (shared by the
+  safetensors path, tests and converters). Three forms of target:
+  `key` renames; `key#N` parts are concatenated along dim 0 in N order;
+  `key@row` / `key@row,col` parts are placed at an offset of the parameter
+  `key`, whose shape comes from `shapes`, with zeros where nothing is placed
+  (fused projections with aligned or padded parts)."""
   state: Dict[str, torch.Tensor] = {}
   packed: Dict[str, Dict[int, torch.Tensor]] = {}
   for hf_key, our in mapping.items():
@@ -103,11 +104,29 @@ def remap_hf_state(sd: Dict[str, torch.Tensor], mapping: Dict[str, str]) -> Dict
     if "#" in our:
       base, part = our.split("#")
       packed.setdefault(base, {})[int(part)] = sd[hf_key]
+    elif "@" in our:
+      base, offset = our.split("@")
+      t = sd[hf_key]
+      if base not in state:
+        state[base] = torch.zeros(shapes[base], dtype=t.dtype, device=t.device)
+      t = t.reshape((1,) * (state[base].dim() - t.dim()) + tuple(t.shape))
+      at = [int(o) for o in offset.split(",")]
+      at += [0] * (t.dim() - len(at))
+      if any(o + n > m for o, n, m in zip(at, t.shape, state[base].shape)):
+        raise RuntimeError(f"{hf_key} {tuple(t.shape)} does not fit {base} {tuple(state[base].shape)} at {at}")
+      state[base][tuple(slice(o, o + n) for o, n in zip(at, t.shape))] = t
     else:
       state[our] = sd[hf_key]
   for base, parts in packed.items():
     state[base] = torch.cat([parts[i] for i in sorted(parts)], dim=0)
   return state
+
+
+def _init_ranges(model) -> Dict[str, tuple]:
+  """Parameters that only make sense in a range of their own (decays, mixing
+  weights, norms of mixers): modules list them in `init_ranges`."""
+  return {f"{mod}.{p}" if mod else p: r for mod, m in model.named_modules()
+          for p, r in getattr(m, "init_ranges", {}).items()}
 
 
 @torch.no_grad()
@@ -119,6 +138,7 @@ def random_init(model: ShardedModel, seed: int = 1234, std: float = 0.02) -> Non
   logits-equality oracle depends on this).
   """
   import zlib
+  ranges = _init_ranges(model)
   for name, p in model.named_parameters():
     # a tied-embedding last shard without the embedding holds a COPY of the
     # embedding matrix as its head: seed it as the embedding so split == full
@@ -131,6 +151,8 @@ def random_init(model: ShardedModel, seed: int = 1234, std: float = 0.02) -> Non
     cpu_t = torch.empty(p.shape, dtype=torch.float32)
     if name.endswith("layernorm.weight") or name.endswith("norm.weight"):
       cpu_t.fill_(1.0)
+    elif name in ranges:
+      cpu_t.uniform_(*ranges[name], generator=g)
     elif name.endswith(".bias"):
       cpu_t.zero_()
     else:
@@ -145,9 +167,12 @@ def fast_random_init_gpu(model: ShardedModel, seed: int = 1234, std: float = 0.0
   affect decode throughput, only shapes do."""
   g = torch.Generator(device="cuda")
   g.manual_seed(seed)
+  ranges = _init_ranges(model)
   for name, p in model.named_parameters():
     if name.endswith("norm.weight"):
       p.fill_(1.0)
+    elif name in ranges:
+      p.copy_(torch.empty(p.shape, dtype=torch.float32, device=p.device).uniform_(*ranges[name], generator=g))
     elif name.endswith(".bias"):
       p.zero_()
     else:

@@ -1,53 +1,75 @@
-"""In-tree build of the CDNA4 HIP extension (no network, no JIT cache).
+"""In-tree build of the CDNA4 HIP extensions (no network, no JIT cache).
 
-Invoked by __graft_entry__.build(). Compiles xotorch_amd/ops/hip/hip_ops.hip
-with hipcc --offload-arch=gfx950 into xotorch_amd/ops/_hip_ops.so so the
-built artifact travels with the repo snapshot to the GPU box.
+Invoked by __graft_entry__.build(). Every hip/*.hip translation unit becomes
+one extension next to this file, compiled with hipcc --offload-arch=gfx950,
+so the built artifacts travel with the repo snapshot to the GPU box. The
+compiler runs are independent and go in parallel.
 """
 from __future__ import annotations
 
+import os
 import subprocess
 import sys
 import sysconfig
 from pathlib import Path
+from typing import List
 
 PKG_DIR = Path(__file__).resolve().parent
-SRC = PKG_DIR / "hip" / "hip_ops.hip"
-OUT = PKG_DIR / "_hip_ops.so"
+# extension module -> its source
+EXTENSIONS = {
+  "_hip_ops": PKG_DIR / "hip" / "hip_ops.hip",
+  "_hip_mixers": PKG_DIR / "hip" / "mixer_ops.hip",
+}
 
 
-def _torch_paths():
+def out_path(name: str) -> Path:
+  return PKG_DIR / f"{name}.so"
+
+
+def needs_build(name: str) -> bool:
+  out = out_path(name)
+  return not out.exists() or EXTENSIONS[name].stat().st_mtime > out.stat().st_mtime
+
+
+def _command(name: str, out: Path) -> List[str]:
   import torch
   from torch.utils import cpp_extension
-  return cpp_extension.include_paths(), cpp_extension.library_paths(), torch._C._GLIBCXX_USE_CXX11_ABI
-
-
-def needs_build() -> bool:
-  if not OUT.exists():
-    return True
-  return SRC.stat().st_mtime > OUT.stat().st_mtime
-
-
-def build(force: bool = False, verbose: bool = True) -> Path:
-  if not force and not needs_build():
-    return OUT
-  includes, libpaths, abi = _torch_paths()
-  py_inc = sysconfig.get_paths()["include"]
+  abi = 1 if torch._C._GLIBCXX_USE_CXX11_ABI else 0
   cmd = [
     "hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared",
-    f"-DTORCH_EXTENSION_NAME=_hip_ops", "-DTORCH_API_INCLUDE_EXTENSION_H",
-    f"-D_GLIBCXX_USE_CXX11_ABI={1 if abi else 0}", "-DUSE_ROCM", "-D__HIP_PLATFORM_AMD__",
+    # packed fp32 instructions stay off: plain fp32 code must not turn into them
+    "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
+    f"-DTORCH_EXTENSION_NAME={name}", "-DTORCH_API_INCLUDE_EXTENSION_H",
+    f"-D_GLIBCXX_USE_CXX11_ABI={abi}", "-DUSE_ROCM", "-D__HIP_PLATFORM_AMD__",
   ]
-  for inc in includes:
+  for inc in [*cpp_extension.include_paths(), sysconfig.get_paths()["include"]]:
     cmd += ["-I", inc]
-  cmd += ["-I", py_inc, str(SRC), "-o", str(OUT)]
-  for lp in libpaths:
+  cmd += [str(EXTENSIONS[name]), "-o", str(out)]
+  for lp in cpp_extension.library_paths():
     cmd += ["-L", lp]
-  cmd += ["-ltorch", "-ltorch_hip", "-lc10", "-lc10_hip", "-ltorch_python"]
-  if verbose:
-    print("[xotorch_amd] building HIP extension:", " ".join(cmd), file=sys.stderr)
-  subprocess.run(cmd, check=True)
-  return OUT
+  return cmd + ["-ltorch", "-ltorch_hip", "-lc10", "-lc10_hip", "-ltorch_python"]
+
+
+def build(force: bool = False, verbose: bool = True, missing_only: bool = False) -> List[Path]:
+  """Compile the extensions that are missing or older than their source;
+  `force` compiles all, `missing_only` trusts what is built already."""
+  names = [n for n in EXTENSIONS if force or (not out_path(n).exists() if missing_only else needs_build(n))]
+  jobs = []
+  for n in names:
+    # compile beside the target and move into place: a concurrent reader sees
+    # the old library or the new one, never half of one
+    tmp = out_path(n).with_suffix(f".so.tmp{os.getpid()}")
+    cmd = _command(n, tmp)
+    if verbose:
+      print(f"[xotorch_amd] building {n}:", " ".join(cmd), file=sys.stderr)
+    jobs.append((n, tmp, cmd, subprocess.Popen(cmd)))
+  for n, tmp, cmd, proc in jobs:
+    proc.wait()
+  for n, tmp, cmd, proc in jobs:
+    if proc.returncode:
+      raise subprocess.CalledProcessError(proc.returncode, cmd)
+    os.replace(tmp, out_path(n))
+  return [out_path(n) for n in names]
 
 
 if __name__ == "__main__":

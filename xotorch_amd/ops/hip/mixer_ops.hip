@@ -1,0 +1,1438 @@
+// CDNA4 (gfx950) kernels of the token mixers in models/mixers.py, and of the
+// norms around an fp32 residual stream:
+//   - sandwich norm: stream += norm(sublayer output), then the stream's norm
+//     for the next sublayer, one pass
+//   - sliding-window attention with a learned distance bias, a zero-score sink
+//     and per-head gates: q/k norm + cache append, flash prefill, split decode
+//   - gated delta rule and WKV recurrences: input preparation (short
+//     convolutions, unit norms, decays), a register-resident scan for prompts,
+//     one fused kernel per decode step
+//
+// Two element types: bf16 (MFMA attention over fragment-packed keys and
+// values) and fp32 (plain layouts, plain fp32 arithmetic). Recurrent state,
+// scores, softmax, norms and everything that feeds a recurrence after its
+// projections are fp32 in both.
+//
+// Rows of a step address state by slot (struct Step): slot -1 is a parked row,
+// which reads and writes no state and yields zeros. A row at position 0
+// ignores what its slot holds.
+
+#include <torch/extension.h>
+#include <c10/hip/HIPStream.h>
+#include <hip/hip_runtime.h>
+#include <hip/hip_bf16.h>
+
+#include <algorithm>
+
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) float floatx4;
+typedef __attribute__((ext_vector_type(4))) unsigned short ushort4_t;
+typedef unsigned short bf16_t;
+
+#define DEVINL __device__ __forceinline__
+
+DEVINL float ld(const bf16_t* p) {
+  union { float f; unsigned int i; } v;
+  v.i = ((unsigned int)*p) << 16;
+  return v.f;
+}
+DEVINL float ld(const float* p) { return *p; }
+DEVINL bf16_t f2b(float f) {
+  __hip_bfloat16 h = __float2bfloat16(f);  // round to nearest even
+  return *reinterpret_cast<bf16_t*>(&h);
+}
+DEVINL void st(bf16_t* p, float f) { *p = f2b(f); }
+DEVINL void st(float* p, float f) { *p = f; }
+// the value as the element type holds it
+DEVINL float rounded(float f, const bf16_t*) { bf16_t b = f2b(f); return ld(&b); }
+DEVINL float rounded(float f, const float*) { return f; }
+
+DEVINL void ld4(const float* p, float* o) {
+  const floatx4 v = *(const floatx4*)p;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) o[i] = v[i];
+}
+DEVINL void ld4(const bf16_t* p, float* o) {
+  const ushort4_t v = *(const ushort4_t*)p;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) { bf16_t u = v[i]; o[i] = ld(&u); }
+}
+DEVINL void st4(float* p, const float* o) {
+  floatx4 v;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = o[i];
+  *(floatx4*)p = v;
+}
+DEVINL void st4(bf16_t* p, const float* o) {
+  ushort4_t v;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = f2b(o[i]);
+  *(ushort4_t*)p = v;
+}
+template <int V, typename T>
+DEVINL void ldv(const T* p, float* o) {
+  if (V == 4) ld4(p, o);
+  else
+#pragma unroll
+    for (int i = 0; i < V; ++i) o[i] = ld(p + i);
+}
+template <int V, typename T>
+DEVINL void stv(T* p, const float* o) {
+  if (V == 4) st4(p, o);
+  else
+#pragma unroll
+    for (int i = 0; i < V; ++i) st(p + i, o[i]);
+}
+
+DEVINL float sigmoidf(float x) { return 1.f / (1.f + expf(-x)); }
+DEVINL float siluf(float x) { return x / (1.f + expf(-x)); }
+DEVINL float softplusf(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+DEVINL float wave_sum(float v) {
+#pragma unroll
+  for (int m = 32; m > 0; m >>= 1) v += __shfl_xor(v, m);
+  return v;
+}
+// sum over a block of 256 threads; `red` holds 4 floats and is free again
+// after the next barrier
+DEVINL float block_sum(float v, float* red) {
+  v = wave_sum(v);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return red[0] + red[1] + red[2] + red[3];
+}
+
+struct Step {
+  const int* slots;      // null: row b is slot b
+  const int* positions;  // decode only
+  const int* lens;       // prefill only; null: every row brings S tokens
+  int npos, start, decode;
+  DEVINL int slot(int b) const { return slots ? slots[b] : b; }
+  DEVINL int first(int b) const { return decode ? positions[npos > 1 ? b : 0] : start; }
+  DEVINL int len(int b, int S) const { return lens ? min(lens[b], S) : S; }
+};
+
+// ---------------------------------------------------------------------------
+// norms around the fp32 stream
+// ---------------------------------------------------------------------------
+
+// y null: h = norm(x; w_next) only. One block per row; the row stays in
+// registers (NC chunks of 256*V elements).
+template <typename T, int V, int NC>
+__global__ __launch_bounds__(256) void sandwich_norm_kernel(
+    const T* __restrict__ y, float* __restrict__ x, const T* __restrict__ w_post,
+    const T* __restrict__ w_next, T* __restrict__ h, int D, float eps) {
+  const size_t off = (size_t)blockIdx.x * D;
+  __shared__ float red[8];
+  float xv[NC * V];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = (c * 256 + threadIdx.x) * V;
+    if (i < D) ldv<V>(x + off + i, xv + c * V);
+    else
+#pragma unroll
+      for (int j = 0; j < V; ++j) xv[c * V + j] = 0.f;
+  }
+  if (y) {
+    float yv[NC * V], acc = 0.f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int i = (c * 256 + threadIdx.x) * V;
+      if (i < D) {
+        ldv<V>(y + off + i, yv + c * V);
+#pragma unroll
+        for (int j = 0; j < V; ++j) acc += yv[c * V + j] * yv[c * V + j];
+      }
+    }
+    const float inv = 1.f / sqrtf(block_sum(acc, red) / (float)D + eps);
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int i = (c * 256 + threadIdx.x) * V;
+      if (i < D) {
+        float w[V];
+        ldv<V>(w_post + i, w);
+#pragma unroll
+        for (int j = 0; j < V; ++j) xv[c * V + j] += yv[c * V + j] * inv * (1.f + w[j]);
+        stv<V>(x + off + i, xv + c * V);
+      }
+    }
+  }
+  if (!w_next) return;
+  float acc = 0.f;
+#pragma unroll
+  for (int i = 0; i < NC * V; ++i) acc += xv[i] * xv[i];
+  const float inv = 1.f / sqrtf(block_sum(acc, red + 4) / (float)D + eps);
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int i = (c * 256 + threadIdx.x) * V;
+    if (i < D) {
+      float w[V], o[V];
+      ldv<V>(w_next + i, w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) o[j] = xv[c * V + j] * inv * (1.f + w[j]);
+      stv<V>(h + off + i, o);
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------
+// elementwise
+// ---------------------------------------------------------------------------
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, long long n, int I) {
+  const long long i = ((long long)blockIdx.x * 256 + threadIdx.x) * V;
+  if (i >= n) return;
+  const long long row = i / I;
+  const int c = (int)(i - row * I);
+  float g[V], u[V];
+  ldv<V>(gu + row * 2 * I + c, g);
+  ldv<V>(gu + row * 2 * I + I + c, u);
+#pragma unroll
+  for (int j = 0; j < V; ++j) u[j] *= siluf(g[j]);
+  stv<V>(out + i, u);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void tanh_kernel(const T* __restrict__ x, T* __restrict__ out, long long n) {
+  const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) st(out + i, tanhf(ld(x + i)));
+}
+
+// ---------------------------------------------------------------------------
+// window attention: cache layouts
+//   bf16, fragment-packed per (slot, kv head):
+//     K [rows/16][KC][64 lanes][8]: lane = (d%32)/8*16 + row%16
+//     V [VG][rows/32][64 lanes][8]: lane = (row%16)/4*16 + c%16,
+//       element = (row%32)/16*4 + row%4
+//     Scores are computed transposed (keys x queries), so the lane that holds
+//     a query's probabilities for keys {4g..4g+3, 16+4g..16+4g+3} feeds them
+//     straight into the second MFMA; V's element order follows that.
+//   fp32: plain rows.
+// ---------------------------------------------------------------------------
+
+struct KVShape { int dim, vdim, kc, vg, rows; };
+
+template <typename T> struct Layout;
+template <> struct Layout<bf16_t> {
+  static DEVINL size_t kbase(const KVShape& s, size_t head) { return head * (size_t)(s.rows >> 4) * s.kc * 512; }
+  static DEVINL size_t vbase(const KVShape& s, size_t head) { return head * (size_t)s.vg * (s.rows >> 5) * 512; }
+  static DEVINL size_t k(const KVShape& s, int row, int d) {
+    return (((size_t)(row >> 4) * s.kc + (d >> 5)) * 64 + ((d & 31) >> 3) * 16 + (row & 15)) * 8 + (d & 7);
+  }
+  static DEVINL size_t v(const KVShape& s, int row, int c) {
+    return (((size_t)(c >> 4) * (s.rows >> 5) + (row >> 5)) * 64 + ((row & 15) >> 2) * 16 + (c & 15)) * 8 +
+           ((row & 31) >> 4) * 4 + (row & 3);
+  }
+};
+template <> struct Layout<float> {
+  static DEVINL size_t kbase(const KVShape& s, size_t head) { return head * s.rows * (size_t)s.dim; }
+  static DEVINL size_t vbase(const KVShape& s, size_t head) { return head * s.rows * (size_t)s.vdim; }
+  static DEVINL size_t k(const KVShape& s, int row, int d) { return (size_t)row * s.dim + d; }
+  static DEVINL size_t v(const KVShape& s, int row, int c) { return (size_t)row * s.vdim + c; }
+};
+
+struct AttnArgs {
+  int S, H, G, N, K;                    // tokens a row, heads, projection and output widths
+  int q_at, k_at, v_at, g_at, out_at;
+  int qd;                               // padded dims of the q workspace
+  float scale, eps, out_scale;
+  int window, nb;                       // nb: entries of the distance table
+};
+
+// Keys of the window before a chunk, ring -> workspace rows [0, hist).
+template <typename T>
+__global__ __launch_bounds__(256) void window_history_kernel(
+    const T* __restrict__ kc, const T* __restrict__ vc, T* __restrict__ kw, T* __restrict__ vw,
+    KVShape ring, KVShape ws, int G, int base, int hist, Step step) {
+  const int row = blockIdx.x, g = blockIdx.y, b = blockIdx.z;
+  const int slot = step.slot(b);
+  const int src = (base + row) % ring.rows;
+  typedef Layout<T> L;
+  const size_t kr = L::kbase(ring, (size_t)max(slot, 0) * G + g), vr = L::vbase(ring, (size_t)max(slot, 0) * G + g);
+  const size_t kd = L::kbase(ws, (size_t)b * G + g), vd = L::vbase(ws, (size_t)b * G + g);
+  const int kdims = sizeof(T) == 2 ? ws.kc * 32 : ws.dim, vdims = sizeof(T) == 2 ? ws.vg * 16 : ws.vdim;
+  for (int d = threadIdx.x; d < kdims + vdims; d += 256) {
+    if (d < kdims) kw[kd + L::k(ws, row, d)] = slot < 0 ? (T)0 : kc[kr + L::k(ring, src, d)];
+    else vw[vd + L::v(ws, row, d - kdims)] = slot < 0 ? (T)0 : vc[vr + L::v(ring, src, d - kdims)];
+  }
+}
+
+// One block per token: RMS norm over the whole q and k projections, q to the
+// workspace [B,S,H,qd] (zero-padded dims), k and v into the ring (the last
+// ring.rows tokens of the chunk) and, in prefill, into the workspace at rows
+// hist+s. Blocks past S fill the workspace's last tile with zeros.
+template <typename T>
+__global__ __launch_bounds__(256) void qk_norm_append_kernel(
+    const T* __restrict__ proj, const T* __restrict__ qn, const T* __restrict__ kn, T* __restrict__ qw,
+    T* __restrict__ kc, T* __restrict__ vc, T* __restrict__ kw, T* __restrict__ vw,
+    KVShape ring, KVShape ws, int hist, AttnArgs a, Step step) {
+  const int s = blockIdx.x, b = blockIdx.y;
+  const int slot = step.slot(b), len = step.decode ? 1 : step.len(b, a.S);
+  typedef Layout<T> L;
+  const bool live = s < len && slot >= 0;
+  const int kdims = sizeof(T) == 2 ? ws.kc * 32 : ws.dim, vdims = sizeof(T) == 2 ? ws.vg * 16 : ws.vdim;
+  if (!live) {
+    if (s < a.S)
+      for (int i = threadIdx.x; i < a.H * a.qd; i += 256) st(qw + ((size_t)b * a.S + s) * a.H * a.qd + i, 0.f);
+    if (kw)
+      for (int g = 0; g < a.G; ++g) {
+        const size_t kd = L::kbase(ws, (size_t)b * a.G + g), vd = L::vbase(ws, (size_t)b * a.G + g);
+        for (int d = threadIdx.x; d < kdims + vdims; d += 256) {
+          if (d < kdims) st(kw + kd + L::k(ws, hist + s, d), 0.f);
+          else st(vw + vd + L::v(ws, hist + s, d - kdims), 0.f);
+        }
+      }
+    return;
+  }
+  const T* row = proj + ((size_t)b * a.S + s) * a.N;
+  __shared__ float red[8];
+  float qs = 0.f, ks = 0.f;
+  for (int i = threadIdx.x; i < a.H * ring.dim; i += 256) { const float f = ld(row + a.q_at + i); qs += f * f; }
+  for (int i = threadIdx.x; i < a.G * ring.dim; i += 256) { const float f = ld(row + a.k_at + i); ks += f * f; }
+  const float qi = 1.f / sqrtf(block_sum(qs, red) / (float)(a.H * ring.dim) + a.eps);
+  const float ki = 1.f / sqrtf(block_sum(ks, red + 4) / (float)(a.G * ring.dim) + a.eps);
+  T* qrow = qw + ((size_t)b * a.S + s) * a.H * a.qd;
+  for (int i = threadIdx.x; i < a.H * a.qd; i += 256) {
+    const int h = i / a.qd, d = i - h * a.qd;
+    const int j = h * ring.dim + d;
+    st(qrow + i, d < ring.dim ? ld(row + a.q_at + j) * qi * ld(qn + j) : 0.f);
+  }
+  const int pos = step.first(b) + s;
+  const bool keep = s >= len - ring.rows;
+  const int rrow = pos % ring.rows;
+  for (int i = threadIdx.x; i < a.G * (kdims + vdims); i += 256) {
+    const int g = i / (kdims + vdims), d = i - g * (kdims + vdims);
+    const size_t rh = (size_t)slot * a.G + g, wh = (size_t)b * a.G + g;
+    if (d < kdims) {
+      const int j = g * ring.dim + d;
+      const float f = d < ring.dim ? ld(row + a.k_at + j) * ki * ld(kn + j) : 0.f;
+      if (keep) st(kc + L::kbase(ring, rh) + L::k(ring, rrow, d), f);
+      if (kw) st(kw + L::kbase(ws, wh) + L::k(ws, hist + s, d), f);
+    } else {
+      const int c = d - kdims;
+      const float f = c < ring.vdim ? ld(row + a.v_at + g * ring.vdim + c) : 0.f;
+      if (keep) st(vc + L::vbase(ring, rh) + L::v(ring, rrow, c), f);
+      if (kw) st(vw + L::vbase(ws, wh) + L::v(ws, hist + s, c), f);
+    }
+  }
+}
+
+// Flash prefill on matrix cores: a wave owns 32 queries of one head and walks
+// the key tiles that their windows touch. EXACT: kc == KC and vg == VG.
+template <int KC, int VG, bool EXACT>
+__global__ __launch_bounds__(256) void attn_window_prefill_kernel(
+    const bf16_t* __restrict__ qw, const bf16_t* __restrict__ kw, const bf16_t* __restrict__ vw,
+    const bf16_t* __restrict__ proj, const int* __restrict__ bucket, const bf16_t* __restrict__ rel,
+    bf16_t* __restrict__ out, KVShape ws, int hist, AttnArgs a, Step step) {
+  extern __shared__ float bias[];  // [nb], this head's bias per distance
+  const int h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G);
+  const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
+  for (int i = threadIdx.x; i < a.nb; i += 256) bias[i] = ld(rel + bucket[i] * a.H + h);
+  __syncthreads();
+  const int s0 = blockIdx.x * 128 + (threadIdx.x >> 6) * 32;
+  if (s0 >= a.S) return;
+  const int kc = EXACT ? KC : ws.kc, vg = EXACT ? VG : ws.vg;
+  bf16x8 qf[2][KC];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const int s = min(s0 + t * 16 + col, a.S - 1);
+    const bf16_t* q = qw + (((size_t)b * a.S + s) * a.H + h) * a.qd + quad * 8;
+#pragma unroll
+    for (int c = 0; c < KC; ++c)
+      if (EXACT || c < kc) qf[t][c] = *(const bf16x8*)(q + c * 32);
+  }
+  float m[2] = {0.f, 0.f}, l[2] = {0.f, 0.f};  // the sink's score bounds the maximum from below
+  floatx4 o[2][VG];
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < VG; ++i) o[t][i] = (floatx4)(0.f);
+  const bf16_t* kb = kw + Layout<bf16_t>::kbase(ws, (size_t)b * a.G + g);
+  const bf16_t* vb = vw + Layout<bf16_t>::vbase(ws, (size_t)b * a.G + g);
+  const int vstride = (ws.rows >> 5) * 512;
+  const int t0 = max(0, hist + s0 - (a.window - 1)) >> 5;
+  const int t1 = (hist + min(s0 + 31, a.S - 1)) >> 5;
+  for (int tile = t0; tile <= t1; ++tile) {
+    floatx4 sc[2][2];
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
+      sc[0][hf] = (floatx4)(0.f);
+      sc[1][hf] = (floatx4)(0.f);
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+        if (EXACT || c < kc) {
+          const bf16x8 kf = *(const bf16x8*)(kb + ((size_t)(tile * 2 + hf) * kc + c) * 512 + lane * 8);
+          sc[0][hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[0][c], sc[0][hf], 0, 0, 0);
+          sc[1][hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[1][c], sc[1][hf], 0, 0, 0);
+        }
+    }
+    bf16x8 pf[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      // distance to this lane's first key of the tile
+      const int dist0 = hist + s0 + t * 16 + col - tile * 32 - quad * 4;
+      float top = m[t];
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int dist = dist0 - hf * 16 - r;
+          const float v = sc[t][hf][r] * a.scale + bias[min(max(dist, 0), a.nb - 1)];
+          sc[t][hf][r] = (dist >= 0 && dist < a.window) ? v : -INFINITY;
+          top = fmaxf(top, sc[t][hf][r]);
+        }
+      top = fmaxf(top, __shfl_xor(top, 16));
+      top = fmaxf(top, __shfl_xor(top, 32));
+      if (__any(top > m[t])) {
+        const float al = __expf(m[t] - top);
+        m[t] = top;
+        l[t] *= al;
+#pragma unroll
+        for (int i = 0; i < VG; ++i) o[t][i] *= al;
+      }
+      float sum = 0.f;
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float p = __expf(sc[t][hf][r] - top);
+          sum += p;
+          pf[t][hf * 4 + r] = (__bf16)p;
+        }
+      l[t] += sum;
+    }
+#pragma unroll
+    for (int i = 0; i < VG; ++i)
+      if (EXACT || i < vg) {
+        const bf16x8 vf = *(const bf16x8*)(vb + (size_t)i * vstride + (size_t)tile * 512 + lane * 8);
+        o[0][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[0], o[0][i], 0, 0, 0);
+        o[1][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[1], o[1][i], 0, 0, 0);
+      }
+  }
+  const int len = step.slot(b) < 0 ? 0 : step.len(b, a.S);
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const int s = s0 + t * 16 + col;
+    float sum = l[t];
+    sum += __shfl_xor(sum, 16);
+    sum += __shfl_xor(sum, 32);
+    if (s >= a.S) continue;
+    const size_t tok = (size_t)b * a.S + s;
+    float f = 0.f;
+    if (s < len) f = a.out_scale * sigmoidf(ld(proj + tok * a.N + a.g_at + h)) / (sum + __expf(-m[t]));
+    bf16_t* dst = out + tok * a.K + a.out_at + h * ws.vdim;
+#pragma unroll
+    for (int i = 0; i < VG; ++i) {
+      const int c = i * 16 + quad * 4;
+      if (c + 3 < ws.vdim && (ws.vdim & 3) == 0) {
+        float v[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = s < len ? o[t][i][r] * f : 0.f;
+        st4(dst + c, v);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (c + r < ws.vdim) st(dst + c + r, s < len ? o[t][i][r] * f : 0.f);
+      }
+    }
+  }
+}
+
+// Split decode: a block scores one row's ring (or a part of it) for up to 16
+// query heads of a kv head; its 4 waves walk 32-row tiles and merge in LDS.
+// part null: the block saw the whole ring and writes the result.
+template <int KC, int VG, bool EXACT>
+__global__ __launch_bounds__(256) void attn_window_decode_kernel(
+    const bf16_t* __restrict__ qw, const bf16_t* __restrict__ kc_, const bf16_t* __restrict__ vc_,
+    const bf16_t* __restrict__ proj, const int* __restrict__ bucket, const bf16_t* __restrict__ rel, int rel_rows,
+    bf16_t* __restrict__ out, float* __restrict__ part, int splits, KVShape ring, AttnArgs a, Step step) {
+  constexpr int OW = VG * 16 + 4;  // row of a wave's partial output (padded)
+  __shared__ float po[4][16 * OW];
+  __shared__ float pm[4][16], pl[4][16];
+  extern __shared__ int tab[];  // [nb] buckets, then [rel_rows][16] bias of these heads
+  const int split = blockIdx.x, b = blockIdx.z;
+  const int per = a.H / a.G, qgs = (per + 15) >> 4;
+  const int g = blockIdx.y / qgs, q0 = (blockIdx.y % qgs) * 16, nq = min(16, per - q0);
+  const int h0 = g * per + q0;
+  const int slot = step.slot(b);
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
+  if (slot < 0) {
+    if (!part)
+      for (int i = threadIdx.x; i < nq * ring.vdim; i += 256)
+        st(out + (size_t)b * a.K + a.out_at + (size_t)h0 * ring.vdim + i, 0.f);
+    return;
+  }
+  float* relb = (float*)(tab + a.nb);
+  for (int i = threadIdx.x; i < a.nb; i += 256) tab[i] = bucket[i];
+  for (int i = threadIdx.x; i < rel_rows * 16; i += 256)
+    relb[i] = (i & 15) < nq ? ld(rel + (i >> 4) * a.H + h0 + (i & 15)) : 0.f;
+  __syncthreads();
+  const int kc = EXACT ? KC : ring.kc, vg = EXACT ? VG : ring.vg;
+  const int pos = step.first(b), cur = pos % ring.rows;
+  const int seen = min(min(a.window, ring.rows), pos + 1);
+  const int ntiles = (min(ring.rows, pos + 1) + 31) >> 5;
+  const int per_split = (ntiles + splits - 1) / splits;
+  bf16x8 qf[KC];
+  const bf16_t* q = qw + ((size_t)b * a.H + h0 + min(col, nq - 1)) * a.qd + quad * 8;
+#pragma unroll
+  for (int c = 0; c < KC; ++c)
+    if (EXACT || c < kc) qf[c] = *(const bf16x8*)(q + c * 32);
+  float m = 0.f, l = 0.f;
+  floatx4 o[VG];
+#pragma unroll
+  for (int i = 0; i < VG; ++i) o[i] = (floatx4)(0.f);
+  const bf16_t* kb = kc_ + Layout<bf16_t>::kbase(ring, (size_t)slot * a.G + g);
+  const bf16_t* vb = vc_ + Layout<bf16_t>::vbase(ring, (size_t)slot * a.G + g);
+  const size_t vstride = (size_t)(ring.rows >> 5) * 512;
+  const int end = min(ntiles, (split + 1) * per_split);
+  for (int tile = split * per_split + wave; tile < end; tile += 4) {
+    bf16x8 vf[VG];
+    floatx4 sc[2];
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
+      sc[hf] = (floatx4)(0.f);
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+        if (EXACT || c < kc) {
+          const bf16x8 kf = *(const bf16x8*)(kb + ((size_t)(tile * 2 + hf) * kc + c) * 512 + lane * 8);
+          sc[hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[c], sc[hf], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < VG; ++i)
+      if (EXACT || i < vg) vf[i] = *(const bf16x8*)(vb + i * vstride + (size_t)tile * 512 + lane * 8);
+    float top = m;
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        int age = cur - (tile * 32 + hf * 16 + quad * 4 + r);
+        if (age < 0) age += ring.rows;
+        const float v = sc[hf][r] * a.scale + relb[tab[min(age, a.nb - 1)] * 16 + col];
+        sc[hf][r] = age < seen ? v : -INFINITY;
+        top = fmaxf(top, sc[hf][r]);
+      }
+    top = fmaxf(top, __shfl_xor(top, 16));
+    top = fmaxf(top, __shfl_xor(top, 32));
+    const float al = __expf(m - top);
+    m = top;
+    l *= al;
+    bf16x8 pf;
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = __expf(sc[hf][r] - top);
+        l += p;
+        pf[hf * 4 + r] = (__bf16)p;
+      }
+#pragma unroll
+    for (int i = 0; i < VG; ++i)
+      if (EXACT || i < vg) {
+        o[i] *= al;
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i], pf, o[i], 0, 0, 0);
+      }
+  }
+  l += __shfl_xor(l, 16);
+  l += __shfl_xor(l, 32);
+  if (quad == 0) { pm[wave][col] = m; pl[wave][col] = l; }
+#pragma unroll
+  for (int i = 0; i < VG; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) po[wave][col * OW + i * 16 + quad * 4 + r] = o[i][r];
+  __syncthreads();
+  for (int i = threadIdx.x; i < nq * ring.vdim; i += 256) {
+    const int qh = i / ring.vdim, c = i - qh * ring.vdim;
+    float M = 0.f, L = 0.f, O = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) M = fmaxf(M, pm[w][qh]);
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float f = __expf(pm[w][qh] - M);
+      L += f * pl[w][qh];
+      O += f * po[w][qh * OW + c];
+    }
+    const int h = h0 + qh;
+    if (part) {
+      float* p = part + (((size_t)b * splits + split) * a.H + h) * (ring.vdim + 2);
+      p[2 + c] = O;
+      if (c == 0) { p[0] = M; p[1] = L; }
+    } else {
+      const float gate = a.out_scale * sigmoidf(ld(proj + (size_t)b * a.N + a.g_at + h));
+      st(out + (size_t)b * a.K + a.out_at + (size_t)h * ring.vdim + c, O / (L + __expf(-M)) * gate);
+    }
+  }
+}
+
+__global__ __launch_bounds__(64) void attn_window_merge_kernel(
+    const float* __restrict__ part, const bf16_t* __restrict__ proj, bf16_t* __restrict__ out, int splits,
+    int vdim, AttnArgs a, Step step) {
+  const int h = blockIdx.x, b = blockIdx.y;
+  const bool live = step.slot(b) >= 0;
+  for (int c = threadIdx.x; c < vdim; c += 64) {
+    float r = 0.f;
+    if (live) {
+      float M = 0.f, L = 0.f, O = 0.f;
+      for (int s = 0; s < splits; ++s) M = fmaxf(M, part[(((size_t)b * splits + s) * a.H + h) * (vdim + 2)]);
+      for (int s = 0; s < splits; ++s) {
+        const float* p = part + (((size_t)b * splits + s) * a.H + h) * (vdim + 2);
+        const float f = __expf(p[0] - M);
+        L += f * p[1];
+        O += f * p[2 + c];
+      }
+      r = O / (L + __expf(-M)) * a.out_scale * sigmoidf(ld(proj + (size_t)b * a.N + a.g_at + h));
+    }
+    st(out + (size_t)b * a.K + a.out_at + (size_t)h * vdim + c, r);
+  }
+}
+
+// 32-bit attention, one wave per (token, head): lanes over keys for the
+// scores, over value columns for the sum. base/rows: where position p lies
+// ((p - base) % rows), so one kernel serves the ring and the workspace.
+__global__ __launch_bounds__(64) void attn_window_f32_kernel(
+    const float* __restrict__ qw, const float* __restrict__ k, const float* __restrict__ v,
+    const float* __restrict__ proj, const int* __restrict__ bucket, const float* __restrict__ rel,
+    float* __restrict__ out, KVShape kv, int base, AttnArgs a, Step step) {
+  __shared__ float q[256];
+  const int s = blockIdx.x, h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G), lane = threadIdx.x;
+  const int slot = step.slot(b), len = step.decode ? 1 : step.len(b, a.S);
+  float* dst = out + ((size_t)b * a.S + s) * a.K + a.out_at + (size_t)h * kv.vdim;
+  if (slot < 0 || s >= len) {
+    for (int c = lane; c < kv.vdim; c += 64) dst[c] = 0.f;
+    return;
+  }
+  for (int d = lane; d < kv.dim; d += 64) q[d] = qw[(((size_t)b * a.S + s) * a.H + h) * a.qd + d];
+  __syncthreads();
+  const size_t head = (size_t)(step.decode ? slot : b) * a.G + g;
+  const float* kb = k + Layout<float>::kbase(kv, head);
+  const float* vb = v + Layout<float>::vbase(kv, head);
+  const int pos = step.first(b) + s, lo = max(0, pos - a.window + 1);
+  float m = 0.f, l = 0.f, acc[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int p0 = lo; p0 <= pos; p0 += 64) {
+    const int p = p0 + lane;
+    float sc = -INFINITY;
+    if (p <= pos) {
+      const float* row = kb + Layout<float>::k(kv, (p - base) % kv.rows, 0);
+      float dot = 0.f;
+      for (int d = 0; d < kv.dim; ++d) dot += q[d] * row[d];
+      sc = dot * a.scale + rel[bucket[min(pos - p, a.nb - 1)] * a.H + h];
+    }
+    float top = sc;
+#pragma unroll
+    for (int x = 32; x > 0; x >>= 1) top = fmaxf(top, __shfl_xor(top, x));
+    top = fmaxf(top, m);
+    const float al = expf(m - top), e = expf(sc - top);
+    m = top;
+    l = l * al + wave_sum(e);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] *= al;
+    const int n = min(64, pos - p0 + 1);
+    for (int j = 0; j < n; ++j) {
+      const float pj = __shfl(e, j);
+      const float* row = vb + Layout<float>::v(kv, (p0 + j - base) % kv.rows, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (lane + i * 64 < kv.vdim) acc[i] += pj * row[lane + i * 64];
+    }
+  }
+  const float f = a.out_scale * sigmoidf(proj[((size_t)b * a.S + s) * a.N + a.g_at + h]) / (l + expf(-m));
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (lane + i * 64 < kv.vdim) dst[lane + i * 64] = acc[i] * f;
+}
+
+// ---------------------------------------------------------------------------
+// recurrences
+// ---------------------------------------------------------------------------
+
+// Last inputs of a chunk into a ring of rows by position (convolutions,
+// token shift). Up to three column ranges of src, side by side in the ring.
+struct Columns { int at[3], n[3]; };
+
+template <typename T>
+__global__ __launch_bounds__(256) void remember_kernel(
+    const T* __restrict__ src, T* __restrict__ ring, int S, int N, int M, int C, Columns cols, Step step) {
+  const int b = blockIdx.y, slot = step.slot(b), len = step.len(b, S);
+  const int s = len - 1 - blockIdx.x;
+  if (slot < 0 || s < 0) return;
+  const T* row = src + ((size_t)b * S + s) * N;
+  T* dst = ring + ((size_t)slot * M + (step.first(b) + s) % M) * C;
+  for (int i = threadIdx.x; i < C; i += 256) {
+    int c = i, r = 0;
+    while (r < 2 && c >= cols.n[r]) c -= cols.n[r++];
+    dst[i] = row[cols.at[r] + c];
+  }
+}
+
+struct RecArgs {
+  int S, H, G, N, K;
+  int dim, vdim, dp, taps;               // dp: padded key channels
+  int q_at, k_at, v_at, b_at, out_at;
+  float eps, out_scale;
+};
+
+// sum over taps of a channel's inputs, then silu; ch: channel in the ring
+template <typename T>
+DEVINL float conv_silu(const T* proj, const T* ring, const T* taps_w, int s, int first, int col, int ch, int wch,
+                       int C, const RecArgs& a) {
+  float y = 0.f;
+  for (int j = 0; j < a.taps; ++j) {
+    const int back = a.taps - 1 - j;
+    float x = 0.f;
+    if (s >= back) x = ld(proj + (long long)(s - back) * a.N + col);
+    else if (first + s >= back) x = ld(ring + (size_t)((first + s - back) % a.taps) * C + ch);
+    y += x * ld(taps_w + wch * a.taps + j);
+  }
+  return siluf(y);
+}
+
+// Prompt side of the delta rule: one wave per (token, q/k head) prepares that
+// head's unit q (scaled) and k, q.k, and for its value heads v, decays, beta.
+template <typename T>
+__global__ __launch_bounds__(256) void delta_prep_kernel(
+    const T* __restrict__ proj, const T* __restrict__ qc, const T* __restrict__ kcv, const T* __restrict__ vcv,
+    const T* __restrict__ pre, const T* __restrict__ a_log, const T* __restrict__ dt, const T* __restrict__ ring,
+    float* __restrict__ q, float* __restrict__ k, float* __restrict__ dot, float* __restrict__ v,
+    float* __restrict__ dec, float* __restrict__ beta, int total, RecArgs a, Step step) {
+  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (id >= total) return;
+  const int g = id % a.G, tok = id / a.G, s = tok % a.S, b = tok / a.S;
+  const int slot = step.slot(b);
+  if (slot < 0 || s >= step.len(b, a.S)) return;
+  const int C = 2 * a.G * a.dim + a.H * a.vdim, first = step.first(b), per = a.H / a.G;
+  const T* rows = proj + (size_t)b * a.S * a.N;
+  const T* hist = ring + (size_t)slot * a.taps * C;
+  float qv[4], kv[4], qq = 0.f, kk = 0.f, qk = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int d = lane + 64 * i, ch = g * a.dim + d;
+    qv[i] = kv[i] = 0.f;
+    if (d < a.dim) {
+      qv[i] = conv_silu(rows, hist, qc, s, first, a.q_at + ch, ch, ch, C, a);
+      kv[i] = conv_silu(rows, hist, kcv, s, first, a.k_at + ch, a.G * a.dim + ch, ch, C, a);
+    }
+    qq += qv[i] * qv[i];
+    kk += kv[i] * kv[i];
+    qk += qv[i] * kv[i];
+  }
+  const float qi = 1.f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)a.dim), ki = 1.f / sqrtf(wave_sum(kk) + 1e-6f);
+  qk = wave_sum(qk) * qi * ki;
+  const size_t qo = ((size_t)tok * a.G + g) * a.dp;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int d = lane + 64 * i;
+    if (d < a.dp) { q[qo + d] = qv[i] * qi; k[qo + d] = kv[i] * ki; }
+  }
+  if (lane == 0) dot[(size_t)tok * a.G + g] = qk;
+  for (int h = g * per; h < (g + 1) * per; ++h) {
+    const float A = expf(ld(a_log + h));
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = lane + 64 * i;
+      if (d < a.dp) {
+        const int ch = h * a.dim + d;
+        dec[((size_t)tok * a.H + h) * a.dp + d] =
+            d < a.dim ? expf(-A * softplusf(ld(pre + (size_t)tok * a.H * a.dim + ch) + ld(dt + ch))) : 1.f;
+      }
+      if (d < a.vdim) {
+        const int ch = h * a.vdim + d;
+        v[(size_t)tok * a.H * a.vdim + ch] =
+            conv_silu(rows, hist, vcv, s, first, a.v_at + ch, 2 * a.G * a.dim + ch, ch, C, a);
+      }
+    }
+    if (lane == 0) beta[(size_t)tok * a.H + h] = sigmoidf(ld(proj + (size_t)tok * a.N + a.b_at + h));
+  }
+}
+
+// Prompt side of WKV: r, k, v in fp32, decays, and r.(u*k) per (token, head).
+template <typename T>
+__global__ __launch_bounds__(256) void wkv_prep_kernel(
+    const T* __restrict__ rr, const T* __restrict__ kk, const T* __restrict__ vv, const T* __restrict__ pre,
+    const T* __restrict__ w0, const T* __restrict__ u, float* __restrict__ q, float* __restrict__ k,
+    float* __restrict__ dot, float* __restrict__ v, float* __restrict__ dec, int total, RecArgs a, Step step) {
+  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (id >= total) return;
+  const int h = id % a.H, tok = id / a.H, s = tok % a.S, b = tok / a.S;
+  if (step.slot(b) < 0 || s >= step.len(b, a.S)) return;
+  const size_t src = ((size_t)tok * a.H + h) * a.dim, dst = ((size_t)tok * a.H + h) * a.dp;
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int d = lane + 64 * i;
+    if (d >= a.dp) continue;
+    float r = 0.f, kx = 0.f, w = 1.f;
+    if (d < a.dim) {
+      r = ld(rr + src + d);
+      kx = ld(kk + src + d);
+      w = expf(-expf(ld(pre + src + d) + ld(w0 + h * a.dim + d)));
+      sum += r * kx * ld(u + h * a.dim + d);
+      v[src + d] = ld(vv + src + d);
+    }
+    q[dst + d] = r;
+    k[dst + d] = kx;
+    dec[dst + d] = w;
+  }
+  sum = wave_sum(sum);
+  if (lane == 0) dot[(size_t)tok * a.H + h] = sum;
+}
+
+// sum over the 16 lanes of a DPP row, in every lane
+DEVINL float row_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, true));  // row_ror:8
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, true));
+  return v;
+}
+
+// rows of the state that lane r (0..15) of a column holds: vectors of V
+template <int RPL> struct Rows {
+  static constexpr int V = RPL % 4 == 0 ? 4 : RPL % 2 == 0 ? 2 : 1;
+  static DEVINL int at(int j, int r) { return j * 16 * V + V * r; }  // j < RPL / V
+};
+template <int RPL>
+DEVINL void load_rows(const float* p, int r, float* o) {
+#pragma unroll
+  for (int j = 0; j < RPL / Rows<RPL>::V; ++j) ldv<Rows<RPL>::V>(p + Rows<RPL>::at(j, r), o + j * Rows<RPL>::V);
+}
+template <int RPL>
+DEVINL void store_rows(float* p, int r, const float* o) {
+#pragma unroll
+  for (int j = 0; j < RPL / Rows<RPL>::V; ++j) stv<Rows<RPL>::V>(p + Rows<RPL>::at(j, r), o + j * Rows<RPL>::V);
+}
+
+// one token of a column; s: the column's rows in this lane. Returns the
+// column's output (in all 16 lanes).
+template <bool DELTA, int RPL>
+DEVINL float rec_step(float* s, const float* q, const float* k, const float* g, float v, float beta, float dot) {
+  float p1 = 0.f, p2 = 0.f;
+  if (DELTA) {
+#pragma unroll
+    for (int i = 0; i < RPL; ++i) {
+      s[i] *= g[i];
+      p1 += s[i] * k[i];
+      p2 += s[i] * q[i];
+    }
+    p1 = row_sum(p1);
+    p2 = row_sum(p2);
+    const float u = beta * (v - p1);
+#pragma unroll
+    for (int i = 0; i < RPL; ++i) s[i] += k[i] * u;
+    return p2 + u * dot;
+  }
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) {
+    p2 += s[i] * q[i];
+    s[i] = g[i] * s[i] + k[i] * v;
+  }
+  return row_sum(p2) + dot * v;
+}
+
+// The scan: 16 lanes hold one column of a head's state in registers (16
+// columns a block) and step through the prompt; q, k and decays of CT tokens
+// at a time pass through LDS, loaded one chunk ahead.
+template <bool DELTA, int RPL>
+__global__ __launch_bounds__(256) void scan_kernel(
+    const float* __restrict__ q, const float* __restrict__ k, const float* __restrict__ dec,
+    const float* __restrict__ v, const float* __restrict__ beta, const float* __restrict__ dot,
+    float* __restrict__ state, float* __restrict__ o, RecArgs a, Step step) {
+  constexpr int CT = 16, DP = 16 * RPL, V4 = CT * DP / 4, NL = (V4 + 255) / 256;
+  __shared__ __attribute__((aligned(16))) float sq[CT * DP], sk[CT * DP], sg[CT * DP];
+  __shared__ float sv[CT * 16], so[CT * 16], sb[CT], sd[CT];
+  const int h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G);
+  const int slot = step.slot(b);
+  if (slot < 0) return;
+  const int len = step.len(b, a.S), tid = threadIdx.x;
+  const int r = tid & 15, cl = tid >> 4, col = blockIdx.x * 16 + cl;
+  float* st_ = state + (((size_t)slot * a.H + h) * a.vdim + min(col, a.vdim - 1)) * DP;
+  float s[RPL];
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) s[i] = 0.f;
+  if (step.first(b) > 0) load_rows<RPL>(st_, r, s);
+  floatx4 rq[NL], rk[NL], rg[NL];
+  float rv = 0.f, rb = 0.f, rd = 0.f;
+  const size_t tok0 = (size_t)b * a.S;
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = (tid + i * 256) * 4, t = t0 + e / DP, d = e % DP;
+      if (e < CT * DP && t < len) {
+        rq[i] = *(const floatx4*)(q + ((tok0 + t) * a.G + g) * DP + d);
+        rk[i] = *(const floatx4*)(k + ((tok0 + t) * a.G + g) * DP + d);
+        rg[i] = *(const floatx4*)(dec + ((tok0 + t) * a.H + h) * DP + d);
+      }
+    }
+    const int tv = t0 + (tid >> 4), cv = blockIdx.x * 16 + (tid & 15);
+    rv = tv < len && cv < a.vdim ? v[((tok0 + tv) * a.H + h) * a.vdim + cv] : 0.f;
+    if (tid < CT && t0 + tid < len) {
+      if (DELTA) rb = beta[(tok0 + t0 + tid) * a.H + h];
+      rd = dot[(tok0 + t0 + tid) * a.G + g];
+    }
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < len; t0 += CT) {
+    __syncthreads();  // the previous chunk's inputs and outputs are done with
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = (tid + i * 256) * 4;
+      if (e < CT * DP) {
+        *(floatx4*)(sq + e) = rq[i];
+        *(floatx4*)(sk + e) = rk[i];
+        *(floatx4*)(sg + e) = rg[i];
+      }
+    }
+    sv[tid] = rv;
+    if (tid < CT) { sb[tid] = rb; sd[tid] = rd; }
+    __syncthreads();
+    if (t0 + CT < len) fetch(t0 + CT);
+    const int n = min(CT, len - t0);
+    for (int t = 0; t < n; ++t) {
+      float qq[RPL], kk[RPL], gg[RPL];
+      load_rows<RPL>(sq + t * DP, r, qq);
+      load_rows<RPL>(sk + t * DP, r, kk);
+      load_rows<RPL>(sg + t * DP, r, gg);
+      const float y = rec_step<DELTA, RPL>(s, qq, kk, gg, sv[t * 16 + cl], DELTA ? sb[t] : 0.f, sd[t]);
+      if (r == 0) so[t * 16 + cl] = y;
+    }
+    __syncthreads();
+    const int t = tid >> 4, c = blockIdx.x * 16 + (tid & 15);
+    if (t < n && c < a.vdim) o[((tok0 + t0 + t) * a.H + h) * a.vdim + c] = so[tid];
+  }
+  if (col < a.vdim) store_rows<RPL>(st_, r, s);
+}
+
+// Per-head RMS norm, weight and gate: one wave per (token, head). DELTA: the
+// weight is shared by heads and the gate a sigmoid; else a weight per head
+// and a silu.
+template <typename T, bool DELTA>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(
+    const float* __restrict__ o, const T* __restrict__ norm, const T* __restrict__ gate, T* __restrict__ out,
+    int total, RecArgs a, Step step) {
+  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (id >= total) return;
+  const int h = id % a.H, tok = id / a.H, s = tok % a.S, b = tok / a.S;
+  const bool live = step.slot(b) >= 0 && s < step.len(b, a.S);
+  const size_t src = ((size_t)tok * a.H + h) * a.vdim;
+  T* dst = out + (size_t)tok * a.K + a.out_at + h * a.vdim;
+  float x[4], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = lane + 64 * i;
+    x[i] = live && c < a.vdim ? o[src + c] : 0.f;
+    ss += x[i] * x[i];
+  }
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = lane + 64 * i;
+    if (c >= a.vdim) continue;
+    float y = 0.f;
+    if (live) {
+      const float gv = ld(gate + src + c);
+      y = x[i] * inv * ld(norm + (DELTA ? c : h * a.vdim + c)) * (DELTA ? sigmoidf(gv) : siluf(gv)) * a.out_scale;
+    }
+    st(dst + c, y);
+  }
+}
+
+// One token of one head, everything from projections to the gated output: a
+// block streams the head's state once. DELTA inputs: q/k/v columns of `in0`
+// (with their convolutions), beta there too; WKV inputs: r, k, v tensors.
+template <typename T, bool DELTA, int RPL>
+__global__ __launch_bounds__(256) void rec_decode_kernel(
+    const T* __restrict__ in0, const T* __restrict__ in1, const T* __restrict__ in2, const T* __restrict__ w0_,
+    const T* __restrict__ w1_, const T* __restrict__ w2_, const T* __restrict__ pre, const T* __restrict__ a_log,
+    const T* __restrict__ dt, const T* __restrict__ norm, const T* __restrict__ gate, float* __restrict__ state,
+    T* __restrict__ ring, T* __restrict__ out, RecArgs a, Step step) {
+  constexpr int DP = 16 * RPL;
+  __shared__ __attribute__((aligned(16))) float sq[DP], sk[DP], sg[DP];
+  __shared__ float sv[256], so[256], red[16];
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, g = h / (a.H / a.G);
+  const int slot = step.slot(b);
+  T* dst = out + (size_t)b * a.K + a.out_at + h * a.vdim;
+  if (slot < 0) {
+    if (tid < a.vdim) st(dst + tid, 0.f);
+    return;
+  }
+  const int pos = step.first(b);
+  // (dim and vdim are at most 256: one channel a thread)
+  float q = 0.f, k = 0.f, dec = 1.f, beta = 0.f, extra = 0.f;
+  if (DELTA) {
+    const int C = 2 * a.G * a.dim + a.H * a.vdim, qch = g * a.dim + tid, vch = h * a.vdim + tid;
+    const T* row = in0 + (size_t)b * a.N;
+    T* hist = ring + (size_t)slot * a.taps * C;
+    T* now = hist + (size_t)(pos % a.taps) * C;  // a row that no convolution of this step reads
+    if (tid < a.dim) {
+      q = conv_silu(row, hist, w0_, 0, pos, a.q_at + qch, qch, qch, C, a);
+      k = conv_silu(row, hist, w1_, 0, pos, a.k_at + qch, a.G * a.dim + qch, qch, C, a);
+      if (h % (a.H / a.G) == 0) {
+        now[qch] = row[a.q_at + qch];
+        now[a.G * a.dim + qch] = row[a.k_at + qch];
+      }
+      const int ch = h * a.dim + tid;
+      dec = expf(-expf(ld(a_log + h)) * softplusf(ld(pre + (size_t)b * a.H * a.dim + ch) + ld(dt + ch)));
+    }
+    if (tid < a.vdim) {
+      sv[tid] = conv_silu(row, hist, w2_, 0, pos, a.v_at + vch, 2 * a.G * a.dim + vch, vch, C, a);
+      now[2 * a.G * a.dim + vch] = row[a.v_at + vch];
+    }
+    beta = sigmoidf(ld(row + a.b_at + h));
+  } else if (tid < a.dim) {
+    const size_t src = ((size_t)b * a.H + h) * a.dim + tid;
+    q = ld(in0 + src);
+    k = ld(in1 + src);
+    sv[tid] = ld(in2 + src);
+    dec = expf(-expf(ld(pre + src) + ld(w0_ + h * a.dim + tid)));
+    extra = q * k * ld(w1_ + h * a.dim + tid);
+  }
+  float dot;
+  if (DELTA) {
+    const float qq = wave_sum(q * q), kk = wave_sum(k * k), qk = wave_sum(q * k);
+    if ((tid & 63) == 0) { red[tid >> 6] = qq; red[4 + (tid >> 6)] = kk; red[8 + (tid >> 6)] = qk; }
+    __syncthreads();
+    const float qi = 1.f / sqrtf(red[0] + red[1] + red[2] + red[3] + 1e-6f) / sqrtf((float)a.dim);
+    const float ki = 1.f / sqrtf(red[4] + red[5] + red[6] + red[7] + 1e-6f);
+    dot = (red[8] + red[9] + red[10] + red[11]) * qi * ki;
+    q *= qi;
+    k *= ki;
+  } else {
+    dot = block_sum(extra, red);
+  }
+  if (tid < DP) { sq[tid] = q; sk[tid] = k; sg[tid] = dec; }
+  __syncthreads();
+  const int r = tid & 15, cl = tid >> 4;
+  float qq[RPL], kk[RPL], gg[RPL];
+  load_rows<RPL>(sq, r, qq);
+  load_rows<RPL>(sk, r, kk);
+  load_rows<RPL>(sg, r, gg);
+  float* base = state + ((size_t)slot * a.H + h) * (size_t)a.vdim * DP;
+  constexpr int NB = RPL <= 8 ? 4 : 2;  // columns in flight per lane group
+  for (int c0 = 0; c0 < a.vdim; c0 += 16 * NB) {
+    float s[NB][RPL];
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      const int col = c0 + i * 16 + cl;
+      if (col < a.vdim && pos > 0) load_rows<RPL>(base + (size_t)col * DP, r, s[i]);
+      else
+#pragma unroll
+        for (int j = 0; j < RPL; ++j) s[i][j] = 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      const int col = c0 + i * 16 + cl;
+      const float y = rec_step<DELTA, RPL>(s[i], qq, kk, gg, sv[min(col, a.vdim - 1)], beta, dot);
+      if (col < a.vdim) {
+        if (r == 0) so[col] = y;
+        store_rows<RPL>(base + (size_t)col * DP, r, s[i]);
+      }
+    }
+  }
+  __syncthreads();
+  const float y = tid < a.vdim ? so[tid] : 0.f;
+  const float inv = 1.f / sqrtf(block_sum(y * y, red + 12) / (float)a.vdim + a.eps);
+  if (tid < a.vdim) {
+    const float gv = ld(gate + ((size_t)b * a.H + h) * a.vdim + tid);
+    st(dst + tid, y * inv * ld(norm + (DELTA ? tid : h * a.vdim + tid)) * (DELTA ? sigmoidf(gv) : siluf(gv)) *
+                      a.out_scale);
+  }
+}
+
+// n blends of the current and the previous token: out [n][B,S,D]
+template <typename T>
+__global__ __launch_bounds__(256) void token_shift_kernel(
+    const T* __restrict__ h, const T* __restrict__ mu, T* __restrict__ ring, T* __restrict__ out, int S, int D,
+    int M, int n, size_t plane, Step step) {
+  const int s = blockIdx.x, b = blockIdx.y;
+  const int slot = step.slot(b), len = step.decode ? 1 : step.len(b, S);
+  const bool live = slot >= 0 && s < len;
+  const int first = live ? step.first(b) : 0;
+  const size_t at = ((size_t)b * S + s) * D;
+  for (int d = threadIdx.x; d < D; d += 256) {
+    float x = 0.f, p = 0.f;
+    if (live) {
+      x = ld(h + at + d);
+      if (s > 0) p = ld(h + at - D + d);
+      else if (first > 0) p = ld(ring + ((size_t)slot * M + (first - 1) % M) * D + d);
+      if (step.decode) st(ring + ((size_t)slot * M + first % M) * D + d, x);  // M >= 2: not the row just read
+    }
+    for (int i = 0; i < n; ++i) st(out + i * plane + at + d, x + (p - x) * ld(mu + (size_t)i * D + d));
+  }
+}
+
+// ===========================================================================
+// host side
+// ===========================================================================
+
+#define CHK(x) TORCH_CHECK(x, #x)
+using torch::Tensor;
+using OptT = c10::optional<Tensor>;
+
+static inline hipStream_t cur_stream() { return (hipStream_t)c10::hip::getCurrentHIPStream().stream(); }
+
+static void check_io(const Tensor& t, torch::ScalarType dt) {
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == dt, "contiguous GPU tensor of type ",
+              c10::toString(dt), " expected, got ", c10::toString(t.scalar_type()), t.sizes());
+}
+static torch::ScalarType io_type(const Tensor& t) {
+  const auto dt = t.scalar_type();
+  TORCH_CHECK(dt == torch::kBFloat16 || dt == torch::kFloat32, "bfloat16 or float32 expected");
+  check_io(t, dt);
+  return dt;
+}
+static Tensor f32(const Tensor& like, std::vector<int64_t> shape) {
+  return torch::empty(shape, like.options().dtype(torch::kFloat32));
+}
+
+static Step make_step(const OptT& slots, const OptT& positions, const OptT& lens, int64_t start, bool decode, int B) {
+  Step s{};
+  if (slots) { check_io(*slots, torch::kInt32); CHK(slots->numel() == B); s.slots = slots->data_ptr<int>(); }
+  if (lens && !decode) { check_io(*lens, torch::kInt32); CHK(lens->numel() == B); s.lens = lens->data_ptr<int>(); }
+  if (decode) {
+    TORCH_CHECK(positions, "a decode step needs positions");
+    check_io(*positions, torch::kInt32);
+    CHK(positions->numel() == 1 || positions->numel() == B);
+    s.positions = positions->data_ptr<int>();
+    s.npos = positions->numel();
+  }
+  CHK(start >= 0);
+  s.start = (int)start;
+  s.decode = decode;
+  return s;
+}
+
+template <typename T> static const T* P(const Tensor& t) { return (const T*)t.data_ptr(); }
+template <typename T> static T* M(Tensor& t) { return (T*)t.data_ptr(); }
+
+#define BY_TYPE(dt, ...)                                              \
+  if (dt == torch::kBFloat16) { typedef bf16_t T; __VA_ARGS__; }      \
+  else { typedef float T; __VA_ARGS__; }
+
+template <typename T, int V>
+static void launch_norm(const T* y, float* x, const T* wp, const T* wn, T* h, int rows, int D, float eps) {
+  const int nc = (D + 256 * V - 1) / (256 * V);
+#define NORM_CASE(NC) \
+  if (nc <= NC) { hipLaunchKernelGGL((sandwich_norm_kernel<T, V, NC>), dim3(rows), dim3(256), 0, cur_stream(), y, x, wp, wn, h, D, eps); return; }
+  NORM_CASE(1) NORM_CASE(2) NORM_CASE(4) NORM_CASE(8) NORM_CASE(16)
+#undef NORM_CASE
+  TORCH_CHECK(false, "row of ", D, " elements is too long");
+}
+
+static OptT norm_host(const OptT& y, Tensor x, const OptT& w_post, const OptT& w_next, double eps,
+                      torch::ScalarType dt) {
+  check_io(x, torch::kFloat32);
+  const int D = x.size(-1), rows = x.numel() / D;
+  if (y) { check_io(*y, dt); CHK(y->numel() == x.numel() && y->size(-1) == D && w_post); check_io(*w_post, dt); CHK(w_post->numel() == D); }
+  OptT h;
+  if (w_next) { check_io(*w_next, dt); CHK(w_next->numel() == D); h = torch::empty(x.sizes(), x.options().dtype(dt)); }
+  if (rows == 0) return h;
+  BY_TYPE(dt, {
+    const T* yp = y ? P<T>(*y) : nullptr;
+    const T* wp = w_post ? P<T>(*w_post) : nullptr;
+    const T* wn = w_next ? P<T>(*w_next) : nullptr;
+    T* hp = h ? M<T>(*h) : nullptr;
+    if (D % 4 == 0) launch_norm<T, 4>(yp, M<float>(x), wp, wn, hp, rows, D, (float)eps);
+    else launch_norm<T, 1>(yp, M<float>(x), wp, wn, hp, rows, D, (float)eps);
+  });
+  return h;
+}
+
+OptT sandwich_norm(Tensor y, Tensor x, Tensor w_post, OptT w_next, double eps) {
+  return norm_host(y, x, w_post, w_next, eps, io_type(y));
+}
+
+Tensor prenorm(Tensor x, Tensor w, double eps, bool bf16) {
+  return *norm_host(c10::nullopt, x, c10::nullopt, w, eps, bf16 ? torch::kBFloat16 : torch::kFloat32);
+}
+
+Tensor swiglu_packed(Tensor gu) {
+  const auto dt = io_type(gu);
+  const int I = gu.size(-1) / 2;
+  CHK(gu.size(-1) == 2 * I);
+  auto shape = gu.sizes().vec();
+  shape.back() = I;
+  auto out = torch::empty(shape, gu.options());
+  const long long n = out.numel();
+  if (n == 0) return out;
+  BY_TYPE(dt, {
+    if (I % 4 == 0)
+      hipLaunchKernelGGL((swiglu_kernel<T, 4>), dim3((n / 4 + 255) / 256), dim3(256), 0, cur_stream(), P<T>(gu), M<T>(out), n, I);
+    else
+      hipLaunchKernelGGL((swiglu_kernel<T, 1>), dim3((n + 255) / 256), dim3(256), 0, cur_stream(), P<T>(gu), M<T>(out), n, I);
+  });
+  return out;
+}
+
+Tensor tanh_op(Tensor x) {
+  const auto dt = io_type(x);
+  auto out = torch::empty_like(x);
+  const long long n = x.numel();
+  if (n == 0) return out;
+  BY_TYPE(dt, { hipLaunchKernelGGL((tanh_kernel<T>), dim3((n + 255) / 256), dim3(256), 0, cur_stream(), P<T>(x), M<T>(out), n); });
+  return out;
+}
+
+template <int KC, int VG>
+static void launch_prefill(bool exact, dim3 grid, size_t lds, const bf16_t* q, const bf16_t* k, const bf16_t* v,
+                           const bf16_t* proj, const int* bucket, const bf16_t* rel, bf16_t* out, KVShape ws, int hist,
+                           AttnArgs a, Step step) {
+  if (exact)
+    hipLaunchKernelGGL((attn_window_prefill_kernel<KC, VG, true>), grid, dim3(256), lds, cur_stream(), q, k, v, proj, bucket, rel, out, ws, hist, a, step);
+  else
+    hipLaunchKernelGGL((attn_window_prefill_kernel<KC, VG, false>), grid, dim3(256), lds, cur_stream(), q, k, v, proj, bucket, rel, out, ws, hist, a, step);
+}
+
+template <int KC, int VG>
+static void launch_decode(bool exact, dim3 grid, size_t lds, const bf16_t* q, const bf16_t* k, const bf16_t* v,
+                          const bf16_t* proj, const int* bucket, const bf16_t* rel, int rel_rows, bf16_t* out,
+                          float* part, int splits, KVShape ring, AttnArgs a, Step step) {
+  if (exact)
+    hipLaunchKernelGGL((attn_window_decode_kernel<KC, VG, true>), grid, dim3(256), lds, cur_stream(), q, k, v, proj, bucket, rel, rel_rows, out, part, splits, ring, a, step);
+  else
+    hipLaunchKernelGGL((attn_window_decode_kernel<KC, VG, false>), grid, dim3(256), lds, cur_stream(), q, k, v, proj, bucket, rel, rel_rows, out, part, splits, ring, a, step);
+}
+
+// template sizes: the smallest that hold both dims
+#define BY_DIMS(kc, vg, FN, ...)                                                 \
+  if (kc <= 1 && vg <= 2) FN<1, 2>(kc == 1 && vg == 2, __VA_ARGS__);             \
+  else if (kc <= 2 && vg <= 4) FN<2, 4>(kc == 2 && vg == 4, __VA_ARGS__);        \
+  else if (kc <= 4 && vg <= 8) FN<4, 8>(kc == 4 && vg == 8, __VA_ARGS__);        \
+  else FN<8, 16>(kc == 8 && vg == 16, __VA_ARGS__);
+
+void window_attn(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t g_at, int64_t H, int64_t G,
+                 int64_t dim, int64_t vdim, Tensor q_norm, Tensor k_norm, Tensor bucket, Tensor rel, double scale,
+                 double eps, int64_t window, Tensor kc, Tensor vc, OptT slots, OptT positions, OptT lens,
+                 int64_t start, bool decode, Tensor out, int64_t out_at, double out_scale) {
+  const auto dt = io_type(proj);
+  const bool bf = dt == torch::kBFloat16;
+  CHK(proj.dim() == 3 && out.dim() == 3 && out.size(0) == proj.size(0) && out.size(1) == proj.size(1));
+  for (const Tensor& t : {q_norm, k_norm, rel, kc, vc, out}) check_io(t, dt);
+  check_io(bucket, torch::kInt32);
+  const int B = proj.size(0), S = proj.size(1), N = proj.size(2);
+  CHK(H > 0 && G > 0 && H % G == 0 && dim > 0 && vdim > 0 && dim <= 256 && vdim <= 256 && window > 0);
+  CHK(q_at + H * dim <= N && k_at + G * dim <= N && v_at + G * vdim <= N && g_at + H <= N);
+  CHK(out_at + H * vdim <= out.size(2) && out_at % 4 == 0 && out.size(2) % 4 == 0);
+  CHK(q_norm.numel() == H * dim && k_norm.numel() == G * dim && rel.dim() == 2 && rel.size(1) == H);
+  CHK(bucket.numel() > 0 && (!decode || S == 1));
+  if (B == 0 || S == 0) return;
+  KVShape ring{(int)dim, (int)vdim, (int)(dim + 31) / 32, (int)(vdim + 15) / 16, 0};
+  CHK(kc.size(1) == G && vc.size(1) == G && kc.size(0) == vc.size(0) && (slots || B <= kc.size(0)));
+  if (bf) {
+    CHK(kc.dim() == 6 && vc.dim() == 6 && kc.size(3) == ring.kc && vc.size(2) == ring.vg);
+    ring.rows = kc.size(2) * 16;
+    CHK(ring.rows % 32 == 0 && vc.size(3) * 32 == ring.rows);
+  } else {
+    CHK(kc.dim() == 4 && vc.dim() == 4 && kc.size(3) == dim && vc.size(3) == vdim && kc.size(2) == vc.size(2));
+    ring.rows = kc.size(2);
+  }
+  CHK(ring.rows > 0);
+  const Step step = make_step(slots, positions, lens, start, decode, B);
+  AttnArgs a{S, (int)H, (int)G, N, (int)out.size(2), (int)q_at, (int)k_at, (int)v_at, (int)g_at, (int)out_at,
+             bf ? ring.kc * 32 : (int)dim, (float)scale, (float)eps, (float)out_scale, (int)window,
+             (int)bucket.numel()};
+  auto qw = torch::empty({B, S, H, a.qd}, proj.options());
+  const hipStream_t stream = cur_stream();
+  // prefill reads keys from one linear workspace: what the window still holds
+  // of earlier chunks, then this chunk
+  KVShape ws = ring;
+  int base = 0, hist = 0, fill = S;
+  Tensor kw, vw;
+  if (!decode) {
+    base = (int)std::max<int64_t>(0, start - (window - 1));
+    hist = (int)start - base;
+    CHK(hist <= ring.rows);
+    ws.rows = (hist + S + 31) / 32 * 32;
+    fill = ws.rows - hist;
+    kw = torch::empty({B, G, (int64_t)ws.rows * (bf ? ws.kc * 32 : ws.dim)}, proj.options());
+    vw = torch::empty({B, G, (int64_t)ws.rows * (bf ? ws.vg * 16 : ws.vdim)}, proj.options());
+  }
+  BY_TYPE(dt, {
+    T* kwp = decode ? nullptr : M<T>(kw);
+    T* vwp = decode ? nullptr : M<T>(vw);
+    if (hist > 0)
+      hipLaunchKernelGGL((window_history_kernel<T>), dim3(hist, G, B), dim3(256), 0, stream, P<T>(kc), P<T>(vc), kwp, vwp, ring, ws, (int)G, base, hist, step);
+    hipLaunchKernelGGL((qk_norm_append_kernel<T>), dim3(fill, B), dim3(256), 0, stream, P<T>(proj), P<T>(q_norm),
+                       P<T>(k_norm), M<T>(qw), M<T>(kc), M<T>(vc), kwp, vwp, ring, ws, hist, a, step);
+  });
+  if (!bf) {
+    const Tensor& k = decode ? kc : kw;
+    const Tensor& v = decode ? vc : vw;
+    hipLaunchKernelGGL(attn_window_f32_kernel, dim3(S, H, B), dim3(64), 0, stream, P<float>(qw), P<float>(k),
+                       P<float>(v), P<float>(proj), bucket.data_ptr<int>(), P<float>(rel), M<float>(out),
+                       decode ? ring : ws, decode ? 0 : base, a, step);
+    return;
+  }
+  const int rel_rows = rel.size(0);
+  if (!decode) {
+    const size_t lds = (size_t)a.nb * 4;
+    TORCH_CHECK(lds <= 60000, "distance table of ", a.nb, " entries does not fit LDS");
+    const dim3 grid((S + 127) / 128, H, B);
+    BY_DIMS(ws.kc, ws.vg, launch_prefill, grid, lds, P<bf16_t>(qw), P<bf16_t>(kw), P<bf16_t>(vw), P<bf16_t>(proj),
+            bucket.data_ptr<int>(), P<bf16_t>(rel), M<bf16_t>(out), ws, hist, a, step);
+    return;
+  }
+  const size_t lds = (size_t)a.nb * 4 + (size_t)rel_rows * 64;
+  TORCH_CHECK(lds <= 60000, "distance table of ", a.nb, " entries does not fit LDS");
+  const int qgs = ((int)(H / G) + 15) / 16;
+  // enough blocks for the chip, at least one 32-row tile per wave
+  const int blocks = B * (int)G * qgs;
+  const int splits = std::max(1, std::min((512 + blocks - 1) / blocks, ring.rows / 128));
+  Tensor part;
+  if (splits > 1) part = f32(proj, {B, splits, H, vdim + 2});
+  const dim3 grid(splits, G * qgs, B);
+  BY_DIMS(ring.kc, ring.vg, launch_decode, grid, lds, P<bf16_t>(qw), P<bf16_t>(kc), P<bf16_t>(vc), P<bf16_t>(proj),
+          bucket.data_ptr<int>(), P<bf16_t>(rel), rel_rows, M<bf16_t>(out), splits > 1 ? M<float>(part) : nullptr,
+          splits, ring, a, step);
+  if (splits > 1)
+    hipLaunchKernelGGL(attn_window_merge_kernel, dim3(H, B), dim3(64), 0, stream, P<float>(part), P<bf16_t>(proj),
+                       M<bf16_t>(out), splits, (int)vdim, a, step);
+}
+
+static int row_pad(int dim) {
+  for (int p : {1, 2, 3, 4, 6, 8, 12, 16})
+    if (dim <= 16 * p) return 16 * p;
+  TORCH_CHECK(false, "recurrent state with ", dim, " key channels");
+}
+
+#define BY_ROWS(dp, ...)                                                                                   \
+  switch (dp / 16) {                                                                                       \
+    case 1: { constexpr int R = 1; __VA_ARGS__; break; }  case 2: { constexpr int R = 2; __VA_ARGS__; break; }   \
+    case 3: { constexpr int R = 3; __VA_ARGS__; break; }  case 4: { constexpr int R = 4; __VA_ARGS__; break; }   \
+    case 6: { constexpr int R = 6; __VA_ARGS__; break; }  case 8: { constexpr int R = 8; __VA_ARGS__; break; }   \
+    case 12: { constexpr int R = 12; __VA_ARGS__; break; } case 16: { constexpr int R = 16; __VA_ARGS__; break; } \
+    default: TORCH_CHECK(false, "padded key channels ", dp);                                               \
+  }
+
+template <bool DELTA>
+static void launch_scan(int B, const Tensor& q, const Tensor& k, const Tensor& dec, const Tensor& v, const Tensor& beta,
+                        const Tensor& dot, Tensor& state, Tensor& o, const RecArgs& a, const Step& step) {
+  BY_ROWS(a.dp, {
+    hipLaunchKernelGGL((scan_kernel<DELTA, R>), dim3((a.vdim + 15) / 16, a.H, B), dim3(256), 0, cur_stream(),
+                       P<float>(q), P<float>(k), P<float>(dec), P<float>(v), DELTA ? P<float>(beta) : nullptr,
+                       P<float>(dot), M<float>(state), M<float>(o), a, step);
+  });
+}
+
+template <typename T>
+static void remember(const Tensor& src, Tensor& ring, int B, int S, int N, Columns cols, const Step& step) {
+  const int Mr = ring.size(1), C = ring.size(2);
+  hipLaunchKernelGGL((remember_kernel<T>), dim3(std::min(Mr, S), B), dim3(256), 0, cur_stream(), P<T>(src), M<T>(ring), S, N, Mr, C, cols, step);
+}
+
+void delta_rule(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t b_at, int64_t H, int64_t G, int64_t dim,
+                int64_t vdim, Tensor qc, Tensor kcv, Tensor vcv, Tensor pre, Tensor pre_gate, Tensor a_log, Tensor dt_,
+                Tensor norm, double eps, Tensor state, Tensor ring, OptT slots, OptT positions, OptT lens,
+                int64_t start, bool decode, Tensor out, int64_t out_at, double out_scale) {
+  const auto dt = io_type(proj);
+  CHK(proj.dim() == 3 && out.dim() == 3 && out.size(0) == proj.size(0) && out.size(1) == proj.size(1));
+  for (const Tensor& t : {qc, kcv, vcv, pre, pre_gate, a_log, dt_, norm, ring, out}) check_io(t, dt);
+  check_io(state, torch::kFloat32);
+  const int B = proj.size(0), S = proj.size(1), N = proj.size(2), taps = qc.size(-1);
+  const int dp = row_pad(dim), C = 2 * G * dim + H * vdim;
+  CHK(H > 0 && G > 0 && H % G == 0 && dim > 0 && vdim > 0 && vdim <= 256 && taps > 0);
+  CHK(q_at + G * dim <= N && k_at + G * dim <= N && v_at + H * vdim <= N && b_at + H <= N);
+  CHK(out_at + H * vdim <= out.size(2) && (!decode || S == 1));
+  CHK(qc.numel() == G * dim * taps && kcv.numel() == G * dim * taps && vcv.numel() == H * vdim * taps);
+  CHK(pre.numel() == (int64_t)B * S * H * dim && pre_gate.numel() == (int64_t)B * S * H * vdim);
+  CHK(a_log.numel() == H && dt_.numel() == H * dim && norm.numel() == vdim);
+  CHK(state.dim() == 4 && state.size(1) == H && state.size(2) == vdim && state.size(3) == dp);
+  CHK(ring.dim() == 3 && ring.size(0) == state.size(0) && ring.size(1) == taps && ring.size(2) == C);
+  CHK(slots || B <= state.size(0));
+  if (B == 0 || S == 0) return;
+  const Step step = make_step(slots, positions, lens, start, decode, B);
+  RecArgs a{S, (int)H, (int)G, N, (int)out.size(2), (int)dim, (int)vdim, dp, taps, (int)q_at, (int)k_at, (int)v_at,
+            (int)b_at, (int)out_at, (float)eps, (float)out_scale};
+  const hipStream_t stream = cur_stream();
+  if (decode) {
+    BY_TYPE(dt, BY_ROWS(dp, {
+      hipLaunchKernelGGL((rec_decode_kernel<T, true, R>), dim3(H, B), dim3(256), 0, stream, P<T>(proj), nullptr,
+                         nullptr, P<T>(qc), P<T>(kcv), P<T>(vcv), P<T>(pre), P<T>(a_log), P<T>(dt_), P<T>(norm),
+                         P<T>(pre_gate), M<float>(state), M<T>(ring), M<T>(out), a, step);
+    }));
+    return;
+  }
+  auto q = f32(proj, {B, S, G, dp}), k = f32(proj, {B, S, G, dp}), dot = f32(proj, {B, S, G});
+  auto v = f32(proj, {B, S, H, vdim}), dec = f32(proj, {B, S, H, dp}), beta = f32(proj, {B, S, H});
+  auto o = f32(proj, {B, S, H, vdim});
+  const int prep = B * S * (int)G, heads = B * S * (int)H;
+  BY_TYPE(dt, {
+    hipLaunchKernelGGL((delta_prep_kernel<T>), dim3((prep + 3) / 4), dim3(256), 0, stream, P<T>(proj), P<T>(qc),
+                       P<T>(kcv), P<T>(vcv), P<T>(pre), P<T>(a_log), P<T>(dt_), P<T>(ring), M<float>(q), M<float>(k),
+                       M<float>(dot), M<float>(v), M<float>(dec), M<float>(beta), prep, a, step);
+    remember<T>(proj, ring, B, S, N, Columns{{(int)q_at, (int)k_at, (int)v_at}, {(int)(G * dim), (int)(G * dim), (int)(H * vdim)}}, step);
+  });
+  launch_scan<true>(B, q, k, dec, v, beta, dot, state, o, a, step);
+  BY_TYPE(dt, {
+    hipLaunchKernelGGL((head_norm_gate_kernel<T, true>), dim3((heads + 3) / 4), dim3(256), 0, stream, P<float>(o),
+                       P<T>(norm), P<T>(pre_gate), M<T>(out), heads, a, step);
+  });
+}
+
+Tensor wkv(Tensor r, Tensor k_, Tensor v_, Tensor gate, Tensor pre, Tensor w0, Tensor u, Tensor norm, int64_t H,
+           int64_t dim, double eps, Tensor state, OptT slots, OptT positions, OptT lens, int64_t start, bool decode) {
+  const auto dt = io_type(r);
+  const int dp = row_pad(dim);
+  CHK(r.dim() == 3 && r.size(2) == H * dim && H > 0 && dim > 0);
+  for (const Tensor& t : {k_, v_, gate, pre}) { check_io(t, dt); CHK(t.sizes() == r.sizes()); }
+  for (const Tensor& t : {w0, u, norm}) { check_io(t, dt); CHK(t.numel() == H * dim); }
+  check_io(state, torch::kFloat32);
+  const int B = r.size(0), S = r.size(1);
+  CHK(state.dim() == 4 && state.size(1) == H && state.size(2) == dim && state.size(3) == dp);
+  CHK((slots || B <= state.size(0)) && (!decode || S == 1));
+  auto out = torch::empty_like(r);
+  if (B == 0 || S == 0) return out;
+  const Step step = make_step(slots, positions, lens, start, decode, B);
+  RecArgs a{S, (int)H, (int)H, 0, (int)(H * dim), (int)dim, (int)dim, dp, 1, 0, 0, 0, 0, 0, (float)eps, 1.f};
+  const hipStream_t stream = cur_stream();
+  if (decode) {
+    BY_TYPE(dt, BY_ROWS(dp, {
+      hipLaunchKernelGGL((rec_decode_kernel<T, false, R>), dim3(H, B), dim3(256), 0, stream, P<T>(r), P<T>(k_),
+                         P<T>(v_), P<T>(w0), P<T>(u), nullptr, P<T>(pre), nullptr, nullptr, P<T>(norm), P<T>(gate),
+                         M<float>(state), nullptr, M<T>(out), a, step);
+    }));
+    return out;
+  }
+  auto q = f32(r, {B, S, H, dp}), k = f32(r, {B, S, H, dp}), dec = f32(r, {B, S, H, dp});
+  auto dot = f32(r, {B, S, H}), v = f32(r, {B, S, H, dim}), o = f32(r, {B, S, H, dim});
+  const int heads = B * S * (int)H;
+  BY_TYPE(dt, {
+    hipLaunchKernelGGL((wkv_prep_kernel<T>), dim3((heads + 3) / 4), dim3(256), 0, stream, P<T>(r), P<T>(k_), P<T>(v_),
+                       P<T>(pre), P<T>(w0), P<T>(u), M<float>(q), M<float>(k), M<float>(dot), M<float>(v),
+                       M<float>(dec), heads, a, step);
+  });
+  launch_scan<false>(B, q, k, dec, v, dot, dot, state, o, a, step);
+  BY_TYPE(dt, {
+    hipLaunchKernelGGL((head_norm_gate_kernel<T, false>), dim3((heads + 3) / 4), dim3(256), 0, stream, P<float>(o),
+                       P<T>(norm), P<T>(gate), M<T>(out), heads, a, step);
+  });
+  return out;
+}
+
+Tensor token_shift(Tensor h, Tensor mu, Tensor ring, OptT slots, OptT positions, OptT lens, int64_t start, bool decode) {
+  const auto dt = io_type(h);
+  check_io(mu, dt);
+  check_io(ring, dt);
+  CHK(h.dim() == 3 && mu.dim() == 2 && mu.size(1) == h.size(2));
+  const int B = h.size(0), S = h.size(1), D = h.size(2), n = mu.size(0);
+  CHK(ring.dim() == 3 && ring.size(1) >= 2 && ring.size(2) == D && (slots || B <= ring.size(0)) && (!decode || S == 1));
+  auto out = torch::empty({n, B, S, D}, h.options());
+  if (B == 0 || S == 0) return out;
+  const Step step = make_step(slots, positions, lens, start, decode, B);
+  BY_TYPE(dt, {
+    hipLaunchKernelGGL((token_shift_kernel<T>), dim3(S, B), dim3(256), 0, cur_stream(), P<T>(h), P<T>(mu), M<T>(ring),
+                       M<T>(out), S, D, (int)ring.size(1), n, (size_t)B * S * D, step);
+    if (!decode) remember<T>(h, ring, B, S, D, Columns{{0, 0, 0}, {D, 0, 0}}, step);
+  });
+  return out;
+}
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("prenorm", &prenorm, "RMS norm with a (1+w) weight of the fp32 stream");
+  m.def("sandwich_norm", &sandwich_norm, "stream += norm(y); norm of the stream for the next sublayer");
+  m.def("swiglu_packed", &swiglu_packed, "SwiGLU on a packed projection, any width, bf16 or fp32");
+  m.def("tanh", &tanh_op, "tanh with fp32 math");
+  m.def("window_attn", &window_attn, "sliding-window attention with distance bias, sink and head gates");
+  m.def("delta_rule", &delta_rule, "gated delta rule with short convolutions and per-channel decay");
+  m.def("wkv", &wkv, "decayed outer-product memory with a current-token bonus");
+  m.def("token_shift", &token_shift, "blends of the current and the previous token");
+}

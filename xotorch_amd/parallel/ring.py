@@ -24,7 +24,7 @@ from typing import List, Optional
 import torch
 import torch.distributed as dist
 
-from xotorch_amd.engine.kvcache import ShardKVCache
+from xotorch_amd.engine.kvcache import make_cache
 from xotorch_amd.models import model_class_for
 from xotorch_amd.models.config import ModelConfig, config_from_hf
 from xotorch_amd.models.registry import builtin_config
@@ -120,10 +120,13 @@ class RingPipeline:
     if device == "cuda":
       # decode-GEMM weight prepack (memory permitting; KV caches below still
       # need room — reserve their size + headroom before packing greedily)
-      kv_bytes = (
-        self.M * 2 * shards[rank].get_layer_count() * mb_batch * self.cfg.n_kv_heads
-        * self.total_len * self.cfg.head_dim * (2 if dtype == torch.bfloat16 else 4)
-      )
+      if self.cfg.layer_specs is not None:
+        kv_bytes = self.M * make_cache(self.cfg, self.shard, mb_batch, self.total_len, dtype, "meta").nbytes()
+      else:
+        kv_bytes = (
+          self.M * 2 * shards[rank].get_layer_count() * mb_batch * self.cfg.n_kv_heads
+          * self.total_len * self.cfg.head_dim * (2 if dtype == torch.bfloat16 else 4)
+        )
       if self.cfg.head_dim == 128 and dtype == torch.bfloat16 \
          and os.getenv("XOT_MFMA_ATTN", "1") == "1":
         kv_bytes *= 2  # the MFMA-packed cache copies double KV residency
@@ -133,19 +136,15 @@ class RingPipeline:
 
     # --- per-micro-batch state ---
     B = mb_batch
-    kv_heads, k_dim, v_dim = self.cfg.kv_cache_dims()
-    self.caches = [
-      ShardKVCache(self.shard.get_layer_count(), B, kv_heads, self.total_len,
-                   k_dim, dtype, device, v_dim=v_dim)
-      for _ in range(self.M)
-    ]
+    self.caches = [make_cache(self.cfg, self.shard, B, self.total_len, dtype, device) for _ in range(self.M)]
     self.positions = [torch.zeros(1, dtype=torch.int32, device=device) for _ in range(self.M)]
     self.seq_lens = [torch.zeros(B, dtype=torch.int32, device=device) for _ in range(self.M)]
     # static I/O buffers (graph + recv targets)
     self.tok_buf = [torch.zeros(B, 1, dtype=torch.int64, device=device) for _ in range(self.M)]
     D = self.cfg.dim
+    self.hid_dtype = getattr(model, "hidden_dtype", dtype)
     if not self.is_first:
-      self.hid_buf = [torch.zeros(B, 1, D, dtype=dtype, device=device) for _ in range(self.M)]
+      self.hid_buf = [torch.zeros(B, 1, D, dtype=self.hid_dtype, device=device) for _ in range(self.M)]
     self.hid_out: List[Optional[torch.Tensor]] = [None] * self.M
     # async handles
     self._tok_recv_req = [None] * self.M
@@ -217,6 +216,10 @@ class RingPipeline:
     outs = []
     for c0 in range(0, B, bc):
       c1 = min(c0 + bc, B)
+      if getattr(self.model, "slot_indexed", False):
+        rows = torch.arange(c0, c1, dtype=torch.int32, device=x.device)
+        outs.append(self.model(x[c0:c1], caches=self.caches[mb].caches, positions=pos, start_pos=start_pos, slots=rows))
+        continue
       sliced = []
       for layer in self.caches[mb].caches:
         if len(layer) > 2 and layer[2] is not None:
@@ -257,7 +260,7 @@ class RingPipeline:
             tokens = torch.randint(0, self.cfg.vocab_size, (B, S), generator=g).to(self.device)
           h = self._prefill_forward(mb, tokens, pos)
         else:
-          hbuf = torch.empty(B, S, self.cfg.dim, dtype=self.dtype, device=self.device)
+          hbuf = torch.empty(B, S, self.cfg.dim, dtype=self.hid_dtype, device=self.device)
           self.comm.recv(hbuf, self.prev_rank)
           h = self._prefill_forward(mb, hbuf, pos)
         if self.is_last:

@@ -14,13 +14,14 @@ RCCL/xGMI, and requests are served with SLOT-BASED CONTINUOUS BATCHING:
   the graph reads, so admission/release never re-captures);
 - prompt prefill is CHUNKED through the ring (stage 0 forwards sequence
   chunks so later stages overlap instead of idling through the whole
-  prompt — request-level TTFT);
+  prompt — request-level TTFT); prompts that are equally far run as one
+  padded batch where the model addresses slots by index;
 - rank 0 hosts the FULL ChatGPT-compatible API (the same ChatGPTAPI as the
   elastic Node path — models/topology/tinychat/encode routes included) via
   a thin Node adapter.
 
-Control plane per tick: rank 0 broadcasts a small header (op, slot, len,
-milli-temperature); ADMIT is followed by the prompt tokens; the last stage
+Control plane per tick: rank 0 broadcasts a small header (op, slot or slot
+bitmask, len or chunk start, milli-temperature); ADMIT is followed by the prompt tokens; the last stage
 samples and broadcasts the per-slot tokens; rank 0 streams them to clients.
 All collectives go through RingComm, so N ranks verify on fewer GPUs (gloo
 staging) while the real deployment runs pure RCCL.
@@ -45,9 +46,9 @@ if __package__ in (None, ""):  # torchrun launches this file by path
 import torch
 import torch.distributed as dist
 
-from xotorch_amd.engine.kvcache import ShardKVCache
+from xotorch_amd.engine.kvcache import make_cache
 from xotorch_amd.models.config import config_from_hf
-from xotorch_amd.models.registry import builtin_config, get_repo
+from xotorch_amd.models.registry import builtin_config, get_repo, register_local_model
 from xotorch_amd.models.weights import fast_random_init_gpu, load_shard_weights, random_init
 from xotorch_amd.parallel.comm import RingComm, init_distributed
 from xotorch_amd.parallel.ring import equal_ring_shards
@@ -93,7 +94,8 @@ class RingSlotWorker:
       raise ValueError(f"slots must be in [1, 63] (release op is an int64 bitmask), got {slots}")
     self.slots, self.max_seq = slots, max_seq
     self.use_graphs = use_graphs and device == "cuda"
-    self.cfg = config_from_hf(builtin_config(model_id) or {}, model_id)
+    own = Path(model_dir) / "config.json" if model_dir else None
+    self.cfg = config_from_hf(own if own is not None and own.exists() else builtin_config(model_id) or {}, model_id)
     self.max_seq = min(self.max_seq, self.cfg.max_seq_len)
     self.shard = equal_ring_shards(model_id, self.cfg.n_layers, world)[rank]
     from xotorch_amd.models import model_class_for
@@ -116,9 +118,12 @@ class RingSlotWorker:
     model.reset_rope()
     model.eval()
     self.model = model
-    heads, k_dim, v_dim = self.cfg.kv_cache_dims()
-    self.cache = ShardKVCache(self.shard.get_layer_count(), slots, heads,
-                              self.max_seq, k_dim, dtype, device, v_dim=v_dim)
+    self.cache = make_cache(self.cfg, self.shard, slots, self.max_seq, dtype, device)
+    # slot-indexed models address any set of slots in one step: their prompts
+    # prefill in batches of unequal length and parked slots are skipped;
+    # the others get views of one slot's cache rows
+    self.slot_indexed = getattr(model, "slot_indexed", False)
+    self.hid_dtype = getattr(model, "hidden_dtype", dtype)
     if device == "cuda":
       torch.cuda.empty_cache()
       model.pack_decode_weights(reserve_bytes=8 << 30)
@@ -134,7 +139,8 @@ class RingSlotWorker:
     self.positions = torch.zeros(slots, dtype=torch.int32, device=dev)
     self.seq_lens = torch.ones(slots, dtype=torch.int32, device=dev)
     self.tok_buf = torch.zeros(slots, 1, dtype=torch.int64, device=dev)
-    self.hid_buf = torch.zeros(slots, 1, D, dtype=dtype, device=dev)
+    self.hid_buf = torch.zeros(slots, 1, D, dtype=self.hid_dtype, device=dev)
+    self.slot_map = torch.full((slots,), -1, dtype=torch.int32, device=dev)  # -1: parked
     self.logits_buf: Optional[torch.Tensor] = None
     self.hid_out: Optional[torch.Tensor] = None
     # control/broadcast buffers
@@ -151,8 +157,9 @@ class RingSlotWorker:
 
   def _decode_forward(self):
     x = self.tok_buf if self.is_first else self.hid_buf
+    kw = {"slots": self.slot_map} if self.slot_indexed else {}
     out = self.model(x, caches=self.cache.caches, positions=self.positions,
-                     start_pos=-1, is_decode=True, seq_lens=self.seq_lens)
+                     start_pos=-1, is_decode=True, seq_lens=self.seq_lens, **kw)
     if self.is_last:
       if self.logits_buf is None:
         self.logits_buf = torch.empty_like(out)
@@ -190,19 +197,26 @@ class RingSlotWorker:
     can take garbage writes without ever clobbering real prefill data
     (prerequisite for interleaving chunked prefill with decode ticks)."""
     idle = [i for i in range(self.slots) if not self.active[i]]
+    if self.slot_indexed:
+      self.slot_map.copy_(torch.tensor([i if on else -1 for i, on in enumerate(self.active)], dtype=torch.int32))
     if idle:
       idx = torch.tensor(idle, dtype=torch.int64, device=self.positions.device)
       self.positions[idx] = self.max_seq - 1
       self.seq_lens[idx] = 1
 
+  def run_decode(self):
+    """This rank's part of a decode tick: every active slot one token on
+    (tokens in tok_buf, logits to logits_buf), nothing sampled."""
+    if self._graph is not None:
+      self._graph.replay()
+    else:
+      self._decode_forward()
+
   def decode_tick(self):
     with torch.inference_mode():
       if not self.is_first and self.world > 1:
         self.comm.recv(self.hid_buf, self.prev_rank)
-      if self._graph is not None:
-        self._graph.replay()
-      else:
-        self._decode_forward()
+      self.run_decode()
       if not self.is_last and self.world > 1:
         self.comm.send(self.hid_out, self.next_rank)
       if self.is_last:
@@ -235,46 +249,75 @@ class RingSlotWorker:
       out.append(type(layer)(*sl) if hasattr(layer, "_fields") else sl)
     return out
 
-  def _prefill_chunk(self, slot: int, caches, tokens, c0: int, c1: int,
-                     plen: int) -> Optional[int]:
-    """One prompt chunk through this rank's layers; returns the first
-    sampled token on the last stage of the last chunk, else None."""
+  def _prefill_hidden(self, group: List[int], c0: int, last_only: bool = True) -> torch.Tensor:
+    """The chunk that starts at c0 of the prompts in `group` through this
+    rank's layers, as one batch (slot-indexed models; else one prompt).
+    Shorter rows are padded at the end. Returns logits on the last stage."""
     dev = self.device
+    pfs = [self._pf[i] for i in group]
+    lens = [min(PREFILL_CHUNK, pf["plen"] - c0) for pf in pfs]
+    S = max(lens)
+    kw = {}
+    if self.slot_indexed:
+      caches = self.cache.caches
+      kw["slots"] = torch.tensor(group, dtype=torch.int32, device=dev)
+      if min(lens) < S:
+        kw["lens"] = torch.tensor(lens, dtype=torch.int32, device=dev)
+    else:
+      (slot,) = group
+      caches = self._pf[slot]["caches"]
+    pos = torch.arange(c0, c0 + S, dtype=torch.int32, device=dev)
+    if self.is_first:
+      x = torch.zeros(len(group), S, dtype=torch.int64, device=dev)
+      for row, (pf, n) in enumerate(zip(pfs, lens)):
+        x[row, :n] = pf["toks"][0, c0:c0 + n]
+    else:
+      x = torch.empty(len(group), S, self.cfg.dim, dtype=self.hid_dtype, device=dev)
+      self.comm.recv(x, self.prev_rank)
+    return self.model(x, caches=caches, positions=pos, start_pos=c0, last_only=last_only, **kw)
+
+  def _prefill_group(self, group: List[int], c0: int) -> Dict[int, int]:
+    """One chunk of the prompts in `group`; returns the first sampled token of
+    every prompt that ends with it (last stage only)."""
     with torch.inference_mode():
-      pos = torch.arange(c0, c1, dtype=torch.int32, device=dev)
-      if self.is_first:
-        x = tokens[:, c0:c1].to(dev)
-        h = self.model(x, caches=caches, positions=pos, start_pos=c0)
-      else:
-        hbuf = torch.empty(1, c1 - c0, self.cfg.dim, dtype=self.dtype, device=dev)
-        self.comm.recv(hbuf, self.prev_rank)
-        h = self.model(hbuf, caches=caches, positions=pos, start_pos=c0)
+      h = self._prefill_hidden(group, c0)
       if not self.is_last:
         if self.world > 1:
           self.comm.send(h.contiguous(), self.next_rank)
-        return None
-      if c1 != plen:
-        return None
-      st = self.slot_state[slot]
-      logits = h[:, -1] if h.dim() == 3 else h
-      if st.temp > 0:
-        from xotorch_amd import ops
-        return int(ops.softmax_sample(logits, temperature=st.temp, top_k=35)[0])
-      return int(logits.argmax(dim=-1)[0])
+        return {}
+      first = {}
+      for row, slot in enumerate(group):
+        if c0 + PREFILL_CHUNK < self._pf[slot]["plen"]:
+          continue
+        logits = h[row:row + 1, -1] if h.dim() == 3 else h[row:row + 1]
+        st = self.slot_state[slot]
+        if st.temp > 0:
+          from xotorch_amd import ops
+          first[slot] = int(ops.softmax_sample(logits, temperature=st.temp, top_k=35)[0])
+        else:
+          first[slot] = int(logits.argmax(dim=-1)[0])
+      return first
 
-  def prefill_slot(self, slot: int, tokens: Optional[torch.Tensor], plen: int) -> Optional[int]:
-    """Run the whole prompt through the ring in chunks (non-interleaved
-    path, used when the ring has nothing decoding)."""
-    caches = self._slot_caches(slot)
-    first_tok = None
-    for c0 in range(0, plen, PREFILL_CHUNK):
-      c1 = min(c0 + PREFILL_CHUNK, plen)
-      tok = self._prefill_chunk(slot, caches, tokens, c0, c1, plen)
-      if tok is not None:
-        first_tok = tok
+  def _begin_prefill(self, slot: int, toks: torch.Tensor):
+    """Hand a prompt [1, S] to a free slot; its chunks run in later ticks."""
+    self._pf[slot] = {"toks": toks, "c0": 0, "plen": toks.shape[1],
+                      "caches": None if self.slot_indexed else self._slot_caches(slot)}
+
+  def _activate(self, slot: int):
+    """A slot whose prompt is in the cache joins the decode ticks."""
+    plen = self._pf.pop(slot)["plen"]
     self.positions[slot] = plen
     self.seq_lens[slot] = plen + 1
-    return first_tok
+    self.slot_map[slot] = slot
+    self.active[slot] = True
+
+  def _release(self, slots: List[int]):
+    """Give slots back; they are parked until their next prompt."""
+    for i in slots:
+      self.active[i] = False
+      self.slot_state[i] = SlotState()
+      self._pf.pop(i, None)
+    self._reset_inactive()
 
   def _log_done(self, st: SlotState):
     dt = max(1e-9, time.perf_counter() - st.t_admit)
@@ -345,10 +388,11 @@ class RingSlotWorker:
           elif self._pf and (self._pf_turn or not any(self.active)):
             # alternate one prompt chunk with one decode tick so slots that
             # are already generating keep emitting during long prefills
-            slot = max(self._pf, key=lambda i: self._pf[i]["c0"])  # finish-first
-            pf = self._pf[slot]
-            op, plen = OP_PREFILL, pf["c0"]
-            extra = min(pf["c0"] + PREFILL_CHUNK, pf["plen"])
+            lead = max(self._pf, key=lambda i: self._pf[i]["c0"])  # finish-first
+            op, plen = OP_PREFILL, self._pf[lead]["c0"]
+            # prompts that are equally far go together where the model can
+            group = [i for i in self._pf if self._pf[i]["c0"] == plen] if self.slot_indexed else [lead]
+            slot = sum(1 << i for i in group)
             self._pf_turn = False
           elif any(self.active):
             op = OP_DECODE
@@ -369,12 +413,7 @@ class RingSlotWorker:
           time.sleep(min(idle_sleep * (1 + idle_ticks // 50), 0.05))
         continue
       if op == OP_RELEASE:
-        for i in range(self.slots):
-          if slot & (1 << i):
-            self.active[i] = False
-            self.slot_state[i] = SlotState()
-            self._pf.pop(i, None)
-        self._reset_inactive()
+        self._release([i for i in range(self.slots) if slot & (1 << i)])
         continue
       if op == OP_ADMIT:
         if self.rank == 0:
@@ -386,8 +425,7 @@ class RingSlotWorker:
           self.comm.broadcast(toks, 0)
         st = SlotState(prompt_len=plen, temp=extra / 1000.0)
         self.slot_state[slot] = st
-        self._pf[slot] = {"toks": toks, "c0": 0, "plen": plen,
-                          "caches": self._slot_caches(slot)}
+        self._begin_prefill(slot, toks)
         if self.rank == 0:
           msg = inflight.pop(slot)
           st.request_id = msg.request_id
@@ -395,36 +433,38 @@ class RingSlotWorker:
           st.t_admit = msg.t_submit
         continue
       if op == OP_PREFILL:
-        c0, c1 = plen, extra
-        pf = self._pf[slot]
-        first = self._prefill_chunk(slot, pf["caches"], pf["toks"], c0, c1, pf["plen"])
-        pf["c0"] = c1
-        if c1 < pf["plen"]:
+        group = [i for i in range(self.slots) if slot & (1 << i)]
+        first = self._prefill_group(group, plen)
+        done = []
+        for i in group:
+          self._pf[i]["c0"] = plen + PREFILL_CHUNK
+          if self._pf[i]["c0"] >= self._pf[i]["plen"]:
+            done.append(i)
+        if not done:
           continue
-        # last chunk: activate the slot and ship the first token to rank 0
-        del self._pf[slot]
-        self.positions[slot] = pf["plen"]
-        self.seq_lens[slot] = pf["plen"] + 1
+        # last chunk: activate the slots and ship the first tokens to rank 0
         self.tok_bcast.zero_()
-        if self.is_last and first is not None:
-          self.tok_bcast[slot] = first
+        for i, tok in first.items():
+          self.tok_bcast[i] = tok
         if self.world > 1:
           self.comm.broadcast(self.tok_bcast, self.world - 1)
-        if self.is_first:
-          self.tok_buf[slot, 0] = self.tok_bcast[slot]
-        self.active[slot] = True
-        if self.rank == 0:
-          st = self.slot_state[slot]
+        for i in done:
+          self._activate(i)
+          if self.is_first:
+            self.tok_buf[i, 0] = self.tok_bcast[i]
+          if self.rank != 0:
+            continue
+          st = self.slot_state[i]
           st.generated = 1
           st.ttft_s = time.perf_counter() - st.t_admit
-          tok = int(self.tok_bcast[slot])
+          tok = int(self.tok_bcast[i])
           fin = (self.eos_token_id is not None and tok == self.eos_token_id) or st.generated >= st.max_new
           if emit:
             emit(st.request_id, tok, fin, {"ttft_s": st.ttft_s})
           if fin:
             st.done = True
             self._log_done(st)
-            pending_release.append(slot)
+            pending_release.append(i)
         continue
       # OP_DECODE
       self.decode_tick()
@@ -525,6 +565,8 @@ def main():
   p.add_argument("--slots", type=int, default=SLOTS)
   p.add_argument("--no-graphs", action="store_true")
   args = p.parse_args()
+  if args.model_dir:
+    register_local_model(args.model, args.model_dir)  # the API resolves models by card
   rank, world = init_distributed()
   device = "cuda" if torch.cuda.is_available() else "cpu"
   dtype = torch.bfloat16 if device == "cuda" else torch.float32

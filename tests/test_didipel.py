@@ -1,0 +1,768 @@
+"""Didipel: every mechanism alone, the model through its cache, and serving,
+against the plain functions of didipel_oracle.py. CPU runs take the torch
+path in 32-bit, GPU runs the HIP kernels in 32-bit and bfloat16."""
+import asyncio
+import io
+import json
+import queue
+import threading
+
+import numpy as np
+import pytest
+import torch
+
+import didipel_cases as cases
+import didipel_oracle as oracle
+from xotorch_amd.engine.kvcache import make_cache
+from xotorch_amd.models.config import config_from_hf
+from xotorch_amd.models.mixers import GatedDeltaRule, WindowBiasAttention, distance_buckets
+from xotorch_amd.ops import mixer_ops as mo
+
+F32, BF16 = torch.float32, torch.bfloat16
+KINDS = [
+  pytest.param(("cpu", F32), id="cpu-f32"),
+  pytest.param(("cuda", F32), id="gpu-f32", marks=pytest.mark.gpu),
+  pytest.param(("cuda", BF16), id="gpu-bf16", marks=pytest.mark.gpu),
+]
+on = pytest.mark.parametrize("kind", KINDS)
+
+
+def close(got, want, dtype, scale=1.0):
+  """Rounding-sized differences only, against the typical size of the expected
+  values: on average, and for the worst element."""
+  got, want = got.detach().cpu().double(), want.double()
+  assert torch.isfinite(got).all()
+  size = max(want.pow(2).mean().sqrt().item(), 1e-6)
+  mean_tol, worst_tol = (1e-2, 8e-2) if dtype == BF16 else (1e-5, 5e-5)
+  err = (got - want).abs()
+  mean, worst = err.pow(2).mean().sqrt().item() / size, err.max().item() / size
+  assert mean <= mean_tol * scale and worst <= worst_tol * scale, f"error {mean:.2e}, worst {worst:.2e}"
+
+
+def rnd(*shape, seed=0, scale=1.0):
+  """Random values that bfloat16 holds exactly."""
+  g = torch.Generator().manual_seed(seed)
+  return (torch.randn(*shape, generator=g) * scale).to(BF16).double()
+
+
+def rows(kind, decode=False, start=0, positions=None, slots=None, lens=None):
+  def dev(t):
+    return None if t is None else torch.tensor(t, dtype=torch.int32, device=kind[0])
+  return mo.StepRows(decode, start, dev(positions), dev(slots), dev(lens))
+
+
+def on_device(kind, *tensors):
+  return [t.to(device=kind[0], dtype=kind[1]) for t in tensors]
+
+
+def state_of(cls, p, kind, slots=3, capacity=512):
+  return tuple(torch.zeros(slots, *shape, dtype=dt, device=kind[0])
+               for shape, dt in cls.state_spec(p, capacity, kind[1], kind[0]).values())
+
+
+# ---------------------------------------------------------------- mechanisms
+
+@on
+@pytest.mark.parametrize("D", [72, 257, 1024, 5000])
+def test_norms(kind, D):
+  x, y, a, b = rnd(3, 2, D), rnd(3, 2, D, seed=1, scale=3), rnd(D, seed=2, scale=.3), rnd(D, seed=3, scale=.3)
+  xd = x.to(kind[0], F32)
+  yd, ad, bd = on_device(kind, y, a, b)
+  close(mo.prenorm(xd, ad, 1e-5, kind[1]), oracle.norm_one_plus(x, a, 1e-5), kind[1])
+  want = x + oracle.norm_one_plus(y, a, 1e-5)
+  got, h = mo.sandwich_norm(yd, xd.clone(), ad, bd, 1e-5)
+  assert got.dtype == F32 and h.dtype == kind[1]
+  close(got, want, F32)
+  close(h, oracle.norm_one_plus(want, b, 1e-5), kind[1])
+  got, h = mo.sandwich_norm(yd, xd.clone(), ad, None, 1e-5)
+  assert h is None
+  close(got, want, F32)
+
+
+@on
+@pytest.mark.parametrize("width", [56, 33])
+def test_elementwise(kind, width):
+  gu = rnd(2, 5, 2 * width, scale=2)
+  (d,) = on_device(kind, gu)
+  close(mo.swiglu_packed(d), oracle.silu(gu[..., :width]) * gu[..., width:], kind[1])
+  close(mo.tanh(d), torch.tanh(gu), kind[1])
+
+
+@pytest.mark.parametrize("n,far", [(8, 17), (16, 200), (32, 128), (4, 1000), (16, 128)])
+def test_distance_buckets(n, far):
+  got = distance_buckets(n, far, 3 * far)
+  assert got.tolist() == [oracle.distance_bucket(d, n, far) for d in range(3 * far)]
+  assert got[-1] == n - 1 and got[far] == n - 1
+
+
+def test_distance_bucket_edges_are_exact():
+  # 8 log steps over a factor 16: each doubling is two buckets, to the token
+  got = distance_buckets(16, 128, 129).tolist()
+  assert [got[n] for n in (15, 16, 31, 32, 63, 64, 127, 128)] == [9, 10, 11, 12, 13, 14, 15, 15]
+
+
+ATTN = [  # heads, kv_heads, dim, vdim, window, far
+  (6, 2, 20, 12, 11, 17),
+  (4, 4, 64, 64, 33, 9),
+  (8, 1, 128, 96, 64, 400),
+  (20, 1, 32, 48, 40, 30),   # more query heads on one key head than a tile holds
+  (2, 1, 256, 256, 70, 50),
+  (3, 3, 40, 8, 1, 5),       # sees itself only
+]
+
+
+class Attention:
+  """One window-attention op with its inputs for T tokens."""
+
+  def __init__(self, kind, shape, T, seed=0):
+    self.kind, self.T = kind, T
+    H, G, d, e, W, far = self.shape = shape
+    self.at = [0, 8 + H * d, 16 + (H + G) * d, 24 + (H + G) * d + G * e]  # parts with gaps
+    self.N = self.at[3] + H + 5
+    self.proj = rnd(T, self.N, seed=seed, scale=1.5)
+    self.qn, self.kn = rnd(H * d, seed=1) * .2 + 1, rnd(G * d, seed=2) * .2 + 1
+    self.qn, self.kn = self.qn.to(BF16).double(), self.kn.to(BF16).double()
+    self.rel = rnd(8, H, seed=3)
+    self.scale = 1.5 / d ** .5
+    self.bucket = distance_buckets(8, far, min(W, far + 1)).to(kind[0])
+
+  def parts(self):
+    H, G, d, e, _, _ = self.shape
+    q, k, v, g = (self.proj[:, a:a + n] for a, n in zip(self.at, (H * d, G * d, G * e, H)))
+    q, k = oracle.rms(q, 1e-5) * self.qn, oracle.rms(k, 1e-5) * self.kn
+    return q.view(-1, H, d), k.view(-1, G, d), v.view(-1, G, e), g
+
+  def expected(self):
+    H, G, d, e, W, far = self.shape
+    q, k, v, g = self.parts()
+    bias = torch.stack([self.rel[oracle.distance_bucket(n, 8, far)] for n in range(min(W, self.T))])
+    o = oracle.window_attention(q, k, v, bias, self.scale, W)
+    return .7 * (o * oracle.sigmoid(g)[:, :, None]).reshape(self.T, H * e)
+
+  def state(self, slots=3, capacity=512):
+    H, G, d, e, W, _ = self.shape
+    return state_of(WindowBiasAttention, {"kv_heads": G, "dim": d, "vdim": e, "mask": {"size": W}}, self.kind,
+                    slots, capacity)
+
+  def __call__(self, x, state, step):
+    H, G, d, e, W, _ = self.shape
+    qn, kn, rel = on_device(self.kind, self.qn, self.kn, self.rel)
+    (x,) = on_device(self.kind, x)
+    out = None
+    if x.is_cuda:  # columns of a wider tensor
+      out = torch.full((*x.shape[:2], 16 + H * e), 9.0, dtype=x.dtype, device=x.device)
+      out = torch.nn.functional.pad(out, (0, -out.shape[2] % 4)).contiguous()
+    y = mo.window_attn(x, self.at, H, G, d, e, qn, kn, self.bucket, rel, self.scale, 1e-5, W, state, step,
+                       out=out, out_at=8 if x.is_cuda else 0, out_scale=.7)
+    if x.is_cuda:
+      assert (y[..., :8] == 9).all() and (y[..., 8 + H * e:16 + H * e] == 9).all()
+      y = y[..., 8:8 + H * e]
+    return y.cpu().double()
+
+  def decode(self, state, slot, first, n):
+    outs = []
+    for t in range(first, first + n):
+      outs.append(self(self.proj[None, t:t + 1], state, rows(self.kind, True, positions=[t], slots=[slot]))[0])
+    return torch.cat(outs)
+
+
+@on
+@pytest.mark.parametrize("shape", ATTN)
+def test_window_attention_prompt_portions_and_decode(kind, shape):
+  a = Attention(kind, shape, 150)
+  want = a.expected()
+  close(a(a.proj[None], a.state(), rows(kind))[0], want, kind[1])
+  state, outs, p = a.state(), [], 0
+  for n in (1, 2, 40, 3, 64):
+    outs.append(a(a.proj[None, p:p + n], state, rows(kind, start=p, slots=[2]))[0])
+    p += n
+  outs.append(a.decode(state, 2, p, 150 - p))
+  close(torch.cat(outs), want, kind[1])
+
+
+@on
+@pytest.mark.parametrize("shape", [(4, 2, 32, 32, 37, 20), (2, 2, 128, 128, 300, 64)])
+@pytest.mark.parametrize("query", [40, 63, 64, 137, 330])
+def test_window_edge_shows(kind, shape, query):
+  """A key that outweighs all others counts at distance window-1 and is gone
+  at distance window, in a prompt, after a cut and decoded."""
+  H, G, d, e, W, far = shape
+  T = 340
+  for age in (0, W - 1, W, W + 1):
+    if query - age < 0:
+      continue
+    a = Attention(kind, shape, T)
+    qa, ka, va, ga = a.at
+    a.proj[:, qa:qa + H * d] = a.proj[:, qa:qa + H * d] * .1
+    a.proj[query, qa:qa + H * d] = 4.0
+    a.proj[query - age, ka:ka + G * d] = 4.0
+    a.scale = 1.0
+    want = a.expected()[query]
+    alone = (.7 * oracle.sigmoid(a.proj[query, ga:ga + H])[:, None]
+             * a.proj[query - age, va:va + G * e].view(G, e).repeat_interleave(H // G, 0)).reshape(-1)
+    assert ((want - alone).abs().max() < 1e-2) == (age < W)
+    close(a(a.proj[None, :query + 1], a.state(), rows(kind))[0, query], want, kind[1])
+    state = a.state()
+    a(a.proj[None, :query - 1], state, rows(kind, slots=[1]))
+    cut = [t.clone() for t in state]
+    close(a(a.proj[None, query - 1:query + 1], cut, rows(kind, start=query - 1, slots=[1]))[0, 1], want, kind[1])
+    close(a.decode(state, 1, query - 1, 2)[1], want, kind[1])
+
+
+@on
+def test_sink_takes_its_share(kind):
+  """Scores far below zero leave everything to the sink: outputs vanish; at
+  score zero it weighs as much as one token."""
+  a = Attention(kind, (2, 1, 32, 16, 8, 5), 6)
+  qa, ka, va, ga = a.at
+  a.qn, a.kn = torch.ones(64).double(), torch.ones(32).double()
+  a.rel = torch.zeros(8, 2).double()
+  a.proj[:, qa:qa + 64], a.proj[:, ka:ka + 32] = 1.0, -1.0
+  a.scale = 2.0
+  assert a(a.proj[None], a.state(), rows(kind)).abs().max() < 1e-6
+  assert a.decode(a.state(), 0, 0, 6).abs().max() < 1e-6
+  a.scale = 0.0
+  got, v = a.decode(a.state(), 0, 0, 6), a.proj[:, va:va + 16]
+  want = torch.stack([v[:t + 1].sum(0) / (t + 2) for t in range(6)]).repeat(1, 2)
+  gate = oracle.sigmoid(a.proj[:, ga:ga + 2]).repeat_interleave(16, 1)
+  close(got, .7 * want * gate, kind[1])
+
+
+@on
+def test_attention_rows_are_independent(kind):
+  """Unequal lengths in one step, arbitrary slots, a parked row in between,
+  ragged decode positions."""
+  a = Attention(kind, (6, 2, 64, 40, 21, 30), 90)
+  b = Attention(kind, (6, 2, 64, 40, 21, 30), 90, seed=7)
+  state = a.state(slots=4)
+  for t in state:
+    t.fill_(3.0)
+  before = [t[0].clone() for t in state]
+  both = torch.stack([a.proj[:70], b.proj[:70], b.proj[:70]])
+  got = a(both, state, rows(kind, slots=[3, -1, 1], lens=[5, 70, 70]))
+  close(got[0, :5], a.expected()[:5], kind[1])
+  assert (got[1] == 0).all() and (got[0, 5:] == 0).all()
+  close(got[2], b.expected()[:70], kind[1])
+  for i in range(12):
+    x = torch.stack([b.proj[70 + i:71 + i], a.proj[:1], a.proj[5 + i:6 + i]])
+    got = a(x, state, rows(kind, True, positions=[70 + i, 0, 5 + i], slots=[1, -1, 3]))
+    close(got[0, 0], b.expected()[70 + i], kind[1])
+    assert (got[1] == 0).all()
+    close(got[2, 0], a.expected()[5 + i], kind[1])
+  assert all((t[0] == u).all() for t, u in zip(state, before))
+
+
+REC = [(4, 2, 12, 20, 4), (3, 3, 40, 16, 2), (2, 1, 64, 64, 3), (1, 1, 128, 128, 1), (2, 2, 90, 33, 4), (2, 2, 256, 200, 3)]
+
+
+class Delta:
+  def __init__(self, kind, shape, T, seed=0):
+    self.kind, self.T = kind, T
+    H, G, d, e, taps = self.shape = shape
+    self.at = [8, 16 + G * d, 24 + 2 * G * d, 32 + 2 * G * d + H * e]
+    self.proj = rnd(T, self.at[3] + H + 3, seed=seed)
+    self.convs = [rnd(n, taps, seed=i, scale=.6) for i, n in enumerate((G * d, G * d, H * e))]
+    self.pre, self.gate = rnd(T, H * d, seed=seed + 11), rnd(T, H * e, seed=12)
+    self.a_log, self.dt = rnd(H, seed=13, scale=.7), rnd(H * d, seed=14, scale=1.5) - 2
+    self.dt = self.dt.to(BF16).double()
+    self.norm = (rnd(e, seed=15, scale=.2) + 1).to(BF16).double()
+
+  def expected(self):
+    H, G, d, e, _ = self.shape
+    T = self.T
+    q, k, v = (oracle.silu(oracle.causal_conv(self.proj[:, a:a + c.shape[0]], c)) for a, c in zip(self.at, self.convs))
+    q, k = oracle.unit(q.view(T, G, d)) * d ** -.5, oracle.unit(k.view(T, G, d))
+    g = torch.exp(-torch.exp(self.a_log)[None, :, None] * oracle.softplus(self.pre + self.dt).view(T, H, d))
+    beta = oracle.sigmoid(self.proj[:, self.at[3]:self.at[3] + H])
+    o = oracle.rms(oracle.delta_scan(q, k, v.view(T, H, e), g, beta), 1e-5) * self.norm
+    return 1.3 * (o * oracle.sigmoid(self.gate).view(T, H, e)).reshape(T, H * e)
+
+  def state(self, slots=3):
+    H, G, d, e, taps = self.shape
+    return state_of(GatedDeltaRule, {"heads": H, "kv_heads": G, "dim": d, "vdim": e, "conv": taps}, self.kind, slots)
+
+  def __call__(self, lo, hi, state, step, pad=0):
+    H, G, d, e, _ = self.shape
+    x, pre, gate, a_log, dt, norm, *convs = on_device(
+      self.kind, self.proj[None, lo:hi], self.pre[None, lo:hi], self.gate[None, lo:hi], self.a_log, self.dt, self.norm,
+      *self.convs)
+    return mo.delta_rule(x, self.at, H, G, d, e, convs, pre, gate, a_log, dt, norm, 1e-5, state, step,
+                         out_scale=1.3)[0].cpu().double()
+
+
+def run_cut(op, kind, T, cuts, slot=2):
+  state, outs, p = op.state(), [], 0
+  for t in state:
+    t.fill_(2.0)  # what an earlier sequence left: a new one must not see it
+  for n in cuts:
+    outs.append(op(p, p + n, state, rows(kind, start=p, slots=[slot])))
+    p += n
+  while p < T:
+    outs.append(op(p, p + 1, state, rows(kind, True, positions=[p], slots=[slot])))
+    p += 1
+  assert all((t[0] == 2.0).all() for t in state)
+  return torch.cat(outs)
+
+
+@on
+@pytest.mark.parametrize("shape", REC)
+def test_delta_rule(kind, shape):
+  T = 60
+  op = Delta(kind, shape, T)
+  want = op.expected()
+  close(op(0, T, op.state(), rows(kind)), want, kind[1])
+  for cuts in ((50,), (2, 3, 1, 16, 17), (1, 2), ()):
+    close(run_cut(op, kind, T, cuts), want, kind[1])
+
+
+class Wkv:
+  def __init__(self, kind, H, d, T):
+    self.kind, self.H, self.d, self.T = kind, H, d, T
+    self.r, self.k, self.v, self.gate, self.pre = (rnd(T, H * d, seed=i) for i in range(5))
+    self.w0, self.u = rnd(H * d, seed=6, scale=1.5) - 2, rnd(H * d, seed=7, scale=.7)
+    self.w0 = self.w0.to(BF16).double()
+    self.norm = (rnd(H * d, seed=8, scale=.2) + 1).to(BF16).double()
+
+  def expected(self):
+    T, H, d = self.T, self.H, self.d
+    w = torch.exp(-torch.exp(self.pre + self.w0)).view(T, H, d)
+    o = oracle.wkv_scan(self.r.view(T, H, d), self.k.view(T, H, d), self.v.view(T, H, d), w, self.u.view(H, d))
+    return oracle.rms(o, 1e-5).reshape(T, H * d) * self.norm * oracle.silu(self.gate)
+
+  def state(self, slots=3):
+    return (torch.zeros(slots, self.H, self.d, mo.row_pad(self.d), device=self.kind[0]),)
+
+  def __call__(self, lo, hi, state, step):
+    x = on_device(self.kind, *(t[None, lo:hi] for t in (self.r, self.k, self.v, self.gate, self.pre)))
+    w = on_device(self.kind, self.w0, self.u, self.norm)
+    return mo.wkv(*x, *w, self.H, self.d, 1e-5, state[0], step)[0].cpu().double()
+
+
+@on
+@pytest.mark.parametrize("H,d", [(3, 28), (2, 64), (1, 128), (2, 18), (1, 250)])
+def test_wkv(kind, H, d):
+  T = 60
+  op = Wkv(kind, H, d, T)
+  want = op.expected()
+  close(op(0, T, op.state(), rows(kind)), want, kind[1])
+  for cuts in ((50,), (2, 3, 1, 16, 17), (1, 2), ()):
+    close(run_cut(op, kind, T, cuts), want, kind[1])
+
+
+@on
+def test_token_shift(kind):
+  T, D = 20, 36
+  h, mu = rnd(T, D), rnd(5, D, seed=1, scale=.5)
+  before = torch.cat([torch.zeros(1, D).double(), h[:-1]])
+  want = torch.stack([h + (before - h) * m for m in mu])
+  hd, mud = on_device(kind, h[None], mu)
+  for cuts in ((20,), (1, 2, 2, 4, 3), (2,), ()):
+    ring, outs, p = torch.full((2, 2, D), 5.0, dtype=kind[1], device=kind[0]), [], 0
+    for n in cuts:
+      outs.append(mo.token_shift(hd[:, p:p + n].contiguous(), mud, ring, rows(kind, start=p, slots=[1])))
+      p += n
+    while p < T:
+      outs.append(mo.token_shift(hd[:, p:p + 1].contiguous(), mud, ring, rows(kind, True, positions=[p], slots=[1])))
+      p += 1
+    close(torch.cat(outs, dim=2)[:, 0], want, kind[1])
+    assert (ring[0] == 5).all()
+
+
+# ---------------------------------------------------------------- model
+
+def variants():
+  one = cases.small(width=40, vocab=37, layers=[
+    {"type": "parallel", "mlp": None, "mixer": {
+      "left": {"heads": 1, "kv_heads": 1, "dim": 16, "vdim": 16, "scale": 1.0, "bias_max": 6, "mask": {"size": 1}},
+      "right": {"heads": 1, "kv_heads": 1, "dim": 16, "vdim": 16, "conv": 1},
+      "left_scale": 1.0, "right_scale": 1.0}},
+    {"type": "wkv", "mlp": {"kind": "dense", "ff": 24}, "mixer": {"heads": 1, "dim": 40}}])
+  wkv_first = cases.small(norm={"eps": 1e-3})
+  wkv_first["layers"] = wkv_first["layers"][::-1]
+  return {"base": cases.small(), "ones": one, "reversed": wkv_first}
+
+
+@pytest.fixture(scope="module")
+def checkpoints(tmp_path_factory):
+  out = {}
+  for name, cfg in variants().items():
+    w = cases.random_weights(cfg, seed=len(name))
+    out[name] = (cases.write_checkpoint(tmp_path_factory.mktemp("didipel") / name, cfg, w), cfg, w)
+  return out
+
+
+TOKENS = torch.randint(0, 37, (90,), generator=torch.Generator().manual_seed(3))
+
+
+@pytest.fixture(scope="module")
+def references(checkpoints):
+  found = {}
+
+  def get(name, tokens):
+    key = (name, tuple(int(t) for t in tokens))
+    if key not in found:
+      folder, cfg, w = checkpoints[name]
+      found[key] = oracle.forward(list(key[1]), w, cfg)
+    return found[key]
+  return get
+
+
+class Session:
+  """A model with a cache of a few slots, stepped by hand."""
+
+  def __init__(self, kind, folder, slots=4, capacity=200, layers=None):
+    self.kind, self.model = kind, cases.load_model(folder, *kind, layers=layers)
+    self.cache = make_cache(self.model.cfg, self.model.shard, slots, capacity, kind[1], kind[0])
+
+  @torch.inference_mode()
+  def prompt(self, prompts, start=0, slots=None, **kw):
+    S = max(len(p) for p in prompts)
+    x = torch.stack([torch.nn.functional.pad(p, (0, S - len(p))) for p in prompts]).to(self.kind[0])
+    r = rows(self.kind, slots=slots, lens=[len(p) for p in prompts])
+    return self.model(x, self.cache.caches, torch.arange(start, start + S), start, slots=r.slots,
+                      lens=r.lens, **{"last_only": False, **kw}).cpu().double()
+
+  @torch.inference_mode()
+  def decode(self, tokens, positions, slots=None):
+    r = rows(self.kind, True, positions=positions, slots=slots)
+    x = torch.tensor(tokens).view(-1, 1).to(self.kind[0])
+    return self.model(x, self.cache.caches, r.positions, -1, is_decode=True, slots=r.slots).cpu().double()
+
+
+@on
+@pytest.mark.parametrize("name", ["base", "ones", "reversed"])
+def test_model_whole_cut_and_decoded(kind, name, checkpoints, references):
+  want = references(name, TOKENS)
+  s = Session(kind, checkpoints[name][0])
+  close(s.prompt([TOKENS])[0], want, kind[1], 3)
+  for cuts in ((2,), (2,) * 10, (33, 1, 31), (1,)):  # the rest token by token: several windows long
+    outs, p = [], 0
+    for n in cuts:
+      outs.append(s.prompt([TOKENS[p:p + n]], p, [2])[0])
+      p += n
+    for t in range(p, len(TOKENS)):
+      outs.append(s.decode([TOKENS[t]], [t], [2]))
+    close(torch.cat(outs), want, kind[1], 3)
+
+
+@on
+def test_layers_one_by_one(kind, checkpoints):
+  folder, cfg, w = checkpoints["base"]
+  want, got = [], []
+  oracle.forward(TOKENS[:30].tolist(), w, cfg, layers_out=want)
+  s = Session(kind, folder)
+  s.prompt([TOKENS[:30]], layers_out=got)
+  assert len(got) == len(want) == 4
+  for g, x in zip(got, want):
+    close(g[0], x, kind[1], 2)
+
+
+@on
+def test_batch_of_unequal_requests_and_slots_used_again(kind, checkpoints, references):
+  s = Session(kind, checkpoints["base"][0])
+  lens = [1, 40, 7]
+  reqs = [TOKENS[:1], TOKENS[10:50], TOKENS[60:67]]
+  follow = [TOKENS[20:45], TOKENS[50:75], TOKENS[:25]]
+  full = [torch.cat([a, b]) for a, b in zip(reqs, follow)]
+  want = [references("base", f) for f in full]
+  for slots in ([3, 0, 1], [0, 1, 3], [1, 3, 0]):  # every slot is used by each request in turn
+    out = s.prompt(reqs, slots=slots)
+    last = s.prompt(reqs, slots=slots, last_only=True)
+    got, exp = [], []  # single rows of a bfloat16 model are noisy: compare them together
+    for i, n in enumerate(lens):
+      got += [*out[i, :n], last[i]]
+      exp += [*want[i][:n], want[i][n - 1]]
+    for t in range(25):
+      live = [i for i in range(3) if t < 10 or i != 1]  # one ends earlier: its row is parked
+      row_slots = [slots[i] if i in live else -1 for i in range(3)]
+      out = s.decode([f[t] for f in follow], [n + t for n in lens], row_slots)
+      got += [out[i] for i in live]
+      exp += [want[i][lens[i] + t] for i in live]
+    close(torch.stack(got), torch.stack(exp), kind[1], 3)
+
+
+@on
+def test_prefill_leaves_other_slots_alone(kind, checkpoints):
+  s = Session(kind, checkpoints["base"][0])
+  s.prompt([TOKENS[:20]], slots=[1])
+  before = [t[[0, 1, 3]].clone() for t in s.cache._tensors()]
+  s.prompt([TOKENS[:33]], slots=[2])
+  s.decode([TOKENS[33], 0], [33, 5], [2, -1])
+  assert all((t[[0, 1, 3]] == u).all() for t, u in zip(s.cache._tensors(), before))
+
+
+@on
+def test_long_decoding(kind, checkpoints, references):
+  tokens = TOKENS.repeat(4)[:300]
+  want = references("ones", tokens)
+  s = Session(kind, checkpoints["ones"][0], capacity=320)
+  got = [s.prompt([tokens[:2]], slots=[1])[0]]
+  got += [s.decode([tokens[t]], [t], [1]) for t in range(2, 300)]
+  close(torch.cat(got), want, kind[1], 3)
+
+
+@on
+def test_capacity_below_the_window(kind, checkpoints, references):
+  s = Session(kind, checkpoints["base"][0], capacity=25)  # a ring shorter than one layer's window
+  want = references("base", TOKENS[:25])
+  got = [s.prompt([TOKENS[:20]])[0]] + [s.decode([TOKENS[t]], [t]) for t in range(20, 25)]
+  close(torch.cat(got), want, kind[1], 3)
+
+
+@on
+def test_shards_pass_the_stream_in_32_bit(kind, checkpoints, references):
+  folder = checkpoints["base"][0]
+  a, b = Session(kind, folder, layers=(0, 1)), Session(kind, folder, layers=(2, 3))
+  want = references("base", TOKENS[:40])
+  with torch.inference_mode():
+    x = TOKENS[None, :39].to(kind[0])
+    mid = a.model(x, a.cache.caches, torch.arange(39), 0)
+    assert mid.dtype == a.model.hidden_dtype == F32
+    kept = mid.clone()
+    got = b.model(mid, b.cache.caches, torch.arange(39), 0, last_only=False)[0]
+    assert (mid == kept).all()
+    pos = torch.tensor([39], dtype=torch.int32, device=kind[0])
+    mid = a.model(TOKENS[None, 39:40].to(kind[0]), a.cache.caches, pos, -1, is_decode=True)
+    got = torch.cat([got, b.model(mid, b.cache.caches, pos, -1, is_decode=True)])
+  close(got, want, kind[1], 3)
+
+
+def test_cacheless_forward_trains(checkpoints, references):
+  model = cases.load_model(checkpoints["base"][0])
+  out = model(TOKENS[None, :20], None, torch.arange(20), 0, last_only=False)
+  close(out[0], references("base", TOKENS[:20]), F32, 3)
+  out.float().pow(2).mean().backward()
+  dead = [n for n, p in model.named_parameters() if p.grad is None or not p.grad.isfinite().all()]
+  assert not dead
+
+
+# ---------------------------------------------------------------- loading
+
+def test_config_reads_sizes_from_tensor_shapes(checkpoints):
+  folder, raw, _ = checkpoints["base"]
+  cfg = config_from_hf(folder / "config.json", "m")
+  assert cfg.model_type == "didipel" and cfg.n_layers == 4 and cfg.dim == 72 and cfg.norm_eps == 1e-5
+  assert cfg.layer_specs[0].params["left"]["buckets"] == cases.RANKS["rel"]
+  assert cfg.layer_specs[2].params["right"]["decay_rank"] == cases.RANKS["a1"]
+  assert cfg.layer_specs[1].params["decay_rank"] == cases.RANKS["w1"] and cfg.layer_specs[1].ff == 0
+  with pytest.raises(ValueError, match="unknown"):
+    config_from_hf(raw, "m")  # no folder, so no tensor shapes
+  with pytest.raises(ValueError, match="unknown architecture"):
+    config_from_hf({"architecture": "Else"}, "m")
+
+
+def test_parameter_count_matches_the_estimate(checkpoints):
+  folder = checkpoints["base"][0]
+  cfg = config_from_hf(folder / "config.json", "m")
+  stored = sum(t.numel() for t in checkpoints["base"][2].values())
+  assert abs(cfg.estimate_param_bytes() / 2 - stored) / stored < 0.02
+
+
+def test_loader_names_what_is_missing(tmp_path, checkpoints):
+  _, cfg, w = checkpoints["base"]
+  for gone in ("l0.mix.right.k", "l1.mix.mu.g", "l3.mix.norm", "final.norm"):
+    folder = cases.write_checkpoint(tmp_path / gone, cfg, {n: t for n, t in w.items() if n != gone})
+    with pytest.raises(RuntimeError, match="missing weights"):
+      cases.load_model(folder)
+
+
+def test_constant_state_per_slot(checkpoints):
+  cfg = config_from_hf(checkpoints["base"][0] / "config.json", "m")
+  from xotorch_amd.shard import Shard
+  shard = Shard("m", 0, 3, 4)
+  small, large = (make_cache(cfg, shard, 2, n, F32, "cpu").nbytes() for n in (64, 100000))
+  assert small == large
+
+
+def test_speculative_decoding_refuses_recurrent_state(checkpoints):
+  from xotorch_amd.engine.spec import SpeculativeDecoder
+  cfg = config_from_hf(checkpoints["base"][0] / "config.json", "m")
+  with pytest.raises(ValueError, match="recurrent"):
+    SpeculativeDecoder(None, None, cfg, cfg, "cpu", F32)
+
+
+# ---------------------------------------------------------------- serving
+
+def plausible(generated, prompt, dtype, ref):
+  """Greedy: every token is the expected logits' best (in bfloat16: as good
+  as the best up to rounding) after what was generated before it."""
+  logits = ref(torch.tensor(list(prompt) + generated[:-1]))[len(prompt) - 1:]
+  slack = 0.15 if dtype == BF16 else 1e-4
+  for row, tok in zip(logits, generated):
+    assert row.max() - row[tok] <= slack
+
+
+@on
+def test_engine_generates(kind, checkpoints, references):
+  from xotorch_amd.download.downloader import NoopShardDownloader
+  from xotorch_amd.engine.torch_engine import TorchEngine
+  from xotorch_amd.shard import Shard
+  eng = TorchEngine(NoopShardDownloader(checkpoints["base"][0]), device=kind[0], dtype=kind[1])
+  prompt = TOKENS[:14].numpy()
+
+  async def go(rid):
+    out, state = await eng.infer_tensor(rid, Shard("m", 0, 3, 4), prompt[None], {"total_len": 60})
+    toks = []
+    for _ in range(20):
+      toks.append(int((await eng.sample(out, temp=0.0))[0]))
+      out, state = await eng.infer_tensor(rid, Shard("m", 0, 3, 4), np.array([[toks[-1]]]), state)
+    return toks
+  loop = asyncio.new_event_loop()
+  toks = loop.run_until_complete(go("a"))
+  plausible(toks, prompt, kind[1], lambda t: references("base", t))
+  assert loop.run_until_complete(go("b")) == toks
+
+
+def serve(worker, reqs):
+  q, got, done = queue.Queue(), {}, threading.Event()
+  left = {r[0] for r in reqs}
+
+  def emit(rid, tok, fin, meta):
+    got.setdefault(rid, []).append(tok)
+    if fin:
+      left.discard(rid)
+      if not left:
+        done.set()
+  from xotorch_amd.serve_ring import AdmitMsg
+  for rid, ids, n in reqs:
+    q.put(AdmitMsg(rid, torch.tensor([list(ids)], dtype=torch.int64), n, 0.0))
+  t = threading.Thread(target=worker.serve_forever, args=(q, emit), daemon=True)
+  t.start()
+  assert done.wait(100), f"unfinished: {left}"
+  q.put(AdmitMsg("stop", None, 0, 0.0))
+  t.join(timeout=30)
+  return got
+
+
+def make_worker(kind, folder, **kw):
+  from xotorch_amd.serve_ring import RingSlotWorker
+  w = RingSlotWorker("m", 0, 1, device=kind[0], dtype=kind[1], model_dir=str(folder), max_seq=160,
+                     **{"slots": 3, **kw})
+  if kind[0] == "cuda":
+    w._build_graph()
+    assert w._graph is not None
+  return w
+
+
+@on
+def test_scheduler_serves_more_requests_than_slots(kind, checkpoints, references, monkeypatch):
+  """Prompts of unequal length in chunks and batches, decode ticks in between,
+  slots handed on."""
+  monkeypatch.setattr("xotorch_amd.serve_ring.PREFILL_CHUNK", 16)
+  w = make_worker(kind, checkpoints["base"][0])
+  reqs = [(f"r{i}", TOKENS[i:i + n].tolist(), m) for i, (n, m) in
+          enumerate([(5, 25), (40, 6), (16, 12), (1, 30), (33, 9), (2, 3), (17, 20)])]
+  got = serve(w, reqs)
+  for rid, ids, n in reqs:
+    assert len(got[rid]) == n
+    plausible(got[rid], ids, kind[1], lambda t: references("base", t))
+
+
+def test_prompts_equally_far_share_a_batch(checkpoints, monkeypatch):
+  monkeypatch.setattr("xotorch_amd.serve_ring.PREFILL_CHUNK", 8)
+  w = make_worker(("cpu", F32), checkpoints["base"][0], slots=4)
+  calls, inner = [], w._prefill_hidden
+  monkeypatch.setattr(w, "_prefill_hidden", lambda group, c0, **kw: (calls.append((list(group), c0)), inner(group, c0, **kw))[1])
+  serve(w, [("a", TOKENS[:12].tolist(), 2), ("b", TOKENS[:9].tolist(), 2), ("c", TOKENS[:3].tolist(), 2)])
+  assert ([0, 1, 2], 0) in calls and ([0, 1], 8) in calls
+
+
+def _ring_rank(rank, world, folder, port, out):
+  import os
+  import torch.distributed as dist
+  from xotorch_amd.serve_ring import AdmitMsg, RingSlotWorker
+  os.environ.update(MASTER_ADDR="127.0.0.1", MASTER_PORT=str(port), RANK=str(rank), WORLD_SIZE=str(world))
+  dist.init_process_group("gloo", rank=rank, world_size=world)
+  try:
+    w = RingSlotWorker("m", rank, world, device="cpu", dtype=F32, model_dir=folder, slots=2, max_seq=120, use_graphs=False)
+    if rank == 0:
+      out.put(serve(w, [("a", TOKENS[:20].tolist(), 12), ("b", TOKENS[5:9].tolist(), 15), ("c", TOKENS[:11].tolist(), 4)]))
+    else:
+      w.serve_forever()
+  finally:
+    dist.destroy_process_group()
+
+
+def test_two_rank_ring_serves_the_same_tokens(checkpoints, references):
+  import torch.multiprocessing as mp
+  from xotorch_amd.helpers import find_available_port
+  ctx = mp.get_context("spawn")
+  out, port = ctx.Queue(), find_available_port("127.0.0.1")
+  procs = [ctx.Process(target=_ring_rank, args=(r, 2, str(checkpoints["base"][0]), port, out)) for r in range(2)]
+  for p in procs:
+    p.start()
+  got = out.get(timeout=110)
+  for p in procs:
+    p.join(timeout=30)
+  for rid, ids in (("a", TOKENS[:20]), ("b", TOKENS[5:9]), ("c", TOKENS[:11])):
+    plausible(got[rid], ids.tolist(), F32, lambda t: references("base", t))
+
+
+@on
+def test_ring_pipeline_prefill_in_slices(kind, monkeypatch):
+  """Batch slices of a prefill address their cache rows by slot."""
+  from xotorch_amd.parallel.ring import RingPipeline
+  got = []
+  for chunk in ("2", "8"):
+    monkeypatch.setenv("XOT_PREFILL_CHUNK", chunk)
+    ring = RingPipeline("didipel-dummy", 0, 1, kind[0], kind[1], mb_batch=5, prompt_len=30, max_gen=12)
+    ring.capture_tokens = True
+    ring.prefill()
+    for _ in range(8):
+      ring.decode_step()
+    got.append(torch.cat(ring.generated[0], dim=1).cpu())
+  assert got[0].shape == (5, 9)
+  if kind[1] == F32:
+    assert (got[0] == got[1]).all()
+
+
+@on
+def test_trace_replay(kind, checkpoints, references, tmp_path, monkeypatch, capsys):
+  """The replay command: whole, cut and ragged steps, slots given back."""
+  from xotorch_amd.engine import trace
+  folder = checkpoints["base"][0]
+  monkeypatch.setattr("xotorch_amd.serve_ring.PREFILL_CHUNK", 32)
+  if kind[0] == "cpu":
+    monkeypatch.setattr(torch.cuda, "is_available", lambda: False)
+  a, b = TOKENS[:75].tolist(), TOKENS[30:50].tolist()
+  steps = [{"entries": [{"id": "a", "tokens": a[:70], "want": [0, 10, 11, 32, 69]}, {"id": "b", "tokens": b[:3], "want": [2]}]}]
+  steps += [{"entries": [{"id": "b", "tokens": [b[t]], "want": [0]}] +
+             ([{"id": "a", "tokens": [a[67 + t]], "want": [0]}] if 3 <= t < 8 else [])} for t in range(3, 8)]
+  steps += [{"entries": [{"id": "b", "tokens": [b[8]], "want": []}], "end": ["a"]},
+            {"entries": [{"id": "b", "tokens": b[9:20], "want": [10]}, {"id": "c", "tokens": a[:40], "want": [39]}], "end": ["b"]}]
+  for i, s in enumerate(steps):
+    s["step"] = i
+  monkeypatch.setattr("sys.stdin", io.StringIO("".join(json.dumps(s) + "\n" for s in steps)))
+  dtype = "bfloat16" if kind[1] == BF16 else "float32"
+  assert trace.main(["--model", str(folder), "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "160"]) == 0
+  assert [x for x in capsys.readouterr().out.splitlines() if x.startswith("done")] == [f"done {i}" for i in range(len(steps))]
+  got, exp = [], []
+  tokens, at = {"a": a, "b": b, "c": a[:40]}, {"a": 0, "b": 0, "c": 0}
+  for s in steps:
+    want = []
+    for e in s["entries"]:
+      ref = references("base", torch.tensor(tokens[e["id"]]))
+      want += [ref[at[e["id"]] + p] for p in e["want"]]
+      at[e["id"]] += len(e["tokens"])
+    file = tmp_path / f"{s['step']}.f32"
+    assert file.exists() == bool(want)
+    if want:
+      got.append(torch.from_numpy(np.fromfile(file, "<f4")).view(len(want), -1))
+      exp += want
+  close(torch.cat(got), torch.stack(exp), kind[1], 3)
+
+
+def test_cli_runs_a_checkpoint_folder(checkpoints, capsys, monkeypatch):
+  from xotorch_amd.cli import build_parser, run_model_cli
+  from xotorch_amd.models import registry
+  monkeypatch.setattr(registry, "model_cards", dict(registry.model_cards))
+  folder = checkpoints["base"][0]
+  args = build_parser().parse_args(
+    ["run", "my-didipel", "--model-dir", str(folder), "--prompt", "AB", "--inference-engine", "torch",
+     "--discovery-module", "none", "--max-generate-tokens", "5", "--disable-tui"])
+  monkeypatch.setenv("XOT_OFFLINE", "1")
+  # the folder has no tokenizer: the fallback's ids must fit this vocabulary
+  from xotorch_amd.engine.tokenizers import DummyTokenizer
+  monkeypatch.setattr(DummyTokenizer, "encode", lambda self, text, **kw: [ord(c) % 100 for c in text])
+  asyncio.new_event_loop().run_until_complete(run_model_cli(args))
+  assert capsys.readouterr().out.strip()

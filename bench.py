@@ -47,6 +47,72 @@ if _tuned.exists() and os.getenv("XOT_TUNABLEOP", "1") == "1":
 import torch  # noqa: E402
 
 
+def _gemma2_like(width, n_layers, ff, vocab, kv_heads, window):
+  return {
+    "model_type": "gemma2", "hidden_size": width, "num_hidden_layers": n_layers,
+    "num_attention_heads": width // 128, "num_key_value_heads": kv_heads, "head_dim": 128,
+    "intermediate_size": ff, "vocab_size": vocab, "rms_norm_eps": 1e-6, "max_position_embeddings": 1 << 20,
+    "tie_word_embeddings": True, "query_pre_attn_scalar": 128, "attn_logit_softcapping": 50.0,
+    "final_logit_softcapping": 30.0, "sliding_window": window,
+  }
+
+
+def _didipel_pair(model_id):
+  """The registry's Didipel of that size, and gemma2 (sandwich norms, sliding
+  windows) with the same width, depth, heads, feed-forward, vocabulary."""
+  from xotorch_amd.models.registry import builtin_config
+  cfg = builtin_config(model_id)
+  left = next(e["mixer"]["left"] for e in cfg["layers"] if e["type"] == "parallel")
+  like = _gemma2_like(cfg["width"], len(cfg["layers"]), cfg["layers"][0]["mlp"]["ff"], cfg["vocab"],
+                      left["kv_heads"], left["mask"]["size"])
+  return [(model_id, cfg), ("gemma2 of that size", like)]
+
+
+DESIGNS = {"didipel": _didipel_pair}
+
+
+def design_bench(args):
+  """One JSON line per (model, batch x prompt): prompt and decode tokens/s on
+  one GPU, random weights. The pair takes turns at every shape."""
+  from xotorch_amd.parallel.comm import init_distributed
+  from xotorch_amd.parallel.ring import RingPipeline
+  init_distributed()
+  device = args.device or ("cuda" if torch.cuda.is_available() else "cpu")
+
+  def sync():
+    if device == "cuda":
+      torch.cuda.synchronize()
+
+  for size in args.sizes.split(","):
+    for shape in args.shapes.split(","):
+      batch, prompt = (int(v) for v in shape.split("x"))
+      for name, cfg in DESIGNS[args.design](f"{args.design}-{size}"):
+        ring = RingPipeline(name, 0, 1, device, torch.bfloat16 if args.dtype == "bf16" else torch.float32,
+                            mb_batch=batch, prompt_len=prompt, max_gen=args.warmup + args.steps + 4,
+                            use_graphs=not args.no_graphs, cfg_override=cfg)
+        ring.prefill()  # first calls: library heuristics, allocator
+        ring.use_graphs = False  # captured; only the prompts run again
+        ms = min(ring.prefill().ttft_ms[0] for _ in range(3))
+        for _ in range(args.warmup):
+          ring.decode_step()
+        sync()
+        t0 = time.perf_counter()
+        for _ in range(args.steps):
+          ring.decode_step()
+        sync()
+        step = (time.perf_counter() - t0) / args.steps
+        print(json.dumps({
+          "model": name, "size": size, "batch": batch, "prompt": prompt, "dtype": args.dtype,
+          "params_b": round(sum(p.numel() for p in ring.model.parameters()) / 1e9, 3),
+          "state_mib": round(ring.caches[0].nbytes() / 2**20, 1),
+          "prefill_tokens_per_s": round(batch * prompt / ms * 1e3), "prefill_ms": round(ms, 2),
+          "decode_tokens_per_s": round(batch / step), "decode_ms_per_step": round(step * 1e3, 3),
+        }), flush=True)
+        del ring
+        if device == "cuda":
+          torch.cuda.empty_cache()
+
+
 def main():
   p = argparse.ArgumentParser()
   p.add_argument("--gpus", type=int, default=1)
@@ -58,7 +124,14 @@ def main():
   p.add_argument("--no-graphs", action="store_true")
   p.add_argument("--device", type=str, default=None)
   p.add_argument("--dtype", type=str, default="bf16", choices=["bf16", "fp32"])
+  p.add_argument("--design", choices=sorted(DESIGNS), default=None,
+                 help="instead: prefill and decode throughput of a design beside the closest other model at equal size")
+  p.add_argument("--sizes", type=str, default="1b,7b", help="with --design: sizes to run")
+  p.add_argument("--shapes", type=str, default="1x4096,32x1024,128x512",
+                 help="with --design: batch x prompt tokens, comma separated")
   args = p.parse_args()
+  if args.design:
+    return design_bench(args)
 
   from xotorch_amd.parallel.comm import init_distributed, max_over_ranks
   import torch.distributed as dist

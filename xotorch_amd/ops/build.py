@@ -67,6 +67,7 @@ def build(force: bool = False, verbose: bool = True, missing_only: bool = False)
     proc.wait()
   for n, tmp, cmd, proc in jobs:
     if proc.returncode:
+      tmp.unlink(missing_ok=True)
       raise subprocess.CalledProcessError(proc.returncode, cmd)
     os.replace(tmp, out_path(n))
   return [out_path(n) for n in names]

@@ -4,9 +4,9 @@
 //     for the next sublayer, one pass
 //   - sliding-window attention with a learned distance bias, a zero-score sink
 //     and per-head gates: q/k norm + cache append, flash prefill, split decode
-//   - gated delta rule and WKV recurrences: input preparation (short
-//     convolutions, unit norms, decays), a register-resident scan for prompts,
-//     one fused kernel per decode step
+//   - gated delta rule and WKV recurrences: for prompts the factors of
+//     16-token chunks (short convolutions, unit norms, decays) and a scan over
+//     chunks on fp32 MFMA, one fused kernel per decode step
 //
 // Two element types: bf16 (MFMA attention over fragment-packed keys and
 // values) and fp32 (plain layouts, plain fp32 arithmetic). Recurrent state,
@@ -57,6 +57,31 @@ DEVINL void ld4(const bf16_t* p, float* o) {
 #pragma unroll
   for (int i = 0; i < 4; ++i) { bf16_t u = v[i]; o[i] = ld(&u); }
 }
+typedef __attribute__((ext_vector_type(2))) float floatx2;
+typedef __attribute__((ext_vector_type(2))) unsigned short ushort2_t;
+DEVINL void ld2(const float* p, float* o) {
+  const floatx2 v = *(const floatx2*)p;
+  o[0] = v[0];
+  o[1] = v[1];
+}
+DEVINL void ld2(const bf16_t* p, float* o) {
+  const ushort2_t v = *(const ushort2_t*)p;
+  bf16_t a = v[0], b = v[1];
+  o[0] = ld(&a);
+  o[1] = ld(&b);
+}
+DEVINL void st2(float* p, const float* o) {
+  floatx2 v;
+  v[0] = o[0];
+  v[1] = o[1];
+  *(floatx2*)p = v;
+}
+DEVINL void st2(bf16_t* p, const float* o) {
+  ushort2_t v;
+  v[0] = f2b(o[0]);
+  v[1] = f2b(o[1]);
+  *(ushort2_t*)p = v;
+}
 DEVINL void st4(float* p, const float* o) {
   floatx4 v;
 #pragma unroll
@@ -88,9 +113,18 @@ DEVINL float sigmoidf(float x) { return 1.f / (1.f + expf(-x)); }
 DEVINL float siluf(float x) { return x / (1.f + expf(-x)); }
 DEVINL float softplusf(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
+// sum over the 16 lanes of a DPP row, in every lane (row_ror:8, 4, 2, 1)
+DEVINL float row_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, true));
+  return v;
+}
 DEVINL float wave_sum(float v) {
-#pragma unroll
-  for (int m = 32; m > 0; m >>= 1) v += __shfl_xor(v, m);
+  v = row_sum(v);
+  v += __shfl_xor(v, 16);
+  v += __shfl_xor(v, 32);
   return v;
 }
 // sum over a block of 256 threads; `red` holds 4 floats and is free again
@@ -687,103 +721,382 @@ DEVINL float conv_silu(const T* proj, const T* ring, const T* taps_w, int s, int
   return siluf(y);
 }
 
-// Prompt side of the delta rule: one wave per (token, q/k head) prepares that
-// head's unit q (scaled) and k, q.k, and for its value heads v, decays, beta.
-template <typename T>
-__global__ __launch_bounds__(256) void delta_prep_kernel(
-    const T* __restrict__ proj, const T* __restrict__ qc, const T* __restrict__ kcv, const T* __restrict__ vcv,
-    const T* __restrict__ pre, const T* __restrict__ a_log, const T* __restrict__ dt, const T* __restrict__ ring,
-    float* __restrict__ q, float* __restrict__ k, float* __restrict__ dot, float* __restrict__ v,
-    float* __restrict__ dec, float* __restrict__ beta, int total, RecArgs a, Step step) {
-  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (id >= total) return;
-  const int g = id % a.G, tok = id / a.G, s = tok % a.S, b = tok / a.S;
-  const int slot = step.slot(b);
-  if (slot < 0 || s >= step.len(b, a.S)) return;
-  const int C = 2 * a.G * a.dim + a.H * a.vdim, first = step.first(b), per = a.H / a.G;
-  const T* rows = proj + (size_t)b * a.S * a.N;
-  const T* hist = ring + (size_t)slot * a.taps * C;
-  float qv[4], kv[4], qq = 0.f, kk = 0.f, qk = 0.f;
+// PER consecutive channels of a lane, those past n as zero; `vec`: the
+// address allows one load
+template <int PER, typename T>
+DEVINL void ld_lane(const T* p, int c, int n, bool vec, float* o) {
+  if (PER == 4 && vec && c + 3 < n) { ld4(p + c, o); return; }
+  if (PER == 2 && vec && c + 1 < n) { ld2(p + c, o); return; }
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int d = lane + 64 * i, ch = g * a.dim + d;
-    qv[i] = kv[i] = 0.f;
-    if (d < a.dim) {
-      qv[i] = conv_silu(rows, hist, qc, s, first, a.q_at + ch, ch, ch, C, a);
-      kv[i] = conv_silu(rows, hist, kcv, s, first, a.k_at + ch, a.G * a.dim + ch, ch, C, a);
-    }
-    qq += qv[i] * qv[i];
-    kk += kv[i] * kv[i];
-    qk += qv[i] * kv[i];
+  for (int i = 0; i < PER; ++i) o[i] = c + i < n ? ld(p + c + i) : 0.f;
+}
+template <int PER, typename T>
+DEVINL void st_lane(T* p, int c, int n, bool vec, const float* o) {
+  if (PER == 4 && vec && c + 3 < n) { st4(p + c, o); return; }
+  if (PER == 2 && vec && c + 1 < n) { st2(p + c, o); return; }
+#pragma unroll
+  for (int i = 0; i < PER; ++i)
+    if (c + i < n) st(p + c + i, o[i]);
+}
+
+// A lane's channels through a causal convolution and silu, token by token:
+// weights and the last inputs stay in registers. TAPS 0: any number of taps,
+// inputs read again for every token.
+template <typename T, int TAPS, int PER>
+struct Conv {
+  static constexpr int NT = TAPS ? TAPS : 1;
+  float w[NT][PER], x[NT][PER];
+  const T *rows, *ring, *tw;
+  int col, ch, c, n, first;
+  bool vec;
+  DEVINL void history(int t, float* o, int C, const RecArgs& a) const {  // input of chunk token t (t < 0: before it)
+    if (t >= 0) ld_lane<PER>(rows + (long long)t * a.N + col, c, n, vec, o);
+    else if (first + t >= 0) ld_lane<PER>(ring + (size_t)((first + t) % a.taps) * C + ch, c, n, false, o);
+    else
+#pragma unroll
+      for (int i = 0; i < PER; ++i) o[i] = 0.f;
   }
-  const float qi = 1.f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)a.dim), ki = 1.f / sqrtf(wave_sum(kk) + 1e-6f);
-  qk = wave_sum(qk) * qi * ki;
-  const size_t qo = ((size_t)tok * a.G + g) * a.dp;
+  DEVINL void begin(int s0, int C, const RecArgs& a) {
+    if (!TAPS) return;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int d = lane + 64 * i;
-    if (d < a.dp) { q[qo + d] = qv[i] * qi; k[qo + d] = kv[i] * ki; }
+    for (int i = 0; i < PER; ++i)
+#pragma unroll
+      for (int j = 0; j < NT; ++j) w[j][i] = c + i < n ? ld(tw + (size_t)(c + i) * TAPS + j) : 0.f;
+#pragma unroll
+    for (int j = 1; j < NT; ++j) history(s0 - NT + j, x[j], C, a);
   }
-  if (lane == 0) dot[(size_t)tok * a.G + g] = qk;
-  for (int h = g * per; h < (g + 1) * per; ++h) {
-    const float A = expf(ld(a_log + h));
+  DEVINL void next(int s, int C, const RecArgs& a, float* y) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = lane + 64 * i;
-      if (d < a.dp) {
-        const int ch = h * a.dim + d;
-        dec[((size_t)tok * a.H + h) * a.dp + d] =
-            d < a.dim ? expf(-A * softplusf(ld(pre + (size_t)tok * a.H * a.dim + ch) + ld(dt + ch))) : 1.f;
+    for (int i = 0; i < PER; ++i) y[i] = 0.f;
+    if (!TAPS) {
+      for (int j = 0; j < a.taps; ++j) {
+        float v[PER];
+        history(s - (a.taps - 1 - j), v, C, a);
+#pragma unroll
+        for (int i = 0; i < PER; ++i) y[i] += v[i] * (c + i < n ? ld(tw + (size_t)(c + i) * a.taps + j) : 0.f);
       }
-      if (d < a.vdim) {
-        const int ch = h * a.vdim + d;
-        v[(size_t)tok * a.H * a.vdim + ch] =
-            conv_silu(rows, hist, vcv, s, first, a.v_at + ch, 2 * a.G * a.dim + ch, ch, C, a);
-      }
+    } else {
+#pragma unroll
+      for (int j = 0; j + 1 < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < PER; ++i) x[j][i] = x[j + 1][i];
+      history(s, x[NT - 1], C, a);
+#pragma unroll
+      for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < PER; ++i) y[i] += x[j][i] * w[j][i];
     }
-    if (lane == 0) beta[(size_t)tok * a.H + h] = sigmoidf(ld(proj + (size_t)tok * a.N + a.b_at + h));
+#pragma unroll
+    for (int i = 0; i < PER; ++i) y[i] = siluf(y[i]);
+  }
+};
+
+// --- prompts, 16 tokens (a chunk) at a time -------------------------------
+// With L_t the log decays summed up to token t of a chunk and S the state
+// before it, the delta rule's 16 sequential updates are
+//   U = T (V - K~ S),  O = Q~ S + B U,  S' = e^{L_15} S + K^T U
+//   K~_t = k_t e^{L_t}   Q~_t = q_t e^{L_t}   K^_s = k_s e^{L_15 - L_s}
+//   A_ts = sum_d k_t k_s e^{L_t - L_s} (s < t),  B_ts = the same with q_t (s <= t)
+//   T = (I + diag(beta) A)^-1 diag(beta)
+// and WKV's, which read before they write, the same with U = V,
+// Q~_t = r_t e^{L_(t-1)}, B_ts = sum_d r_t k_s e^{L_(t-1) - L_s} (s < t) and
+// B_tt the bonus. Every exponent is <= 0, so nothing overflows however strong
+// the decays are. chunk_prep_kernel makes the factors of all chunks in
+// parallel, chunk_scan_kernel walks the chunks with fp32 MFMA.
+//
+// Factors of a (row, chunk, head), in floats: Q~ [16][dp] | K^ transposed
+// [dp][16] | e^{L_15} [dp] | B [16][16] | T [16][16] | K~ [16][dp] (the last
+// two only for the delta rule).
+constexpr int CHUNK = 16;
+DEVINL int chunk_floats(bool delta, int dp) { return delta ? 49 * dp + 512 : 33 * dp + 256; }
+
+// One block per (head, chunk, row). DELTA: x0 is the fused projection, x1 and
+// x2 unused; c0..c2 the taps of q, k, v; d0 = A_log, d1 = dt_bias. WKV: x0..x2
+// are r, k, v; d0 = w0, d1 = u.
+template <typename T, bool DELTA, int TAPS, int PER>
+__global__ __launch_bounds__(256) void chunk_prep_kernel(
+    const T* __restrict__ x0, const T* __restrict__ x1, const T* __restrict__ x2, const T* __restrict__ c0,
+    const T* __restrict__ c1, const T* __restrict__ c2, const T* __restrict__ pre, const T* __restrict__ d0,
+    const T* __restrict__ d1, const T* __restrict__ ring, float* __restrict__ factors, float* __restrict__ v,
+    int chunks, RecArgs a, Step step) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int dps = a.dp + 4;
+  float *sq = lds, *sk = sq + CHUNK * dps, *sl = sk + CHUNK * dps;
+  float *sA = sl + CHUNK * dps, *sB = sA + 256, *sb = sB + 256;  // sb: beta or bonus per token
+  const int h = blockIdx.x, b = blockIdx.z, tid = threadIdx.x, g = h / (a.H / a.G);
+  const int slot = step.slot(b), len = step.len(b, a.S), s0 = blockIdx.y * CHUNK;
+  if (slot < 0 || s0 >= len) return;
+  const int c = (tid & 63) * PER, t0 = (tid >> 6) * 4;  // a wave takes 4 tokens
+  float* out = factors + (((size_t)b * chunks + blockIdx.y) * a.H + h) * chunk_floats(DELTA, a.dp);
+  float bias[PER];
+  if (DELTA) {
+    const int C = 2 * a.G * a.dim + a.H * a.vdim, first = step.first(b), kw = a.G * a.dim;
+    const int qch = g * a.dim, vch = h * a.vdim;
+    const T* rows = x0 + (size_t)b * a.S * a.N;
+    const T* hist = ring + (size_t)slot * a.taps * C;
+    const bool vd = ((a.dim | a.N | a.q_at | a.k_at) & 3) == 0, ve = ((a.vdim | a.N | a.v_at) & 3) == 0;
+    Conv<T, TAPS, PER> cq{{}, {}, rows, hist, c0 + (size_t)qch * a.taps, a.q_at + qch, qch, c, a.dim, first, vd};
+    Conv<T, TAPS, PER> ck{{}, {}, rows, hist, c1 + (size_t)qch * a.taps, a.k_at + qch, kw + qch, c, a.dim, first, vd};
+    Conv<T, TAPS, PER> cv{{}, {}, rows, hist, c2 + (size_t)vch * a.taps, a.v_at + vch, 2 * kw + vch, c, a.vdim, first, ve};
+    const bool any = s0 + t0 < len;
+    if (any) {
+      cq.begin(s0 + t0, C, a);
+      ck.begin(s0 + t0, C, a);
+      cv.begin(s0 + t0, C, a);
+    }
+    const float A = expf(ld(d0 + h)), qscale = 1.f / sqrtf((float)a.dim);
+    ld_lane<PER>(d1 + (size_t)h * a.dim, c, a.dim, (a.dim & 3) == 0, bias);
+    for (int t = t0; t < t0 + 4; ++t) {
+      const int s = s0 + t;
+      float q[PER], k[PER], y[PER], lg[PER], beta = 0.f;
+#pragma unroll
+      for (int i = 0; i < PER; ++i) q[i] = k[i] = lg[i] = 0.f;
+      if (s < len) {
+        const size_t head = ((size_t)b * a.S + s) * a.H + h;
+        cq.next(s, C, a, q);
+        ck.next(s, C, a, k);
+        cv.next(s, C, a, y);
+        st_lane<PER>(v + head * a.vdim, c, a.vdim, (a.vdim & 3) == 0, y);
+        float qq = 0.f, kk = 0.f;
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+          qq += q[i] * q[i];
+          kk += k[i] * k[i];
+        }
+        const float qi = qscale / sqrtf(wave_sum(qq) + 1e-6f), ki = 1.f / sqrtf(wave_sum(kk) + 1e-6f);
+        ld_lane<PER>(pre + head * a.dim, c, a.dim, (a.dim & 3) == 0, lg);
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+          q[i] *= qi;
+          k[i] *= ki;
+          lg[i] = c + i < a.dim ? -A * softplusf(lg[i] + bias[i]) : 0.f;
+        }
+        beta = sigmoidf(ld(rows + (size_t)s * a.N + a.b_at + h));
+      }
+      st_lane<PER>(sq + t * dps, c, a.dp, true, q);
+      st_lane<PER>(sk + t * dps, c, a.dp, true, k);
+      st_lane<PER>(sl + t * dps, c, a.dp, true, lg);
+      if (c == 0) sb[t] = beta;
+    }
+  } else {
+    const bool vec = (a.dim & 3) == 0;
+    float u[PER];
+    ld_lane<PER>(d0 + (size_t)h * a.dim, c, a.dim, vec, bias);
+    ld_lane<PER>(d1 + (size_t)h * a.dim, c, a.dim, vec, u);
+#pragma unroll
+    for (int t = t0; t < t0 + 4; ++t) {
+      const int s = s0 + t;
+      float q[PER], k[PER], y[PER], lg[PER], bonus = 0.f;
+#pragma unroll
+      for (int i = 0; i < PER; ++i) q[i] = k[i] = lg[i] = 0.f;
+      if (s < len) {
+        const size_t src = (((size_t)b * a.S + s) * a.H + h) * a.dim;
+        ld_lane<PER>(x0 + src, c, a.dim, vec, q);
+        ld_lane<PER>(x1 + src, c, a.dim, vec, k);
+        ld_lane<PER>(x2 + src, c, a.dim, vec, y);
+        ld_lane<PER>(pre + src, c, a.dim, vec, lg);
+        st_lane<PER>(v + src, c, a.dim, vec, y);
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+          lg[i] = c + i < a.dim ? -expf(lg[i] + bias[i]) : 0.f;
+          bonus += q[i] * k[i] * u[i];
+        }
+      }
+      bonus = wave_sum(bonus);
+      st_lane<PER>(sq + t * dps, c, a.dp, true, q);
+      st_lane<PER>(sk + t * dps, c, a.dp, true, k);
+      st_lane<PER>(sl + t * dps, c, a.dp, true, lg);
+      if (c == 0) sb[t] = bonus;
+    }
+  }
+  __syncthreads();
+  for (int d = tid; d < a.dp; d += 256) {
+    float run = 0.f;
+#pragma unroll
+    for (int t = 0; t < CHUNK; ++t) {
+      run += sl[t * dps + d];
+      sl[t * dps + d] = run;
+    }
+    out[32 * a.dp + d] = expf(run);
+  }
+  __syncthreads();
+  if (tid < 136) {  // pairs s <= t
+    int t = (int)((sqrtf(8.f * tid + 1.f) - 1.f) * .5f);
+    if ((t + 1) * (t + 2) / 2 <= tid) ++t;
+    if (t * (t + 1) / 2 > tid) --t;
+    const int s = tid - t * (t + 1) / 2;
+    float A = 0.f, B = 0.f;
+    if (DELTA || s < t) {
+      const float *kt = sk + t * dps, *ks = sk + s * dps, *qt = sq + t * dps;
+      const float *lt = sl + (DELTA ? t : t - 1) * dps, *ls = sl + s * dps;
+      for (int d = 0; d < a.dp; d += 4) {
+        float xt[4], xs[4], xq[4], et[4], es[4];
+        ld4(ks + d, xs);
+        ld4(qt + d, xq);
+        ld4(lt + d, et);
+        ld4(ls + d, es);
+        if (DELTA) ld4(kt + d, xt);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float w = xs[i] * __expf(et[i] - es[i]);
+          if (DELTA) A += xt[i] * w;
+          B += xq[i] * w;
+        }
+      }
+    } else {
+      B = sb[t];
+    }
+    sA[t * 16 + s] = A;
+    sB[t * 16 + s] = B;
+  } else {
+    int p = tid - 136, s = 1;  // pairs s > t
+    while (p >= s) p -= s++;
+    sA[p * 16 + s] = 0.f;
+    sB[p * 16 + s] = 0.f;
+  }
+  const int row4 = a.dp >> 2;
+  for (int e = tid; e < CHUNK * row4; e += 256) {
+    const int t = e / row4, d = (e - t * row4) * 4;
+    float q[4], l[4] = {0.f, 0.f, 0.f, 0.f};
+    ld4(sq + t * dps + d, q);
+    if (DELTA || t > 0) ld4(sl + (DELTA ? t : t - 1) * dps + d, l);
+    if (DELTA) {
+      float k[4];
+      ld4(sk + t * dps + d, k);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        l[i] = expf(l[i]);
+        k[i] *= l[i];
+        q[i] *= l[i];
+      }
+      st4(out + 33 * a.dp + 512 + t * a.dp + d, k);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) q[i] *= expf(l[i]);
+    }
+    st4(out + t * a.dp + d, q);
+  }
+  for (int e = tid; e < a.dp * 4; e += 256) {
+    const int d = e >> 2, t = (e & 3) * 4;
+    const float end = sl[(CHUNK - 1) * dps + d];
+    float k[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) k[i] = sk[(t + i) * dps + d] * expf(end - sl[(t + i) * dps + d]);
+    st4(out + 16 * a.dp + e * 4, k);
+  }
+  __syncthreads();
+  out[33 * a.dp + tid] = sB[tid];
+  if (DELTA && tid < CHUNK) {  // column tid of T by forward substitution
+    float x[CHUNK];
+#pragma unroll
+    for (int t = 0; t < CHUNK; ++t) {
+      float r = t == tid ? 1.f : 0.f;
+#pragma unroll
+      for (int s = 0; s < CHUNK; ++s)
+        if (s < t) r -= sA[t * 16 + s] * x[s];
+      x[t] = r * sb[t];
+      out[33 * a.dp + 256 + t * 16 + tid] = x[t];
+    }
   }
 }
 
-// Prompt side of WKV: r, k, v in fp32, decays, and r.(u*k) per (token, head).
-template <typename T>
-__global__ __launch_bounds__(256) void wkv_prep_kernel(
-    const T* __restrict__ rr, const T* __restrict__ kk, const T* __restrict__ vv, const T* __restrict__ pre,
-    const T* __restrict__ w0, const T* __restrict__ u, float* __restrict__ q, float* __restrict__ k,
-    float* __restrict__ dot, float* __restrict__ v, float* __restrict__ dec, int total, RecArgs a, Step step) {
-  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (id >= total) return;
-  const int h = id % a.H, tok = id / a.H, s = tok % a.S, b = tok / a.S;
-  if (step.slot(b) < 0 || s >= step.len(b, a.S)) return;
-  const size_t src = ((size_t)tok * a.H + h) * a.dim, dst = ((size_t)tok * a.H + h) * a.dp;
-  float sum = 0.f;
+// A wave holds 16 columns of a head's state as MFMA accumulators (NI tiles of
+// 16 key channels). A lane's accumulator element r of tile i is channel
+// i*16 + quad*4 + r of its column, so the accumulators are at the same time
+// the right-hand operands of the products with S: step (i, r) of an
+// f32 16x16x4 MFMA contracts the four channels its quads hold.
+template <bool DELTA, int NI>
+__global__ __launch_bounds__(256) void chunk_scan_kernel(
+    const float* __restrict__ factors, const float* __restrict__ v, float* __restrict__ state, float* __restrict__ o,
+    int chunks, RecArgs a, Step step) {
+  constexpr int DP = 16 * NI, QS = DP + 4, TS = 20;  // padded LDS rows: no bank conflicts
+  constexpr int FLOATS = DELTA ? 49 * DP + 512 : 33 * DP + 256, NL = (FLOATS / 4 + 255) / 256;
+  constexpr int AT_KT = 16 * QS, AT_E = AT_KT + DP * TS, AT_B = AT_E + DP, AT_T = AT_B + 16 * TS, AT_K = AT_T + 16 * TS;
+  __shared__ __attribute__((aligned(16))) float lds[DELTA ? AT_K + 16 * QS : AT_T];
+  const int h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x;
+  const int slot = step.slot(b), len = step.len(b, a.S);
+  if (slot < 0) return;
+  const int lane = tid & 63, m = lane & 15, quad = lane >> 4, col = (blockIdx.x * 4 + (tid >> 6)) * 16 + m;
+  const bool mine = col < a.vdim;
+  // where this thread's float4s of a chunk's factors go
+  int dst[NL];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int d = lane + 64 * i;
-    if (d >= a.dp) continue;
-    float r = 0.f, kx = 0.f, w = 1.f;
-    if (d < a.dim) {
-      r = ld(rr + src + d);
-      kx = ld(kk + src + d);
-      w = expf(-expf(ld(pre + src + d) + ld(w0 + h * a.dim + d)));
-      sum += r * kx * ld(u + h * a.dim + d);
-      v[src + d] = ld(vv + src + d);
-    }
-    q[dst + d] = r;
-    k[dst + d] = kx;
-    dec[dst + d] = w;
+  for (int i = 0; i < NL; ++i) {
+    int e = (tid + i * 256) * 4;
+    if (e < 16 * DP) dst[i] = e / DP * QS + e % DP;
+    else if (e < 32 * DP) { e -= 16 * DP; dst[i] = AT_KT + e / 16 * TS + e % 16; }
+    else if (e < 33 * DP) dst[i] = AT_E + e - 32 * DP;
+    else if (e < 33 * DP + 256) { e -= 33 * DP; dst[i] = AT_B + e / 16 * TS + e % 16; }
+    else if (e < 33 * DP + 512) { e -= 33 * DP + 256; dst[i] = AT_T + e / 16 * TS + e % 16; }
+    else { e -= 33 * DP + 512; dst[i] = AT_K + e / DP * QS + e % DP; }
   }
-  sum = wave_sum(sum);
-  if (lane == 0) dot[(size_t)tok * a.H + h] = sum;
-}
-
-// sum over the 16 lanes of a DPP row, in every lane
-DEVINL float row_sum(float v) {
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x128, 0xf, 0xf, true));  // row_ror:8
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x124, 0xf, 0xf, true));
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x122, 0xf, 0xf, true));
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x121, 0xf, 0xf, true));
-  return v;
+  floatx4 S[NI];
+  float* base = state + (((size_t)slot * a.H + h) * a.vdim + (mine ? col : 0)) * DP + quad * 4;
+  const bool fresh = step.first(b) == 0;
+#pragma unroll
+  for (int i = 0; i < NI; ++i) S[i] = fresh || !mine ? (floatx4)(0.f) : *(const floatx4*)(base + i * 16);
+  const size_t tok0 = (size_t)b * a.S, vstride = (size_t)a.H * a.vdim, vcol = (size_t)h * a.vdim + col;
+  floatx4 rf[NL], rv;
+  auto fetch = [&](int t0) {
+    const float* src = factors + (((size_t)b * chunks + t0 / CHUNK) * a.H + h) * FLOATS;
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int e = (tid + i * 256) * 4;
+      if (e < FLOATS) rf[i] = *(const floatx4*)(src + e);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = t0 + quad * 4 + r;
+      rv[r] = mine && t < len ? v[(tok0 + t) * vstride + vcol] : 0.f;
+    }
+  };
+  if (len > 0) fetch(0);
+  for (int t0 = 0; t0 < len; t0 += CHUNK) {
+    __syncthreads();  // everyone is done with the previous chunk's factors
+#pragma unroll
+    for (int i = 0; i < NL; ++i)
+      if ((tid + i * 256) * 4 < FLOATS) *(floatx4*)(lds + dst[i]) = rf[i];
+    const floatx4 V = rv;
+    __syncthreads();
+    if (t0 + CHUNK < len) fetch(t0 + CHUNK);
+    floatx4 O = (floatx4)(0.f), P = (floatx4)(0.f);
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const floatx4 q4 = *(const floatx4*)(lds + m * QS + i * 16 + quad * 4);
+      floatx4 k4;
+      if (DELTA) k4 = *(const floatx4*)(lds + AT_K + m * QS + i * 16 + quad * 4);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        if (DELTA) P = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[r], S[i][r], P, 0, 0, 0);
+        O = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[r], S[i][r], O, 0, 0, 0);
+      }
+    }
+    floatx4 U = V;
+    if (DELTA) {
+      const floatx4 W = V - P, t4 = *(const floatx4*)(lds + AT_T + m * TS + quad * 4);
+      U = (floatx4)(0.f);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) U = __builtin_amdgcn_mfma_f32_16x16x4f32(t4[r], W[r], U, 0, 0, 0);
+    }
+    const floatx4 b4 = *(const floatx4*)(lds + AT_B + m * TS + quad * 4);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(b4[r], U[r], O, 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < NI; ++i) S[i] *= *(const floatx4*)(lds + AT_E + i * 16 + quad * 4);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)  // tiles innermost: consecutive MFMAs are independent
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+        S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(lds[AT_KT + (i * 16 + m) * TS + quad * 4 + r], U[r], S[i], 0, 0, 0);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = t0 + quad * 4 + r;
+      if (mine && t < len) o[(tok0 + t) * vstride + vcol] = O[r];
+    }
+  }
+  if (mine && len > 0)
+#pragma unroll
+    for (int i = 0; i < NI; ++i) *(floatx4*)(base + i * 16) = S[i];
 }
 
 // rows of the state that lane r (0..15) of a column holds: vectors of V
@@ -829,111 +1142,43 @@ DEVINL float rec_step(float* s, const float* q, const float* k, const float* g, 
   return row_sum(p2) + dot * v;
 }
 
-// The scan: 16 lanes hold one column of a head's state in registers (16
-// columns a block) and step through the prompt; q, k and decays of CT tokens
-// at a time pass through LDS, loaded one chunk ahead.
-template <bool DELTA, int RPL>
-__global__ __launch_bounds__(256) void scan_kernel(
-    const float* __restrict__ q, const float* __restrict__ k, const float* __restrict__ dec,
-    const float* __restrict__ v, const float* __restrict__ beta, const float* __restrict__ dot,
-    float* __restrict__ state, float* __restrict__ o, RecArgs a, Step step) {
-  constexpr int CT = 16, DP = 16 * RPL, V4 = CT * DP / 4, NL = (V4 + 255) / 256;
-  __shared__ __attribute__((aligned(16))) float sq[CT * DP], sk[CT * DP], sg[CT * DP];
-  __shared__ float sv[CT * 16], so[CT * 16], sb[CT], sd[CT];
-  const int h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G);
-  const int slot = step.slot(b);
-  if (slot < 0) return;
-  const int len = step.len(b, a.S), tid = threadIdx.x;
-  const int r = tid & 15, cl = tid >> 4, col = blockIdx.x * 16 + cl;
-  float* st_ = state + (((size_t)slot * a.H + h) * a.vdim + min(col, a.vdim - 1)) * DP;
-  float s[RPL];
-#pragma unroll
-  for (int i = 0; i < RPL; ++i) s[i] = 0.f;
-  if (step.first(b) > 0) load_rows<RPL>(st_, r, s);
-  floatx4 rq[NL], rk[NL], rg[NL];
-  float rv = 0.f, rb = 0.f, rd = 0.f;
-  const size_t tok0 = (size_t)b * a.S;
-  auto fetch = [&](int t0) {
-#pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int e = (tid + i * 256) * 4, t = t0 + e / DP, d = e % DP;
-      if (e < CT * DP && t < len) {
-        rq[i] = *(const floatx4*)(q + ((tok0 + t) * a.G + g) * DP + d);
-        rk[i] = *(const floatx4*)(k + ((tok0 + t) * a.G + g) * DP + d);
-        rg[i] = *(const floatx4*)(dec + ((tok0 + t) * a.H + h) * DP + d);
-      }
-    }
-    const int tv = t0 + (tid >> 4), cv = blockIdx.x * 16 + (tid & 15);
-    rv = tv < len && cv < a.vdim ? v[((tok0 + tv) * a.H + h) * a.vdim + cv] : 0.f;
-    if (tid < CT && t0 + tid < len) {
-      if (DELTA) rb = beta[(tok0 + t0 + tid) * a.H + h];
-      rd = dot[(tok0 + t0 + tid) * a.G + g];
-    }
-  };
-  fetch(0);
-  for (int t0 = 0; t0 < len; t0 += CT) {
-    __syncthreads();  // the previous chunk's inputs and outputs are done with
-#pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int e = (tid + i * 256) * 4;
-      if (e < CT * DP) {
-        *(floatx4*)(sq + e) = rq[i];
-        *(floatx4*)(sk + e) = rk[i];
-        *(floatx4*)(sg + e) = rg[i];
-      }
-    }
-    sv[tid] = rv;
-    if (tid < CT) { sb[tid] = rb; sd[tid] = rd; }
-    __syncthreads();
-    if (t0 + CT < len) fetch(t0 + CT);
-    const int n = min(CT, len - t0);
-    for (int t = 0; t < n; ++t) {
-      float qq[RPL], kk[RPL], gg[RPL];
-      load_rows<RPL>(sq + t * DP, r, qq);
-      load_rows<RPL>(sk + t * DP, r, kk);
-      load_rows<RPL>(sg + t * DP, r, gg);
-      const float y = rec_step<DELTA, RPL>(s, qq, kk, gg, sv[t * 16 + cl], DELTA ? sb[t] : 0.f, sd[t]);
-      if (r == 0) so[t * 16 + cl] = y;
-    }
-    __syncthreads();
-    const int t = tid >> 4, c = blockIdx.x * 16 + (tid & 15);
-    if (t < n && c < a.vdim) o[((tok0 + t0 + t) * a.H + h) * a.vdim + c] = so[tid];
-  }
-  if (col < a.vdim) store_rows<RPL>(st_, r, s);
-}
-
 // Per-head RMS norm, weight and gate: one wave per (token, head). DELTA: the
 // weight is shared by heads and the gate a sigmoid; else a weight per head
 // and a silu.
-template <typename T, bool DELTA>
+template <typename T, bool DELTA, int PER>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(
     const float* __restrict__ o, const T* __restrict__ norm, const T* __restrict__ gate, T* __restrict__ out,
     int total, RecArgs a, Step step) {
-  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int id = blockIdx.x * 4 + (threadIdx.x >> 6), c = (threadIdx.x & 63) * PER;
   if (id >= total) return;
   const int h = id % a.H, tok = id / a.H, s = tok % a.S, b = tok / a.S;
-  const bool live = step.slot(b) >= 0 && s < step.len(b, a.S);
+  const bool live = step.slot(b) >= 0 && s < step.len(b, a.S), vec = (a.vdim & 3) == 0;
   const size_t src = ((size_t)tok * a.H + h) * a.vdim;
-  T* dst = out + (size_t)tok * a.K + a.out_at + h * a.vdim;
-  float x[4], ss = 0.f;
+  float x[PER], g[PER], w[PER], ss = 0.f;
+  ld_lane<PER>(o + src, c, live ? a.vdim : 0, vec, x);
+  ld_lane<PER>(gate + src, c, a.vdim, vec, g);
+  ld_lane<PER>(norm + (DELTA ? 0 : h * a.vdim), c, a.vdim, vec, w);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int c = lane + 64 * i;
-    x[i] = live && c < a.vdim ? o[src + c] : 0.f;
-    ss += x[i] * x[i];
-  }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+  for (int i = 0; i < PER; ++i) ss += x[i] * x[i];
+  const float inv = a.out_scale / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int c = lane + 64 * i;
-    if (c >= a.vdim) continue;
-    float y = 0.f;
-    if (live) {
-      const float gv = ld(gate + src + c);
-      y = x[i] * inv * ld(norm + (DELTA ? c : h * a.vdim + c)) * (DELTA ? sigmoidf(gv) : siluf(gv)) * a.out_scale;
-    }
-    st(dst + c, y);
-  }
+  for (int i = 0; i < PER; ++i) x[i] = live ? x[i] * inv * w[i] * (DELTA ? sigmoidf(g[i]) : siluf(g[i])) : 0.f;
+  st_lane<PER>(out + (size_t)tok * a.K + a.out_at + h * a.vdim, c, a.vdim, vec && ((a.K | a.out_at) & 3) == 0, x);
+}
+
+template <bool DELTA>
+static void launch_head_norm_gate(bool bf16, const torch::Tensor& o, const torch::Tensor& norm,
+                                  const torch::Tensor& gate, torch::Tensor& out, int heads, const RecArgs& a,
+                                  const Step& step, hipStream_t stream) {
+#define GATE(T, PER)                                                                                             \
+  hipLaunchKernelGGL((head_norm_gate_kernel<T, DELTA, PER>), dim3((heads + 3) / 4), dim3(256), 0, stream,       \
+                     (const float*)o.data_ptr(), (const T*)norm.data_ptr(), (const T*)gate.data_ptr(),          \
+                     (T*)out.data_ptr(), heads, a, step)
+#define GATE_WIDTH(T) \
+  if (a.vdim <= 64) GATE(T, 1); else if (a.vdim <= 128) GATE(T, 2); else GATE(T, 4);
+  if (bf16) { GATE_WIDTH(bf16_t) } else { GATE_WIDTH(float) }
+#undef GATE_WIDTH
+#undef GATE
 }
 
 // One token of one head, everything from projections to the gated output: a
@@ -1039,7 +1284,7 @@ __global__ __launch_bounds__(256) void rec_decode_kernel(
 }
 
 // n blends of the current and the previous token: out [n][B,S,D]
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void token_shift_kernel(
     const T* __restrict__ h, const T* __restrict__ mu, T* __restrict__ ring, T* __restrict__ out, int S, int D,
     int M, int n, size_t plane, Step step) {
@@ -1048,15 +1293,25 @@ __global__ __launch_bounds__(256) void token_shift_kernel(
   const bool live = slot >= 0 && s < len;
   const int first = live ? step.first(b) : 0;
   const size_t at = ((size_t)b * S + s) * D;
-  for (int d = threadIdx.x; d < D; d += 256) {
-    float x = 0.f, p = 0.f;
+  for (int d = threadIdx.x * V; d < D; d += 256 * V) {
+    float x[V], p[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) x[i] = p[i] = 0.f;
     if (live) {
-      x = ld(h + at + d);
-      if (s > 0) p = ld(h + at - D + d);
-      else if (first > 0) p = ld(ring + ((size_t)slot * M + (first - 1) % M) * D + d);
-      if (step.decode) st(ring + ((size_t)slot * M + first % M) * D + d, x);  // M >= 2: not the row just read
+      ldv<V>(h + at + d, x);
+      if (s > 0) ldv<V>(h + at - D + d, p);
+      else if (first > 0) ldv<V>(ring + ((size_t)slot * M + (first - 1) % M) * D + d, p);
+      if (step.decode) stv<V>(ring + ((size_t)slot * M + first % M) * D + d, x);  // M >= 2: not the row just read
     }
-    for (int i = 0; i < n; ++i) st(out + i * plane + at + d, x + (p - x) * ld(mu + (size_t)i * D + d));
+#pragma unroll
+    for (int i = 0; i < V; ++i) p[i] -= x[i];
+    for (int j = 0; j < n; ++j) {
+      float m[V];
+      ldv<V>(mu + (size_t)j * D + d, m);
+#pragma unroll
+      for (int i = 0; i < V; ++i) m[i] = x[i] + p[i] * m[i];
+      stv<V>(out + j * plane + at + d, m);
+    }
   }
 }
 
@@ -1303,14 +1558,34 @@ static int row_pad(int dim) {
     default: TORCH_CHECK(false, "padded key channels ", dp);                                               \
   }
 
+static int64_t chunk_count(int S) { return (S + CHUNK - 1) / CHUNK; }
+static int64_t chunk_size(bool delta, int dp) { return delta ? 49 * dp + 512 : 33 * dp + 256; }
+
 template <bool DELTA>
-static void launch_scan(int B, const Tensor& q, const Tensor& k, const Tensor& dec, const Tensor& v, const Tensor& beta,
-                        const Tensor& dot, Tensor& state, Tensor& o, const RecArgs& a, const Step& step) {
+static void launch_scan(int B, const Tensor& factors, const Tensor& v, Tensor& state, Tensor& o, const RecArgs& a,
+                        const Step& step) {
   BY_ROWS(a.dp, {
-    hipLaunchKernelGGL((scan_kernel<DELTA, R>), dim3((a.vdim + 15) / 16, a.H, B), dim3(256), 0, cur_stream(),
-                       P<float>(q), P<float>(k), P<float>(dec), P<float>(v), DELTA ? P<float>(beta) : nullptr,
-                       P<float>(dot), M<float>(state), M<float>(o), a, step);
+    hipLaunchKernelGGL((chunk_scan_kernel<DELTA, R>), dim3((a.vdim + 63) / 64, a.H, B), dim3(256), 0, cur_stream(),
+                       P<float>(factors), P<float>(v), M<float>(state), M<float>(o), (int)chunk_count(a.S), a, step);
   });
+}
+
+// channels per lane and, for the delta rule, taps as template arguments
+template <typename T, bool DELTA, int TAPS>
+static void launch_prep_width(int B, const T* x0, const T* x1, const T* x2, const T* c0, const T* c1, const T* c2,
+                              const T* pre, const T* d0, const T* d1, const T* ring, Tensor& factors, Tensor& v,
+                              const RecArgs& a, const Step& step) {
+  const int chunks = chunk_count(a.S), widest = std::max(a.vdim, a.dp);
+  TORCH_CHECK(chunks <= 65535 && B <= 65535, "a prefill step of ", B, " x ", a.S, " tokens is too large");
+  const dim3 grid(a.H, chunks, B);
+  const size_t lds = (3 * CHUNK * (a.dp + 4) + 512 + CHUNK) * sizeof(float);
+#define PREP(PER)                                                                                              \
+  hipLaunchKernelGGL((chunk_prep_kernel<T, DELTA, TAPS, PER>), grid, dim3(256), lds, cur_stream(), x0, x1, x2, c0, c1, \
+                     c2, pre, d0, d1, ring, M<float>(factors), M<float>(v), chunks, a, step)
+  if (widest <= 64) PREP(1);
+  else if (widest <= 128) PREP(2);
+  else PREP(4);
+#undef PREP
 }
 
 template <typename T>
@@ -1351,21 +1626,22 @@ void delta_rule(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t b
     }));
     return;
   }
-  auto q = f32(proj, {B, S, G, dp}), k = f32(proj, {B, S, G, dp}), dot = f32(proj, {B, S, G});
-  auto v = f32(proj, {B, S, H, vdim}), dec = f32(proj, {B, S, H, dp}), beta = f32(proj, {B, S, H});
-  auto o = f32(proj, {B, S, H, vdim});
-  const int prep = B * S * (int)G, heads = B * S * (int)H;
+  auto factors = f32(proj, {B, chunk_count(S), H, chunk_size(true, dp)});
+  auto v = f32(proj, {B, S, H, vdim}), o = f32(proj, {B, S, H, vdim});
+  const int heads = B * S * (int)H;
   BY_TYPE(dt, {
-    hipLaunchKernelGGL((delta_prep_kernel<T>), dim3((prep + 3) / 4), dim3(256), 0, stream, P<T>(proj), P<T>(qc),
-                       P<T>(kcv), P<T>(vcv), P<T>(pre), P<T>(a_log), P<T>(dt_), P<T>(ring), M<float>(q), M<float>(k),
-                       M<float>(dot), M<float>(v), M<float>(dec), M<float>(beta), prep, a, step);
+    auto prep = [&](auto launch) {
+      launch(B, P<T>(proj), (const T*)nullptr, (const T*)nullptr, P<T>(qc), P<T>(kcv), P<T>(vcv), P<T>(pre),
+             P<T>(a_log), P<T>(dt_), (const T*)P<T>(ring), factors, v, a, step);
+    };
+    if (taps == 2) prep(launch_prep_width<T, true, 2>);
+    else if (taps == 3) prep(launch_prep_width<T, true, 3>);
+    else if (taps == 4) prep(launch_prep_width<T, true, 4>);
+    else prep(launch_prep_width<T, true, 0>);
     remember<T>(proj, ring, B, S, N, Columns{{(int)q_at, (int)k_at, (int)v_at}, {(int)(G * dim), (int)(G * dim), (int)(H * vdim)}}, step);
   });
-  launch_scan<true>(B, q, k, dec, v, beta, dot, state, o, a, step);
-  BY_TYPE(dt, {
-    hipLaunchKernelGGL((head_norm_gate_kernel<T, true>), dim3((heads + 3) / 4), dim3(256), 0, stream, P<float>(o),
-                       P<T>(norm), P<T>(pre_gate), M<T>(out), heads, a, step);
-  });
+  launch_scan<true>(B, factors, v, state, o, a, step);
+  launch_head_norm_gate<true>(dt == torch::kBFloat16, o, norm, pre_gate, out, heads, a, step, stream);
 }
 
 Tensor wkv(Tensor r, Tensor k_, Tensor v_, Tensor gate, Tensor pre, Tensor w0, Tensor u, Tensor norm, int64_t H,
@@ -1392,19 +1668,16 @@ Tensor wkv(Tensor r, Tensor k_, Tensor v_, Tensor gate, Tensor pre, Tensor w0, T
     }));
     return out;
   }
-  auto q = f32(r, {B, S, H, dp}), k = f32(r, {B, S, H, dp}), dec = f32(r, {B, S, H, dp});
-  auto dot = f32(r, {B, S, H}), v = f32(r, {B, S, H, dim}), o = f32(r, {B, S, H, dim});
+  auto factors = f32(r, {B, chunk_count(S), H, chunk_size(false, dp)});
+  auto v = f32(r, {B, S, H, dim}), o = f32(r, {B, S, H, dim});
   const int heads = B * S * (int)H;
   BY_TYPE(dt, {
-    hipLaunchKernelGGL((wkv_prep_kernel<T>), dim3((heads + 3) / 4), dim3(256), 0, stream, P<T>(r), P<T>(k_), P<T>(v_),
-                       P<T>(pre), P<T>(w0), P<T>(u), M<float>(q), M<float>(k), M<float>(dot), M<float>(v),
-                       M<float>(dec), heads, a, step);
+    const T* none = nullptr;
+    launch_prep_width<T, false, 1>(B, P<T>(r), P<T>(k_), P<T>(v_), none, none, none, P<T>(pre), P<T>(w0), P<T>(u), none,
+                                   factors, v, a, step);
   });
-  launch_scan<false>(B, q, k, dec, v, dot, dot, state, o, a, step);
-  BY_TYPE(dt, {
-    hipLaunchKernelGGL((head_norm_gate_kernel<T, false>), dim3((heads + 3) / 4), dim3(256), 0, stream, P<float>(o),
-                       P<T>(norm), P<T>(gate), M<T>(out), heads, a, step);
-  });
+  launch_scan<false>(B, factors, v, state, o, a, step);
+  launch_head_norm_gate<false>(dt == torch::kBFloat16, o, norm, gate, out, heads, a, step, stream);
   return out;
 }
 
@@ -1419,8 +1692,12 @@ Tensor token_shift(Tensor h, Tensor mu, Tensor ring, OptT slots, OptT positions,
   if (B == 0 || S == 0) return out;
   const Step step = make_step(slots, positions, lens, start, decode, B);
   BY_TYPE(dt, {
-    hipLaunchKernelGGL((token_shift_kernel<T>), dim3(S, B), dim3(256), 0, cur_stream(), P<T>(h), P<T>(mu), M<T>(ring),
-                       M<T>(out), S, D, (int)ring.size(1), n, (size_t)B * S * D, step);
+    if (D % 4 == 0)
+      hipLaunchKernelGGL((token_shift_kernel<T, 4>), dim3(S, B), dim3(256), 0, cur_stream(), P<T>(h), P<T>(mu),
+                         M<T>(ring), M<T>(out), S, D, (int)ring.size(1), n, (size_t)B * S * D, step);
+    else
+      hipLaunchKernelGGL((token_shift_kernel<T, 1>), dim3(S, B), dim3(256), 0, cur_stream(), P<T>(h), P<T>(mu),
+                         M<T>(ring), M<T>(out), S, D, (int)ring.size(1), n, (size_t)B * S * D, step);
     if (!decode) remember<T>(h, ring, B, S, D, Columns{{0, 0, 0}, {D, 0, 0}}, step);
   });
   return out;

@@ -109,9 +109,14 @@ DEVINL void stv(T* p, const float* o) {
     for (int i = 0; i < V; ++i) st(p + i, o[i]);
 }
 
-DEVINL float sigmoidf(float x) { return 1.f / (1.f + expf(-x)); }
-DEVINL float siluf(float x) { return x / (1.f + expf(-x)); }
-DEVINL float softplusf(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+// hardware exp2/log2/rcp (about one ulp each)
+DEVINL float sigmoidf(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+DEVINL float siluf(float x) { return x * sigmoidf(x); }
+// log1p(e) = log(u) e / (u - 1) with u = 1 + e as rounded: exact where e is tiny
+DEVINL float softplusf(float x) {
+  const float e = __expf(-fabsf(x)), u = 1.f + e;
+  return fmaxf(x, 0.f) + (u == 1.f ? e : __logf(u) * e * __builtin_amdgcn_rcpf(u - 1.f));
+}
 
 // sum over the 16 lanes of a DPP row, in every lane (row_ror:8, 4, 2, 1)
 DEVINL float row_sum(float v) {
@@ -844,7 +849,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(
       ck.begin(s0 + t0, C, a);
       cv.begin(s0 + t0, C, a);
     }
-    const float A = expf(ld(d0 + h)), qscale = 1.f / sqrtf((float)a.dim);
+    const float A = __expf(ld(d0 + h)), qscale = 1.f / sqrtf((float)a.dim);
     ld_lane<PER>(d1 + (size_t)h * a.dim, c, a.dim, (a.dim & 3) == 0, bias);
     for (int t = t0; t < t0 + 4; ++t) {
       const int s = s0 + t;
@@ -898,7 +903,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(
         st_lane<PER>(v + src, c, a.dim, vec, y);
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
-          lg[i] = c + i < a.dim ? -expf(lg[i] + bias[i]) : 0.f;
+          lg[i] = c + i < a.dim ? -__expf(lg[i] + bias[i]) : 0.f;
           bonus += q[i] * k[i] * u[i];
         }
       }
@@ -917,7 +922,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(
       run += sl[t * dps + d];
       sl[t * dps + d] = run;
     }
-    out[32 * a.dp + d] = expf(run);
+    out[32 * a.dp + d] = __expf(run);
   }
   __syncthreads();
   if (tid < 136) {  // pairs s <= t
@@ -965,14 +970,14 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(
       ld4(sk + t * dps + d, k);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        l[i] = expf(l[i]);
+        l[i] = __expf(l[i]);
         k[i] *= l[i];
         q[i] *= l[i];
       }
       st4(out + 33 * a.dp + 512 + t * a.dp + d, k);
     } else {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) q[i] *= expf(l[i]);
+      for (int i = 0; i < 4; ++i) q[i] *= __expf(l[i]);
     }
     st4(out + t * a.dp + d, q);
   }
@@ -981,7 +986,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(
     const float end = sl[(CHUNK - 1) * dps + d];
     float k[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) k[i] = sk[(t + i) * dps + d] * expf(end - sl[(t + i) * dps + d]);
+    for (int i = 0; i < 4; ++i) k[i] = sk[(t + i) * dps + d] * __expf(end - sl[(t + i) * dps + d]);
     st4(out + 16 * a.dp + e * 4, k);
   }
   __syncthreads();
@@ -1005,18 +1010,24 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(
 // i*16 + quad*4 + r of its column, so the accumulators are at the same time
 // the right-hand operands of the products with S: step (i, r) of an
 // f32 16x16x4 MFMA contracts the four channels its quads hold.
-template <bool DELTA, int NI>
+// KS > 1: KS of a block's 4 waves share a column group, each holding its part
+// of the channels, and add their partial products through LDS (more blocks and
+// shorter chunks where there are few sequences).
+template <bool DELTA, int NI, int KS>
 __global__ __launch_bounds__(256) void chunk_scan_kernel(
     const float* __restrict__ factors, const float* __restrict__ v, float* __restrict__ state, float* __restrict__ o,
     int chunks, RecArgs a, Step step) {
   constexpr int DP = 16 * NI, QS = DP + 4, TS = 20;  // padded LDS rows: no bank conflicts
   constexpr int FLOATS = DELTA ? 49 * DP + 512 : 33 * DP + 256, NL = (FLOATS / 4 + 255) / 256;
+  constexpr int NT = NI / KS;  // tiles of this wave
   constexpr int AT_KT = 16 * QS, AT_E = AT_KT + DP * TS, AT_B = AT_E + DP, AT_T = AT_B + 16 * TS, AT_K = AT_T + 16 * TS;
   __shared__ __attribute__((aligned(16))) float lds[DELTA ? AT_K + 16 * QS : AT_T];
+  __shared__ floatx4 part_p[KS > 1 && DELTA ? 256 : 1], part_o[KS > 1 ? 256 : 1];
   const int h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x;
   const int slot = step.slot(b), len = step.len(b, a.S);
   if (slot < 0) return;
-  const int lane = tid & 63, m = lane & 15, quad = lane >> 4, col = (blockIdx.x * 4 + (tid >> 6)) * 16 + m;
+  const int lane = tid & 63, m = lane & 15, quad = lane >> 4, ks = (tid >> 6) % KS;
+  const int col = (blockIdx.x * (4 / KS) + (tid >> 6) / KS) * 16 + m, d0 = ks * NT * 16 + quad * 4;
   const bool mine = col < a.vdim;
   // where this thread's float4s of a chunk's factors go
   int dst[NL];
@@ -1030,11 +1041,11 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
     else if (e < 33 * DP + 512) { e -= 33 * DP + 256; dst[i] = AT_T + e / 16 * TS + e % 16; }
     else { e -= 33 * DP + 512; dst[i] = AT_K + e / DP * QS + e % DP; }
   }
-  floatx4 S[NI];
-  float* base = state + (((size_t)slot * a.H + h) * a.vdim + (mine ? col : 0)) * DP + quad * 4;
+  floatx4 S[NT];
+  float* base = state + (((size_t)slot * a.H + h) * a.vdim + (mine ? col : 0)) * DP + d0;
   const bool fresh = step.first(b) == 0;
 #pragma unroll
-  for (int i = 0; i < NI; ++i) S[i] = fresh || !mine ? (floatx4)(0.f) : *(const floatx4*)(base + i * 16);
+  for (int i = 0; i < NT; ++i) S[i] = fresh || !mine ? (floatx4)(0.f) : *(const floatx4*)(base + i * 16);
   const size_t tok0 = (size_t)b * a.S, vstride = (size_t)a.H * a.vdim, vcol = (size_t)h * a.vdim + col;
   floatx4 rf[NL], rv;
   auto fetch = [&](int t0) {
@@ -1061,14 +1072,25 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
     if (t0 + CHUNK < len) fetch(t0 + CHUNK);
     floatx4 O = (floatx4)(0.f), P = (floatx4)(0.f);
 #pragma unroll
-    for (int i = 0; i < NI; ++i) {
-      const floatx4 q4 = *(const floatx4*)(lds + m * QS + i * 16 + quad * 4);
+    for (int i = 0; i < NT; ++i) {
+      const floatx4 q4 = *(const floatx4*)(lds + m * QS + i * 16 + d0);
       floatx4 k4;
-      if (DELTA) k4 = *(const floatx4*)(lds + AT_K + m * QS + i * 16 + quad * 4);
+      if (DELTA) k4 = *(const floatx4*)(lds + AT_K + m * QS + i * 16 + d0);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         if (DELTA) P = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[r], S[i][r], P, 0, 0, 0);
         O = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[r], S[i][r], O, 0, 0, 0);
+      }
+    }
+    if (KS > 1) {
+      if (DELTA) part_p[tid] = P;
+      part_o[tid] = O;
+      __syncthreads();
+#pragma unroll
+      for (int i = 1; i < KS; ++i) {
+        const int other = tid + (((ks + i) % KS) - ks) * 64;
+        if (DELTA) P += part_p[other];
+        O += part_o[other];
       }
     }
     floatx4 U = V;
@@ -1082,21 +1104,21 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(b4[r], U[r], O, 0, 0, 0);
 #pragma unroll
-    for (int i = 0; i < NI; ++i) S[i] *= *(const floatx4*)(lds + AT_E + i * 16 + quad * 4);
+    for (int i = 0; i < NT; ++i) S[i] *= *(const floatx4*)(lds + AT_E + i * 16 + d0);
 #pragma unroll
     for (int r = 0; r < 4; ++r)  // tiles innermost: consecutive MFMAs are independent
 #pragma unroll
-      for (int i = 0; i < NI; ++i)
-        S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(lds[AT_KT + (i * 16 + m) * TS + quad * 4 + r], U[r], S[i], 0, 0, 0);
+      for (int i = 0; i < NT; ++i)
+        S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(lds[AT_KT + ((ks * NT + i) * 16 + m) * TS + quad * 4 + r], U[r], S[i], 0, 0, 0);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = t0 + quad * 4 + r;
-      if (mine && t < len) o[(tok0 + t) * vstride + vcol] = O[r];
+      if (mine && ks == 0 && t < len) o[(tok0 + t) * vstride + vcol] = O[r];
     }
   }
   if (mine && len > 0)
 #pragma unroll
-    for (int i = 0; i < NI; ++i) *(floatx4*)(base + i * 16) = S[i];
+    for (int i = 0; i < NT; ++i) *(floatx4*)(base + i * 16) = S[i];
 }
 
 // rows of the state that lane r (0..15) of a column holds: vectors of V
@@ -1564,10 +1586,19 @@ static int64_t chunk_size(bool delta, int dp) { return delta ? 49 * dp + 512 : 3
 template <bool DELTA>
 static void launch_scan(int B, const Tensor& factors, const Tensor& v, Tensor& state, Tensor& o, const RecArgs& a,
                         const Step& step) {
+  const int groups = (a.vdim + 15) / 16 * a.H * B;  // of 16 columns
+#define SCAN(KS)                                                                                                    \
+  hipLaunchKernelGGL((chunk_scan_kernel<DELTA, R, KS>), dim3((a.vdim + 64 / KS - 1) / (64 / KS), a.H, B), dim3(256), 0, \
+                     cur_stream(), P<float>(factors), P<float>(v), M<float>(state), M<float>(o),                    \
+                     (int)chunk_count(a.S), a, step)
   BY_ROWS(a.dp, {
-    hipLaunchKernelGGL((chunk_scan_kernel<DELTA, R>), dim3((a.vdim + 63) / 64, a.H, B), dim3(256), 0, cur_stream(),
-                       P<float>(factors), P<float>(v), M<float>(state), M<float>(o), (int)chunk_count(a.S), a, step);
+    constexpr int TWO = R % 2 ? 1 : 2, FOUR = R % 4 ? TWO : 4;
+    // split channels while the chip's 1024 SIMDs are not covered
+    if (groups * 4 <= 1024) SCAN(FOUR);
+    else if (groups * 2 <= 1024) SCAN(TWO);
+    else SCAN(1);
   });
+#undef SCAN
 }
 
 // channels per lane and, for the delta rule, taps as template arguments

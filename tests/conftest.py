@@ -11,7 +11,7 @@ os.environ.setdefault("XOT_OFFLINE", "1")
 
 
 def pytest_configure(config):
-  config.addinivalue_line("markers", "gpu: needs a real MI355X GPU (run via gpurun)")
+  config.addinivalue_line("markers", "gpu: needs a real MI355X GPU")
 
 
 def pytest_collection_modifyitems(config, items):

@@ -252,7 +252,7 @@ def test_attention_rows_are_independent(kind):
   assert all((t[0] == u).all() for t, u in zip(state, before))
 
 
-REC = [(4, 2, 12, 20, 4), (3, 3, 40, 16, 2), (2, 1, 64, 64, 3), (1, 1, 128, 128, 1), (2, 2, 90, 33, 4), (2, 2, 256, 200, 3)]
+REC = [(4, 2, 12, 20, 4), (3, 3, 40, 16, 2), (2, 1, 64, 64, 3), (1, 1, 128, 128, 1), (2, 2, 90, 33, 4), (2, 2, 256, 200, 3), (2, 1, 20, 24, 6)]
 
 
 class Delta:

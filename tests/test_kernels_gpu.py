@@ -466,7 +466,7 @@ def test_rope_qkv_append_qk_norm(hip, hd, H, KVH, S):
   assert torch.equal(vc, vc_ref)
 
 
-# ---------------- round 2: xreg GEMM + gemma2 attention semantics ----------------
+# ---------------- xreg GEMM + gemma2 attention semantics ----------------
 
 @pytest.mark.parametrize("M,K,N", [(64, 512, 256), (128, 4096, 1280), (128, 2048, 512), (256, 1024, 384)])
 def test_skinny_gemm_packed_xreg(hip, M, K, N):
@@ -1012,7 +1012,7 @@ def test_spec_self_draft_full_acceptance():
   """Draft == target (same seed -> identical weights): acceptance must stay
   ~1.0 across MANY rounds. Catches the draft-cache hole regression (a fully
   accepted round used to leave one unwritten KV row in the draft cache,
-  collapsing acceptance to ~0.06 from round 2 on)."""
+  collapsing acceptance to ~0.06 after the first proposal round)."""
   import torch
   from xotorch_amd.engine.spec import SpeculativeDecoder
   sd = SpeculativeDecoder.from_model_ids("llama-3-8b", "llama-3-8b",

@@ -297,7 +297,7 @@ def test_registry_consistency():
 
 def test_pack_decode_weight_is_a_permutation():
   """The MFMA prepack is a pure permutation of W: inverting the documented
-  index map (docs/KERNELS.md) must recover W exactly, and every element must
+  index map must recover W exactly, and every element must
   land where the kernel's A-fragment load expects it:
   packed[n32][kt][half][n][e] == W[n32*32+n][kt*16+half*8+e]."""
   import torch

@@ -1,5 +1,5 @@
 """Node orchestration tests: single-node decode, two-node TCP ring (the
-reference's multi-node-without-cluster pattern — SURVEY.md §4), elastic
+reference's multi-node-without-cluster pattern), elastic
 topology, ring training over the wire."""
 import torch
 import asyncio

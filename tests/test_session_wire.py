@@ -49,7 +49,7 @@ async def _make_tcp_pair(tmp_path, engine_cls):
 @pytest.mark.timeout(120)
 def test_sessions_cleared_on_both_stages(tmp_path):
   """After a request finishes, NO stage of the ring may still hold its KV
-  session (round-1 leak: only the sampling stage cleared)."""
+  session (not only of the sampling stage)."""
   async def go():
     nodes = await _make_tcp_pair(tmp_path, lambda: TorchEngine(device="cpu", dtype=torch.float32))
     a, b = nodes
@@ -76,7 +76,7 @@ def test_sessions_cleared_on_both_stages(tmp_path):
 @pytest.mark.timeout(120)
 def test_training_sessions_cleared(tmp_path):
   """Ring training forwards create KV sessions per example on non-last
-  stages; they must be cleared after each example (ADVICE medium)."""
+  stages; they must be cleared after each example."""
   async def go():
     nodes = await _make_tcp_pair(tmp_path, lambda: TorchEngine(device="cpu", dtype=torch.float32))
     a, b = nodes
@@ -123,7 +123,7 @@ def test_bf16_hidden_on_wire():
 
 def test_evaluate_leaves_no_grads():
   """evaluate() must not backward: grads stay None so the next optimizer
-  step only sees its own batch (ADVICE low)."""
+  step only sees its own batch."""
   async def go():
     eng = TorchEngine(device="cpu", dtype=torch.float32)
     shard = build_full_shard("dummy", "TorchEngine")

@@ -4,7 +4,7 @@ Parity with the reference's engine ABC
 (/root/reference/xotorch/inference/inference_engine.py:11-74) with the
 capability gap closed: `train`/`evaluate` are part of the contract and are
 actually implemented by the engines here (the reference declares the calls at
-node.py:317-333 but ships no implementation — SURVEY.md §3.4).
+node.py:317-333 but ships no implementation).
 """
 from __future__ import annotations
 

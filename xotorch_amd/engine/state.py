@@ -2,7 +2,7 @@
 
 The reference serializes tokens + the FULL causal mask + input_pos as JSON
 lists on every pipeline hop (/root/reference/xotorch/inference/torch/llm_utils.py:593-631
-— O(T·max_seq) per token, SURVEY.md §5 "known absurdity"). Here each stage
+— O(T·max_seq) per token). Here each stage
 keeps positions/caches device-resident and only {curr_pos, seq_len} metadata
 travels on the control plane.
 """

@@ -10,7 +10,7 @@ with e-score correction bias, group-limited top-k (n_group/topk_group),
 routed scaling and always-on shared experts; the first k layers are dense.
 
 The reference lists deepseek-v3 / r1 cards its torchtune GQA assembly cannot
-run (SURVEY.md appendix); here the family runs the absorbed-latent
+run; here the family runs the absorbed-latent
 MLA MFMA decode path on GPU (hip_ops.hip: mla_prep_append / mla_q_prep /
 attn_decode_mla) and a plain-torch path on CPU, both validated against
 transformers' DeepseekV3ForCausalLM on tiny random configs (the full 671B

@@ -200,7 +200,7 @@ class Attention(nn.Module):
     """Cache-free causal attention (training/eval): the SAME modules and
     weights as the inference path, autograd-safe ops (fp32 sdpa). This is
     the one and only training forward — the engine calls the model, so the
-    two paths cannot drift (round-1 VERDICT weak #7)."""
+    two paths cannot drift."""
     import torch.nn.functional as F
     B, S, _ = x.shape
     cfg = self.cfg

@@ -269,8 +269,8 @@ model_cards: Dict[str, dict] = {
   "nemotron-70b": {"layers": 80, "repo": {"TorchEngine": "nvidia/Llama-3.1-Nemotron-70B-Instruct-HF", "HIPEngine": "nvidia/Llama-3.1-Nemotron-70B-Instruct-HF"}},
   # Listed for registry parity with the reference but with NO supported
   # engine here: llava needs a vision tower + image path (the reference
-  # lists it too; its torchtune GQA assembly cannot run it either —
-  # SURVEY.md appendix). get_supported_models() filters it out.
+  # lists it too; its torchtune GQA assembly cannot run it either).
+  # get_supported_models() filters it out.
   "qwen-3-0.6b": {"layers": 28, "repo": {"TorchEngine": "Qwen/Qwen3-0.6B", "HIPEngine": "Qwen/Qwen3-0.6B"}},
   "qwen-3-8b": {"layers": 36, "repo": {"TorchEngine": "Qwen/Qwen3-8B", "HIPEngine": "Qwen/Qwen3-8B"}},
   "qwen-3-32b": {"layers": 64, "repo": {"TorchEngine": "Qwen/Qwen3-32B", "HIPEngine": "Qwen/Qwen3-32B"}},
@@ -287,7 +287,7 @@ model_cards: Dict[str, dict] = {
   # modes instead); listed for id parity, filtered like llava
   "llama-3.1-405b-8bit": {"layers": 126, "repo": {}},
   # llava needs PIL for the image path (not present in this environment);
-  # the reference's vision handling is also vestigial (SURVEY.md appendix)
+  # the reference's vision handling is also vestigial
   "llava-1.5-7b-hf": {"layers": 32, "repo": {}},
   "didipel-1b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "didipel-7b": {"layers": 24, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},

@@ -1,7 +1,7 @@
 // xotorch_amd CDNA4 (gfx950 / MI355X) kernels for the transformer hot path.
 //
 // These replace the ops the reference delegates to torchtune
-// (SURVEY.md §2.2 op table; reference call sites cited per kernel below):
+// (reference call sites cited per kernel below):
 //   - fused residual-add + RMSNorm      (llm_utils.py:465-476)
 //   - fused RoPE rotate + KV-cache append, dual layout (general_mha.py:78-106)
 //   - GQA attention, prefill AND decode, on matrix cores
@@ -16,7 +16,7 @@
 //     TunableOp-tuned hipBLASLt at runtime
 //   - SwiGLU activation                  (llm_utils.py:491-500)
 //
-// Design notes (per /opt/skills/guides/cdna_hip_programming.md):
+// Design notes:
 //   * wave = 64 lanes; all block sizes are multiples of 64
 //   * bf16 is loaded vectorized (ushort8 = 16 B per lane); the big streamed
 //     operands (weights, KV) are pre-shuffled ONCE into MFMA fragment order
@@ -1733,7 +1733,7 @@ __global__ __launch_bounds__(256) void skinny_gemm_kernel(
 // and read back as B fragments.  K % 64 == 0 required.
 // ---------------------------------------------------------------------------
 
-// Also the MoE grouped-GEMM kernel (SURVEY.md §2.2: the reference's latent
+// Also the MoE grouped-GEMM kernel (the reference's latent
 // MOEExpert/MOELayer scaffolding, llm_utils.py:502-590, never executed): for
 // Mixtral-class decode each expert e (blockIdx.y) computes its own
 // [C, N] = [C, K] @ Wp_e^T over a fixed per-expert token capacity C — one

@@ -2,8 +2,7 @@
 
 These are the numerics oracle for the HIP kernels (tests compare the HIP path
 against these in fp32) and the CPU execution path for the plumbing tests.
-They implement the same ops the reference delegates to torchtune
-(SURVEY.md §2.2 table), with HF "rotate-half" RoPE convention so HF
+They implement the same ops the reference delegates to torchtune, with HF "rotate-half" RoPE convention so HF
 safetensors load without the q/k permute torchtune needs
 (/root/reference/xotorch/inference/torch/llm_utils.py:175-183).
 """

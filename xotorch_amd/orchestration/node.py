@@ -372,7 +372,7 @@ class Node:
     callbacks, and when the request is finished release OUR stage's state:
     on a multi-node ring the first/middle stages hold KV sessions that only
     the sampling stage used to clear — at 70B/B=128 that is GBs per request
-    accumulating forever (round-1 VERDICT weak #4)."""
+    accumulating forever."""
     self.trigger_on_token_callbacks(request_id, result or [], is_finished)
     if is_finished:
       self.outstanding_requests.pop(request_id, None)

@@ -1,8 +1,8 @@
 """Request tracing: per-request spans, token-group spans, W3C traceparent.
 
 The reference ships an OpenTelemetry tracer that is never imported by the
-main path (/root/reference/xotorch/orchestration/tracing.py — latent,
-SURVEY.md §5). Here tracing is wired in for real: Node opens a request span
+main path (/root/reference/xotorch/orchestration/tracing.py — latent).
+Here tracing is wired in for real: Node opens a request span
 on process_prompt, token-group spans every TOKEN_GROUP_SIZE sampled tokens,
 and the traceparent string travels on the wire so multi-host rings correlate.
 Spans export to OpenTelemetry when the SDK is importable, else to an

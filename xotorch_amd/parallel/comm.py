@@ -1,6 +1,6 @@
 """torch.distributed (RCCL on GPU / gloo on CPU) process-group helpers.
 
-This replaces the reference's gRPC-per-hop transport (SURVEY.md §2.4): stage
+This replaces the reference's gRPC-per-hop transport: stage
 hops are point-to-point send/recv of resident bf16 hidden states over a
 single xGMI link; token wrap-around is a tiny int send; gradient all-reduce
 for the DP train path uses the communicator's topology-aware algorithms.
@@ -19,12 +19,11 @@ def init_distributed(backend: Optional[str] = None) -> tuple[int, int]:
   """Initialize from torchrun env vars; no-op single-process if absent.
 
   Backend selection: RCCL ("nccl") whenever every rank can own its own GPU.
-  RCCL refuses two ranks on one device ("Duplicate GPU detected" — that is
-  what killed the round-1 2-ranks/1-GPU attempt, gpurun_out/b8_2rank.log),
+  RCCL refuses two ranks on one device ("Duplicate GPU detected"),
   so when WORLD_SIZE exceeds the visible GPU count we fall back to gloo for
   the process group while compute stays on the GPU (tensors are staged
   through pinned CPU buffers for the hops — see RingComm). That makes
-  multi-rank verification runnable in a 1-GPU lease; on the driver's 8-GPU
+  multi-rank verification runnable in a 1-GPU lease; on an 8-GPU
   node each rank gets its own device and the path is pure RCCL over xGMI.
 
   Returns (rank, world_size).

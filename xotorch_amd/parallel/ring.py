@@ -1,7 +1,7 @@
 """Ring pipeline-parallel decode: one process per GPU, RCCL p2p over xGMI.
 
 This is the MI355X-native replacement for the reference's per-hop gRPC
-serialization (SURVEY.md §2.4): contiguous layer shards per rank (the ring
+serialization: contiguous layer shards per rank (the ring
 memory-weighted partitioning degenerates to equal layer counts on equal-HBM
 GPUs), bf16 hidden states moved rank→rank with torch.distributed send/recv
 (one xGMI link per hop, full bandwidth), sampled tokens looped back to stage

@@ -1,7 +1,7 @@
 """LoRA adapters for the sharded decoder.
 
-The reference's train CLI is LoRA-flavored (sample data under train/data/lora,
-SURVEY.md §3.4) but ships no engine implementation. Here: low-rank A/B
+The reference's train CLI is LoRA-flavored (sample data under train/data/lora)
+but ships no engine implementation. Here: low-rank A/B
 adapters wrap the projection Linears of a ShardedModel; base weights freeze;
 merge/unmerge supported for inference; adapter state dicts save/load
 separately (small checkpoints).

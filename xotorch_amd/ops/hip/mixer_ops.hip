@@ -43,9 +43,6 @@ DEVINL bf16_t f2b(float f) {
 }
 DEVINL void st(bf16_t* p, float f) { *p = f2b(f); }
 DEVINL void st(float* p, float f) { *p = f; }
-// the value as the element type holds it
-DEVINL float rounded(float f, const bf16_t*) { bf16_t b = f2b(f); return ld(&b); }
-DEVINL float rounded(float f, const float*) { return f; }
 
 DEVINL void ld4(const float* p, float* o) {
   const floatx4 v = *(const floatx4*)p;
@@ -326,34 +323,79 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(
   }
   const T* row = proj + ((size_t)b * a.S + s) * a.N;
   __shared__ float red[8];
+  const int dim = ring.dim, nq = a.H * dim, nk = a.G * dim;
+  const bool vec = ((dim | a.q_at | a.k_at | a.N) & 7) == 0;
   float qs = 0.f, ks = 0.f;
-  for (int i = threadIdx.x; i < a.H * ring.dim; i += 256) { const float f = ld(row + a.q_at + i); qs += f * f; }
-  for (int i = threadIdx.x; i < a.G * ring.dim; i += 256) { const float f = ld(row + a.k_at + i); ks += f * f; }
-  const float qi = 1.f / sqrtf(block_sum(qs, red) / (float)(a.H * ring.dim) + a.eps);
-  const float ki = 1.f / sqrtf(block_sum(ks, red + 4) / (float)(a.G * ring.dim) + a.eps);
-  T* qrow = qw + ((size_t)b * a.S + s) * a.H * a.qd;
-  for (int i = threadIdx.x; i < a.H * a.qd; i += 256) {
-    const int h = i / a.qd, d = i - h * a.qd;
-    const int j = h * ring.dim + d;
-    st(qrow + i, d < ring.dim ? ld(row + a.q_at + j) * qi * ld(qn + j) : 0.f);
+  if (vec) {
+    for (int i = threadIdx.x * 4; i < nq + nk; i += 1024) {
+      float x[4];
+      ld4(row + (i < nq ? a.q_at + i : a.k_at + i - nq), x);
+      const float f = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+      if (i < nq) qs += f;
+      else ks += f;
+    }
+  } else {
+    for (int i = threadIdx.x; i < nq; i += 256) { const float f = ld(row + a.q_at + i); qs += f * f; }
+    for (int i = threadIdx.x; i < nk; i += 256) { const float f = ld(row + a.k_at + i); ks += f * f; }
   }
+  const float qi = 1.f / sqrtf(block_sum(qs, red) / (float)nq + a.eps);
+  const float ki = 1.f / sqrtf(block_sum(ks, red + 4) / (float)nk + a.eps);
+  T* qrow = qw + ((size_t)b * a.S + s) * a.H * a.qd;
   const int pos = step.first(b) + s;
   const bool keep = s >= len - ring.rows;
   const int rrow = pos % ring.rows;
-  for (int i = threadIdx.x; i < a.G * (kdims + vdims); i += 256) {
-    const int g = i / (kdims + vdims), d = i - g * (kdims + vdims);
-    const size_t rh = (size_t)slot * a.G + g, wh = (size_t)b * a.G + g;
-    if (d < kdims) {
-      const int j = g * ring.dim + d;
-      const float f = d < ring.dim ? ld(row + a.k_at + j) * ki * ld(kn + j) : 0.f;
-      if (keep) st(kc + L::kbase(ring, rh) + L::k(ring, rrow, d), f);
-      if (kw) st(kw + L::kbase(ws, wh) + L::k(ws, hist + s, d), f);
-    } else {
-      const int c = d - kdims;
-      const float f = c < ring.vdim ? ld(row + a.v_at + g * ring.vdim + c) : 0.f;
-      if (keep) st(vc + L::vbase(ring, rh) + L::v(ring, rrow, c), f);
-      if (kw) st(vw + L::vbase(ws, wh) + L::v(ws, hist + s, c), f);
+  if (vec) {
+    // 8 channels at a time: they lie side by side in q rows and in both key
+    // layouts; padded channels are zero
+    const int gq = a.qd >> 3, gk = kdims >> 3;
+    for (int i = threadIdx.x; i < a.H * gq + a.G * gk; i += 256) {
+      const bool is_q = i < a.H * gq;
+      const int e = is_q ? i : i - a.H * gq, h = e / (is_q ? gq : gk), d = (e - h * (is_q ? gq : gk)) * 8;
+      float x[8], w[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = 0.f;
+      if (d < dim) {
+        const T *src = row + (is_q ? a.q_at : a.k_at) + h * dim + d, *wt = (is_q ? qn : kn) + h * dim + d;
+        ld4(src, x);
+        ld4(src + 4, x + 4);
+        ld4(wt, w);
+        ld4(wt + 4, w + 4);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] *= (is_q ? qi : ki) * w[j];
+      }
+      if (is_q) {
+        st4(qrow + h * a.qd + d, x);
+        st4(qrow + h * a.qd + d + 4, x + 4);
+        continue;
+      }
+      if (keep) {
+        T* dst = kc + L::kbase(ring, (size_t)slot * a.G + h) + L::k(ring, rrow, d);
+        st4(dst, x);
+        st4(dst + 4, x + 4);
+      }
+      if (kw) {
+        T* dst = kw + L::kbase(ws, (size_t)b * a.G + h) + L::k(ws, hist + s, d);
+        st4(dst, x);
+        st4(dst + 4, x + 4);
+      }
     }
+  } else {
+    for (int i = threadIdx.x; i < a.H * a.qd; i += 256) {
+      const int h = i / a.qd, d = i - h * a.qd, j = h * dim + d;
+      st(qrow + i, d < dim ? ld(row + a.q_at + j) * qi * ld(qn + j) : 0.f);
+    }
+    for (int i = threadIdx.x; i < a.G * kdims; i += 256) {
+      const int g = i / kdims, d = i - g * kdims, j = g * dim + d;
+      const float f = d < dim ? ld(row + a.k_at + j) * ki * ld(kn + j) : 0.f;
+      if (keep) st(kc + L::kbase(ring, (size_t)slot * a.G + g) + L::k(ring, rrow, d), f);
+      if (kw) st(kw + L::kbase(ws, (size_t)b * a.G + g) + L::k(ws, hist + s, d), f);
+    }
+  }
+  for (int i = threadIdx.x; i < a.G * vdims; i += 256) {
+    const int g = i / vdims, c = i - g * vdims;
+    const float f = c < ring.vdim ? ld(row + a.v_at + g * ring.vdim + c) : 0.f;
+    if (keep) st(vc + L::vbase(ring, (size_t)slot * a.G + g) + L::v(ring, rrow, c), f);
+    if (kw) st(vw + L::vbase(ws, (size_t)b * a.G + g) + L::v(ws, hist + s, c), f);
   }
 }
 

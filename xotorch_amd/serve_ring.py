@@ -141,6 +141,7 @@ class RingSlotWorker:
     self.tok_buf = torch.zeros(slots, 1, dtype=torch.int64, device=dev)
     self.hid_buf = torch.zeros(slots, 1, D, dtype=self.hid_dtype, device=dev)
     self.slot_map = torch.full((slots,), -1, dtype=torch.int32, device=dev)  # -1: parked
+    self._mapped = [-1] * slots  # what slot_map holds
     self.logits_buf: Optional[torch.Tensor] = None
     self.hid_out: Optional[torch.Tensor] = None
     # control/broadcast buffers
@@ -198,7 +199,10 @@ class RingSlotWorker:
     (prerequisite for interleaving chunked prefill with decode ticks)."""
     idle = [i for i in range(self.slots) if not self.active[i]]
     if self.slot_indexed:
-      self.slot_map.copy_(torch.tensor([i if on else -1 for i, on in enumerate(self.active)], dtype=torch.int32))
+      mapped = [i if on else -1 for i, on in enumerate(self.active)]
+      if mapped != self._mapped:
+        self.slot_map.copy_(torch.tensor(mapped, dtype=torch.int32))
+        self._mapped = mapped
     if idle:
       idx = torch.tensor(idle, dtype=torch.int64, device=self.positions.device)
       self.positions[idx] = self.max_seq - 1
@@ -309,6 +313,7 @@ class RingSlotWorker:
     self.positions[slot] = plen
     self.seq_lens[slot] = plen + 1
     self.slot_map[slot] = slot
+    self._mapped[slot] = slot
     self.active[slot] = True
 
   def _release(self, slots: List[int]):

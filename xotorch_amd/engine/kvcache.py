@@ -125,8 +125,7 @@ class MixerStateCache:
     from xotorch_amd.models.mixers import MIXERS
     self.batch, self.capacity = slots, capacity
     self.caches: List[list] = []
-    for lid in range(shard.start_layer, shard.end_layer + 1):
-      spec = cfg.layer_specs[lid]
+    for spec in cfg.shard_specs(shard).values():
       self.caches.append([
         tuple(torch.zeros(slots, *shape, dtype=dt, device=device) for shape, dt in branch.values())
         for branch in MIXERS[spec.mixer].state_spec(spec.params, capacity, dtype, device)

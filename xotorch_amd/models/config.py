@@ -11,7 +11,7 @@ from __future__ import annotations
 import json
 import math
 import os
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from pathlib import Path
 from typing import Dict, List, Optional, Tuple
 
@@ -107,7 +107,13 @@ class ModelConfig:
   # designs whose layers differ (models/layered.py); None → n_layers alike
   layer_specs: Optional[List[LayerSpec]] = None
   residual_mult: float = 1.0  # what a sublayer's output is scaled with
-  carried_dim: int = 0        # channels that travel with the stream (an early layer's values)
+  embed_scale: float = 1.0    # what embeddings are scaled with
+  # what travels with the stream between ring stages besides it: name -> channels
+  carried: Dict[str, int] = field(default_factory=dict)
+
+  @property
+  def carried_dim(self) -> int:
+    return sum(self.carried.values())
 
   @property
   def hidden_dim(self) -> int:
@@ -117,6 +123,20 @@ class ModelConfig:
   @property
   def kv_mult(self) -> int:
     return self.n_heads // self.n_kv_heads
+
+  def shard_specs(self, shard) -> Dict[int, LayerSpec]:
+    """The listed layers of a shard. A layer that reads the keys and values of
+    an earlier one ("kv_from") keeps a copy of them if that one is in another
+    shard and no layer before it here does."""
+    specs, kept = {}, set()
+    for i in range(shard.start_layer, shard.end_layer + 1):
+      spec = self.layer_specs[i]
+      j = spec.params.get("kv_from")
+      if j is not None and j < shard.start_layer and j not in kept:
+        kept.add(j)
+        spec = replace(spec, params={**spec.params, "keeps": True})
+      specs[i] = spec
+    return specs
 
   def estimate_param_bytes(self) -> int:
     """Rough bf16 parameter footprint — used by the partitioner for sizing."""
@@ -171,6 +191,9 @@ def config_from_hf(config_path: Path | str | dict, model_id: str = "unknown") ->
     if raw["architecture"] == "Lebotar":
       from xotorch_amd.models.lebotar import lebotar_config
       return lebotar_config(raw, model_id, shapes)
+    if raw["architecture"] == "Tapupel":
+      from xotorch_amd.models.tapupel import tapupel_config
+      return tapupel_config(raw, model_id, shapes)
     raise ValueError(f"unknown architecture {raw['architecture']!r}")
 
   n_heads = raw.get("num_attention_heads", 32)

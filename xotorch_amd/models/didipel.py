@@ -85,8 +85,8 @@ class DidipelLayer(nn.Module):
 
 
 class DidipelModel(LayeredModel):
-  def make_layer(self, cfg: ModelConfig, index: int) -> nn.Module:
-    return DidipelLayer(cfg, cfg.layer_specs[index])
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
+    return DidipelLayer(cfg, spec)
 
 
 def key_map_didipel(shard: Shard, cfg: ModelConfig) -> Dict[str, str]:

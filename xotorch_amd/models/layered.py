@@ -19,7 +19,7 @@ from typing import Dict, List, Optional
 import torch
 import torch.nn as nn
 
-from xotorch_amd.models.config import ModelConfig
+from xotorch_amd.models.config import LayerSpec, ModelConfig
 from xotorch_amd.models.llama import ShardedModel, XotLinear
 from xotorch_amd.ops import mixer_ops as mo
 from xotorch_amd.shard import Shard
@@ -37,23 +37,27 @@ def max_positions(raw: dict) -> int:
 class LayeredModel(nn.Module):
   """Layer range [shard.start_layer .. shard.end_layer] of such a model.
 
-  A layer has `norm1` (what the stream is normed with before it), `mix`, `mlp`
-  or None, `step(x, h, cache, rows, after)` -> (stream, its norm with `after`
-  or None) and `key_map(src, dst)`."""
+  A layer has `norm1`, `mix`, `mlp` or None, `key_map(src, dst)` and `step(x,
+  h, cache, rows, after)` -> (stream, what is read next): `after` is the weight
+  of the stream's next norm, mo.STREAM for the stream as it is, or None."""
 
   slot_indexed = True
   hidden_dtype = torch.float32
 
-  def make_layer(self, cfg: ModelConfig, index: int) -> nn.Module:
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
     raise NotImplementedError
+
+  @staticmethod
+  def entry(layer):
+    """What a layer reads: the stream normed with this weight, or mo.STREAM."""
+    return layer.norm1
 
   def __init__(self, cfg: ModelConfig, shard: Shard):
     super().__init__()
     self.cfg, self.shard = cfg, shard
     if shard.is_first_layer:
       self.embed_tokens = nn.Embedding(cfg.vocab_size, cfg.dim)
-    self.layers = nn.ModuleDict({str(i): self.make_layer(cfg, i)
-                                 for i in range(shard.start_layer, shard.end_layer + 1)})
+    self.layers = nn.ModuleDict({str(i): self.make_layer(cfg, spec) for i, spec in cfg.shard_specs(shard).items()})
     self.init_ranges = {}
     if shard.is_last_layer:
       self.norm = nn.Parameter(torch.zeros(cfg.dim))
@@ -94,18 +98,20 @@ class LayeredModel(nn.Module):
                        positions.reshape(-1) if is_decode else None, slots, lens)
     if x.dtype in (torch.int32, torch.int64):
       x = self.embed_tokens(x).float()
+      if cfg.embed_scale != 1.0:
+        x = x * cfg.embed_scale
     else:
       if cfg.carried_dim:
-        x, carried = x.split([cfg.dim, cfg.carried_dim], dim=-1)
-        rows.first_values = carried.to(dtype)
+        x, *carried = x.split([cfg.dim, *cfg.carried.values()], dim=-1)
+        rows.carried = {name: t.to(dtype) for name, t in zip(cfg.carried, carried)}
       if not (torch.is_grad_enabled() and x.requires_grad):
         x = x.float().clone(memory_format=torch.contiguous_format)  # updated in place; the caller keeps its own
     layers = [self.layers[str(i)] for i in self.local_layer_ids]
-    h = mo.prenorm(x, layers[0].norm1, eps, dtype)
+    h = mo.prenorm(x, self.entry(layers[0]), eps, dtype)
     whole = is_decode or not last_only or S == 1  # the head reads every row
     for i, layer in enumerate(layers):
       if i + 1 < len(layers):
-        after = layers[i + 1].norm1
+        after = self.entry(layers[i + 1])
       else:
         after = self.norm if self.shard.is_last_layer and whole else None
       x, h = layer.step(x, h, caches[i] if caches is not None else None, rows, after)
@@ -113,9 +119,8 @@ class LayeredModel(nn.Module):
         layers_out.append(x.clone())
     if not self.shard.is_last_layer:
       if cfg.carried_dim:
-        carried = rows.first_values
-        carried = x.new_zeros(B, S, cfg.carried_dim) if carried is None else carried.float()
-        x = torch.cat([x, carried], dim=-1)
+        x = torch.cat([x, *(rows.carried[name].float() if name in rows.carried else x.new_zeros(B, S, width)
+                            for name, width in cfg.carried.items())], dim=-1)
       return x
     if not whole:
       if lens is None:

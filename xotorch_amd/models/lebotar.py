@@ -45,7 +45,7 @@ def lebotar_config(raw: dict, model_id: str, shapes: Dict[str, tuple]) -> ModelC
   return ModelConfig(
     model_id=model_id, model_type="lebotar", vocab_size=raw["vocab"], dim=raw["width"], n_layers=len(specs),
     norm_eps=float(raw["norm"]["eps"]), max_seq_len=max_positions(raw), layer_specs=specs,
-    residual_mult=float(raw["residual_mult"]), carried_dim=shared,
+    residual_mult=float(raw["residual_mult"]), carried={"values": shared} if shared else {},
     n_experts=max((m["router"]["experts"] for m in moes), default=0),
     moe_intermediate_dim=max((m["expert"]["ff"] for m in moes), default=0),
     intermediate_dim=max((m["expert"]["ff"] for m in moes), default=0),
@@ -82,8 +82,8 @@ class LebotarLayer(nn.Module):
 
 
 class LebotarModel(LayeredModel):
-  def make_layer(self, cfg: ModelConfig, index: int) -> nn.Module:
-    return LebotarLayer(cfg, cfg.layer_specs[index])
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
+    return LebotarLayer(cfg, spec)
 
 
 def key_map_lebotar(shard: Shard, cfg: ModelConfig) -> Dict[str, str]:

@@ -5,7 +5,7 @@ each; MIXERS maps that name to a class here. Every constant of a mechanism is
 a parameter of its branch, so another design can use it with its own.
 
 Branches that read projections of the layer's input (the attentions,
-`GatedDeltaRule`, `SelectiveScan`) are combined by `BranchMixer`: ONE fused input GEMM over
+`GatedDeltaRule`, `SelectiveScan`, `GatedLinearUnit`) are combined by `BranchMixer`: ONE fused input GEMM over
 the parts of all branches and ONE output GEMM over their concatenated
 activations (branch weights fold into the activations in fp32), however many
 branches run side by side. `WKVMixer` shifts its input per projection and so
@@ -332,13 +332,51 @@ class ChunkAttention(nn.Module):
 
   def forward(self, h, proj, at, state, rows, **out):
     if self.shares:
-      rows.first_values = proj[..., at["v"]:at["v"] + self.G * self.vdim]
-    mix = (rows.first_values, self.v_mix) if self.mixes else None
+      rows.carried["values"] = proj[..., at["v"]:at["v"] + self.G * self.vdim]
+    mix = (rows.carried["values"], self.v_mix) if self.mixes else None
     return mo.chunk_attn(proj, [at[n] for n, _ in self.parts], self.H, self.G, self.dim, self.vdim, self.q_norm,
                          self.k_norm, self.sink, mix, self.scale, self.eps, self.chunk, state, rows, **out)
 
 
-class LatentAttention(nn.Module):
+def turn_rates(rot: dict) -> List[float]:
+  """Radians per position of every pair of turned dimensions. With `scaling`,
+  wavelengths beyond original / low are stretched by `factor`, those below
+  original / high stay, and the ones between blend."""
+  out, s = [], rot.get("scaling")
+  for i in range(rot["dims"] // 2):
+    f = float(rot["base"]) ** (-2.0 * i / rot["dims"])
+    if s is not None:
+      turns = s["original"] * f / (2 * math.pi)  # within the original length
+      blend = min(1.0, max(0.0, (turns - s["low"]) / (s["high"] - s["low"])))
+      f = f * (blend + (1 - blend) / s["factor"])
+    out.append(f)
+  return out
+
+
+class Turning(nn.Module):
+  """A module with a table of turn rates, which stays in 32-bit whatever the
+  model is cast to."""
+
+  def __init__(self):
+    super().__init__()
+    self.register_buffer("freq", torch.empty(0), persistent=False)
+
+  def rates(self) -> List[float]:
+    return turn_rates(self.rot)
+
+  def reset_tables(self, device=None):
+    self.freq = torch.tensor(self.rates(), dtype=torch.float32, device=device or self.freq.device)
+
+  def _apply(self, fn, recurse=True):
+    super()._apply(fn, recurse)
+    if self.freq.dtype != torch.float32:
+      self.freq = self.freq.float()
+      if self.freq.device.type != "meta":
+        self.reset_tables(self.freq.device)
+    return self
+
+
+class LatentAttention(Turning):
   """Latent attention: keys and values of all heads come out of one normed
   latent per token, plus one rotated key part that the heads share. Only these
   two are cached; decode folds the expansion into query and output."""
@@ -354,22 +392,12 @@ class LatentAttention(nn.Module):
     self.kv_norm = nn.Parameter(torch.ones(self.rank))
     self.kv_up = XotLinear(self.rank, self.H * (self.dim + self.vdim), bias=False)  # all keys, then all values
     self.init_ranges = {"kv_norm": (0.8, 1.2)}
-    self.register_buffer("freq", torch.empty(0), persistent=False)
     self.reset_tables()
 
-  def reset_tables(self, device=None):
-    """Turns per position of every pair; pairs that do not rotate have none."""
-    n = self.rot["dims"]
-    freq = [float(self.rot["base"]) ** (-2.0 * i / n) if 2 * i < n else 0.0 for i in range(self.rot_dim // 2)]
-    self.freq = torch.tensor(freq, dtype=torch.float32, device=device or self.freq.device)
-
-  def _apply(self, fn, recurse=True):
-    super()._apply(fn, recurse)
-    if self.freq.dtype != torch.float32:  # a cast of the model leaves angles in 32-bit
-      self.freq = self.freq.float()
-      if self.freq.device.type != "meta":
-        self.reset_tables(self.freq.device)
-    return self
+  def rates(self) -> List[float]:
+    """Pairs that do not rotate have a rate of zero."""
+    rates = turn_rates(self.rot)
+    return rates + [0.0] * (self.rot_dim // 2 - len(rates))
 
   @staticmethod
   def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> StateSpec:
@@ -388,6 +416,159 @@ class LatentAttention(nn.Module):
   def forward(self, h, proj, at, state, rows, **out):
     return mo.latent_attn(proj, at["q"], at["dkv"], self.H, self.dim, self.rot_dim, self.rank, self.vdim, self.kv_norm,
                           self.kv_up, self.freq, self.scale, self.eps, state, rows, **out)
+
+
+class RotaryAttention(Turning):
+  """GQA attention with rotary positions, causal or over a sliding window that
+  keeps the first tokens in sight.
+
+  p: heads, kv_heads, dim, vdim, rot {base, dims, scaling}, scale and
+  - mask {size, keep_first}: the window; none: causal
+  - softcap: scores become softcap * tanh(score / softcap)
+  - pairs: neighbours turn together (else dimensions half the turned ones apart)
+  - norm: "before" the rotation, an RMS norm per head with a weight, or "after"
+    it, one without
+  - values: "own" projection, or the "keys" as projected
+  - diff: two maps per head over the same values; the output is the first minus
+    lambda times the second, RMS-normed per head and scaled by 1 - diff
+  - kv_from: the layer whose cached keys and values this one reads instead of
+    having its own; lent: another layer reads this one's; keeps: the layer read
+    from is in another shard, so this one caches what travels with the stream
+  """
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__()
+    self.H, self.G, self.dim, self.vdim = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    self.rot, self.maps = p["rot"], 2 if p.get("diff") is not None else 1
+    if self.H % self.G:
+      raise ValueError(f"{self.H} query heads do not divide into {self.G} key/value heads")
+    if self.rot["dims"] % 2 or self.rot["dims"] > self.dim:
+      raise ValueError(f"rotation of {self.rot['dims']} of {self.dim} dimensions")
+    if p["values"] == "keys" and (self.vdim != self.dim or self.maps != 1):
+      raise ValueError(f"keys of {self.dim} dimensions are no values of {self.vdim}")
+    mask = p.get("mask") or {"size": 0, "keep_first": 0}
+    if p.get("mask") and mask["size"] < 1:
+      raise ValueError(f"window of {mask['size']} tokens")
+    self.layer, self.source = p.get("layer"), p.get("kv_from")
+    self.lent, self.keeps = bool(p.get("lent")), bool(p.get("keeps"))
+    if (self.lent or self.source is not None) and (p.get("mask") or p["values"] == "keys"):
+      raise ValueError("only causal attention with values of its own shares them")
+    self.rule = mo.AttnRule(
+      self.H, self.G, self.dim, self.vdim, self.maps, float(p["scale"]), float(p.get("softcap") or 0.0),
+      int(mask["size"]), int(mask.get("keep_first", 0)), bool(p["pairs"]), p["norm"] == "after", eps,
+      1.0 - p["diff"] if self.maps == 2 else 1.0)
+    q, k = ("q", self.H * self.maps * self.dim), ("k", self.G * self.maps * self.dim)
+    self.parts = [q] if self.source is not None else [q, k] if p["values"] == "keys" else [q, k, ("v", self.G * self.vdim)]
+    self.width = self.H * self.vdim
+    self.init_ranges = {}
+    self.q_norm = self.k_norm = None
+    if p["norm"] == "before":
+      self.q_norm = nn.Parameter(torch.ones(self.dim))
+      self.init_ranges["q_norm"] = (0.8, 1.2)
+      if self.source is None or self.keeps:
+        self.k_norm = nn.Parameter(torch.ones(self.dim))
+        self.init_ranges["k_norm"] = (0.8, 1.2)
+    if self.maps == 2:
+      self.diff = float(p["diff"])
+      self.contrast = nn.Parameter(torch.zeros(4, self.dim))  # the vectors of lambda: q1, k1, q2, k2
+      self.init_ranges["contrast"] = (-0.1, 0.1)
+    self.reset_tables()
+
+  @staticmethod
+  def lent_width(p: dict) -> int:
+    """Channels of what travels with the stream: keys and values as projected."""
+    return _up(2 * p["kv_heads"] * p["dim"], 8) + p["kv_heads"] * p["vdim"]
+
+  @staticmethod
+  def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> StateSpec:
+    if p.get("kv_from") is not None and not p.get("keeps"):
+      return {}
+    G, d, e, mask = p["kv_heads"], p["dim"], p["vdim"], p.get("mask")
+    maps = 2 if p.get("diff") is not None else 1
+    # the kept tokens' rows, then a ring of the window's
+    n = min(capacity, mask["size"] + mask.get("keep_first", 0)) if mask else capacity
+    if mo.packed_kv(dtype, device):
+      n = _up(n, 32)  # MFMA fragment order, as for WindowBiasAttention
+      return {"k": ((G * maps, n // 16, _up(d, 32) // 32, 64, 8), dtype),
+              "v": ((G, _up(e, 16) // 16, n // 32, 64, 8), dtype)}
+    return {"k": ((G * maps, n, d), dtype), "v": ((G, n, e), dtype)}
+
+  @staticmethod
+  def param_count(dim: int, p: dict) -> int:
+    H, G, d, e = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
+    maps = 2 if p.get("diff") is not None else 1
+    own = 0 if p.get("kv_from") is not None else G * maps * d + (G * e if p["values"] == "own" else 0)
+    return dim * (H * maps * d + own + H * e) + (2 * d if p["norm"] == "before" else 0) + (4 * d if maps == 2 else 0)
+
+  def contrast_weight(self):
+    """lambda as a 32-bit tensor; outside of training kept with the module."""
+    if self.maps == 1:
+      return None
+
+    def value():
+      q1, k1, q2, k2 = self.contrast.float()
+      return torch.exp((q1 * k1).sum()) - torch.exp((q2 * k2).sum()) + self.diff
+    if torch.is_grad_enabled() and self.contrast.requires_grad:
+      return value()
+    key = (self.contrast.data_ptr(), self.contrast._version)
+    if getattr(self, "_lambda_key", None) != key:
+      self._lambda, self._lambda_key = value().reshape(1), key
+    return self._lambda
+
+  def forward(self, h, proj, at, state, rows, **out):
+    source, k_norm, append = None, self.k_norm, True
+    if self.source is None:
+      source = (proj, at["k"], at.get("v", at["k"]))
+      if self.lent:
+        rows.carried[f"kv{self.layer}"] = proj[..., at["k"]:at["v"] + self.G * self.vdim]
+    elif self.keeps:
+      source = (rows.carried[f"kv{self.source}"].contiguous(), 0, _up(self.G * self.maps * self.dim, 8))
+    else:
+      state, source, k_norm = rows.kept[self.source]
+      append = False
+    if self.lent or self.keeps:
+      rows.kept[self.layer if self.lent else self.source] = (state, source, k_norm)
+    return mo.rotary_attn(proj, at["q"], source, self.rule, self.q_norm, k_norm, self.freq, self.contrast_weight(), state,
+                          rows, append, **out)
+
+
+class GatedLinearUnit(nn.Module):
+  """Recurrent block of a gated linear unit: a short causal convolution, gates
+  of recurrence and input through block-diagonal products, an fp32 state per
+  channel, and a gelu branch that multiplies the result."""
+
+  RATE = 8.0  # the decay's exponent at an open gate, in softplus(lam)
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__()
+    self.width, self.blocks = p["width"], p["blocks"]
+    if self.width % self.blocks:
+      raise ValueError(f"{self.width} channels do not divide into {self.blocks} blocks")
+    W, n = self.width, self.width // self.blocks
+    self.parts = [("y", W), ("x", W)]
+    self.in_bias = nn.Parameter(torch.zeros(2, W))
+    self.conv = nn.Parameter(torch.zeros(W, p["conv"]))
+    self.conv_bias = nn.Parameter(torch.zeros(W))
+    self.gates = nn.Parameter(torch.zeros(2, self.blocks, n, n))  # of the recurrence, of the input
+    self.gate_bias = nn.Parameter(torch.zeros(2, self.blocks, n))
+    self.lam = nn.Parameter(torch.zeros(W))
+    self.init_ranges = {"in_bias": (-0.1, 0.1), "conv": (-0.5, 0.5), "conv_bias": (-0.1, 0.1), "gate_bias": (-1.0, 1.0),
+                        "lam": (-6.0, -2.0)}
+
+  @staticmethod
+  def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> StateSpec:
+    return {"s": ((p["width"],), torch.float32),
+            # the convolution's last inputs, position t in row t % taps
+            "conv": ((p["conv"], p["width"]), dtype)}
+
+  @staticmethod
+  def param_count(dim: int, p: dict) -> int:
+    W, n = p["width"], p["width"] // p["blocks"]
+    return W * (3 * dim + 2 * n + p["conv"] + 6)
+
+  def forward(self, h, proj, at, state, rows, **out):
+    return mo.gated_unit(proj, at["y"], at["x"], self.in_bias, self.conv, self.conv_bias, self.gates, self.gate_bias,
+                         self.lam, self.RATE, state, rows, **out)
 
 
 class SelectiveScan(nn.Module):
@@ -476,5 +657,34 @@ class SelectiveScanMixer(SingleMixer):
              "A_log": "a_log", "D": "skip"}
 
 
-MIXERS = {"parallel": ParallelMixer, "wkv": WKVMixer, "chunk_attention": ChunkAttentionMixer,
+class KeptAttentionMixer(SingleMixer):
+  BRANCH = RotaryAttention
+  TENSORS = {"q.norm": "q_norm", "k.norm": "k_norm"}
+
+
+class DifferenceAttentionMixer(KeptAttentionMixer):
+  def key_map(self, src: str, dst: str) -> Dict[str, str]:
+    m, own = super().key_map(src, dst), self.branches["only"]
+    for i, n in enumerate(("lq1", "lk1", "lq2", "lk2")):
+      m[src + n] = f"{dst}branches.only.contrast@{i}"
+    if own.keeps:  # the norm of the keys it caches is the other layer's
+      del m[f"{src}k.norm"]
+      m[f"l{own.source}.mix.k.norm"] = f"{dst}branches.only.k_norm"
+    return m
+
+
+class GatedLinearUnitMixer(SingleMixer):
+  BRANCH = GatedLinearUnit
+  TENSORS = {"conv": "conv", "conv.b": "conv_bias", "lam": "lam"}
+
+  def key_map(self, src: str, dst: str) -> Dict[str, str]:
+    m, own = super().key_map(src, dst), f"{dst}branches.only."
+    for i, (branch, gate) in enumerate((("y", "ra"), ("x", "ri"))):
+      m[f"{src}{branch}.b"] = f"{own}in_bias@{i}"
+      m[f"{src}{gate}"], m[f"{src}{gate}.b"] = f"{own}gates@{i}", f"{own}gate_bias@{i}"
+    return m
+
+
+MIXERS = {"kept_attention": KeptAttentionMixer, "difference_attention": DifferenceAttentionMixer,
+          "rglru": GatedLinearUnitMixer, "parallel": ParallelMixer, "wkv": WKVMixer, "chunk_attention": ChunkAttentionMixer,
           "latent_attention": LatentAttentionMixer, "mamba1": SelectiveScanMixer}

@@ -34,6 +34,9 @@ def hf_key_map(shard, cfg):
   if mtype == "lebotar":
     from xotorch_amd.models.lebotar import key_map_lebotar
     return key_map_lebotar(shard, cfg)
+  if mtype == "tapupel":
+    from xotorch_amd.models.tapupel import key_map_tapupel
+    return key_map_tapupel(shard, cfg)
   return _hf_key_map_llama(shard, cfg)
 
 
@@ -98,7 +101,8 @@ def remap_hf_state(sd: Dict[str, torch.Tensor], mapping: Dict[str, str],
   `key` renames; `key#N` parts are concatenated along dim 0 in N order;
   `key@row` / `key@row,col` parts are placed at an offset of the parameter
   `key`, whose shape comes from `shapes`, with zeros where nothing is placed
-  (fused projections with aligned or padded parts)."""
+  (fused projections with aligned or padded parts). `key@row<axis,lo:hi` places
+  that range of the tensor only; several such targets are joined by `;`."""
   state: Dict[str, torch.Tensor] = {}
   packed: Dict[str, Dict[int, torch.Tensor]] = {}
   for hf_key, our in mapping.items():
@@ -108,16 +112,21 @@ def remap_hf_state(sd: Dict[str, torch.Tensor], mapping: Dict[str, str],
       base, part = our.split("#")
       packed.setdefault(base, {})[int(part)] = sd[hf_key]
     elif "@" in our:
-      base, offset = our.split("@")
-      t = sd[hf_key]
-      if base not in state:
-        state[base] = torch.zeros(shapes[base], dtype=t.dtype, device=t.device)
-      t = t.reshape((1,) * (state[base].dim() - t.dim()) + tuple(t.shape))
-      at = [int(o) for o in offset.split(",")]
-      at += [0] * (t.dim() - len(at))
-      if any(o + n > m for o, n, m in zip(at, t.shape, state[base].shape)):
-        raise RuntimeError(f"{hf_key} {tuple(t.shape)} does not fit {base} {tuple(state[base].shape)} at {at}")
-      state[base][tuple(slice(o, o + n) for o, n in zip(at, t.shape))] = t
+      for target in our.split(";"):
+        target, _, part = target.partition("<")
+        base, offset = target.split("@")
+        t = sd[hf_key]
+        if part:
+          axis, lo, hi = (int(v) for v in part.replace(":", ",").split(","))
+          t = t.narrow(axis, lo, hi - lo)
+        if base not in state:
+          state[base] = torch.zeros(shapes[base], dtype=t.dtype, device=t.device)
+        t = t.reshape((1,) * (state[base].dim() - t.dim()) + tuple(t.shape))
+        at = [int(o) for o in offset.split(",")]
+        at += [0] * (t.dim() - len(at))
+        if any(o + n > m for o, n, m in zip(at, t.shape, state[base].shape)):
+          raise RuntimeError(f"{hf_key} {tuple(t.shape)} does not fit {base} {tuple(state[base].shape)} at {at}")
+        state[base][tuple(slice(o, o + n) for o, n in zip(at, t.shape))] = t
     else:
       state[our] = sd[hf_key]
   for base, parts in packed.items():

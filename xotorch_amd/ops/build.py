@@ -20,6 +20,8 @@ EXTENSIONS = {
   "_hip_ops": PKG_DIR / "hip" / "hip_ops.hip",
   "_hip_mixers": PKG_DIR / "hip" / "mixer_ops.hip",
   "_hip_attn": PKG_DIR / "hip" / "attn_rows.hip",
+  "_hip_rotary": PKG_DIR / "hip" / "rotary_attn.hip",
+  "_hip_lru": PKG_DIR / "hip" / "lru_ops.hip",
   "_hip_experts": PKG_DIR / "hip" / "expert_ops.hip",
   "_hip_scan": PKG_DIR / "hip" / "scan_ops.hip",
   "_hip_latent": PKG_DIR / "hip" / "latent_ops.hip",

@@ -1,48 +1,9 @@
-// CDNA4 (gfx950) kernels of softmax attention over rows of a cache, one flash
-// kernel for prompts and one split kernel for decode steps, in three modes:
-//   WINDOW: sliding window, learned bias per distance bucket, a zero-score
-//           sink, a sigmoid gate per head, norms over whole projections
-//   CHUNK:  keys of the query's own chunk of the sequence, a bias that falls
-//           linearly with the distance, a learned sink per head, norms per
-//           head, values mixed with an earlier layer's
-//   CAUSAL: all earlier keys, plain softmax (prompts only)
-//
-// Two element types: bf16 (MFMA over fragment-packed keys and values) and fp32
-// (plain layouts, plain fp32 arithmetic). Scores, softmax and norms are fp32
-// in both. Rows address caches by slot (struct Step): slot -1 is a parked row.
+// Attention over a window of the sequence with a bias per distance, and within
+// chunks of it (modes WINDOW and CHUNK of attn_rows.h): what norms, appends and
+// copies rows, and the entry points. Norms are over whole projections (WINDOW)
+// or per head (CHUNK, whose values may be mixed with an earlier layer's).
 
-#include "common.h"
-
-struct AttnArgs {
-  int S, H, G, N, K;                    // tokens a row, heads, projection and output widths
-  int q_at, k_at, v_at, g_at, out_at;
-  int qd;                               // padded dims of the q workspace
-  float scale, eps, out_scale;
-  int window, nb;                       // window or chunk length; entries of the distance table
-};
-
-enum Mode { WINDOW, CHUNK, CAUSAL };
-
-// Keys that position pos sees: itself and the reach - 1 before it.
-template <int MODE>
-DEVINL int reach_of(const AttnArgs& a, int pos) {
-  return MODE == WINDOW ? a.window : MODE == CHUNK ? pos % a.window + 1 : pos + 1;
-}
-// Slope of the linear distance bias: halves 8 times over the heads.
-DEVINL float slope_of(const AttnArgs& a, int h) { return exp2f(-8.f * (float)(h + 1) / (float)a.H); }
-
-// What joins the softmax beside the keys, and what scales a head's output.
-template <int MODE, typename T>
-struct Side {
-  const T *proj, *sinks;
-  // score of the extra entry in the denominator
-  DEVINL float sink(int h) const { return MODE == WINDOW ? 0.f : MODE == CHUNK ? ld(sinks + h) : -INFINITY; }
-  // where the running maximum starts: finite, so that fully masked tiles are harmless
-  DEVINL float start(int h) const { return MODE == CAUSAL ? -1e30f : sink(h); }
-  DEVINL float gate(const AttnArgs& a, size_t tok, int h) const {
-    return MODE == WINDOW ? a.out_scale * sigmoidf(ld(proj + tok * a.N + a.g_at + h)) : a.out_scale;
-  }
-};
+#include "attn_rows.h"
 
 // Keys of the window before a chunk, ring -> workspace rows [0, hist).
 template <typename T>
@@ -257,471 +218,9 @@ __global__ __launch_bounds__(256) void head_norm_append_kernel(
   }
 }
 
-// Flash prefill on matrix cores: a wave owns 32 queries of one head and walks
-// the key tiles that their windows touch. EXACT: kc == KC and vg == VG.
-template <int KC, int VG, bool EXACT, int MODE>
-__global__ __launch_bounds__(256) void attn_rows_prefill_kernel(
-    const bf16_t* __restrict__ qw, const bf16_t* __restrict__ kw, const bf16_t* __restrict__ vw,
-    Side<MODE, bf16_t> side, const int* __restrict__ bucket, const bf16_t* __restrict__ rel,
-    bf16_t* __restrict__ out, KVShape ws, int hist, AttnArgs a, Step step) {
-  extern __shared__ float bias[];  // [nb], this head's bias per distance
-  const int h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G);
-  const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
-  if (MODE == WINDOW) {
-    for (int i = threadIdx.x; i < a.nb; i += 256) bias[i] = ld(rel + bucket[i] * a.H + h);
-    __syncthreads();
-  }
-  const float slope = MODE == CHUNK ? slope_of(a, h) : 0.f, sink = side.sink(h);
-  const int s0 = blockIdx.x * 128 + (threadIdx.x >> 6) * 32;
-  if (s0 >= a.S) return;
-  const int kc = EXACT ? KC : ws.kc, vg = EXACT ? VG : ws.vg;
-  bf16x8 qf[2][KC];
-#pragma unroll
-  for (int t = 0; t < 2; ++t) {
-    const int s = min(s0 + t * 16 + col, a.S - 1);
-    const bf16_t* q = qw + (((size_t)b * a.S + s) * a.H + h) * a.qd + quad * 8;
-#pragma unroll
-    for (int c = 0; c < KC; ++c)
-      if (EXACT || c < kc) qf[t][c] = *(const bf16x8*)(q + c * 32);
-  }
-  // the sink's score bounds the maximum from below
-  float m[2] = {side.start(h), side.start(h)}, l[2] = {0.f, 0.f};
-  int reach[2];
-#pragma unroll
-  for (int t = 0; t < 2; ++t) reach[t] = reach_of<MODE>(a, step.start + s0 + t * 16 + col);
-  floatx4 o[2][VG];
-#pragma unroll
-  for (int t = 0; t < 2; ++t)
-#pragma unroll
-    for (int i = 0; i < VG; ++i) o[t][i] = (floatx4)(0.f);
-  const bf16_t* kb = kw + Layout<bf16_t>::kbase(ws, (size_t)b * a.G + g);
-  const bf16_t* vb = vw + Layout<bf16_t>::vbase(ws, (size_t)b * a.G + g);
-  const int vstride = (ws.rows >> 5) * 512;
-  const int t0 = max(0, hist + s0 + 1 - reach_of<MODE>(a, step.start + s0)) >> 5;
-  const int t1 = (hist + min(s0 + 31, a.S - 1)) >> 5;
-  for (int tile = t0; tile <= t1; ++tile) {
-    floatx4 sc[2][2];
-#pragma unroll
-    for (int hf = 0; hf < 2; ++hf) {
-      sc[0][hf] = (floatx4)(0.f);
-      sc[1][hf] = (floatx4)(0.f);
-#pragma unroll
-      for (int c = 0; c < KC; ++c)
-        if (EXACT || c < kc) {
-          const bf16x8 kf = *(const bf16x8*)(kb + ((size_t)(tile * 2 + hf) * kc + c) * 512 + lane * 8);
-          sc[0][hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[0][c], sc[0][hf], 0, 0, 0);
-          sc[1][hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[1][c], sc[1][hf], 0, 0, 0);
-        }
-    }
-    bf16x8 pf[2];
-#pragma unroll
-    for (int t = 0; t < 2; ++t) {
-      // distance to this lane's first key of the tile
-      const int dist0 = hist + s0 + t * 16 + col - tile * 32 - quad * 4;
-      float top = m[t];
-#pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int dist = dist0 - hf * 16 - r;
-          float v = sc[t][hf][r] * a.scale;
-          if (MODE == WINDOW) v += bias[min(max(dist, 0), a.nb - 1)];
-          if (MODE == CHUNK) v -= slope * (float)dist;
-          sc[t][hf][r] = (dist >= 0 && dist < reach[t]) ? v : -INFINITY;
-          top = fmaxf(top, sc[t][hf][r]);
-        }
-      top = fmaxf(top, __shfl_xor(top, 16));
-      top = fmaxf(top, __shfl_xor(top, 32));
-      if (__any(top > m[t])) {
-        const float al = __expf(m[t] - top);
-        m[t] = top;
-        l[t] *= al;
-#pragma unroll
-        for (int i = 0; i < VG; ++i) o[t][i] *= al;
-      }
-      float sum = 0.f;
-#pragma unroll
-      for (int hf = 0; hf < 2; ++hf)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const float p = __expf(sc[t][hf][r] - top);
-          sum += p;
-          pf[t][hf * 4 + r] = (__bf16)p;
-        }
-      l[t] += sum;
-    }
-#pragma unroll
-    for (int i = 0; i < VG; ++i)
-      if (EXACT || i < vg) {
-        const bf16x8 vf = *(const bf16x8*)(vb + (size_t)i * vstride + (size_t)tile * 512 + lane * 8);
-        o[0][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[0], o[0][i], 0, 0, 0);
-        o[1][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[1], o[1][i], 0, 0, 0);
-      }
-  }
-  const int len = step.slot(b) < 0 ? 0 : step.len(b, a.S);
-#pragma unroll
-  for (int t = 0; t < 2; ++t) {
-    const int s = s0 + t * 16 + col;
-    float sum = l[t];
-    sum += __shfl_xor(sum, 16);
-    sum += __shfl_xor(sum, 32);
-    if (s >= a.S) continue;
-    const size_t tok = (size_t)b * a.S + s;
-    float f = 0.f;
-    if (s < len) f = side.gate(a, tok, h) / (sum + __expf(sink - m[t]));
-    bf16_t* dst = out + tok * a.K + a.out_at + h * ws.vdim;
-#pragma unroll
-    for (int i = 0; i < VG; ++i) {
-      const int c = i * 16 + quad * 4;
-      if (c + 3 < ws.vdim && (ws.vdim & 3) == 0) {
-        float v[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = s < len ? o[t][i][r] * f : 0.f;
-        st4(dst + c, v);
-      } else {
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          if (c + r < ws.vdim) st(dst + c + r, s < len ? o[t][i][r] * f : 0.f);
-      }
-    }
-  }
-}
-
-// Split decode: a block scores one row's ring (or a part of it) for up to 16
-// query heads of a kv head; its 4 waves walk 32-row tiles and merge in LDS.
-// part null: the block saw the whole ring and writes the result.
-template <int KC, int VG, bool EXACT, int MODE>
-__global__ __launch_bounds__(256) void attn_rows_decode_kernel(
-    const bf16_t* __restrict__ qw, const bf16_t* __restrict__ kc_, const bf16_t* __restrict__ vc_,
-    Side<MODE, bf16_t> side, const int* __restrict__ bucket, const bf16_t* __restrict__ rel, int rel_rows,
-    bf16_t* __restrict__ out, float* __restrict__ part, int splits, KVShape ring, AttnArgs a, Step step) {
-  constexpr int OW = VG * 16 + 4;  // row of a wave's partial output (padded)
-  __shared__ float po[4][16 * OW];
-  __shared__ float pm[4][16], pl[4][16];
-  extern __shared__ int tab[];  // [nb] buckets, then [rel_rows][16] bias of these heads
-  const int split = blockIdx.x, b = blockIdx.z;
-  const int per = a.H / a.G, qgs = (per + 15) >> 4;
-  const int g = blockIdx.y / qgs, q0 = (blockIdx.y % qgs) * 16, nq = min(16, per - q0);
-  const int h0 = g * per + q0;
-  const int slot = step.slot(b);
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
-  if (slot < 0) {
-    if (!part)
-      for (int i = threadIdx.x; i < nq * ring.vdim; i += 256)
-        st(out + (size_t)b * a.K + a.out_at + (size_t)h0 * ring.vdim + i, 0.f);
-    return;
-  }
-  float* relb = (float*)(tab + a.nb);
-  if (MODE == WINDOW) {
-    for (int i = threadIdx.x; i < a.nb; i += 256) tab[i] = bucket[i];
-    for (int i = threadIdx.x; i < rel_rows * 16; i += 256)
-      relb[i] = (i & 15) < nq ? ld(rel + (i >> 4) * a.H + h0 + (i & 15)) : 0.f;
-    __syncthreads();
-  }
-  const int hc = h0 + min(col, nq - 1);  // this lane's head
-  const float slope = MODE == CHUNK ? slope_of(a, hc) : 0.f;
-  const int kc = EXACT ? KC : ring.kc, vg = EXACT ? VG : ring.vg;
-  const int pos = step.first(b), cur = pos % ring.mod;
-  // CHUNK: rows past the current one still hold an earlier chunk
-  const int seen = MODE == CHUNK ? min(cur + 1, ring.rows) : min(min(a.window, ring.rows), pos + 1);
-  const int ntiles = ((MODE == CHUNK ? seen : min(ring.rows, pos + 1)) + 31) >> 5;
-  const int per_split = (ntiles + splits - 1) / splits;
-  bf16x8 qf[KC];
-  const bf16_t* q = qw + ((size_t)b * a.H + hc) * a.qd + quad * 8;
-#pragma unroll
-  for (int c = 0; c < KC; ++c)
-    if (EXACT || c < kc) qf[c] = *(const bf16x8*)(q + c * 32);
-  float m = side.start(hc), l = 0.f;
-  floatx4 o[VG];
-#pragma unroll
-  for (int i = 0; i < VG; ++i) o[i] = (floatx4)(0.f);
-  const bf16_t* kb = kc_ + Layout<bf16_t>::kbase(ring, (size_t)slot * a.G + g);
-  const bf16_t* vb = vc_ + Layout<bf16_t>::vbase(ring, (size_t)slot * a.G + g);
-  const size_t vstride = (size_t)(ring.rows >> 5) * 512;
-  const int end = min(ntiles, (split + 1) * per_split);
-  for (int tile = split * per_split + wave; tile < end; tile += 4) {
-    bf16x8 vf[VG];
-    floatx4 sc[2];
-#pragma unroll
-    for (int hf = 0; hf < 2; ++hf) {
-      sc[hf] = (floatx4)(0.f);
-#pragma unroll
-      for (int c = 0; c < KC; ++c)
-        if (EXACT || c < kc) {
-          const bf16x8 kf = *(const bf16x8*)(kb + ((size_t)(tile * 2 + hf) * kc + c) * 512 + lane * 8);
-          sc[hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[c], sc[hf], 0, 0, 0);
-        }
-    }
-#pragma unroll
-    for (int i = 0; i < VG; ++i)
-      if (EXACT || i < vg) vf[i] = *(const bf16x8*)(vb + i * vstride + (size_t)tile * 512 + lane * 8);
-    float top = m;
-#pragma unroll
-    for (int hf = 0; hf < 2; ++hf)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        int age = cur - (tile * 32 + hf * 16 + quad * 4 + r);
-        if (age < 0) age += ring.rows;
-        float v = sc[hf][r] * a.scale;
-        if (MODE == WINDOW) v += relb[tab[min(age, a.nb - 1)] * 16 + col];
-        if (MODE == CHUNK) v -= slope * (float)age;
-        sc[hf][r] = age < seen ? v : -INFINITY;
-        top = fmaxf(top, sc[hf][r]);
-      }
-    top = fmaxf(top, __shfl_xor(top, 16));
-    top = fmaxf(top, __shfl_xor(top, 32));
-    const float al = __expf(m - top);
-    m = top;
-    l *= al;
-    bf16x8 pf;
-#pragma unroll
-    for (int hf = 0; hf < 2; ++hf)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float p = __expf(sc[hf][r] - top);
-        l += p;
-        pf[hf * 4 + r] = (__bf16)p;
-      }
-#pragma unroll
-    for (int i = 0; i < VG; ++i)
-      if (EXACT || i < vg) {
-        o[i] *= al;
-        o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i], pf, o[i], 0, 0, 0);
-      }
-  }
-  l += __shfl_xor(l, 16);
-  l += __shfl_xor(l, 32);
-  if (quad == 0) { pm[wave][col] = m; pl[wave][col] = l; }
-#pragma unroll
-  for (int i = 0; i < VG; ++i)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) po[wave][col * OW + i * 16 + quad * 4 + r] = o[i][r];
-  __syncthreads();
-  for (int i = threadIdx.x; i < nq * ring.vdim; i += 256) {
-    const int qh = i / ring.vdim, c = i - qh * ring.vdim;
-    const int h = h0 + qh;
-    float M = side.start(h), L = 0.f, O = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) M = fmaxf(M, pm[w][qh]);
-#pragma unroll
-    for (int w = 0; w < 4; ++w) {
-      const float f = __expf(pm[w][qh] - M);
-      L += f * pl[w][qh];
-      O += f * po[w][qh * OW + c];
-    }
-    if (part) {
-      float* p = part + (((size_t)b * splits + split) * a.H + h) * (ring.vdim + 2);
-      p[2 + c] = O;
-      if (c == 0) { p[0] = M; p[1] = L; }
-    } else {
-      st(out + (size_t)b * a.K + a.out_at + (size_t)h * ring.vdim + c,
-         O / (L + __expf(side.sink(h) - M)) * side.gate(a, b, h));
-    }
-  }
-}
-
-template <int MODE>
-__global__ __launch_bounds__(64) void attn_rows_merge_kernel(
-    const float* __restrict__ part, Side<MODE, bf16_t> side, bf16_t* __restrict__ out, int splits,
-    int vdim, AttnArgs a, Step step) {
-  const int h = blockIdx.x, b = blockIdx.y;
-  const bool live = step.slot(b) >= 0;
-  for (int c = threadIdx.x; c < vdim; c += 64) {
-    float r = 0.f;
-    if (live) {
-      float M = side.start(h), L = 0.f, O = 0.f;
-      for (int s = 0; s < splits; ++s) M = fmaxf(M, part[(((size_t)b * splits + s) * a.H + h) * (vdim + 2)]);
-      for (int s = 0; s < splits; ++s) {
-        const float* p = part + (((size_t)b * splits + s) * a.H + h) * (vdim + 2);
-        const float f = __expf(p[0] - M);
-        L += f * p[1];
-        O += f * p[2 + c];
-      }
-      r = O / (L + __expf(side.sink(h) - M)) * side.gate(a, b, h);
-    }
-    st(out + (size_t)b * a.K + a.out_at + (size_t)h * vdim + c, r);
-  }
-}
-
-// 32-bit attention, one wave per (token, head): lanes over keys for the
-// scores, over value columns for the sum. base/rows: where position p lies
-// ((p - base) % mod), so one kernel serves caches and workspaces. NC: value
-// columns per lane.
-template <int MODE, int NC>
-__global__ __launch_bounds__(64) void attn_rows_f32_kernel(
-    const float* __restrict__ qw, const float* __restrict__ k, const float* __restrict__ v,
-    Side<MODE, float> side, const int* __restrict__ bucket, const float* __restrict__ rel,
-    float* __restrict__ out, KVShape kv, int base, AttnArgs a, Step step) {
-  extern __shared__ float q[];  // [dim]
-  const int s = blockIdx.x, h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G), lane = threadIdx.x;
-  const int slot = step.slot(b), len = step.decode ? 1 : step.len(b, a.S);
-  float* dst = out + ((size_t)b * a.S + s) * a.K + a.out_at + (size_t)h * kv.vdim;
-  if (slot < 0 || s >= len) {
-    for (int c = lane; c < kv.vdim; c += 64) dst[c] = 0.f;
-    return;
-  }
-  for (int d = lane; d < kv.dim; d += 64) q[d] = qw[(((size_t)b * a.S + s) * a.H + h) * a.qd + d];
-  __syncthreads();
-  const size_t head = (size_t)(step.decode ? slot : b) * a.G + g;
-  const float* kb = k + Layout<float>::kbase(kv, head);
-  const float* vb = v + Layout<float>::vbase(kv, head);
-  const int pos = min(step.first(b) + s, MODE == CAUSAL ? kv.rows - 1 : INT_MAX);
-  const int lo = max(0, pos - reach_of<MODE>(a, pos) + 1);
-  const float slope = MODE == CHUNK ? slope_of(a, h) : 0.f;
-  float m = side.start(h), l = 0.f, acc[NC];
-#pragma unroll
-  for (int i = 0; i < NC; ++i) acc[i] = 0.f;
-  for (int p0 = lo; p0 <= pos; p0 += 64) {
-    const int p = p0 + lane;
-    float sc = -INFINITY;
-    if (p <= pos) {
-      const float* row = kb + Layout<float>::k(kv, min((p - base) % kv.mod, kv.rows - 1), 0);
-      float dot = 0.f;
-      for (int d = 0; d < kv.dim; ++d) dot += q[d] * row[d];
-      sc = dot * a.scale;
-      if (MODE == WINDOW) sc += rel[bucket[min(pos - p, a.nb - 1)] * a.H + h];
-      if (MODE == CHUNK) sc -= slope * (float)(pos - p);
-    }
-    float top = sc;
-#pragma unroll
-    for (int x = 32; x > 0; x >>= 1) top = fmaxf(top, __shfl_xor(top, x));
-    top = fmaxf(top, m);
-    const float al = expf(m - top), e = expf(sc - top);
-    m = top;
-    l = l * al + wave_sum(e);
-#pragma unroll
-    for (int i = 0; i < NC; ++i) acc[i] *= al;
-    const int n = min(64, pos - p0 + 1);
-    for (int j = 0; j < n; ++j) {
-      const float pj = __shfl(e, j);
-      const float* row = vb + Layout<float>::v(kv, min((p0 + j - base) % kv.mod, kv.rows - 1), 0);
-#pragma unroll
-      for (int i = 0; i < NC; ++i)
-        if (lane + i * 64 < kv.vdim) acc[i] += pj * row[lane + i * 64];
-    }
-  }
-  const float f = side.gate(a, (size_t)b * a.S + s, h) / (l + expf(side.sink(h) - m));
-#pragma unroll
-  for (int i = 0; i < NC; ++i)
-    if (lane + i * 64 < kv.vdim) dst[lane + i * 64] = acc[i] * f;
-}
-
 // ===========================================================================
 // host side
 // ===========================================================================
-
-// template sizes: the smallest that hold both dims
-#define BY_DIMS(kc, vg, RUN)                                           \
-  if (kc <= 1 && vg <= 2) RUN(1, 2, (kc == 1 && vg == 2))              \
-  else if (kc <= 2 && vg <= 4) RUN(2, 4, (kc == 2 && vg == 4))         \
-  else if (kc <= 4 && vg <= 8) RUN(4, 8, (kc == 4 && vg == 8))         \
-  else if (kc <= 6 && vg <= 8) RUN(6, 8, (kc == 6 && vg == 8))         \
-  else RUN(8, 16, (kc == 8 && vg == 16))
-
-// Prompt rows [B,S,H,qd] against workspaces of rows [0, hist + S).
-template <int MODE>
-static void prefill_rows(bool bf, int B, const Tensor& qw, const Tensor& kw, const Tensor& vw, const void* proj,
-                         const void* sinks, const int* bucket, const void* rel, Tensor& out, const KVShape& ws,
-                         int hist, int base, const AttnArgs& a, const Step& step) {
-  const hipStream_t stream = cur_stream();
-  TORCH_CHECK(B <= 65535 && a.H <= 65535, "a prefill step of ", B, " rows and ", a.H, " heads is too large");
-  if (!bf) {
-    const Side<MODE, float> side{(const float*)proj, (const float*)sinks};
-    CHK(ws.vdim <= 256);
-    hipLaunchKernelGGL((attn_rows_f32_kernel<MODE, 4>), dim3(a.S, a.H, B), dim3(64), ws.dim * sizeof(float), stream,
-                       P<float>(qw), P<float>(kw), P<float>(vw), side, bucket, (const float*)rel, M<float>(out), ws,
-                       base, a, step);
-    return;
-  }
-  const Side<MODE, bf16_t> side{(const bf16_t*)proj, (const bf16_t*)sinks};
-  const size_t lds = MODE == WINDOW ? (size_t)a.nb * 4 : 0;
-  TORCH_CHECK(lds <= 60000, "distance table of ", a.nb, " entries does not fit LDS");
-  const dim3 grid((a.S + 127) / 128, a.H, B);
-#define RUN(KC, VG, EXACT)                                                                                          \
-  {                                                                                                                 \
-    if (EXACT)                                                                                                      \
-      hipLaunchKernelGGL((attn_rows_prefill_kernel<KC, VG, true, MODE>), grid, dim3(256), lds, stream, P<bf16_t>(qw), \
-                         P<bf16_t>(kw), P<bf16_t>(vw), side, bucket, (const bf16_t*)rel, M<bf16_t>(out), ws, hist, a, step); \
-    else                                                                                                            \
-      hipLaunchKernelGGL((attn_rows_prefill_kernel<KC, VG, false, MODE>), grid, dim3(256), lds, stream, P<bf16_t>(qw), \
-                         P<bf16_t>(kw), P<bf16_t>(vw), side, bucket, (const bf16_t*)rel, M<bf16_t>(out), ws, hist, a, step); \
-  }
-  BY_DIMS(ws.kc, ws.vg, RUN)
-#undef RUN
-}
-
-// One token a row [B,1,H,qd] against the cache.
-template <int MODE>
-static void decode_rows(bool bf, int B, const Tensor& qw, const Tensor& kc, const Tensor& vc, const void* proj,
-                        const void* sinks, const int* bucket, const void* rel, int rel_rows, Tensor& out,
-                        const KVShape& ring, const AttnArgs& a, const Step& step) {
-  const hipStream_t stream = cur_stream();
-  if (!bf) {
-    const Side<MODE, float> side{(const float*)proj, (const float*)sinks};
-    hipLaunchKernelGGL((attn_rows_f32_kernel<MODE, 4>), dim3(1, a.H, B), dim3(64), ring.dim * sizeof(float), stream,
-                       P<float>(qw), P<float>(kc), P<float>(vc), side, bucket, (const float*)rel, M<float>(out), ring,
-                       0, a, step);
-    return;
-  }
-  const Side<MODE, bf16_t> side{(const bf16_t*)proj, (const bf16_t*)sinks};
-  const size_t lds = MODE == WINDOW ? (size_t)a.nb * 4 + (size_t)rel_rows * 64 : 0;
-  TORCH_CHECK(lds <= 60000, "distance table of ", a.nb, " entries does not fit LDS");
-  const int qgs = (a.H / a.G + 15) / 16;
-  // enough blocks for the chip, at least one 32-row tile per wave
-  const int blocks = B * a.G * qgs;
-  const int splits = std::max(1, std::min((512 + blocks - 1) / blocks, ring.rows / 128));
-  Tensor part;
-  if (splits > 1) part = f32(qw, {B, splits, a.H, ring.vdim + 2});
-  float* pp = splits > 1 ? M<float>(part) : nullptr;
-  const dim3 grid(splits, a.G * qgs, B);
-#define RUN(KC, VG, EXACT)                                                                                          \
-  {                                                                                                                 \
-    if (EXACT)                                                                                                      \
-      hipLaunchKernelGGL((attn_rows_decode_kernel<KC, VG, true, MODE>), grid, dim3(256), lds, stream, P<bf16_t>(qw), \
-                         P<bf16_t>(kc), P<bf16_t>(vc), side, bucket, (const bf16_t*)rel, rel_rows, M<bf16_t>(out), pp, \
-                         splits, ring, a, step);                                                                    \
-    else                                                                                                            \
-      hipLaunchKernelGGL((attn_rows_decode_kernel<KC, VG, false, MODE>), grid, dim3(256), lds, stream, P<bf16_t>(qw), \
-                         P<bf16_t>(kc), P<bf16_t>(vc), side, bucket, (const bf16_t*)rel, rel_rows, M<bf16_t>(out), pp, \
-                         splits, ring, a, step);                                                                    \
-  }
-  BY_DIMS(ring.kc, ring.vg, RUN)
-#undef RUN
-  if (splits > 1)
-    hipLaunchKernelGGL((attn_rows_merge_kernel<MODE>), dim3(a.H, B), dim3(64), 0, stream, pp, side, M<bf16_t>(out),
-                       splits, ring.vdim, a, step);
-}
-
-static KVShape cache_shape(bool bf, int64_t G, int64_t dim, int64_t vdim, const Tensor& kc, const Tensor& vc) {
-  KVShape ring{(int)dim, (int)vdim, (int)(dim + 31) / 32, (int)(vdim + 15) / 16, 0, 0};
-  CHK(kc.size(1) == G && vc.size(1) == G && kc.size(0) == vc.size(0));
-  if (bf) {
-    CHK(kc.dim() == 6 && vc.dim() == 6 && kc.size(3) == ring.kc && vc.size(2) == ring.vg);
-    ring.rows = kc.size(2) * 16;
-    CHK(ring.rows % 32 == 0 && vc.size(3) * 32 == ring.rows);
-  } else {
-    CHK(kc.dim() == 4 && vc.dim() == 4 && kc.size(3) == dim && vc.size(3) == vdim && kc.size(2) == vc.size(2));
-    ring.rows = kc.size(2);
-  }
-  CHK(ring.rows > 0);
-  ring.mod = ring.rows;
-  return ring;
-}
-
-// One linear workspace of keys and values for a prompt chunk: `hist` earlier
-// rows, then the chunk, padded to whole tiles.
-struct Workspace {
-  KVShape shape;
-  Tensor k, v;
-  int fill;
-  Workspace(bool bf, const KVShape& ring, const Tensor& like, int B, int G, int hist, int S) : shape(ring) {
-    shape.rows = (hist + S + 31) / 32 * 32;
-    shape.mod = INT_MAX;
-    fill = shape.rows - hist;
-    k = torch::empty({B, G, (int64_t)shape.rows * (bf ? shape.kc * 32 : shape.dim)}, like.options());
-    v = torch::empty({B, G, (int64_t)shape.rows * (bf ? shape.vg * 16 : shape.vdim)}, like.options());
-  }
-};
 
 void window_attn(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t g_at, int64_t H, int64_t G,
                  int64_t dim, int64_t vdim, Tensor q_norm, Tensor k_norm, Tensor bucket, Tensor rel, double scale,
@@ -754,7 +253,7 @@ void window_attn(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t 
       hipLaunchKernelGGL((qk_norm_append_kernel<T>), dim3(1, B), dim3(256), 0, stream, P<T>(proj), P<T>(q_norm),
                          P<T>(k_norm), M<T>(qw), M<T>(kc), M<T>(vc), (T*)nullptr, (T*)nullptr, ring, ring, 0, a, step);
     });
-    decode_rows<WINDOW>(bf, B, qw, kc, vc, proj.data_ptr(), nullptr, bk, rel.data_ptr(), rel_rows, out, ring, a, step);
+    decode_rows<WINDOW>(bf, B, qw, kc, vc, proj.data_ptr(), nullptr, bk, rel.data_ptr(), rel_rows, out, ring, 0, a, step);
     return;
   }
   // the workspace: what the window still holds of earlier chunks, then this chunk
@@ -811,7 +310,7 @@ void chunk_attn(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t H
                          P<T>(k_norm), mix, M<T>(qw), M<T>(kc), M<T>(vc), (T*)nullptr, (T*)nullptr, ring, ring, 0, a,
                          step);
     });
-    decode_rows<CHUNK>(bf, B, qw, kc, vc, nullptr, sinks.data_ptr(), nullptr, nullptr, 0, out, ring, a, step);
+    decode_rows<CHUNK>(bf, B, qw, kc, vc, nullptr, sinks.data_ptr(), nullptr, nullptr, 0, out, ring, 0, a, step);
     return;
   }
   // the workspace begins with the chunk that `start` lies in

@@ -138,6 +138,36 @@ DEVINL float block_sum(float v, float* red) {
   return red[0] + red[1] + red[2] + red[3];
 }
 
+// operands of 16x16 matrix products in either element type (fp32 throughout)
+template <typename T> struct Frag;
+template <> struct Frag<bf16_t> {
+  typedef bf16x8 V;
+  static constexpr int K = 32, PER = 8;  // k of a step, elements of a lane
+};
+template <> struct Frag<float> {
+  typedef floatx4 V;
+  static constexpr int K = 16, PER = 4;
+};
+// D[16 rows of a][16 rows of b] += over one k step
+DEVINL floatx4 mma(const bf16x8& a, const bf16x8& b, floatx4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+DEVINL floatx4 mma(const floatx4& a, const floatx4& b, floatx4 c) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
+  return c;
+}
+// a lane's elements k.. of a row of n; WHOLE: n is a multiple of the step
+template <typename T, bool WHOLE>
+DEVINL typename Frag<T>::V ld_frag(const T* row, int k, int n) {
+  typedef typename Frag<T>::V V;
+  if (WHOLE) return *(const V*)(row + k);
+  union { V v; T e[Frag<T>::PER]; } u;
+#pragma unroll
+  for (int i = 0; i < Frag<T>::PER; ++i) u.e[i] = k + i < n ? row[k + i] : (T)0;
+  return u.v;
+}
+
 struct Step {
   const int* slots;      // null: row b is slot b
   const int* positions;  // decode only

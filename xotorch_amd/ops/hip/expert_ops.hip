@@ -1,7 +1,8 @@
 // CDNA4 (gfx950) kernels of sparse feed-forwards: a mixture of small experts,
 // routed and computed without the host seeing a count.
 //   - router: logits on matrix cores (fp32 accumulation), sigmoid scores, a
-//     correction that only chooses, group-limited top-k, counts per block
+//     correction that only chooses, group-limited top-k, or a softmax over the
+//     chosen logits; experts that every token uses; counts per block
 //   - place: every (token, expert) pair gets a row; rows of an expert lie
 //     together, in token order
 //   - grouped products: gate and up of a pair's token with the gated activation
@@ -14,37 +15,6 @@
 
 #include "common.h"
 
-typedef __attribute__((ext_vector_type(16))) float floatx16;
-
-template <typename T> struct Frag;
-template <> struct Frag<bf16_t> {
-  typedef bf16x8 V;
-  static constexpr int K = 32, PER = 8;  // k of a step, elements of a lane
-};
-template <> struct Frag<float> {
-  typedef floatx4 V;
-  static constexpr int K = 16, PER = 4;
-};
-// D[16 rows of a][16 rows of b] += over one k step
-DEVINL floatx4 mma(const bf16x8& a, const bf16x8& b, floatx4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
-}
-DEVINL floatx4 mma(const floatx4& a, const floatx4& b, floatx4 c) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
-  return c;
-}
-// a lane's elements k.. of a row of n; WHOLE: n is a multiple of the step
-template <typename T, bool WHOLE>
-DEVINL typename Frag<T>::V ld_frag(const T* row, int k, int n) {
-  typedef typename Frag<T>::V V;
-  if (WHOLE) return *(const V*)(row + k);
-  union { V v; T e[Frag<T>::PER]; } u;
-#pragma unroll
-  for (int i = 0; i < Frag<T>::PER; ++i) u.e[i] = k + i < n ? row[k + i] : (T)0;
-  return u.v;
-}
-
 // ---------------------------------------------------------------------------
 // router
 // ---------------------------------------------------------------------------
@@ -52,7 +22,9 @@ DEVINL typename Frag<T>::V ld_frag(const T* row, int k, int n) {
 constexpr int RT = 16;          // tokens of a router block
 constexpr int MAX_EXPERTS = 512, MAX_TOP = 16;
 
-struct RouteArgs { int T, D, E, top, groups, keep, nblk, tile; float scale; };  // tile: rows of a tile
+// pick of E experts are chosen, then come top - pick that every token uses, all
+// in all; tile: rows of a tile
+struct RouteArgs { int T, D, E, top, groups, keep, nblk, tile; float scale; int pick, all, softmax; };
 
 // RW waves share k. Sixteen lanes choose for a token, J experts each.
 template <typename T, bool WHOLE, int J, int RW>
@@ -60,21 +32,23 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
     const T* __restrict__ x, const T* __restrict__ w, const T* __restrict__ correction, int* __restrict__ idx,
     float* __restrict__ weight, int* __restrict__ rank, int* __restrict__ counts, RouteArgs a) {
   typedef Frag<T> F;
-  extern __shared__ float lds[];  // choice, scores [RT][E]; partial sums [RW][RT][65]; chosen [RT][top]
+  extern __shared__ float lds[];  // choice, scores [RT][E]; partial sums [RW][RT][65]; chosen [RT][top]; open [RT]
   float* choice = lds;
   float* score = choice + RT * a.E;
   float* part = score + RT * a.E;
   int* chosen = (int*)(part + RW * RT * 65);
+  float* open = (float*)(chosen + RT * a.top);  // [RT], the gate of the experts that every token uses
+  const int Z = a.E + (a.all > a.E);
   const int t0 = blockIdx.x * RT, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
   const T* xr = x + (size_t)min(t0 + col, a.T - 1) * a.D;
   const int steps = (a.D + F::K - 1) / F::K;
-  for (int e0 = 0; e0 < a.E; e0 += 64) {
+  for (int e0 = 0; e0 < Z; e0 += 64) {
     floatx4 acc[4];
     const T* wr[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       acc[i] = (floatx4)(0.f);
-      wr[i] = w + (size_t)min(e0 + i * 16 + col, a.E - 1) * a.D;
+      wr[i] = w + (size_t)min(e0 + i * 16 + col, Z - 1) * a.D;
     }
     auto run = [&](int c, auto count) {  // `count` steps from c on, loads first
       constexpr int UN = decltype(count)::value;
@@ -101,13 +75,15 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
     __syncthreads();
     for (int i = threadIdx.x; i < RT * 64; i += 64 * RW) {
       const int t = i >> 6, e = e0 + (i & 63);
-      if (e < a.E) {
+      if (e < Z) {
         float z = 0.f;
 #pragma unroll
         for (int v = 0; v < RW; ++v) z += part[(v * RT + t) * 65 + (i & 63)];
-        const float s = 1.f / (1.f + expf(-z));
-        score[t * a.E + e] = s;
-        choice[t * a.E + e] = s + ld(correction + e);
+        const float s = a.softmax && e < a.E ? z : 1.f / (1.f + expf(-z));
+        if (e < a.E) {
+          score[t * a.E + e] = s;
+          choice[t * a.E + e] = correction ? s + ld(correction + e) : s;
+        } else open[t] = s;
       }
     }
     __syncthreads();
@@ -143,7 +119,8 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
 #pragma unroll
     for (int j = 0; j < J; ++j) v[j] = l + j * 16 < a.E ? ch[l + j * 16] : -INFINITY;
     const bool valid = t0 + t < a.T;
-    for (int k = 0; k < a.top; ++k) {
+    float mine = 0.f;  // score of the choice that lane l weighs
+    for (int k = 0; k < a.pick; ++k) {
       float best = v[0];
 #pragma unroll
       for (int j = 1; j < J; ++j) best = fmaxf(best, v[j]);
@@ -156,12 +133,23 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
 #pragma unroll
       for (int j = 0; j < J; ++j)
         if (at == l + j * 16) v[j] = -INFINITY;
+      if (l == k) mine = score[t * a.E + at];
       if (l == 0) {
         chosen[t * a.top + k] = valid ? at : -1;
-        if (valid) {
-          idx[(size_t)(t0 + t) * a.top + k] = at;
-          weight[(size_t)(t0 + t) * a.top + k] = score[t * a.E + at] * a.scale;
-        }
+        if (valid) idx[(size_t)(t0 + t) * a.top + k] = at;
+      }
+    }
+    if (a.softmax) {
+      const float e = l < a.pick ? expf(mine - row_max(l < a.pick ? mine : -INFINITY)) : 0.f;
+      mine = e / row_sum(e);
+    }
+    if (valid && l < a.pick) weight[(size_t)(t0 + t) * a.top + l] = mine * a.scale;
+    if (l >= a.pick && l < a.top) {
+      const int e = a.E + l - a.pick;
+      chosen[t * a.top + l] = valid ? e : -1;
+      if (valid) {
+        idx[(size_t)(t0 + t) * a.top + l] = e;
+        weight[(size_t)(t0 + t) * a.top + l] = open[t];
       }
     }
   }
@@ -170,7 +158,7 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
   // chosen holds RT * top entries, a multiple of four
   const int4* four = (const int4*)chosen;
   const int pairs = (min(RT, a.T - t0) * a.top + 3) >> 2;  // fours of them
-  for (int e = threadIdx.x; e < a.E; e += 64 * RW) {
+  for (int e = threadIdx.x; e < a.all; e += 64 * RW) {
     int n = 0;
     int* dst = rank + (size_t)t0 * a.top;
     for (int o = 0; o < pairs; ++o) {
@@ -216,10 +204,10 @@ __global__ __launch_bounds__(256) void place_kernel(
     int2* __restrict__ tiles, int max_tiles, RouteArgs a) {
   __shared__ int at[MAX_EXPERTS], cnt[MAX_EXPERTS], tile_at[MAX_EXPERTS], ends[2];
   // a single block of the router needs no scan: its counts are the totals
-  for (int e = threadIdx.x; e < a.E; e += 256) cnt[e] = a.nblk == 1 ? before[e] : total[e];
+  for (int e = threadIdx.x; e < a.all; e += 256) cnt[e] = a.nblk == 1 ? before[e] : total[e];
   __syncthreads();
   if (threadIdx.x < 64) {  // one wave scans, E/64 each
-    const int per = (a.E + 63) / 64, lo = threadIdx.x * per, hi = min(lo + per, a.E);
+    const int per = (a.all + 63) / 64, lo = threadIdx.x * per, hi = min(lo + per, a.all);
     int n = 0, m = 0;
     for (int e = lo; e < hi; ++e) { n += cnt[e]; m += (cnt[e] + a.tile - 1) / a.tile; }
     int sn = n, sm = m;
@@ -247,12 +235,12 @@ __global__ __launch_bounds__(256) void place_kernel(
     token[r] = t;
   }
   if (blockIdx.x) return;
-  for (int e = threadIdx.x; e < a.E; e += 256) {
+  for (int e = threadIdx.x; e < a.all; e += 256) {
     first[e] = at[e];
     for (int i = 0; i * a.tile < cnt[e]; ++i) tiles[tile_at[e] + i] = make_int2(e, at[e] + i * a.tile);
   }
   for (int i = ends[1] + threadIdx.x; i < max_tiles; i += 256) tiles[i] = make_int2(-1, 0);
-  if (threadIdx.x == 0) first[a.E] = ends[0];
+  if (threadIdx.x == 0) first[a.all] = ends[0];
 }
 
 // ---------------------------------------------------------------------------
@@ -528,34 +516,40 @@ __global__ __launch_bounds__(256) void add_norm_kernel(
 // ===========================================================================
 
 // x [.., D] -> (weights [T, top] fp32, row of every pair [T, top], token of
-// every row, first row of every expert [E + 1], tiles [max, 2], rows of a tile)
-std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tensor w, Tensor correction, int64_t top, int64_t groups, int64_t keep,
-                          double scale) {
+// every row, first row of every expert [E + 1], tiles [max, 2], rows of a tile).
+// `shared` experts follow the routed ones in every token's list (top counts
+// them then); their weight is the sigmoid of one more row of w.
+std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tensor w, OptT correction, int64_t pick,
+                                                                  int64_t groups, int64_t keep, double scale,
+                                                                  bool softmax, int64_t shared) {
   const auto dt = io_type(x);
   check_io(w, dt);
-  check_io(correction, dt);
-  const int D = x.size(-1), T_ = x.numel() / D, E = w.size(0);
-  CHK(w.dim() == 2 && w.size(1) == D && correction.numel() == E && T_ > 0);
-  TORCH_CHECK(E >= 1 && E <= MAX_EXPERTS && top >= 1 && top <= MAX_TOP && top <= E, "routing to ", top, " of ", E, " experts");
-  TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
-              "routing to ", top, " experts of ", keep, " of ", groups, " groups of ", E, " experts");
+  const int D = x.size(-1), T_ = x.numel() / D, E = w.size(0) - (shared > 0);
+  if (correction) { check_io(*correction, dt); CHK(correction->numel() == E); }
+  CHK(w.dim() == 2 && w.size(1) == D && T_ > 0 && shared >= 0);
+  const int64_t top = pick + shared, all = E + shared;
+  TORCH_CHECK(E >= 1 && all <= MAX_EXPERTS && pick >= 1 && top <= MAX_TOP && pick <= E, "routing to ", pick, " of ", E,
+              " experts and ", shared, " shared ones");
+  TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && pick <= keep * (E / groups),
+              "routing to ", pick, " experts of ", keep, " of ", groups, " groups of ", E, " experts");
   CHK((int64_t)T_ * top < INT_MAX);
   const int nblk = (T_ + RT - 1) / RT, pairs = T_ * (int)top;
-  const int tile = pairs >= 320 * E ? 256 : 128, max_tiles = pairs / tile + std::min(pairs, E);
+  const int tile = pairs >= 320 * all ? 256 : 128, max_tiles = pairs / tile + std::min(pairs, (int)all);
   const auto ints = x.options().dtype(torch::kInt32);
   auto weight = f32(x, {T_, top});
   auto idx = torch::empty({T_, top}, ints), rank = torch::empty({T_, top}, ints), row = torch::empty({T_, top}, ints);
-  auto counts = torch::empty({E, nblk}, ints), total = torch::empty({E}, ints), first = torch::empty({E + 1}, ints);
+  auto counts = torch::empty({all, nblk}, ints), total = torch::empty({all}, ints), first = torch::empty({all + 1}, ints);
   auto token = torch::empty({pairs}, ints), tiles = torch::empty({max_tiles, 2}, ints);
-  const RouteArgs a{T_, D, E, (int)top, (int)groups, (int)keep, nblk, tile, (float)scale};
+  const RouteArgs a{T_, D, E, (int)top, (int)groups, (int)keep, nblk, tile, (float)scale, (int)pick, (int)all, softmax};
   const hipStream_t stream = cur_stream();
   CHK(groups <= 4 * 65);
   BY_TYPE(dt, {
+    const T* cp = correction ? P<T>(*correction) : nullptr;
     auto run = [&](auto kernel, int waves) {
       static const hipError_t err = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
       TORCH_CHECK(err == hipSuccess, "no LDS for the router");
-      const size_t lds = (2 * RT * E + waves * RT * 65) * sizeof(float) + RT * top * sizeof(int);  // parts of 16 bytes
-      hipLaunchKernelGGL(kernel, dim3(nblk), dim3(64 * waves), lds, stream, P<T>(x), P<T>(w), P<T>(correction),
+      const size_t lds = (2 * RT * E + waves * RT * 65) * sizeof(float) + RT * (top + 1) * sizeof(int);  // parts of 16 bytes
+      hipLaunchKernelGGL(kernel, dim3(nblk), dim3(64 * waves), lds, stream, P<T>(x), P<T>(w), cp,
                          idx.data_ptr<int>(), M<float>(weight), rank.data_ptr<int>(), counts.data_ptr<int>(), a);
     };
     // few tokens: more waves on each
@@ -566,7 +560,7 @@ std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tens
     else run(route_kernel<T, true, MAX_EXPERTS / 16, 4>, 4);
   });
   if (nblk > 1)
-    hipLaunchKernelGGL(count_scan_kernel, dim3(E), dim3(256), 0, stream, counts.data_ptr<int>(), total.data_ptr<int>(), nblk);
+    hipLaunchKernelGGL(count_scan_kernel, dim3(all), dim3(256), 0, stream, counts.data_ptr<int>(), total.data_ptr<int>(), nblk);
   hipLaunchKernelGGL(place_kernel, dim3((pairs + 255) / 256), dim3(256), 0, stream, idx.data_ptr<int>(),
                      rank.data_ptr<int>(), counts.data_ptr<int>(), total.data_ptr<int>(), row.data_ptr<int>(),
                      token.data_ptr<int>(), first.data_ptr<int>(), (int2*)tiles.data_ptr<int>(), max_tiles, a);
@@ -669,7 +663,9 @@ OptT add_norm(Tensor y, OptT rows, OptT weight, Tensor x, OptT w_next, double mu
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
-  m.def("route", &route, "sigmoid router with a choosing correction and group-limited top-k; rows of all pairs");
+  m.def("route", &route, "router: sigmoid scores or a softmax over the chosen, group-limited top-k, shared experts; rows of all pairs",
+        py::arg("x"), py::arg("w"), py::arg("correction"), py::arg("top"), py::arg("groups"), py::arg("keep"),
+        py::arg("scale"), py::arg("softmax") = false, py::arg("shared") = 0);
   m.def("expert_product", &expert_product, "grouped product of all (token, expert) pairs, gated or plain");
   m.def("add_norm", &add_norm, "stream += mult * (output or weighted expert rows); norm of the stream");
 }

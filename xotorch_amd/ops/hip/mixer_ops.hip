@@ -19,12 +19,14 @@
 // norms around the fp32 stream
 // ---------------------------------------------------------------------------
 
-// y null: h = norm(x; w_next) only. One block per row; the row stays in
-// registers (NC chunks of 256*V elements).
+// y null: h = norm(x; w_next) only. With `rows`, a row of y is the weighted sum
+// of `top` of its rows. copy: h is the stream as it is. One block per row; the
+// row stays in registers (NC chunks of 256*V elements).
 template <typename T, int V, int NC>
 __global__ __launch_bounds__(256) void sandwich_norm_kernel(
-    const T* __restrict__ y, float* __restrict__ x, const T* __restrict__ w_post,
-    const T* __restrict__ w_next, T* __restrict__ h, int D, float eps) {
+    const T* __restrict__ y, const int* __restrict__ rows, const float* __restrict__ weight, int top, int ys,
+    float* __restrict__ x, const T* __restrict__ w_post, const T* __restrict__ w_next, T* __restrict__ h, int copy,
+    int D, float eps) {
   const size_t off = (size_t)blockIdx.x * D;
   __shared__ float red[8];
   float xv[NC * V];
@@ -42,7 +44,17 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(
     for (int c = 0; c < NC; ++c) {
       const int i = (c * 256 + threadIdx.x) * V;
       if (i < D) {
-        ldv<V>(y + off + i, yv + c * V);
+        if (!rows) ldv<V>(y + (size_t)blockIdx.x * ys + i, yv + c * V);
+        else
+#pragma unroll
+          for (int j = 0; j < V; ++j) yv[c * V + j] = 0.f;
+        for (int k = 0; rows && k < top; ++k) {
+          const float wk = weight[(size_t)blockIdx.x * top + k];
+          float v[V];
+          ldv<V>(y + (size_t)rows[(size_t)blockIdx.x * top + k] * ys + i, v);
+#pragma unroll
+          for (int j = 0; j < V; ++j) yv[c * V + j] += wk * v[j];
+        }
 #pragma unroll
         for (int j = 0; j < V; ++j) acc += yv[c * V + j] * yv[c * V + j];
       }
@@ -57,6 +69,7 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(
 #pragma unroll
         for (int j = 0; j < V; ++j) xv[c * V + j] += yv[c * V + j] * inv * (1.f + w[j]);
         stv<V>(x + off + i, xv + c * V);
+        if (copy) stv<V>(h + off + i, xv + c * V);
       }
     }
   }
@@ -762,41 +775,69 @@ __global__ __launch_bounds__(256) void token_shift_kernel(
 // host side
 // ===========================================================================
 
+// what a sublayer's output row is made of: itself, or weighted rows (rows set)
+struct Gather { const int* rows; const float* weight; int top, ys; };
+
 template <typename T, int V>
-static void launch_norm(const T* y, float* x, const T* wp, const T* wn, T* h, int rows, int D, float eps) {
+static void launch_norm(const T* y, const Gather& from, float* x, const T* wp, const T* wn, T* h, int copy, int rows,
+                        int D, float eps) {
   const int nc = (D + 256 * V - 1) / (256 * V);
-#define NORM_CASE(NC) \
-  if (nc <= NC) { hipLaunchKernelGGL((sandwich_norm_kernel<T, V, NC>), dim3(rows), dim3(256), 0, cur_stream(), y, x, wp, wn, h, D, eps); return; }
+#define NORM_CASE(NC)                                                                                              \
+  if (nc <= NC) {                                                                                                  \
+    hipLaunchKernelGGL((sandwich_norm_kernel<T, V, NC>), dim3(rows), dim3(256), 0, cur_stream(), y, from.rows,     \
+                       from.weight, from.top, from.ys, x, wp, wn, h, copy, D, eps);                                \
+    return;                                                                                                        \
+  }
   NORM_CASE(1) NORM_CASE(2) NORM_CASE(4) NORM_CASE(8) NORM_CASE(16)
 #undef NORM_CASE
   TORCH_CHECK(false, "row of ", D, " elements is too long");
 }
 
-static OptT norm_host(const OptT& y, Tensor x, const OptT& w_post, const OptT& w_next, double eps,
-                      torch::ScalarType dt) {
+static OptT norm_host(const OptT& y, Tensor x, const OptT& w_post, const OptT& w_next, double eps, bool copy,
+                      const OptT& take, const OptT& weight, torch::ScalarType dt) {
   check_io(x, torch::kFloat32);
   const int D = x.size(-1), rows = x.numel() / D;
-  if (y) { check_io(*y, dt); CHK(y->numel() == x.numel() && y->size(-1) == D && w_post); check_io(*w_post, dt); CHK(w_post->numel() == D); }
+  Gather from{nullptr, nullptr, 0, D};
+  CHK(!copy || (y && !w_next));
+  if (y) {
+    check_io(*y, dt);
+    CHK(w_post);
+    check_io(*w_post, dt);
+    CHK(w_post->numel() == D);
+  }
+  if (take) {
+    CHK(y && weight);
+    check_io(*take, torch::kInt32);
+    check_io(*weight, torch::kFloat32);
+    from = Gather{take->data_ptr<int>(), weight->data_ptr<float>(), (int)take->size(-1), (int)y->size(-1)};
+    CHK(take->numel() == (int64_t)rows * from.top && weight->numel() == take->numel() && from.ys >= D &&
+        y->numel() == take->numel() * from.ys);
+  } else if (y) {
+    CHK(y->numel() == x.numel() && y->size(-1) == D);
+  }
   OptT h;
-  if (w_next) { check_io(*w_next, dt); CHK(w_next->numel() == D); h = torch::empty(x.sizes(), x.options().dtype(dt)); }
+  if (w_next) { check_io(*w_next, dt); CHK(w_next->numel() == D); }
+  if (w_next || copy) h = torch::empty(x.sizes(), x.options().dtype(dt));
   if (rows == 0) return h;
   BY_TYPE(dt, {
     const T* yp = y ? P<T>(*y) : nullptr;
     const T* wp = w_post ? P<T>(*w_post) : nullptr;
     const T* wn = w_next ? P<T>(*w_next) : nullptr;
     T* hp = h ? M<T>(*h) : nullptr;
-    if (D % 4 == 0) launch_norm<T, 4>(yp, M<float>(x), wp, wn, hp, rows, D, (float)eps);
-    else launch_norm<T, 1>(yp, M<float>(x), wp, wn, hp, rows, D, (float)eps);
+    if (((D | from.ys) & 3) == 0) launch_norm<T, 4>(yp, from, M<float>(x), wp, wn, hp, copy, rows, D, (float)eps);
+    else launch_norm<T, 1>(yp, from, M<float>(x), wp, wn, hp, copy, rows, D, (float)eps);
   });
   return h;
 }
 
-OptT sandwich_norm(Tensor y, Tensor x, Tensor w_post, OptT w_next, double eps) {
-  return norm_host(y, x, w_post, w_next, eps, io_type(y));
+// take, weight [tokens, top]: y is not yet summed, row take[t, k] counts weight[t, k]
+OptT sandwich_norm(Tensor y, Tensor x, Tensor w_post, OptT w_next, double eps, bool copy, OptT take, OptT weight) {
+  return norm_host(y, x, w_post, w_next, eps, copy, take, weight, io_type(y));
 }
 
 Tensor prenorm(Tensor x, Tensor w, double eps, bool bf16) {
-  return *norm_host(c10::nullopt, x, c10::nullopt, w, eps, bf16 ? torch::kBFloat16 : torch::kFloat32);
+  return *norm_host(c10::nullopt, x, c10::nullopt, w, eps, false, c10::nullopt, c10::nullopt,
+                    bf16 ? torch::kBFloat16 : torch::kFloat32);
 }
 
 Tensor swiglu_packed(Tensor gu) {
@@ -997,7 +1038,9 @@ Tensor token_shift(Tensor h, Tensor mu, Tensor ring, OptT slots, OptT positions,
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("prenorm", &prenorm, "RMS norm with a (1+w) weight of the fp32 stream");
-  m.def("sandwich_norm", &sandwich_norm, "stream += norm(y); norm of the stream for the next sublayer");
+  m.def("sandwich_norm", &sandwich_norm, "stream += norm(y); norm or copy of the stream for the next sublayer",
+        py::arg("y"), py::arg("x"), py::arg("w_post"), py::arg("w_next"), py::arg("eps"), py::arg("copy") = false,
+        py::arg("take") = py::none(), py::arg("weight") = py::none());
   m.def("swiglu_packed", &swiglu_packed, "SwiGLU on a packed projection, any width, bf16 or fp32");
   m.def("tanh", &tanh_op, "tanh with fp32 math");
   m.def("delta_rule", &delta_rule, "gated delta rule with short convolutions and per-channel decay");

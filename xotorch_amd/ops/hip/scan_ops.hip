@@ -1,5 +1,5 @@
-// CDNA4 (gfx950) kernels of selective state spaces: a short causal convolution
-// with bias and silu, and the scan
+// CDNA4 (gfx950) kernels of short causal convolutions (also used by other
+// recurrences) and of selective state spaces: the scan
 //   S[c,n] = exp(dt_c A[c,n]) S[c,n] + dt_c x_c B_n,  y_c = sum_n S[c,n] C_n + D_c x_c
 // with the gate y silu(z). Step sizes (softplus), decays and the state are
 // fp32; inputs and outputs are bf16 or fp32.
@@ -10,15 +10,17 @@
 
 #include "common.h"
 
-struct ConvArgs { int S, C, N, at, taps; };  // tokens, channels, input row, first column
+struct ConvArgs { int S, C, N, at, taps, silu; };  // tokens, channels, input row, first column
 
 constexpr int RUN = 16;  // tokens a thread walks
 
 // Thread: V channels, RUN tokens. TAPS 0: any number of taps, inputs read
-// again. A decode step also stores its input (row p % taps of the ring).
+// again. in_bias joins the input of every token there is. A decode step also
+// stores its input (row p % taps of the ring).
 template <typename T, int V, int TAPS>
-__global__ __launch_bounds__(256) void conv_silu_kernel(
-    const T* __restrict__ x, const T* __restrict__ w, const T* __restrict__ bias, T* __restrict__ ring,
+__global__ __launch_bounds__(256) void short_conv_kernel(
+    const T* __restrict__ x, const T* __restrict__ w, const T* __restrict__ bias, const T* __restrict__ in_bias,
+    T* __restrict__ ring,
     T* __restrict__ out, ConvArgs a, Step step) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * V, b = blockIdx.z, s0 = blockIdx.y * RUN;
   if (c >= a.C) return;
@@ -26,12 +28,20 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(
   const int first = len ? step.first(b) : 0;
   const T* rows = x + (size_t)b * a.S * a.N + a.at + c;
   T* hist = ring + (size_t)max(slot, 0) * a.taps * a.C + c;
+  float ib[V];
+#pragma unroll
+  for (int i = 0; i < V; ++i) ib[i] = 0.f;
+  if (in_bias) ldv<V>(in_bias + c, ib);
   auto input = [&](int s, float* o) {  // of token s of this step; s < 0: before it
-    if (s >= 0) ldv<V>(rows + (size_t)s * a.N, o);
-    else if (first + s >= 0) ldv<V>(hist + (size_t)((first + s) % a.taps) * a.C, o);
-    else
+    if (first + s < 0) {
 #pragma unroll
       for (int i = 0; i < V; ++i) o[i] = 0.f;
+      return;
+    }
+    if (s >= 0) ldv<V>(rows + (size_t)s * a.N, o);
+    else ldv<V>(hist + (size_t)((first + s) % a.taps) * a.C, o);
+#pragma unroll
+    for (int i = 0; i < V; ++i) o[i] += ib[i];
   };
   constexpr int NT = TAPS ? TAPS : 1;
   float tw[NT][V], in[NT][V], bs[V];
@@ -69,11 +79,12 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(
           for (int i = 0; i < V; ++i) y[i] += v[i] * ld(w + (size_t)(c + i) * a.taps + j);
         }
       }
+      if (a.silu)
 #pragma unroll
-      for (int i = 0; i < V; ++i) y[i] = siluf(y[i]);
+        for (int i = 0; i < V; ++i) y[i] = siluf(y[i]);
       if (step.decode) {
         float v[V];
-        input(0, v);
+        ldv<V>(rows, v);
         stv<V>(hist + (size_t)(first % a.taps) * a.C, v);  // the oldest input: no tap reaches it any more
       }
     }
@@ -322,8 +333,8 @@ __global__ __launch_bounds__(256) void scan_step_kernel(
 // ===========================================================================
 
 // x: C columns of proj [B,S,N] from column `at` on
-Tensor conv_silu(Tensor proj, int64_t at, Tensor w, Tensor bias, Tensor ring, OptT slots, OptT positions, OptT lens,
-                 int64_t start, bool decode) {
+Tensor short_conv(Tensor proj, int64_t at, Tensor w, Tensor bias, OptT in_bias, bool silu, Tensor ring, OptT slots,
+                  OptT positions, OptT lens, int64_t start, bool decode) {
   const auto dt = io_type(proj);
   for (const Tensor& t : {w, bias, ring}) check_io(t, dt);
   CHK(proj.dim() == 3 && w.dim() == 2 && ring.dim() == 3);
@@ -333,14 +344,15 @@ Tensor conv_silu(Tensor proj, int64_t at, Tensor w, Tensor bias, Tensor ring, Op
   auto out = torch::empty({B, S, C}, proj.options());
   if (B == 0 || S == 0) return out;
   const Step step = make_step(slots, positions, lens, start, decode, B);
-  const ConvArgs a{S, C, N, (int)at, taps};
+  if (in_bias) { check_io(*in_bias, dt); CHK(in_bias->numel() == C); }
+  const ConvArgs a{S, C, N, (int)at, taps, silu};
   const hipStream_t stream = cur_stream();
   const bool vec = ((C | N | (int)at) & 3) == 0;
   CHK((S + RUN - 1) / RUN <= 65535);
   const dim3 grid((C + (vec ? 1023 : 255)) / (vec ? 1024 : 256), (S + RUN - 1) / RUN, B);
 #define CONV(V, TAPS)                                                                                            \
-  hipLaunchKernelGGL((conv_silu_kernel<T, V, TAPS>), grid, dim3(256), 0, stream, P<T>(proj), P<T>(w), P<T>(bias), \
-                     M<T>(ring), M<T>(out), a, step)
+  hipLaunchKernelGGL((short_conv_kernel<T, V, TAPS>), grid, dim3(256), 0, stream, P<T>(proj), P<T>(w), P<T>(bias), \
+                     in_bias ? P<T>(*in_bias) : nullptr, M<T>(ring), M<T>(out), a, step)
 #define CONV_TAPS(V)               \
   if (taps == 4) CONV(V, 4);       \
   else if (taps == 3) CONV(V, 3);  \
@@ -430,6 +442,6 @@ void selective_scan(Tensor x, Tensor pre, Tensor bc, int64_t b_at, int64_t c_at,
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
-  m.def("conv_silu", &conv_silu, "short causal convolution with bias and silu");
+  m.def("short_conv", &short_conv, "short causal convolution with bias, and silu");
   m.def("selective_scan", &selective_scan, "selective state space scan with skip and gate");
 }

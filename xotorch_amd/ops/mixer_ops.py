@@ -1,8 +1,9 @@
 """Dispatch of the token mixers' ops and of the fp32-residual norms.
 
 CUDA tensors run the HIP kernels of `_hip_mixers`, `_hip_attn`, `_hip_latent`,
-`_hip_scan` and `_hip_experts` (hip/*.hip) in bfloat16 or true 32-bit, CPU tensors and training run torch_ref_mixers. A
-CUDA tensor never falls back: without the extension the op raises.
+`_hip_scan`, `_hip_rotary`, `_hip_lru` and `_hip_experts` (hip/*.hip) in
+bfloat16 or true 32-bit, CPU tensors and training run torch_ref_mixers. A CUDA
+tensor never falls back: without the extension the op raises.
 
 A mixer's state is one tuple of tensors per layer whose first dimension is
 the slot (engine/kvcache.py, MixerStateCache). `StepRows` says which slot and
@@ -10,8 +11,8 @@ which positions a step's rows have, so a step may address any set of slots.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import NamedTuple, Optional, Tuple, Union
+from dataclasses import dataclass, field
+from typing import Dict, NamedTuple, Optional, Tuple, Union
 
 import torch
 
@@ -45,8 +46,10 @@ class StepRows:
   positions: Optional[torch.Tensor] = None
   slots: Optional[torch.Tensor] = None
   lens: Optional[torch.Tensor] = None
-  # values [B, S, *] of the layer that later layers mix theirs with
-  first_values: Optional[torch.Tensor] = None
+  # what of a layer [B, S, *] later layers and ring stages read, by name
+  carried: Dict[str, torch.Tensor] = field(default_factory=dict)
+  # (state, source, key norm) of layers whose keys and values others read
+  kept: Dict[int, tuple] = field(default_factory=dict)
 
 
 def row_pad(dim: int) -> int:
@@ -64,20 +67,21 @@ def packed_kv(dtype: torch.dtype, device) -> bool:
 
 # ---------------------------------------------------------------- norms
 
+class _Stream:
+  """In the place of a norm's weight: the stream is read as it is."""
+
+
+STREAM = _Stream()
+
+
 def prenorm(x, weight, eps: float, dtype: torch.dtype):
-  """x fp32 -> RMS norm with a weight around zero, in `dtype`."""
+  """x fp32 -> RMS norm with a weight around zero (STREAM: x itself), in
+  `dtype`."""
+  if weight is STREAM:
+    return x.to(dtype)
   if _on_hip(x):
     return load_hip().prenorm(x, weight, eps, dtype == torch.bfloat16)
   return ref.prenorm(x, weight, eps, dtype)
-
-
-def sandwich_norm(y, x, w_post, w_next, eps: float) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
-  """x + norm(y; w_post), and that stream's norm for the next sublayer
-  (w_next None: no norm). The stream is fp32; on the HIP path it is updated
-  in place."""
-  if _on_hip(y):
-    return x, load_hip().sandwich_norm(y, x, w_post, w_next, eps)
-  return ref.sandwich_norm(y, x, w_post, w_next, eps)
 
 
 class Weighted(NamedTuple):
@@ -85,6 +89,20 @@ class Weighted(NamedTuple):
   y: torch.Tensor
   row: torch.Tensor
   weight: torch.Tensor
+
+
+def sandwich_norm(y: Union[torch.Tensor, Weighted], x, w_post, w_next,
+                  eps: float) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+  """x + norm(y; w_post), and that stream's norm for the next sublayer
+  (w_next None: no norm; STREAM: the stream as it is). The stream is fp32; on
+  the HIP path it is updated in place."""
+  copy = w_next is STREAM
+  if isinstance(y, Weighted):
+    return x, load_hip().sandwich_norm(y.y, x, w_post, None if copy else w_next, eps, copy, y.row, y.weight)
+  if _on_hip(y):
+    return x, load_hip().sandwich_norm(y, x, w_post, None if copy else w_next, eps, copy)
+  x = ref.sandwich_norm(y, x, w_post, eps)
+  return x, None if w_next is None else prenorm(x, w_next, eps, y.dtype)
 
 
 def add_norm(y: Union[torch.Tensor, Weighted], x, mult: float, w_next, eps: float):
@@ -220,13 +238,72 @@ def _value_weights(up, H: int, dim: int):
   return up._values
 
 
-def conv_silu(proj, at: int, taps, bias, ring, rows: StepRows):
-  """Causal convolution per channel and silu over the columns of `proj` from
-  `at` on: [B, S, channels]."""
+class AttnRule(NamedTuple):
+  """Sizes and constants of rotary attention (models.mixers.RotaryAttention)."""
+  H: int
+  G: int
+  dim: int
+  vdim: int
+  maps: int          # 2: differential
+  scale: float
+  cap: float         # 0: scores are not capped
+  window: int        # 0: causal
+  keep: int          # first tokens that stay in sight of the window
+  pairs: bool        # neighbours turn together
+  late_norm: bool    # a norm without a weight after the rotation
+  eps: float
+  gain: float        # of the normed difference of the maps
+
+
+def rotary_attn(proj, q_at: int, source, rule: AttnRule, q_norm, k_norm, freq, lam, state, rows: StepRows, append: bool,
+                out=None, out_at: int = 0, out_scale: float = 1.0):
+  """Attention with rotary positions over `state`'s keys and values. source:
+  (tensor, column of the keys, column of the values), appended to the state
+  first, unless another layer has done so (`append` False). freq: radians per
+  position of each pair. lam: what the second map is weighed with."""
+  if not _on_hip(proj):
+    return ref.rotary_attn(proj, q_at, source, rule, q_norm, k_norm, freq, lam, state, rows, append) * out_scale
+  out = _out(out, proj, rule.H * rule.vdim)
+  kv, k_at, v_at = source if append else (None, 0, 0)
+  load_hip("_hip_rotary").rotary_attn(proj, q_at, kv, k_at, v_at, *rule, q_norm, k_norm, freq, lam, state[0], state[1],
+                                      rows.slots, rows.positions, rows.lens, rows.start, rows.decode, out, out_at,
+                                      out_scale)
+  return out
+
+
+def short_conv(proj, at: int, taps, bias, ring, rows: StepRows, in_bias=None, silu: bool = False):
+  """Causal convolution per channel over the columns of `proj` from `at` on
+  (plus `in_bias`; zeros come before the first token), and silu: [B, S,
+  channels]."""
   if _on_hip(proj):
-    return load_hip("_hip_scan").conv_silu(proj, at, taps, bias, ring, rows.slots, rows.positions, rows.lens,
-                                           rows.start, rows.decode)
-  return ref.conv_silu(proj, at, taps, bias, ring, rows)
+    return load_hip("_hip_scan").short_conv(proj, at, taps, bias, in_bias, silu, ring, rows.slots, rows.positions,
+                                            rows.lens, rows.start, rows.decode)
+  return ref.short_conv(proj, at, taps, bias, ring, rows, in_bias, silu)
+
+
+def conv_silu(proj, at: int, taps, bias, ring, rows: StepRows):
+  return short_conv(proj, at, taps, bias, ring, rows, silu=True)
+
+
+def gated_unit(proj, y_at: int, x_at: int, in_bias, taps, bias, gates, gate_bias, lam, rate: float, state,
+               rows: StepRows, out=None, out_at: int = 0, out_scale: float = 1.0):
+  """S = a S + sqrt(1 - a^2) i u per channel, times gelu(y). u: the convolution
+  of the columns from x_at on; y: those from y_at on; both with a row of
+  in_bias [2, W] (y, x). Gates r and i: sigmoid of block-diagonal products of u
+  (gates [2, blocks, n, n], gate_bias [2, blocks, n]); log a = -rate r
+  softplus(lam)."""
+  if not _on_hip(proj):
+    return ref.gated_unit(proj, y_at, x_at, in_bias, taps, bias, gates, gate_bias, lam, rate, state, rows) * out_scale
+  hip = load_hip("_hip_lru")
+  out = _out(out, proj, lam.numel())
+  if rows.decode:
+    hip.gated_unit_step(proj, y_at, x_at, in_bias, taps, bias, gates, gate_bias, lam, rate, state[0], state[1],
+                        rows.slots, rows.positions, out, out_at, out_scale)
+    return out
+  u = short_conv(proj, x_at, taps, bias, state[1], rows, in_bias[1])
+  hip.gated_unit(u, proj, y_at, in_bias, gates, gate_bias, lam, rate, state[0], rows.slots, rows.lens, rows.start, out,
+                 out_at, out_scale)
+  return out
 
 
 def selective_scan(x, pre, bc, b_at: int, c_at: int, z, z_at: int, a_log, dt_bias, skip, state, rows: StepRows,
@@ -244,9 +321,19 @@ def selective_scan(x, pre, bc, b_at: int, c_at: int, z, z_at: int, a_log, dt_bia
 
 # ---------------------------------------------------------------- experts
 
-def expert_mixture(h, router, correction, gate_up, down, ff: int, rule, act):
-  """Weighted sum of each token's best experts. rule: (top, groups, groups
-  kept, scale of the weights); act: (alpha, limit, plus), the gated activation
+class Routing(NamedTuple):
+  """How tokens choose experts and weigh them (models.experts)."""
+  top: int
+  groups: int
+  keep: int               # groups that stay open
+  scale: float
+  softmax: bool = False   # weights are the softmax over the chosen logits
+  shared: int = 0         # experts after the routed ones that every token uses
+
+
+def expert_mixture(h, router, correction, gate_up, down, ff: int, rule: Routing, act):
+  """Weighted sum of each token's best experts and, weighed with the sigmoid of
+  the router's last row, of the shared ones. act: (alpha, limit, plus), the gated activation
   min(g, limit) sigmoid(alpha min(g, limit)) (clamp(u, +-limit) + plus).
   gate_up [E, 2, F, K] and down [E, D, F] are padded with zeros past the model's
   width and `ff`."""

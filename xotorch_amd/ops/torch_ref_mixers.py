@@ -17,9 +17,8 @@ def prenorm(x, weight, eps, dtype):
   return (_rms(x.float(), eps) * (1.0 + weight.float())).to(dtype)
 
 
-def sandwich_norm(y, x, w_post, w_next, eps):
-  x = x + _rms(y.float(), eps) * (1.0 + w_post.float())
-  return x, None if w_next is None else prenorm(x, w_next, eps, y.dtype)
+def sandwich_norm(y, x, w_post, eps):
+  return x + _rms(y.float(), eps) * (1.0 + w_post.float())
 
 
 def add_norm(y, x, mult, w_next, eps):
@@ -253,7 +252,100 @@ def latent_attn(proj, q_at, c_at, H, dim, rot_dim, rank, vdim, norm, up, freq, s
   return _scatter(parts, proj, H * vdim)
 
 
-def conv_silu(proj, at, taps, bias, ring, rows):
+def _rotate(x, start, freq, pairs):
+  """The first 2 * len(freq) of x's last axis turn by position * freq."""
+  n = freq.numel()
+  turned, rest = x[..., :2 * n], x[..., 2 * n:]
+  if not pairs:
+    turned = turned.unflatten(-1, (2, n)).transpose(-1, -2).flatten(-2)
+  turned = _rotate_pairs(turned, start, freq)
+  if not pairs:
+    turned = turned.unflatten(-1, (n, 2)).transpose(-1, -2).flatten(-2)
+  return torch.cat([turned, rest], dim=-1)
+
+
+def _place(p, keep, rows):
+  """Row of position p: the first `keep` have their own, the rest a ring."""
+  return torch.where(p < keep, p, keep + (p - keep) % max(rows - keep, 1))
+
+
+def rotary_attn(proj, q_at, source, rule, q_norm, k_norm, freq, lam, state, rows, append):
+  r = rule
+  B, S, _ = proj.shape
+  window = r.window or 1 << 62
+
+  def heads(x, n, norm, start):
+    x = x.reshape(x.shape[0], n * r.maps, r.dim)
+    if norm is not None:
+      x = _rms(x, r.eps) * norm.float()
+    x = _rotate(x, start, freq, r.pairs)
+    return (_rms(x, r.eps) if r.late_norm else x).to(proj.dtype).float()
+
+  parts = {}
+  for b, slot, start, n in _each_row(rows, B, S):
+    q = heads(proj[b, :n, q_at:q_at + r.H * r.maps * r.dim].float(), r.H, q_norm, start)
+    at = torch.arange(start, start + n, device=proj.device)
+    if state is None or append:
+      kv, k_at, v_at = source
+      k = heads(kv[b, :n, k_at:k_at + r.G * r.maps * r.dim].float(), r.G, k_norm, start)
+      v = kv[b, :n, v_at:v_at + r.G * r.vdim].float().view(n, r.G, r.vdim)
+    seen = at
+    if state is not None:
+      kc, vc = state
+      R = kc.shape[2]
+      first = max(0, start - window + 1)
+      seen = torch.cat([torch.arange(0, min(r.keep, first), device=proj.device),
+                        torch.arange(first, start + n, device=proj.device)])
+      if append:  # of earlier tokens what the cache holds, before newer ones take their rows
+        old = _place(seen[:-n], r.keep, R)
+        k, v = (torch.cat([c[slot][:, old].transpose(0, 1).float(), t]) for c, t in ((kc, k), (vc, v)))
+        stay = (at < r.keep) | (at >= start + n - max(R - r.keep, 1))
+        new, row = torch.where(stay)[0], _place(at[stay], r.keep, R)
+        kc[slot][:, row] = k[len(old):][new].transpose(0, 1).to(kc.dtype)
+        vc[slot][:, row] = v[len(old):][new].transpose(0, 1).to(vc.dtype)
+      else:
+        here = _place(seen, r.keep, R)
+        k, v = (c[slot][:, here].transpose(0, 1).float() for c in (kc, vc))
+    dist = at[:, None] - seen[None, :]
+    open_ = (dist >= 0) & ((dist < window) | (seen < r.keep)[None])
+    per = r.H // r.G
+    k = k.unflatten(1, (r.G, r.maps)).repeat_interleave(per, dim=1)
+    s = torch.einsum("nhmd,thmd->nthm", q.unflatten(1, (r.H, r.maps)), k) * r.scale
+    if r.cap:
+      s = r.cap * torch.tanh(s / r.cap)
+    p = torch.softmax(s.masked_fill(~open_[:, :, None, None], float("-inf")), dim=1)
+    o = torch.einsum("nthm,the->nhme", p, v.repeat_interleave(per, dim=1))
+    o = o[:, :, 0] if r.maps == 1 else _rms(o[:, :, 0] - lam * o[:, :, 1], r.eps) * r.gain
+    parts[b] = o.reshape(n, r.H * r.vdim)
+  return _scatter(parts, proj, r.H * r.vdim)
+
+
+def gated_unit(proj, y_at, x_at, in_bias, taps, bias, gates, gate_bias, lam, rate, state, rows):
+  B, S, _ = proj.shape
+  W = lam.numel()
+  s, ring = state if state is not None else (None, None)
+  u_all = short_conv(proj, x_at, taps, bias, ring, rows, in_bias[1], False)
+  parts = {}
+  for b, slot, start, n in _each_row(rows, B, S):
+    u = u_all[b, :n].float()
+    blocks = u.view(n, gates.shape[1], -1)
+    r, i = (torch.sigmoid(torch.einsum("nbk,bjk->nbj", blocks, g.float()) + c.float()).reshape(n, W)
+            for g, c in zip(gates, gate_bias))
+    log_a = -rate * r * F.softplus(lam.float())
+    a, x = torch.exp(log_a), torch.sqrt(-torch.expm1(2 * log_a)) * i * u
+    M = x.new_zeros(W) if s is None or start == 0 else s[slot].clone()
+    outs = []
+    for t in range(n):
+      M = a[t] * M + x[t]
+      outs.append(M)
+    y = proj[b, :n, y_at:y_at + W].float() + in_bias[0].float()
+    parts[b] = torch.stack(outs) * F.gelu(y, approximate="tanh")
+    if s is not None:
+      s[slot] = M
+  return _scatter(parts, proj, W)
+
+
+def short_conv(proj, at, taps, bias, ring, rows, in_bias, silu):
   B, S, _ = proj.shape
   C, n_taps = taps.shape
   parts = {}
@@ -264,7 +356,11 @@ def conv_silu(proj, at, taps, bias, ring, rows):
     else:
       hist = _history(ring, slot, start, n_taps - 1)
     full = torch.cat([hist, x.float()])
-    parts[b] = F.silu(sum(full[j:j + n] * taps[:, j].float() for j in range(n_taps)) + bias.float())
+    if in_bias is not None:
+      before = min(n_taps - 1, 0 if ring is None else start)  # tokens there are
+      full = torch.cat([full[:n_taps - 1 - before], full[n_taps - 1 - before:] + in_bias.float()])
+    y = sum(full[j:j + n] * taps[:, j].float() for j in range(n_taps)) + bias.float()
+    parts[b] = F.silu(y) if silu else y
     if ring is not None:
       _remember(ring, slot, start, x)
   return _scatter(parts, proj, C)
@@ -292,27 +388,33 @@ def selective_scan(x, pre, bc, b_at, c_at, z, z_at, a_log, dt_bias, skip, state,
 
 
 def expert_mixture(h, router, correction, gate_up, down, ff, rule, act):
-  top, groups, keep, scale = rule
+  top, groups, keep, scale, softmax, shared = rule
   alpha, limit, plus = act
-  D, E = h.shape[-1], router.shape[0]
+  D, E = h.shape[-1], router.shape[0] - bool(shared)
   flat = h.reshape(-1, D)
-  scores = torch.sigmoid(flat.float() @ router.float().t())
-  choice = scores.detach() + correction.float()
+  z = flat.float() @ router.float().t()
+  z, open_ = z[:, :E], torch.sigmoid(z[:, E:])
+  scores = z if softmax else torch.sigmoid(z)
+  choice = scores.detach() if correction is None else scores.detach() + correction.float()
   if keep < groups:
     by_group = choice.view(-1, groups, E // groups)
     score = by_group.topk(min(2, E // groups), dim=-1).values.sum(-1)
     kept = torch.zeros_like(score, dtype=torch.bool).scatter_(1, score.topk(keep, dim=-1).indices, True)
     choice = by_group.masked_fill(~kept[:, :, None], float("-inf")).flatten(1)
   idx = choice.topk(top, dim=-1).indices
-  weight = scores.gather(1, idx) * scale
+  weight = scores.gather(1, idx)
+  weight = (torch.softmax(weight, dim=-1) if softmax else weight) * scale
+  if shared:
+    idx = torch.cat([idx, torch.arange(E, E + shared, device=h.device).expand(len(idx), -1)], dim=1)
+    weight = torch.cat([weight, open_.expand(-1, shared)], dim=1)
   out = torch.zeros(flat.shape[0], D, dtype=torch.float32, device=h.device)
-  for e in range(E):
+  for e in range(E + shared):
     tok, k = torch.where(idx == e)
     if tok.numel() == 0:
       continue
-    x = flat[tok]
-    g, u = (F.linear(x, gate_up[e, i, :ff, :D]).float() for i in (0, 1))
+    x, F_ = flat[tok], ff if e < E else gate_up.shape[2]
+    g, u = (F.linear(x, gate_up[e, i, :F_, :D]).float() for i in (0, 1))
     g, u = g.clamp(max=limit), u.clamp(-limit, limit)
     a = (g * torch.sigmoid(alpha * g) * (u + plus)).to(h.dtype)
-    out = out.index_add(0, tok, F.linear(a, down[e, :D, :ff]).float() * weight[tok, k, None])
+    out = out.index_add(0, tok, F.linear(a, down[e, :D, :F_]).float() * weight[tok, k, None])
   return out.to(h.dtype).view(h.shape)

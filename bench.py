@@ -90,7 +90,31 @@ def _lebotar_pair(model_id):
   return [(model_id, cfg), ("deepseek of that size", like)]
 
 
-DESIGNS = {"didipel": _didipel_pair, "lebotar": _lebotar_pair}
+def _tapupel_pair(model_id):
+  """The registry's Tapupel of that size, and lebotar (local attention, latent
+  attention, selective scan, sparse feed-forwards) with the same width, depth,
+  heads, experts, vocabulary. It has no shared experts."""
+  from xotorch_amd.models.registry import builtin_config
+  cfg = builtin_config(model_id)
+  att = next(e["mixer"] for e in cfg["layers"] if e["type"] == "attention")
+  moe = cfg["layers"][0]["mlp"]
+  width, dim = cfg["width"], att["dim"]
+  like = {
+    "attention": ("attention", {"heads": att["heads"], "kv_heads": att["kv_heads"], "dim": dim, "vdim": dim,
+                                "scale": dim ** -0.5, "v_mix": False, "mask": {"size": att["mask"]["size"]}}),
+    "attention_2": ("latent_attention", {"heads": att["heads"], "dim": dim, "rot_dim": dim // 2, "vdim": dim,
+                                         "kv_rank": 4 * dim, "rot": {"base": 10000.0, "dims": dim // 2},
+                                         "scale": (dim + dim // 2) ** -0.5}),
+    "rglru": ("mamba1", {"inner": 2 * width, "state": 16, "conv": 4, "dt_rank": width // 16}),
+  }
+  mlp = {"kind": "moe", "expert": {"ff": moe["expert"]["ff"], "limit": 7.0},
+         "router": {**moe["router"], "scale": 2.5, "groups": {"count": 8, "keep": 4}}}
+  return [(model_id, cfg), ("lebotar of that size", {
+    "architecture": "Lebotar", "vocab": cfg["vocab"], "width": width, "norm": cfg["norm"], "residual_mult": 0.5,
+    "layers": [{"type": like[e["type"]][0], "mixer": like[e["type"]][1], "mlp": mlp} for e in cfg["layers"]]})]
+
+
+DESIGNS = {"didipel": _didipel_pair, "lebotar": _lebotar_pair, "tapupel": _tapupel_pair}
 
 
 def design_bench(args):

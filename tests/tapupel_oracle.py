@@ -77,16 +77,16 @@ def attention(q, k, v, scale, mask=None, cap=None):
   """q [T,H,d], k [T,G,d], v [T,G,e]."""
   T, H, _ = q.shape
   per = H // k.shape[1]
-  out = q.new_zeros(T, H, v.shape[2])
-  for i in range(T):
-    js = torch.tensor([j for j in range(i + 1) if sees(i, j, mask)])
-    for h in range(H):
-      s = k[js, h // per] @ q[i, h] * scale
-      if cap is not None:
-        s = cap * torch.tanh(s / cap)
-      e = torch.exp(s - s.max())
-      out[i, h] = (e / e.sum()) @ v[js, h // per]
-  return out
+  open_ = torch.tensor([[sees(i, j, mask) for j in range(T)] for i in range(T)])
+  out = []
+  for h in range(H):
+    s = q[:, h] @ k[:, h // per].T * scale
+    if cap is not None:
+      s = cap * torch.tanh(s / cap)
+    s = torch.where(open_, s, -torch.inf)
+    e = torch.exp(s - s.max(dim=1, keepdim=True).values)
+    out.append((e / e.sum(dim=1, keepdim=True)) @ v[:, h // per])
+  return torch.stack(out, dim=1)
 
 
 def window_mixer(h, w, p, m, eps, kept):

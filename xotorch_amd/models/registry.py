@@ -168,6 +168,36 @@ def _lebotar_sized(width, order, experts, top, ff=1408, vocab=32000, dim=128, ch
          "router": {"experts": experts, "top": top, "scale": 2.5, "groups": {"count": 8, "keep": 4}}})
 
 
+def _tapupel_cfg(width, order, vocab, attention, difference, rglru, moe, dense=None, scale=1.0, eps=1e-6):
+  """order: one letter a layer, a(ttention), d(ifference attention), x (the
+  same with the keys and values of the last d) or r(glru); capitals have the
+  dense feed-forward or none."""
+  kinds = {"a": ("attention", attention), "d": ("attention_2", difference), "r": ("rglru", rglru)}
+  layers = []
+  for i, c in enumerate(order):
+    kind, mixer = kinds["d" if c in "xX" else c.lower()]
+    if c in "xX":
+      mixer = {**mixer, "kv_from": max(order.rfind(d, 0, i) for d in "dD")}
+    layers.append({"type": kind, "mixer": mixer, "mlp": dense if c.isupper() else moe})
+  return {"architecture": "Tapupel", "vocab": vocab, "width": width, "norm": {"eps": eps},
+          "embedding": {"scale": scale}, "layers": layers}
+
+
+def _tapupel_sized(width, order, experts, top, ff=1408, vocab=32000, dim=128, window=1024):
+  """Real-model proportions: heads and the recurrence span the width."""
+  heads = width // dim
+  return _tapupel_cfg(
+    width, order, vocab,
+    attention={"heads": heads, "kv_heads": heads // 4, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "softcap": 50.0,
+               "mask": {"size": window, "keep_first": 16},
+               "rot": {"base": 500000.0, "dims": dim,
+                       "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+    difference={"heads": heads // 2, "kv_heads": heads // 8, "dim": dim, "vdim": 2 * dim, "scale": dim ** -0.5, "diff": 0.8,
+                "rot": {"base": 500000.0, "dims": dim}},
+    rglru={"width": width, "blocks": heads, "conv": 4},
+    moe={"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff}})
+
+
 BUILTIN_CONFIGS: Dict[str, dict] = {
   # llama 3.x family
   "llama-3.2-1b": _llama_cfg(2048, 16, 32, 8, 8192, tie=True, llama3_scaling=True, head_dim=64),
@@ -261,6 +291,19 @@ BUILTIN_CONFIGS: Dict[str, dict] = {
     latent={"heads": 3, "dim": 20, "rot_dim": 8, "vdim": 28, "kv_rank": 36, "rot": {"base": 1000.0, "dims": 8}, "scale": 0.19},
     moe={"kind": "moe", "expert": {"ff": 40, "limit": 2.0},
          "router": {"experts": 6, "top": 2, "scale": 1.2, "groups": {"count": 3, "keep": 2}}}),
+  # tapupel, likewise (3B: 32 experts, 9B: 64 experts a layer)
+  "tapupel-3b": _tapupel_sized(2048, "rradrrax", 32, 4),
+  "tapupel-9b": _tapupel_sized(2048, "rradrrax" * 2, 64, 6),
+  "tapupel-dummy": _tapupel_cfg(
+    80, "drAxR", 256, scale=3.0,
+    attention={"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 24, "scale": 0.2, "softcap": 20.0,
+               "mask": {"size": 12, "keep_first": 2},
+               "rot": {"base": 1000.0, "dims": 16, "scaling": {"factor": 4.0, "low": 1.0, "high": 3.0, "original": 64}}},
+    difference={"heads": 4, "kv_heads": 2, "dim": 20, "vdim": 28, "scale": 0.22, "diff": 0.3,
+                "rot": {"base": 1000.0, "dims": 12}},
+    rglru={"width": 96, "blocks": 6, "conv": 4},
+    moe={"kind": "moe", "expert": {"ff": 40}, "router": {"experts": 6, "top": 2}, "shared": {"ff": 72}},
+    dense={"kind": "dense", "ff": 104}),
   "dummy": _llama_cfg(64, 4, 4, 2, 128, vocab=256, theta=10000.0, max_pos=256, tie=True),
 }
 # DeepSeek-Coder-V2-Lite shares the V2-Lite architecture exactly
@@ -330,6 +373,9 @@ model_cards: Dict[str, dict] = {
   "lebotar-3b": {"layers": 8, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "lebotar-9b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "lebotar-dummy": {"layers": 4, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "tapupel-3b": {"layers": 8, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "tapupel-9b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "tapupel-dummy": {"layers": 5, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "dummy": {"layers": 4, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy", "DummyEngine": "dummy"}},
 }
 
@@ -386,6 +432,9 @@ pretty_names = {
   "lebotar-3b": "Lebotar 3B (random weights)",
   "lebotar-9b": "Lebotar 9B (random weights)",
   "lebotar-dummy": "Lebotar dummy (test)",
+  "tapupel-3b": "Tapupel 3B (random weights)",
+  "tapupel-9b": "Tapupel 9B (random weights)",
+  "tapupel-dummy": "Tapupel dummy (test)",
   "dummy": "Dummy (test)",
 }
 

@@ -20,7 +20,7 @@
 // ---------------------------------------------------------------------------
 
 constexpr int RT = 16;          // tokens of a router block
-constexpr int MAX_EXPERTS = 512, MAX_TOP = 16;
+constexpr int MAX_EXPERTS = 512, MAX_PICK = 16;  // shared ones among the experts
 
 // pick of E experts are chosen, then come top - pick that every token uses, all
 // in all; tile: rows of a tile
@@ -144,12 +144,12 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
       mine = e / row_sum(e);
     }
     if (valid && l < a.pick) weight[(size_t)(t0 + t) * a.top + l] = mine * a.scale;
-    if (l >= a.pick && l < a.top) {
-      const int e = a.E + l - a.pick;
-      chosen[t * a.top + l] = valid ? e : -1;
+    for (int k = a.pick + l; k < a.top; k += 16) {
+      const int e = a.E + k - a.pick;
+      chosen[t * a.top + k] = valid ? e : -1;
       if (valid) {
-        idx[(size_t)(t0 + t) * a.top + l] = e;
-        weight[(size_t)(t0 + t) * a.top + l] = open[t];
+        idx[(size_t)(t0 + t) * a.top + k] = e;
+        weight[(size_t)(t0 + t) * a.top + k] = open[t];
       }
     }
   }
@@ -528,7 +528,7 @@ std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tens
   if (correction) { check_io(*correction, dt); CHK(correction->numel() == E); }
   CHK(w.dim() == 2 && w.size(1) == D && T_ > 0 && shared >= 0);
   const int64_t top = pick + shared, all = E + shared;
-  TORCH_CHECK(E >= 1 && all <= MAX_EXPERTS && pick >= 1 && top <= MAX_TOP && pick <= E, "routing to ", pick, " of ", E,
+  TORCH_CHECK(E >= 1 && all <= MAX_EXPERTS && pick >= 1 && pick <= MAX_PICK && pick <= E, "routing to ", pick, " of ", E,
               " experts and ", shared, " shared ones");
   TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && pick <= keep * (E / groups),
               "routing to ", pick, " experts of ", keep, " of ", groups, " groups of ", E, " experts");

@@ -315,7 +315,7 @@ def test_reading_the_keys_and_values_of_another(kind):
 # ---------------------------------------------------------------- gated linear recurrence
 
 UNIT = [  # channels, blocks, taps
-  (40, 4, 3), (64, 1, 1), (96, 3, 4), (33, 11, 2), (128, 2, 5), (512, 1, 4), (260, 2, 4), (70, 7, 6), (12, 12, 2)]
+  (40, 4, 3), (64, 1, 1), (96, 3, 4), (33, 11, 2), (128, 2, 5), (512, 1, 4), (260, 2, 4), (256, 2, 4), (70, 7, 6), (12, 12, 2)]
 
 
 class Unit:
@@ -390,12 +390,13 @@ def test_gated_unit_rows_are_independent(kind, shape):
 
 
 @on
+@pytest.mark.parametrize("shape", [(24, 2, 4), (256, 2, 3)])
 @pytest.mark.parametrize("cuts", [(), (70,), (250,)])
-def test_gated_unit_of_long_prompts_in_segments(kind, cuts):
+def test_gated_unit_of_long_prompts_in_segments(kind, shape, cuts):
   """Few channels and many tokens: rows are walked in segments side by side,
   also rows that end in an early one."""
   T = 400
-  ops = [Unit(kind, (24, 2, 4), T, seed=s) for s in (0, 9)]
+  ops = [Unit(kind, shape, T, seed=s) for s in (0, 9)]
   want = [op.expected() for op in ops]
   state, p = ops[0].state(), 0
   for t in state:

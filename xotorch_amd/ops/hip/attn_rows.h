@@ -111,7 +111,26 @@ __global__ __launch_bounds__(256) void attn_rows_prefill_kernel(
   const int t0 = max(0, hist + s0 + 1 - reach_of<MODE>(a, step.start + s0)) >> 5;
   const int t1 = (hist + min(s0 + QT * 16 - 1, a.S - 1)) >> 5;
   const int kept = MODE == KEPT ? (a.keep + 31) >> 5 : 0;  // tiles of the first tokens
-  for (int tile = kept ? 0 : t0; tile <= t1; tile = MODE == KEPT && tile + 1 >= kept && tile + 1 < t0 ? t0 : tile + 1) {
+  // two maps leave room for one wave a SIMD: keys are loaded a tile ahead, values
+  // before the softmax
+  constexpr bool AHEAD = MAPS == 2 && KC <= 4;
+  bf16x8 kf[2][MAPS][KC];
+  auto load_keys = [&](int tile) {
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+        if (EXACT || c < kc)
+#pragma unroll
+          for (int mp = 0; mp < MAPS; ++mp)
+            kf[hf][mp][c] = *(const bf16x8*)(kb[mp] + ((size_t)(tile * 2 + hf) * kc + c) * 512 + lane * 8);
+  };
+  int next = kept ? 0 : t0;
+  if (AHEAD) load_keys(next);
+  while (next <= t1) {
+    const int tile = next;
+    if (!AHEAD) load_keys(tile);
+    next = MODE == KEPT && tile + 1 >= kept && tile + 1 < t0 ? t0 : tile + 1;
     floatx4 sc[NT][2];
 #pragma unroll
     for (int hf = 0; hf < 2; ++hf) {
@@ -121,12 +140,19 @@ __global__ __launch_bounds__(256) void attn_rows_prefill_kernel(
       for (int c = 0; c < KC; ++c)
         if (EXACT || c < kc)
 #pragma unroll
-          for (int mp = 0; mp < MAPS; ++mp) {
-            const bf16x8 kf = *(const bf16x8*)(kb[mp] + ((size_t)(tile * 2 + hf) * kc + c) * 512 + lane * 8);
+          for (int mp = 0; mp < MAPS; ++mp)
 #pragma unroll
             for (int t = mp * QT; t < mp * QT + QT; ++t)
-              sc[t][hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[t][c], sc[t][hf], 0, 0, 0);
-          }
+              sc[t][hf] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[hf][mp][c], qf[t][c], sc[t][hf], 0, 0, 0);
+    }
+    bf16x8 vf[VG];
+    auto load_value = [&](int i) { vf[i] = *(const bf16x8*)(vb + (size_t)i * vstride + (size_t)tile * 512 + lane * 8); };
+    if (AHEAD) {
+#pragma unroll
+      for (int i = 0; i < VG; ++i)
+        if (EXACT || i < vg) load_value(i);
+      load_keys(min(next, t1));
+      __builtin_amdgcn_sched_barrier(0);
     }
     bf16x8 pf[NT];
 #pragma unroll
@@ -170,9 +196,9 @@ __global__ __launch_bounds__(256) void attn_rows_prefill_kernel(
 #pragma unroll
     for (int i = 0; i < VG; ++i)
       if (EXACT || i < vg) {
-        const bf16x8 vf = *(const bf16x8*)(vb + (size_t)i * vstride + (size_t)tile * 512 + lane * 8);
+        if (!AHEAD) load_value(i);
 #pragma unroll
-        for (int t = 0; t < NT; ++t) o[t][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[t], o[t][i], 0, 0, 0);
+        for (int t = 0; t < NT; ++t) o[t][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i], pf[t], o[t][i], 0, 0, 0);
       }
   }
   const int len = step.slot(b) < 0 ? 0 : step.len(b, a.S);
@@ -387,48 +413,51 @@ __global__ __launch_bounds__(256) void attn_rows_decode_kernel(
   }
 }
 
+// Partial results of a head's splits -> its output. Four waves take splits in
+// turn, then a thread has a value column.
 template <int MODE, int MAPS = 1>
-__global__ __launch_bounds__(64) void attn_rows_merge_kernel(
+__global__ __launch_bounds__(256) void attn_rows_merge_kernel(
     const float* __restrict__ part, Side<MODE, bf16_t> side, bf16_t* __restrict__ out, int splits,
     int vdim, AttnArgs a, Step step) {
-  const int h = blockIdx.x, b = blockIdx.y;
-  const bool live = step.slot(b) >= 0;
+  __shared__ float po[4][256], pl[4], sums[4];
+  const int h = blockIdx.x, b = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   constexpr int NC = 4;  // value columns of a lane
-  float v[NC], ss = 0.f;
-#pragma unroll
-  for (int i = 0; i < NC; ++i) v[i] = 0.f;
-  if (live)
+  float v = 0.f;
+  if (step.slot(b) >= 0)
 #pragma unroll
     for (int mp = 0; mp < MAPS; ++mp) {
+      const size_t row = ((size_t)b * splits * a.H + h) * MAPS + mp, stride = (size_t)a.H * MAPS;
       float M = side.start(h), L = 0.f, O[NC];
+      for (int s = lane; s < splits; s += 64) M = fmaxf(M, part[(row + s * stride) * (vdim + 2)]);
+#pragma unroll
+      for (int d = 1; d < 64; d <<= 1) M = fmaxf(M, __shfl_xor(M, d));
 #pragma unroll
       for (int i = 0; i < NC; ++i) O[i] = 0.f;
-      const size_t row = ((size_t)b * splits * a.H + h) * MAPS + mp, stride = (size_t)a.H * MAPS;
-      for (int s = 0; s < splits; ++s) M = fmaxf(M, part[(row + s * stride) * (vdim + 2)]);
-      for (int s = 0; s < splits; ++s) {
+#pragma unroll 4
+      for (int s = wave; s < splits; s += 4) {
         const float* p = part + (row + s * stride) * (vdim + 2);
         const float f = __expf(p[0] - M);
         L += f * p[1];
 #pragma unroll
-        for (int i = 0; i < NC; ++i)
-          if (threadIdx.x + i * 64 < vdim) O[i] += f * p[2 + threadIdx.x + i * 64];
+        for (int i = 0; i < NC; ++i) O[i] += f * p[2 + min(lane + i * 64, vdim - 1)];
       }
-      const float f = MAPS == 1 ? side.gate(a, b, h) / (L + __expf(side.sink(h) - M)) : mp ? -*a.lam / L : 1.f / L;
+      if (mp) __syncthreads();
 #pragma unroll
-      for (int i = 0; i < NC; ++i) v[i] += O[i] * f;
+      for (int i = 0; i < NC; ++i) po[wave][i * 64 + lane] = O[i];
+      if (lane == 0) pl[wave] = L;
+      __syncthreads();
+      L = pl[0] + pl[1] + pl[2] + pl[3];
+      const float f = MAPS == 1 ? side.gate(a, b, h) / (L + __expf(side.sink(h) - M)) : mp ? -*a.lam / L : 1.f / L;
+      v += f * (po[0][threadIdx.x] + po[1][threadIdx.x] + po[2][threadIdx.x] + po[3][threadIdx.x]);
     }
   if (MAPS == 2) {
-#pragma unroll
-    for (int i = 0; i < NC; ++i) ss += v[i] * v[i];
-    const float f = a.gain / sqrtf(wave_sum(ss) / (float)vdim + a.eps) * side.gate(a, b, h);
-#pragma unroll
-    for (int i = 0; i < NC; ++i) v[i] *= f;
+    const float ss = wave_sum(threadIdx.x < vdim ? v * v : 0.f);
+    if (lane == 0) sums[wave] = ss;
+    __syncthreads();
+    v *= a.gain / sqrtf((sums[0] + sums[1] + sums[2] + sums[3]) / (float)vdim + a.eps) * side.gate(a, b, h);
   }
-#pragma unroll
-  for (int i = 0; i < NC; ++i) {
-    const int c = threadIdx.x + i * 64;
-    if (c < vdim) st(out + (size_t)b * a.K + a.out_at + (size_t)h * vdim + c, v[i]);
-  }
+  const int c = threadIdx.x;
+  if (c < vdim) st(out + (size_t)b * a.K + a.out_at + (size_t)h * vdim + c, v);
 }
 
 // 32-bit attention, one wave per (token, head): lanes over keys for the
@@ -609,7 +638,7 @@ static inline void decode_rows(bool bf, int B, const Tensor& qw, const Tensor& k
   else { BY_DIMS(ring.kc, ring.vg, RUN) }
 #undef RUN
   if (splits > 1)
-    hipLaunchKernelGGL((attn_rows_merge_kernel<MODE, MAPS>), dim3(a.H, B), dim3(64), 0, stream, pp, side, M<bf16_t>(out),
+    hipLaunchKernelGGL((attn_rows_merge_kernel<MODE, MAPS>), dim3(a.H, B), dim3(256), 0, stream, pp, side, M<bf16_t>(out),
                        splits, ring.vdim, a, step);
 }
 

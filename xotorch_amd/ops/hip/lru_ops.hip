@@ -20,88 +20,135 @@ struct UnitArgs { int S, W, n, N, y_at, x_at, taps, K, out_at; float rate, out_s
 // 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) as z sigmoid(2 sqrt(2/pi) (..))
 DEVINL float gelu_tanh(float z) { return z * sigmoidf(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
 
-// gates before the sigmoid -> decay and what enters the state
-DEVINL void decay_of(float zr, float zi, float u, float lam, float rate, float& a, float& x) {
-  const float r = 1.f / (1.f + expf(-zr)), i = 1.f / (1.f + expf(-zi));
-  const float log_a = -rate * r * (fmaxf(lam, 0.f) + log1pf(expf(-fabsf(lam))));
-  a = expf(log_a);
-  x = sqrtf(-expm1f(2.f * log_a)) * i * u;
+DEVINL float softplus_of(float lam) { return fmaxf(lam, 0.f) + log1pf(expf(-fabsf(lam))); }
+
+// 1 - exp(-x), x >= 0: the series where the difference would cancel
+DEVINL float one_minus_exp(float x) {
+  const float series = x * (1.f - x * (1.f / 2) * (1.f - x * (1.f / 3) * (1.f - x * (1.f / 4) * (1.f - x * (1.f / 5) *
+                       (1.f - x * (1.f / 6))))));
+  return x < 0.25f ? series : 1.f - __expf(-x);
 }
 
-// A wave makes both gates of 32 channels of a part for 32 tokens; the block's
-// four waves take tokens side by side. u [T, W]; gates [2, parts, n, n].
-template <typename T, bool WHOLE>
+// gates before the sigmoid -> decay and what enters the state; most: the
+// decay's logarithm at an open gate, negated
+DEVINL void decay_of(float zr, float zi, float u, float most, float& a, float& x) {
+  const float fall = most * sigmoidf(zr);
+  a = __expf(-fall);
+  x = __builtin_amdgcn_sqrtf(one_minus_exp(2.f * fall)) * sigmoidf(zi) * u;
+}
+
+// A wave makes both gates of 32 channels of a part for GROUPS times 32 tokens;
+// the block's four waves take neighbouring channels, so that the tokens they
+// read are the same and what they write is contiguous. u [T, W]; gates [2,
+// parts, n, n]. HELD: k steps whose gate rows stay in registers (0: none).
+constexpr int GROUPS = 4;
+template <typename T, bool WHOLE, int HELD>
 __global__ __launch_bounds__(256) void gates_kernel(
     const T* __restrict__ u, const T* __restrict__ gates, const T* __restrict__ bias, const T* __restrict__ lam,
     float* __restrict__ decay, float* __restrict__ input, int tokens, UnitArgs a) {
   typedef Frag<T> F;
-  const int tiles = (a.n + 31) / 32, part = blockIdx.x / tiles, c0 = blockIdx.x % tiles * 32;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
-  const int t0 = (blockIdx.y * 4 + wave) * 32;
-  if (t0 >= tokens) return;
-  const T *ur[2], *wr[2][2];
+  const int tiles = (a.n + 31) / 32, unit = blockIdx.y * 4 + wave, part = unit / tiles, c0 = unit % tiles * 32;
+  if (unit >= a.W / a.n * tiles) return;
+  const T* wr[2][2];
 #pragma unroll
-  for (int j = 0; j < 2; ++j) {
-    ur[j] = u + (size_t)min(t0 + j * 16 + col, tokens - 1) * a.W + part * a.n;
+  for (int j = 0; j < 2; ++j)
 #pragma unroll
     for (int g = 0; g < 2; ++g)
       wr[g][j] = gates + ((size_t)g * a.W + part * a.n + min(c0 + j * 16 + col, a.n - 1)) * a.n;
-  }
-  floatx4 acc[2][2][2];  // gate, channels, tokens
+  typename F::V held[HELD ? HELD : 1][2][2];
+  if (HELD)
 #pragma unroll
-  for (int g = 0; g < 2; ++g)
+    for (int s = 0; s < HELD; ++s)
+#pragma unroll
+      for (int g = 0; g < 2; ++g)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) held[s][g][j] = ld_frag<T, WHOLE>(wr[g][j], s * F::K + quad * F::PER, a.n);
+  float br[2][4], bi[2][4], most[2][4];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int c = part * a.n + min(c0 + i * 16 + quad * 4 + r, a.n - 1);
+      br[i][r] = ld(bias + c);
+      bi[i][r] = ld(bias + a.W + c);
+      most[i][r] = a.rate * softplus_of(ld(lam + c));
+    }
+  const bool vec = WHOLE || (a.n & 3) == 0;
+  for (int group = 0; group < GROUPS; ++group) {
+    const int t0 = (blockIdx.x * GROUPS + group) * 32;
+    if (t0 >= tokens) return;
+    const T* ur[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) ur[j] = u + (size_t)min(t0 + j * 16 + col, tokens - 1) * a.W + part * a.n;
+    float uv[2][2][4];  // u of this lane's channels and tokens
 #pragma unroll
     for (int i = 0; i < 2; ++i)
 #pragma unroll
-      for (int j = 0; j < 2; ++j) acc[g][i][j] = (floatx4)(0.f);
-#pragma unroll 2
-  for (int k = quad * F::PER; k - quad * F::PER < a.n; k += F::K) {
-    typename F::V uf[2], wf[2][2];
+      for (int j = 0; j < 2; ++j) {
+        const int cl = c0 + i * 16 + quad * 4;
+        if (vec) ld4(ur[j] + min(cl, a.n - 4), uv[i][j]);
+        else
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      uf[j] = ld_frag<T, WHOLE>(ur[j], k, a.n);
-#pragma unroll
-      for (int g = 0; g < 2; ++g) wf[g][j] = ld_frag<T, WHOLE>(wr[g][j], k, a.n);
-    }
+          for (int r = 0; r < 4; ++r) uv[i][j][r] = ld(ur[j] + min(cl + r, a.n - 1));
+      }
+    floatx4 acc[2][2][2];  // gate, channels, tokens
 #pragma unroll
     for (int g = 0; g < 2; ++g)
 #pragma unroll
       for (int i = 0; i < 2; ++i)
 #pragma unroll
-        for (int j = 0; j < 2; ++j) acc[g][i][j] = mma(wf[g][i], uf[j], acc[g][i][j]);
-  }
+        for (int j = 0; j < 2; ++j) acc[g][i][j] = (floatx4)(0.f);
+    auto step = [&](const typename F::V (&wf)[2][2], const typename F::V (&uf)[2]) {
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int cl = c0 + i * 16 + quad * 4, c = part * a.n + cl;
-    if (cl >= a.n) continue;
-    const bool vec = WHOLE || ((a.n & 3) == 0);
-    float br[4], bi[4], lm[4];
+      for (int g = 0; g < 2; ++g)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int cc = min(c + r, a.W - 1);
-      br[r] = ld(bias + cc);
-      bi[r] = ld(bias + a.W + cc);
-      lm[r] = ld(lam + cc);
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int j = 0; j < 2; ++j) acc[g][i][j] = mma(wf[g][i], uf[j], acc[g][i][j]);
+    };
+    if (HELD) {
+      typename F::V uf[HELD ? HELD : 1][2];
+#pragma unroll
+      for (int s = 0; s < HELD; ++s)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) uf[s][j] = ld_frag<T, WHOLE>(ur[j], s * F::K + quad * F::PER, a.n);
+#pragma unroll
+      for (int s = 0; s < HELD; ++s) step(held[s], uf[s]);
+    } else {
+#pragma unroll 2
+      for (int k = quad * F::PER; k - quad * F::PER < a.n; k += F::K) {
+        typename F::V uf[2], wf[2][2];
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+          uf[j] = ld_frag<T, WHOLE>(ur[j], k, a.n);
+#pragma unroll
+          for (int g = 0; g < 2; ++g) wf[g][j] = ld_frag<T, WHOLE>(wr[g][j], k, a.n);
+        }
+        step(wf, uf);
+      }
     }
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
       const int t = t0 + j * 16 + col;
       if (t >= tokens) continue;
-      const size_t at = (size_t)t * a.W + c;
-      float uv[4], dv[4], xv[4];
-      if (vec) ld4(u + at, uv);
-      else
 #pragma unroll
-        for (int r = 0; r < 4; ++r) uv[r] = cl + r < a.n ? ld(u + at + r) : 0.f;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) decay_of(acc[0][i][j][r] + br[r], acc[1][i][j][r] + bi[r], uv[r], lm[r], a.rate, dv[r], xv[r]);
-      if (vec) {
-        st4(decay + at, dv);
-        st4(input + at, xv);
-      } else
+      for (int i = 0; i < 2; ++i) {
+        const int cl = c0 + i * 16 + quad * 4;
+        if (cl >= a.n) continue;
+        const size_t at = (size_t)t * a.W + part * a.n + cl;
+        float dv[4], xv[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (cl + r < a.n) { decay[at + r] = dv[r]; input[at + r] = xv[r]; }
+          decay_of(acc[0][i][j][r] + br[i][r], acc[1][i][j][r] + bi[i][r], uv[i][j][r], most[i][r], dv[r], xv[r]);
+        if (vec) {
+          st4(decay + at, dv);
+          st4(input + at, xv);
+        } else
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            if (cl + r < a.n) { decay[at + r] = dv[r]; input[at + r] = xv[r]; }
+      }
     }
   }
 }
@@ -173,80 +220,119 @@ __global__ __launch_bounds__(256) void segment_starts_kernel(const float* __rest
   const int c = blockIdx.x * 256 + threadIdx.x, b = blockIdx.y, slot = step.slot(b);
   if (c >= W) return;
   float S = slot >= 0 && step.start > 0 ? state[(size_t)slot * W + c] : 0.f;
-#pragma unroll 4
-  for (int s = 0; s < nseg; ++s) {
-    const size_t at = ((size_t)b * nseg + s) * W + c;
-    const float own = seg_state[at], d = seg_decay[at];
-    seg_state[at] = S;
-    S = d * S + own;
+  constexpr int AHEAD = 16;  // segments in flight
+  for (int s0 = 0; s0 < nseg; s0 += AHEAD) {
+    float own[AHEAD], d[AHEAD];
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j) {
+      const size_t at = ((size_t)b * nseg + min(s0 + j, nseg - 1)) * W + c;
+      own[j] = seg_state[at];
+      d[j] = seg_decay[at];
+    }
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (s0 + j < nseg) {
+        seg_state[((size_t)b * nseg + s0 + j) * W + c] = S;
+        S = d[j] * S + own[j];
+      }
   }
 }
 
 // Decode: 16 rows x 64 channels of a part. The convolution of the part's
 // channels goes through LDS 256 at a time; a wave makes both gates of 16
-// channels for all rows.
-template <typename T>
+// channels for all rows. What does not hang on the convolution is loaded before
+// it. TAPS 0: any number of taps.
+template <typename T, int TAPS>
 __global__ __launch_bounds__(256) void unit_step_kernel(
     const T* __restrict__ proj, const T* __restrict__ in_bias, const T* __restrict__ taps, const T* __restrict__ conv_bias,
     const T* __restrict__ gates, const T* __restrict__ bias, const T* __restrict__ lam, float* __restrict__ state,
     T* __restrict__ ring, T* __restrict__ out, int B, UnitArgs a, Step step) {
   typedef Frag<T> F;
-  constexpr int CH = 256, LD = CH + 16 / (int)sizeof(T);
+  constexpr int CH = 256, LD = CH + 16 / (int)sizeof(T), PRE = 4;
   __shared__ __attribute__((aligned(16))) T us[16][LD];
   __shared__ int slots[16], pos[16];
   const int tiles = (a.n + 63) / 64, part = blockIdx.x / tiles, b0 = blockIdx.y * 16;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
   const int cl0 = blockIdx.x % tiles * 64 + wave * 16;  // this wave's first channel of the part
+  const int nt = TAPS ? TAPS : a.taps;
   if (threadIdx.x < 16) {
     const int b = b0 + threadIdx.x;
     slots[threadIdx.x] = b < B ? step.slot(b) : -1;
     pos[threadIdx.x] = b < B ? step.first(b) : 0;
   }
   __syncthreads();
-  auto conv = [&](int r, int c) {  // u of row r, channel c (of all)
-    const int slot = slots[r], p = pos[r];
-    if (slot < 0) return 0.f;
-    const float ib = ld(in_bias + a.W + c);
-    float y = ld(conv_bias + c);
-    for (int j = 0; j < a.taps; ++j) {
-      const int back = a.taps - 1 - j;
-      if (p - back < 0) continue;
-      const float x = back ? ld(ring + ((size_t)slot * a.taps + (p - back) % a.taps) * a.W + c)
-                           : ld(proj + (size_t)(b0 + r) * a.N + a.x_at + c);
-      y += (x + ib) * ld(taps + (size_t)c * a.taps + j);
-    }
-    return y;
-  };
+  const int b = b0 + col, slot = slots[col], p = pos[col];
   floatx4 acc[2] = {(floatx4)(0.f), (floatx4)(0.f)};
   const T* wr[2];
 #pragma unroll
   for (int g = 0; g < 2; ++g) wr[g] = gates + ((size_t)g * a.W + part * a.n + min(cl0 + col, a.n - 1)) * a.n;
-  float uo[4] = {0.f, 0.f, 0.f, 0.f};  // u of this lane's row and channels
   const bool whole = a.n % F::K == 0;
+  auto gate_row = [&](int g, int k) { return whole ? ld_frag<T, true>(wr[g], k, a.n) : ld_frag<T, false>(wr[g], k, a.n); };
+  // of this lane's row and channels
+  float uo[4], br[4], bi[4], most[4], S[4], y[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int c = part * a.n + min(cl0 + quad * 4 + r, a.n - 1);
+    uo[r] = 0.f;
+    br[r] = ld(bias + c);
+    bi[r] = ld(bias + a.W + c);
+    most[r] = ld(lam + c);
+    S[r] = slot >= 0 && p > 0 ? state[(size_t)slot * a.W + c] : 0.f;
+    y[r] = (b < B ? ld(proj + (size_t)b * a.N + a.y_at + c) : 0.f) + ld(in_bias + c);
+  }
   for (int k0 = 0; k0 < a.n; k0 += CH) {
     const int n = min(CH, a.n - k0);
-#pragma unroll 4
-    for (int i = threadIdx.x; i < 16 * CH; i += 256) {
-      const int r = i / CH, k = i % CH;
-      st(&us[r][k], k < n ? conv(r, part * a.n + k0 + k) : 0.f);
+    typename F::V wf[PRE][2];
+#pragma unroll
+    for (int s = 0; s < PRE; ++s)
+      if (s * F::K < n)
+#pragma unroll
+        for (int g = 0; g < 2; ++g) wf[s][g] = gate_row(g, k0 + s * F::K + quad * F::PER);
+    // a thread has one channel, and every (256 / width)th row
+    const int width = n <= 32 ? 32 : n <= 64 ? 64 : n <= 128 ? 128 : 256;
+    const int k = threadIdx.x & (width - 1), c = part * a.n + k0 + min(k, n - 1);
+    const float ib = ld(in_bias + a.W + c), cb = ld(conv_bias + c);
+    float tw[TAPS ? TAPS : 1];
+    if (TAPS)
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) tw[j] = ld(taps + (size_t)c * TAPS + j);
+#pragma unroll 8
+    for (int r = threadIdx.x / width; r < 16; r += 256 / width) {
+      // parked rows load something valid, so that no load waits for a branch
+      const int at = max(slots[r], 0), q = pos[r];
+      float v = cb + (ld(proj + (size_t)min(b0 + r, B - 1) * a.N + a.x_at + c) + ib) * (TAPS ? tw[TAPS ? TAPS - 1 : 0] : ld(taps + (size_t)c * nt + nt - 1));
+#pragma unroll
+      for (int back = 1; back < nt; ++back) {
+        const float x = ld(ring + ((size_t)at * nt + max(q - back, 0) % nt) * a.W + c) + ib;
+        const float w = TAPS ? tw[TAPS ? TAPS - 1 - back : 0] : ld(taps + (size_t)c * nt + nt - 1 - back);
+        v += q >= back ? x * w : 0.f;
+      }
+      st(&us[r][k], slots[r] >= 0 && k < n ? v : 0.f);
     }
     __syncthreads();
-    if (cl0 < a.n)
-      for (int s = 0; s * F::K < n; ++s) {
-        const int k = s * F::K + quad * F::PER;
-        const typename F::V uf = *(const typename F::V*)&us[col][k];
+    if (cl0 < a.n) {
 #pragma unroll
-        for (int g = 0; g < 2; ++g)
-          acc[g] = mma(whole ? ld_frag<T, true>(wr[g], k0 + k, a.n) : ld_frag<T, false>(wr[g], k0 + k, a.n), uf, acc[g]);
+      for (int s = 0; s < PRE; ++s)
+        if (s * F::K < n) {
+          const typename F::V uf = *(const typename F::V*)&us[col][s * F::K + quad * F::PER];
+#pragma unroll
+          for (int g = 0; g < 2; ++g) acc[g] = mma(wf[s][g], uf, acc[g]);
+        }
+#pragma unroll 2
+      for (int s = PRE; s * F::K < n; ++s) {
+        const int at = s * F::K + quad * F::PER;
+        const typename F::V uf = *(const typename F::V*)&us[col][at];
+#pragma unroll
+        for (int g = 0; g < 2; ++g) acc[g] = mma(gate_row(g, k0 + at), uf, acc[g]);
       }
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int k = cl0 + quad * 4 + r - k0;
-      if (k >= 0 && k < n) uo[r] = ld(&us[col][k]);
+      const int own = cl0 + quad * 4 + r - k0;
+      if (own >= 0 && own < n) uo[r] = ld(&us[col][own]);
     }
     __syncthreads();
   }
-  const int b = b0 + col, slot = slots[col], p = pos[col];
   if (b >= B) return;
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -255,13 +341,12 @@ __global__ __launch_bounds__(256) void unit_step_kernel(
     float o = 0.f;
     if (slot >= 0) {
       float d, x;
-      decay_of(acc[0][r] + ld(bias + c), acc[1][r] + ld(bias + a.W + c), uo[r], ld(lam + c), a.rate, d, x);
-      float* cell = state + (size_t)slot * a.W + c;
-      const float S = p > 0 ? d * *cell + x : x;
-      *cell = S;
+      decay_of(acc[0][r] + br[r], acc[1][r] + bi[r], uo[r], a.rate * softplus_of(most[r]), d, x);
+      const float now = d * S[r] + x;
+      state[(size_t)slot * a.W + c] = now;
       // the row of the oldest input: no tap of this step reaches it
-      ring[((size_t)slot * a.taps + p % a.taps) * a.W + c] = proj[(size_t)b * a.N + a.x_at + c];
-      o = S * gelu_tanh(ld(proj + (size_t)b * a.N + a.y_at + c) + ld(in_bias + c)) * a.out_scale;
+      ring[((size_t)slot * nt + p % nt) * a.W + c] = proj[(size_t)b * a.N + a.x_at + c];
+      o = now * gelu_tanh(y[r]) * a.out_scale;
     }
     st(out + (size_t)b * a.K + a.out_at + c, o);
   }
@@ -300,8 +385,8 @@ void gated_unit(Tensor u, Tensor proj, int64_t y_at, Tensor in_bias, Tensor gate
   const hipStream_t stream = cur_stream();
   const int tokens = B * S, tiles = W / a.n * ((a.n + 31) / 32);
   auto decay = f32(u, {B, S, W}), input = f32(u, {B, S, W});
-  const int groups = (tokens + 127) / 128;
-  CHK(groups <= 65535);
+  const dim3 gate_grid((tokens + 32 * GROUPS - 1) / (32 * GROUPS), (tiles + 3) / 4);
+  CHK(gate_grid.y <= 65535);
   const int V = ((W | a.N | a.y_at | a.K | a.out_at) & 3) == 0 ? 4 : 1;
   // segments where rows and channels are too few to hide the loads
   const int64_t threads = (int64_t)B * (W / V);
@@ -327,12 +412,13 @@ void gated_unit(Tensor u, Tensor proj, int64_t y_at, Tensor in_bias, Tensor gate
     SCAN(V, OUTPUTS);                                                                                                 \
   }
   BY_TYPE(dt, {
-    if (a.n % Frag<T>::K == 0)
-      hipLaunchKernelGGL((gates_kernel<T, true>), dim3(tiles, groups), dim3(256), 0, stream, P<T>(u), P<T>(gates), P<T>(bias),
-                         P<T>(lam), M<float>(decay), M<float>(input), tokens, a);
-    else
-      hipLaunchKernelGGL((gates_kernel<T, false>), dim3(tiles, groups), dim3(256), 0, stream, P<T>(u), P<T>(gates), P<T>(bias),
-                         P<T>(lam), M<float>(decay), M<float>(input), tokens, a);
+    auto make = [&](auto kernel) {
+      hipLaunchKernelGGL(kernel, gate_grid, dim3(256), 0, stream, P<T>(u), P<T>(gates), P<T>(bias), P<T>(lam),
+                         M<float>(decay), M<float>(input), tokens, a);
+    };
+    if (a.n == 4 * Frag<T>::K) make(gates_kernel<T, true, 4>);
+    else if (a.n % Frag<T>::K == 0) make(gates_kernel<T, true, 0>);
+    else make(gates_kernel<T, false, 0>);
     if (V == 4) { SCANS(4) } else { SCANS(1) }
   });
 #undef SCANS
@@ -355,9 +441,12 @@ void gated_unit_step(Tensor proj, int64_t y_at, int64_t x_at, Tensor in_bias, Te
   const Step step = make_step(slots, positions, c10::nullopt, 0, true, B);
   const dim3 grid(a.W / a.n * ((a.n + 63) / 64), (B + 15) / 16);
   BY_TYPE(dt, {
-    hipLaunchKernelGGL((unit_step_kernel<T>), grid, dim3(256), 0, cur_stream(), P<T>(proj), P<T>(in_bias), P<T>(taps),
-                       P<T>(conv_bias), P<T>(gates), P<T>(bias), P<T>(lam), M<float>(state), M<T>(ring), M<T>(out), B, a,
-                       step);
+    auto run = [&](auto kernel) {
+      hipLaunchKernelGGL(kernel, grid, dim3(256), 0, cur_stream(), P<T>(proj), P<T>(in_bias), P<T>(taps), P<T>(conv_bias),
+                         P<T>(gates), P<T>(bias), P<T>(lam), M<float>(state), M<T>(ring), M<T>(out), B, a, step);
+    };
+    if (a.taps == 4) run(unit_step_kernel<T, 4>);
+    else run(unit_step_kernel<T, 0>);
   });
 }
 

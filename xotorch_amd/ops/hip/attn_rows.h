@@ -414,49 +414,84 @@ __global__ __launch_bounds__(256) void attn_rows_decode_kernel(
 }
 
 // Partial results of a head's splits -> its output. Four waves take splits in
-// turn, then a thread has a value column.
+// turn, a few in flight; then a thread has a value column.
 template <int MODE, int MAPS = 1>
 __global__ __launch_bounds__(256) void attn_rows_merge_kernel(
     const float* __restrict__ part, Side<MODE, bf16_t> side, bf16_t* __restrict__ out, int splits,
     int vdim, AttnArgs a, Step step) {
-  __shared__ float po[4][256], pl[4], sums[4];
+  constexpr int NC = 4, AHEAD = 4;  // value columns of a lane; splits in flight
+  __shared__ float po[MAPS][4][NC * 64], pm[MAPS][4], pl[MAPS][4], sums[4];
   const int h = blockIdx.x, b = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  constexpr int NC = 4;  // value columns of a lane
+  const int c = threadIdx.x;
   float v = 0.f;
-  if (step.slot(b) >= 0)
+  if (step.slot(b) >= 0) {
+    float M[MAPS], L[MAPS], O[MAPS][NC];
 #pragma unroll
     for (int mp = 0; mp < MAPS; ++mp) {
-      const size_t row = ((size_t)b * splits * a.H + h) * MAPS + mp, stride = (size_t)a.H * MAPS;
-      float M = side.start(h), L = 0.f, O[NC];
-      for (int s = lane; s < splits; s += 64) M = fmaxf(M, part[(row + s * stride) * (vdim + 2)]);
+      M[mp] = side.start(h);
+      L[mp] = 0.f;
 #pragma unroll
-      for (int d = 1; d < 64; d <<= 1) M = fmaxf(M, __shfl_xor(M, d));
-#pragma unroll
-      for (int i = 0; i < NC; ++i) O[i] = 0.f;
-#pragma unroll 4
-      for (int s = wave; s < splits; s += 4) {
-        const float* p = part + (row + s * stride) * (vdim + 2);
-        const float f = __expf(p[0] - M);
-        L += f * p[1];
-#pragma unroll
-        for (int i = 0; i < NC; ++i) O[i] += f * p[2 + min(lane + i * 64, vdim - 1)];
-      }
-      if (mp) __syncthreads();
-#pragma unroll
-      for (int i = 0; i < NC; ++i) po[wave][i * 64 + lane] = O[i];
-      if (lane == 0) pl[wave] = L;
-      __syncthreads();
-      L = pl[0] + pl[1] + pl[2] + pl[3];
-      const float f = MAPS == 1 ? side.gate(a, b, h) / (L + __expf(side.sink(h) - M)) : mp ? -*a.lam / L : 1.f / L;
-      v += f * (po[0][threadIdx.x] + po[1][threadIdx.x] + po[2][threadIdx.x] + po[3][threadIdx.x]);
+      for (int i = 0; i < NC; ++i) O[mp][i] = 0.f;
     }
+    for (int s0 = wave; s0 < splits; s0 += 4 * AHEAD) {
+      float m[MAPS][AHEAD], l[MAPS][AHEAD], o[MAPS][AHEAD][NC];
+#pragma unroll
+      for (int mp = 0; mp < MAPS; ++mp)
+#pragma unroll
+        for (int j = 0; j < AHEAD; ++j) {
+          const int s = s0 + 4 * j;
+          const float* p = part + ((((size_t)b * splits + min(s, splits - 1)) * a.H + h) * MAPS + mp) * (vdim + 2);
+          m[mp][j] = s < splits ? p[0] : -INFINITY;
+          l[mp][j] = p[1];
+#pragma unroll
+          for (int i = 0; i < NC; ++i) o[mp][j][i] = p[2 + min(lane + i * 64, vdim - 1)];
+        }
+#pragma unroll
+      for (int mp = 0; mp < MAPS; ++mp) {
+        float top = M[mp];
+#pragma unroll
+        for (int j = 0; j < AHEAD; ++j) top = fmaxf(top, m[mp][j]);
+        const float al = __expf(M[mp] - top);
+        M[mp] = top;
+        L[mp] *= al;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) O[mp][i] *= al;
+#pragma unroll
+        for (int j = 0; j < AHEAD; ++j) {
+          const float f = __expf(m[mp][j] - top);
+          L[mp] += f * l[mp][j];
+#pragma unroll
+          for (int i = 0; i < NC; ++i) O[mp][i] += f * o[mp][j][i];
+        }
+      }
+    }
+#pragma unroll
+    for (int mp = 0; mp < MAPS; ++mp) {
+#pragma unroll
+      for (int i = 0; i < NC; ++i) po[mp][wave][i * 64 + lane] = O[mp][i];
+      if (lane == 0) { pm[mp][wave] = M[mp]; pl[mp][wave] = L[mp]; }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int mp = 0; mp < MAPS; ++mp) {
+      float top = pm[mp][0], sum = 0.f, all = 0.f;
+#pragma unroll
+      for (int w = 1; w < 4; ++w) top = fmaxf(top, pm[mp][w]);
+#pragma unroll
+      for (int w = 0; w < 4; ++w) {
+        const float f = __expf(pm[mp][w] - top);
+        all += f * pl[mp][w];
+        sum += f * po[mp][w][c];
+      }
+      v += sum * (MAPS == 1 ? side.gate(a, b, h) / (all + __expf(side.sink(h) - top)) : mp ? -*a.lam / all : 1.f / all);
+    }
+  }
   if (MAPS == 2) {
-    const float ss = wave_sum(threadIdx.x < vdim ? v * v : 0.f);
+    const float ss = wave_sum(c < vdim ? v * v : 0.f);
     if (lane == 0) sums[wave] = ss;
     __syncthreads();
     v *= a.gain / sqrtf((sums[0] + sums[1] + sums[2] + sums[3]) / (float)vdim + a.eps) * side.gate(a, b, h);
   }
-  const int c = threadIdx.x;
   if (c < vdim) st(out + (size_t)b * a.K + a.out_at + (size_t)h * vdim + c, v);
 }
 

@@ -241,8 +241,8 @@ __global__ __launch_bounds__(256) void segment_starts_kernel(const float* __rest
 // Decode: 16 rows x 64 channels of a part. The convolution of the part's
 // channels goes through LDS 256 at a time; a wave makes both gates of 16
 // channels for all rows. What does not hang on the convolution is loaded before
-// it. TAPS 0: any number of taps.
-template <typename T, int TAPS>
+// it. TAPS 0: any number of taps. WHOLE: a part is whole k steps.
+template <typename T, int TAPS, bool WHOLE>
 __global__ __launch_bounds__(256) void unit_step_kernel(
     const T* __restrict__ proj, const T* __restrict__ in_bias, const T* __restrict__ taps, const T* __restrict__ conv_bias,
     const T* __restrict__ gates, const T* __restrict__ bias, const T* __restrict__ lam, float* __restrict__ state,
@@ -266,8 +266,7 @@ __global__ __launch_bounds__(256) void unit_step_kernel(
   const T* wr[2];
 #pragma unroll
   for (int g = 0; g < 2; ++g) wr[g] = gates + ((size_t)g * a.W + part * a.n + min(cl0 + col, a.n - 1)) * a.n;
-  const bool whole = a.n % F::K == 0;
-  auto gate_row = [&](int g, int k) { return whole ? ld_frag<T, true>(wr[g], k, a.n) : ld_frag<T, false>(wr[g], k, a.n); };
+  auto gate_row = [&](int g, int k) { return ld_frag<T, WHOLE>(wr[g], k, a.n); };
   // of this lane's row and channels
   float uo[4], br[4], bi[4], most[4], S[4], y[4];
 #pragma unroll
@@ -288,27 +287,46 @@ __global__ __launch_bounds__(256) void unit_step_kernel(
       if (s * F::K < n)
 #pragma unroll
         for (int g = 0; g < 2; ++g) wf[s][g] = gate_row(g, k0 + s * F::K + quad * F::PER);
-    // a thread has one channel, and every (256 / width)th row
-    const int width = n <= 32 ? 32 : n <= 64 ? 64 : n <= 128 ? 128 : 256;
-    const int k = threadIdx.x & (width - 1), c = part * a.n + k0 + min(k, n - 1);
-    const float ib = ld(in_bias + a.W + c), cb = ld(conv_bias + c);
-    float tw[TAPS ? TAPS : 1];
-    if (TAPS)
+    // a thread has one of 16 * RUNS channels, and RUNS of the rows
+    auto convolve = [&](auto runs) {
+      constexpr int RUNS = decltype(runs)::value, BATCH = RUNS < 8 ? RUNS : 8;
+      const int k = threadIdx.x % (16 * RUNS), r0 = threadIdx.x / (16 * RUNS), c = part * a.n + k0 + min(k, n - 1);
+      const float ib = ld(in_bias + a.W + c), cb = ld(conv_bias + c);
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) tw[j] = ld(taps + (size_t)c * TAPS + j);
-#pragma unroll 8
-    for (int r = threadIdx.x / width; r < 16; r += 256 / width) {
-      // parked rows load something valid, so that no load waits for a branch
-      const int at = max(slots[r], 0), q = pos[r];
-      float v = cb + (ld(proj + (size_t)min(b0 + r, B - 1) * a.N + a.x_at + c) + ib) * (TAPS ? tw[TAPS ? TAPS - 1 : 0] : ld(taps + (size_t)c * nt + nt - 1));
+      for (int j0 = 0; j0 < RUNS; j0 += BATCH) {
+        float v[BATCH];
+        auto tap = [&](int back) {  // of all rows of the batch, loads first
+          float x[BATCH];
 #pragma unroll
-      for (int back = 1; back < nt; ++back) {
-        const float x = ld(ring + ((size_t)at * nt + max(q - back, 0) % nt) * a.W + c) + ib;
-        const float w = TAPS ? tw[TAPS ? TAPS - 1 - back : 0] : ld(taps + (size_t)c * nt + nt - 1 - back);
-        v += q >= back ? x * w : 0.f;
+          for (int j = 0; j < BATCH; ++j) {
+            // parked rows load something valid, so that no load waits for a branch
+            const int r = r0 + (j0 + j) * (16 / RUNS), at = max(slots[r], 0);
+            x[j] = back ? ld(ring + ((size_t)at * nt + max(pos[r] - back, 0) % nt) * a.W + c)
+                        : ld(proj + (size_t)min(b0 + r, B - 1) * a.N + a.x_at + c);
+          }
+          const float w = ld(taps + (size_t)c * nt + nt - 1 - back);
+#pragma unroll
+          for (int j = 0; j < BATCH; ++j)
+            if (pos[r0 + (j0 + j) * (16 / RUNS)] >= back) v[j] += (x[j] + ib) * w;
+        };
+#pragma unroll
+        for (int j = 0; j < BATCH; ++j) v[j] = cb;
+        if (TAPS) {
+#pragma unroll
+          for (int back = 0; back < TAPS; ++back) tap(back);
+        } else
+          for (int back = 0; back < nt; ++back) tap(back);
+#pragma unroll
+        for (int j = 0; j < BATCH; ++j) {
+          const int r = r0 + (j0 + j) * (16 / RUNS);
+          st(&us[r][k], slots[r] >= 0 && k < n ? v[j] : 0.f);
+        }
       }
-      st(&us[r][k], slots[r] >= 0 && k < n ? v : 0.f);
-    }
+    };
+    if (n <= 32) convolve(std::integral_constant<int, 2>());
+    else if (n <= 64) convolve(std::integral_constant<int, 4>());
+    else if (n <= 128) convolve(std::integral_constant<int, 8>());
+    else convolve(std::integral_constant<int, 16>());
     __syncthreads();
     if (cl0 < a.n) {
 #pragma unroll
@@ -445,8 +463,9 @@ void gated_unit_step(Tensor proj, int64_t y_at, int64_t x_at, Tensor in_bias, Te
       hipLaunchKernelGGL(kernel, grid, dim3(256), 0, cur_stream(), P<T>(proj), P<T>(in_bias), P<T>(taps), P<T>(conv_bias),
                          P<T>(gates), P<T>(bias), P<T>(lam), M<float>(state), M<T>(ring), M<T>(out), B, a, step);
     };
-    if (a.taps == 4) run(unit_step_kernel<T, 4>);
-    else run(unit_step_kernel<T, 0>);
+    const bool whole = a.n % Frag<T>::K == 0;
+    if (a.taps == 4) whole ? run(unit_step_kernel<T, 4, true>) : run(unit_step_kernel<T, 4, false>);
+    else whole ? run(unit_step_kernel<T, 0, true>) : run(unit_step_kernel<T, 0, false>);
   });
 }
 

@@ -116,7 +116,9 @@ class ShardKVCache:
 class MixerStateCache:
   """State of the layers of a design whose mixers differ (cfg.layer_specs):
   per local layer a list with one tuple of tensors per branch of its mixer,
-  each tensor [slots, ...] as the mixer's `state_spec` says. Slots are
+  each tensor [slots, ...] as the mixer's `state_spec` says; after these, the
+  last inputs of the layer's input convolution (position p in row p % taps) and,
+  in the first layer of a design that embeds token pairs, the last token. Slots are
   independent and constant in size; a sequence that starts at position 0
   ignores what its slot held before."""
 
@@ -125,10 +127,14 @@ class MixerStateCache:
     from xotorch_amd.models.mixers import MIXERS
     self.batch, self.capacity = slots, capacity
     self.caches: List[list] = []
-    for spec in cfg.shard_specs(shard).values():
+    for i, spec in cfg.shard_specs(shard).items():
+      parts = list(MIXERS[spec.mixer].state_spec(spec.params, capacity, dtype, device))
+      if spec.conv:
+        parts.append({"inputs": ((spec.conv, cfg.dim), dtype)})
+      if cfg.bigram is not None and i == 0:
+        parts.append({"token": ((1,), torch.int32)})
       self.caches.append([
-        tuple(torch.zeros(slots, *shape, dtype=dt, device=device) for shape, dt in branch.values())
-        for branch in MIXERS[spec.mixer].state_spec(spec.params, capacity, dtype, device)
+        tuple(torch.zeros(slots, *shape, dtype=dt, device=device) for shape, dt in part.values()) for part in parts
       ])
 
   def __getitem__(self, i):

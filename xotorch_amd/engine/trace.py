@@ -107,6 +107,18 @@ class TraceRunner:
     return torch.stack(rows).cpu() if rows else torch.empty(0, self.worker.cfg.vocab_size)
 
 
+def build_extensions(model_dir: str):
+  """Compiles what is missing of the HIP extensions that the model runs on."""
+  from xotorch_amd.models import config_from_hf, model_class_for
+  from xotorch_amd.ops import build as hip_build
+  from xotorch_amd.shard import Shard
+  cfg = config_from_hf(Path(model_dir) / "config.json", "model")
+  with torch.device("meta"):
+    model = model_class_for(cfg)(cfg, Shard("model", 0, cfg.n_layers - 1, cfg.n_layers))
+  needed = model.extensions() if hasattr(model, "extensions") else ["_hip_ops"]
+  hip_build.build(verbose=False, missing_only=True, only=needed)
+
+
 def build_worker(model_dir: str, dtype: torch.dtype, max_tokens: int):
   from xotorch_amd.serve_ring import RingSlotWorker
   device = "cuda" if torch.cuda.is_available() else "cpu"
@@ -125,8 +137,7 @@ def main(argv=None) -> int:
   p.add_argument("--max-tokens", type=int, default=4096, help="most tokens that live requests hold at any time")
   args = p.parse_args(argv)
   if torch.cuda.is_available():
-    from xotorch_amd.ops import build as hip_build
-    hip_build.build(verbose=False, missing_only=True)
+    build_extensions(args.model)
   torch.backends.cuda.matmul.allow_tf32 = False
   runner = TraceRunner(build_worker(args.model, getattr(torch, args.dtype), args.max_tokens))
   for line in sys.stdin:

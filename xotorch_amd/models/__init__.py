@@ -11,7 +11,10 @@ from xotorch_amd.models.registry import (  # noqa: F401
 
 def model_class_for(cfg: ModelConfig):
   """Decoder class for a parsed config (ShardedModel / Gemma2 / DeepSeek-MLA /
-  Didipel / Lebotar / Tapupel)."""
+  Didipel / Lebotar / Tapupel / Dupolorn)."""
+  if cfg.model_type == "dupolorn":
+    from xotorch_amd.models.dupolorn import DupolornModel
+    return DupolornModel
   if cfg.model_type == "tapupel":
     from xotorch_amd.models.tapupel import TapupelModel
     return TapupelModel

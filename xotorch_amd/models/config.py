@@ -45,11 +45,13 @@ class LayerSpec:
   """One layer of a design whose layers are listed one by one: the kind of
   its mixer (a key of models.mixers.MIXERS), that mixer's sizes and constants,
   and its feed-forward: the width of a dense one (0: none) or the parameters
-  of a sparse one (models.experts)."""
+  of a sparse one (models.experts). conv: taps of a convolution that the
+  mixer's input passes through (0: none)."""
   mixer: str
   params: dict
   ff: int = 0
   moe: Optional[dict] = None
+  conv: int = 0
 
 
 @dataclass
@@ -108,6 +110,8 @@ class ModelConfig:
   layer_specs: Optional[List[LayerSpec]] = None
   residual_mult: float = 1.0  # what a sublayer's output is scaled with
   embed_scale: float = 1.0    # what embeddings are scaled with
+  # embeddings of token pairs, {buckets, mul_prev, mul_cur}; None: none
+  bigram: Optional[dict] = None
   # what travels with the stream between ring stages besides it: name -> channels
   carried: Dict[str, int] = field(default_factory=dict)
 
@@ -143,7 +147,9 @@ class ModelConfig:
     if self.layer_specs is not None:
       from xotorch_amd.models.mixers import MIXERS
       mixers = sum(MIXERS[s.mixer].param_count(self.dim, s.params) for s in self.layer_specs)
-      ff = sum(3 * self.dim * s.ff for s in self.layer_specs)
+      ff = sum(self.dim * (3 * s.ff + s.conv) for s in self.layer_specs)
+      if self.bigram is not None:
+        ff += (self.bigram["buckets"] + 1) * self.dim
       if any(s.moe is not None for s in self.layer_specs):
         from xotorch_amd.models.experts import GroupedExperts
         ff += sum(GroupedExperts.param_count(self.dim, s.moe) for s in self.layer_specs if s.moe is not None)
@@ -194,6 +200,9 @@ def config_from_hf(config_path: Path | str | dict, model_id: str = "unknown") ->
     if raw["architecture"] == "Tapupel":
       from xotorch_amd.models.tapupel import tapupel_config
       return tapupel_config(raw, model_id, shapes)
+    if raw["architecture"] == "Dupolorn":
+      from xotorch_amd.models.dupolorn import dupolorn_config
+      return dupolorn_config(raw, model_id, shapes)
     raise ValueError(f"unknown architecture {raw['architecture']!r}")
 
   n_heads = raw.get("num_attention_heads", 32)

@@ -55,6 +55,13 @@ class DenseMLP(MLP):
     return mo.swiglu_packed(gu)
 
 
+class DenseGeluMLP(DenseMLP):
+  """The same block with the tanh form of gelu."""
+
+  def forward(self, x):
+    return self.down_proj(mo.gated_packed(self.gate_up_proj(x), "gelu_tanh"))
+
+
 class DidipelLayer(nn.Module):
   def __init__(self, cfg: ModelConfig, spec: LayerSpec):
     super().__init__()
@@ -85,7 +92,7 @@ class DidipelLayer(nn.Module):
 
 
 class DidipelModel(LayeredModel):
-  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec, place: int) -> nn.Module:
     return DidipelLayer(cfg, spec)
 
 

@@ -43,26 +43,57 @@ class LayeredModel(nn.Module):
 
   slot_indexed = True
   hidden_dtype = torch.float32
+  hip = ("_hip_ops", "_hip_mixers")
 
-  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec, place: int) -> nn.Module:
     raise NotImplementedError
 
   @staticmethod
-  def entry(layer):
+  def entry(layer, cache=None):
     """What a layer reads: the stream normed with this weight, or mo.STREAM."""
     return layer.norm1
+
+  def embed(self, tokens, caches, rows):
+    x = self.embed_tokens(tokens).float()
+    return x * self.cfg.embed_scale if self.cfg.embed_scale != 1.0 else x
+
+  def receive(self, x, rows, dtype):
+    """What an earlier ring stage handed on -> the stream."""
+    if self.cfg.carried_dim:
+      x, *carried = x.split([self.cfg.dim, *self.cfg.carried.values()], dim=-1)
+      rows.carried = {name: t.to(dtype) for name, t in zip(self.cfg.carried, carried)}
+    if not (torch.is_grad_enabled() and x.requires_grad):
+      x = x.float().clone(memory_format=torch.contiguous_format)  # updated in place; the caller keeps its own
+    return x
+
+  def hand_on(self, x, rows):
+    if not self.cfg.carried_dim:
+      return x
+    return torch.cat([x, *(rows.carried[name].float() if name in rows.carried else x.new_zeros(*x.shape[:-1], width)
+                           for name, width in self.cfg.carried.items())], dim=-1)
+
+  def read(self, x, what, rows, dtype):
+    """The stream as a layer or the head reads it."""
+    return mo.prenorm(x, what, self.cfg.norm_eps, dtype)
+
+  def extensions(self) -> List[str]:
+    """HIP extensions that a forward pass loads (ops/build.py)."""
+    return sorted({name for m in self.modules() for name in getattr(m, "hip", ())})
 
   def __init__(self, cfg: ModelConfig, shard: Shard):
     super().__init__()
     self.cfg, self.shard = cfg, shard
     if shard.is_first_layer:
       self.embed_tokens = nn.Embedding(cfg.vocab_size, cfg.dim)
-    self.layers = nn.ModuleDict({str(i): self.make_layer(cfg, spec) for i, spec in cfg.shard_specs(shard).items()})
+    self.layers = nn.ModuleDict({str(i): self.make_layer(cfg, spec, i) for i, spec in cfg.shard_specs(shard).items()})
     self.init_ranges = {}
     if shard.is_last_layer:
-      self.norm = nn.Parameter(torch.zeros(cfg.dim))
-      self.init_ranges["norm"] = (-0.2, 0.2)
+      self.make_final_norm()
       self.lm_head = XotLinear(cfg.dim, cfg.vocab_size, bias=False)
+
+  def make_final_norm(self):
+    self.norm = nn.Parameter(torch.zeros(self.cfg.dim))
+    self.init_ranges["norm"] = (-0.2, 0.2)
 
   def reset_rope(self):
     """Position tables of the mixers after meta construction."""
@@ -92,43 +123,36 @@ class LayeredModel(nn.Module):
     (None: row b is slot b; -1: parked). layers_out collects the stream after
     every local layer."""
     dtype = self.layers[str(self.shard.start_layer)].norm1.dtype
-    cfg, eps = self.cfg, self.cfg.norm_eps
     B, S = x.shape[0], x.shape[1]
     rows = mo.StepRows(is_decode, 0 if is_decode else int(start_pos),
                        positions.reshape(-1) if is_decode else None, slots, lens)
     if x.dtype in (torch.int32, torch.int64):
-      x = self.embed_tokens(x).float()
-      if cfg.embed_scale != 1.0:
-        x = x * cfg.embed_scale
+      x = self.embed(x, caches, rows)
     else:
-      if cfg.carried_dim:
-        x, *carried = x.split([cfg.dim, *cfg.carried.values()], dim=-1)
-        rows.carried = {name: t.to(dtype) for name, t in zip(cfg.carried, carried)}
-      if not (torch.is_grad_enabled() and x.requires_grad):
-        x = x.float().clone(memory_format=torch.contiguous_format)  # updated in place; the caller keeps its own
+      x = self.receive(x, rows, dtype)
     layers = [self.layers[str(i)] for i in self.local_layer_ids]
-    h = mo.prenorm(x, self.entry(layers[0]), eps, dtype)
+    states = caches if caches is not None else [None] * len(layers)
+    h = self.read(x, self.entry(layers[0], states[0]), rows, dtype)
     whole = is_decode or not last_only or S == 1  # the head reads every row
     for i, layer in enumerate(layers):
       if i + 1 < len(layers):
-        after = self.entry(layers[i + 1])
+        after = self.entry(layers[i + 1], states[i + 1])
       else:
         after = self.norm if self.shard.is_last_layer and whole else None
-      x, h = layer.step(x, h, caches[i] if caches is not None else None, rows, after)
+      x, h = layer.step(x, h, states[i], rows, after)
       if layers_out is not None:
         layers_out.append(x.clone())
     if not self.shard.is_last_layer:
-      if cfg.carried_dim:
-        x = torch.cat([x, *(rows.carried[name].float() if name in rows.carried else x.new_zeros(B, S, width)
-                            for name, width in cfg.carried.items())], dim=-1)
-      return x
+      return self.hand_on(x, rows)
     if not whole:
       if lens is None:
         x = x[:, -1:].contiguous()
       else:
         x = x[torch.arange(B, device=x.device), lens.long() - 1][:, None].contiguous()
-      h = mo.prenorm(x, self.norm, eps, dtype)
+      h = self.read(x, self.norm, rows, dtype)
     logits = self.lm_head(h)
+    if self.cfg.final_logit_softcapping:
+      logits = mo.soft_cap(logits, self.cfg.final_logit_softcapping)
     return logits[:, -1] if is_decode or last_only else logits
 
 

@@ -82,7 +82,7 @@ class LebotarLayer(nn.Module):
 
 
 class LebotarModel(LayeredModel):
-  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec, place: int) -> nn.Module:
     return LebotarLayer(cfg, spec)
 
 

@@ -5,7 +5,7 @@ each; MIXERS maps that name to a class here. Every constant of a mechanism is
 a parameter of its branch, so another design can use it with its own.
 
 Branches that read projections of the layer's input (the attentions,
-`GatedDeltaRule`, `SelectiveScan`, `GatedLinearUnit`) are combined by `BranchMixer`: ONE fused input GEMM over
+`GatedDeltaRule`, `SelectiveScan`, `GatedLinearUnit`, `MatrixMemory`) are combined by `BranchMixer`: ONE fused input GEMM over
 the parts of all branches and ONE output GEMM over their concatenated
 activations (branch weights fold into the activations in fp32), however many
 branches run side by side. `WKVMixer` shifts its input per projection and so
@@ -51,6 +51,8 @@ class WindowBiasAttention(nn.Module):
   """GQA attention over a sliding window: RMS norm over the whole q and k
   projections, no rotation, a learned bias per distance bucket, a sink of
   score zero in the softmax, one sigmoid output gate per head."""
+
+  hip = ("_hip_attn",)
 
   def __init__(self, dim: int, p: dict, eps: float):
     super().__init__()
@@ -301,6 +303,8 @@ class ChunkAttention(nn.Module):
   the distance, a learned sink per head. With `v_mix`, all but the first such
   layer blend their values with the first one's for the same token."""
 
+  hip = ("_hip_attn",)
+
   def __init__(self, dim: int, p: dict, eps: float):
     super().__init__()
     self.H, self.G, self.dim, self.vdim = p["heads"], p["kv_heads"], p["dim"], p["vdim"]
@@ -379,7 +383,11 @@ class Turning(nn.Module):
 class LatentAttention(Turning):
   """Latent attention: keys and values of all heads come out of one normed
   latent per token, plus one rotated key part that the heads share. Only these
-  two are cached; decode folds the expansion into query and output."""
+  two are cached; decode folds the expansion into query and output. With `sink`,
+  a learned score per head joins the softmax's denominator; with `gate`, the
+  heads' outputs are multiplied with the sigmoid of one more projection."""
+
+  hip = ("_hip_latent", "_hip_attn")
 
   def __init__(self, dim: int, p: dict, eps: float):
     super().__init__()
@@ -387,11 +395,14 @@ class LatentAttention(Turning):
     self.rot, self.scale, self.eps = p["rot"], float(p["scale"]), eps
     if self.rot_dim % 2 or self.rot["dims"] % 2 or self.rot["dims"] > self.rot_dim:
       raise ValueError(f"rotation of {self.rot['dims']} of {self.rot_dim} dimensions")
-    self.parts = [("q", self.H * (self.dim + self.rot_dim)), ("dkv", self.rank + self.rot_dim)]
     self.width = self.H * self.vdim
+    self.parts = [("q", self.H * (self.dim + self.rot_dim)), ("dkv", self.rank + self.rot_dim)]
+    if p.get("gate"):
+      self.parts.append(("g", self.width))
     self.kv_norm = nn.Parameter(torch.ones(self.rank))
     self.kv_up = XotLinear(self.rank, self.H * (self.dim + self.vdim), bias=False)  # all keys, then all values
-    self.init_ranges = {"kv_norm": (0.8, 1.2)}
+    self.sink = nn.Parameter(torch.zeros(self.H)) if p.get("sink") else None
+    self.init_ranges = {"kv_norm": (0.8, 1.2), "sink": (-1.0, 1.0)}
     self.reset_tables()
 
   def rates(self) -> List[float]:
@@ -411,11 +422,12 @@ class LatentAttention(Turning):
   @staticmethod
   def param_count(dim: int, p: dict) -> int:
     H, d, r, e, R = (p[n] for n in ("heads", "dim", "rot_dim", "vdim", "kv_rank"))
-    return dim * (H * (d + r) + R + r + H * e) + R * (H * (d + e) + 1)
+    extra = dim * H * e * bool(p.get("gate")) + H * bool(p.get("sink"))
+    return dim * (H * (d + r) + R + r + H * e) + R * (H * (d + e) + 1) + extra
 
   def forward(self, h, proj, at, state, rows, **out):
     return mo.latent_attn(proj, at["q"], at["dkv"], self.H, self.dim, self.rot_dim, self.rank, self.vdim, self.kv_norm,
-                          self.kv_up, self.freq, self.scale, self.eps, state, rows, **out)
+                          self.kv_up, self.freq, self.scale, self.eps, state, rows, self.sink, at.get("g"), **out)
 
 
 class RotaryAttention(Turning):
@@ -435,6 +447,8 @@ class RotaryAttention(Turning):
     having its own; lent: another layer reads this one's; keeps: the layer read
     from is in another shard, so this one caches what travels with the stream
   """
+
+  hip = ("_hip_rotary",)
 
   def __init__(self, dim: int, p: dict, eps: float):
     super().__init__()
@@ -539,6 +553,8 @@ class GatedLinearUnit(nn.Module):
 
   RATE = 8.0  # the decay's exponent at an open gate, in softplus(lam)
 
+  hip = ("_hip_lru", "_hip_scan",)
+
   def __init__(self, dim: int, p: dict, eps: float):
     super().__init__()
     self.width, self.blocks = p["width"], p["blocks"]
@@ -571,9 +587,48 @@ class GatedLinearUnit(nn.Module):
                          self.lam, self.RATE, state, rows, **out)
 
 
+class MatrixMemory(nn.Module):
+  """Matrix memory with exponential gates (the mLSTM of xLSTM): per head an fp32
+  state that decays by a forget gate and takes in the outer product of key and
+  value by an input gate, both kept as logarithms (capped) relative to a running
+  maximum; the read-out is divided by what the queries find of the keys, then
+  RMS-normed per head, weighted and gated."""
+
+  hip = ("_hip_mlstm",)
+
+  def __init__(self, dim: int, p: dict, eps: float):
+    super().__init__()
+    self.H, self.dim, self.vdim, self.cap, self.eps = p["heads"], p["dim"], p["vdim"], float(p["gate_cap"]), eps
+    if self.cap <= 0:
+      raise ValueError(f"gates capped at {self.cap}")
+    self.width = self.H * self.vdim
+    self.parts = [("q", self.H * self.dim), ("k", self.H * self.dim), ("v", self.width), ("g", self.width),
+                  ("i", self.H), ("f", self.H)]
+    self.gate_bias = nn.Parameter(torch.zeros(2, self.H))  # of the input gate, of the forget gate
+    self.norm = nn.Parameter(torch.ones(self.width))
+    self.init_ranges = {"gate_bias": (1.0, 5.0), "norm": (0.8, 1.2)}
+
+  @staticmethod
+  def state_spec(p: dict, capacity: int, dtype: torch.dtype, device) -> StateSpec:
+    # a row of key channels per value channel; the last one sums the keys alone
+    return {"s": ((p["heads"], p["vdim"] + 1, mo.row_pad(p["dim"])), torch.float32),
+            "m": ((p["heads"],), torch.float32)}
+
+  @staticmethod
+  def param_count(dim: int, p: dict) -> int:
+    H, d, e = p["heads"], p["dim"], p["vdim"]
+    return dim * H * (2 * d + 3 * e + 2) + H * (e + 2)
+
+  def forward(self, h, proj, at, state, rows, **out):
+    return mo.matrix_memory(proj, [at[n] for n, _ in self.parts], self.H, self.dim, self.vdim, self.gate_bias, self.cap,
+                            self.norm, self.eps, state, rows, **out)
+
+
 class SelectiveScan(nn.Module):
   """Selective state space: short causal convolution and silu, step sizes
   through a low-rank pair, an fp32 state [inner, state], skip and silu gate."""
+
+  hip = ("_hip_scan",)
 
   def __init__(self, dim: int, p: dict, eps: float):
     super().__init__()
@@ -643,12 +698,23 @@ class ChunkAttentionMixer(SingleMixer):
 
 class LatentAttentionMixer(SingleMixer):
   BRANCH = LatentAttention
-  TENSORS = {"dkv.norm": "kv_norm"}
+  TENSORS = {"dkv.norm": "kv_norm", "sink": "sink"}
 
   def key_map(self, src: str, dst: str) -> Dict[str, str]:
     own = self.branches["only"]
     up = f"{dst}branches.only.kv_up.weight"
     return {**super().key_map(src, dst), f"{src}uk": f"{up}@0", f"{src}uv": f"{up}@{own.H * own.dim}"}
+
+
+class MatrixMemoryMixer(SingleMixer):
+  BRANCH = MatrixMemory
+  TENSORS = {"norm": "norm"}
+
+  def key_map(self, src: str, dst: str) -> Dict[str, str]:
+    m = super().key_map(src, dst)
+    for i, gate in enumerate(("i", "f")):
+      m[f"{src}{gate}.b"] = f"{dst}branches.only.gate_bias@{i}"
+    return m
 
 
 class SelectiveScanMixer(SingleMixer):
@@ -687,4 +753,4 @@ class GatedLinearUnitMixer(SingleMixer):
 
 MIXERS = {"kept_attention": KeptAttentionMixer, "difference_attention": DifferenceAttentionMixer,
           "rglru": GatedLinearUnitMixer, "parallel": ParallelMixer, "wkv": WKVMixer, "chunk_attention": ChunkAttentionMixer,
-          "latent_attention": LatentAttentionMixer, "mamba1": SelectiveScanMixer}
+          "latent_attention": LatentAttentionMixer, "mamba1": SelectiveScanMixer, "mlstm": MatrixMemoryMixer}

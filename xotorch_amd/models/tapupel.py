@@ -107,11 +107,11 @@ class TapupelLayer(nn.Module):
 
 
 class TapupelModel(LayeredModel):
-  def make_layer(self, cfg: ModelConfig, spec: LayerSpec) -> nn.Module:
+  def make_layer(self, cfg: ModelConfig, spec: LayerSpec, place: int) -> nn.Module:
     return TapupelLayer(cfg, spec)
 
   @staticmethod
-  def entry(layer):
+  def entry(layer, cache=None):
     return mo.STREAM
 
 

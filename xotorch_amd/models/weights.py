@@ -37,6 +37,9 @@ def hf_key_map(shard, cfg):
   if mtype == "tapupel":
     from xotorch_amd.models.tapupel import key_map_tapupel
     return key_map_tapupel(shard, cfg)
+  if mtype == "dupolorn":
+    from xotorch_amd.models.dupolorn import key_map_dupolorn
+    return key_map_dupolorn(shard, cfg)
   return _hf_key_map_llama(shard, cfg)
 
 

@@ -12,7 +12,7 @@ import subprocess
 import sys
 import sysconfig
 from pathlib import Path
-from typing import List
+from typing import List, Optional, Sequence
 
 PKG_DIR = Path(__file__).resolve().parent
 # extension module -> its source
@@ -25,6 +25,8 @@ EXTENSIONS = {
   "_hip_experts": PKG_DIR / "hip" / "expert_ops.hip",
   "_hip_scan": PKG_DIR / "hip" / "scan_ops.hip",
   "_hip_latent": PKG_DIR / "hip" / "latent_ops.hip",
+  "_hip_stream": PKG_DIR / "hip" / "stream_ops.hip",
+  "_hip_mlstm": PKG_DIR / "hip" / "mlstm_ops.hip",
 }
 
 
@@ -57,10 +59,11 @@ def _command(name: str, out: Path) -> List[str]:
   return cmd + ["-ltorch", "-ltorch_hip", "-lc10", "-lc10_hip", "-ltorch_python"]
 
 
-def build(force: bool = False, verbose: bool = True, missing_only: bool = False) -> List[Path]:
-  """Compile the extensions that are missing or older than their source;
-  `force` compiles all, `missing_only` trusts what is built already."""
-  names = [n for n in EXTENSIONS if force or (not out_path(n).exists() if missing_only else needs_build(n))]
+def build(force: bool = False, verbose: bool = True, missing_only: bool = False,
+          only: Optional[Sequence[str]] = None) -> List[Path]:
+  """Compile the extensions (`only`: of these) that are missing or older than their
+  source; `force` compiles all, `missing_only` trusts what is built already."""
+  names = [n for n in (EXTENSIONS if only is None else only) if force or (not out_path(n).exists() if missing_only else needs_build(n))]
   jobs = []
   for n in names:
     # compile beside the target and move into place: a concurrent reader sees

@@ -4,7 +4,8 @@
 //           sink, a sigmoid gate per head
 //   CHUNK:  keys of the query's own chunk of the sequence, a bias that falls
 //           linearly with the distance, a learned sink per head
-//   CAUSAL: all earlier keys, plain softmax (prompts only)
+//   CAUSAL: all earlier keys; a learned sink per head or none; a sigmoid gate per
+//           value channel or none (prompts only)
 //   KEPT:   sliding window (or none) that keeps the first tokens in sight,
 //           capped scores, one or two maps over the same values, of which the
 //           second is subtracted and the difference normed
@@ -54,11 +55,17 @@ template <int MODE, typename T>
 struct Side {
   const T *proj, *sinks;
   // score of the extra entry in the denominator
-  DEVINL float sink(int h) const { return MODE == WINDOW ? 0.f : MODE == CHUNK ? ld(sinks + h) : -INFINITY; }
+  DEVINL float sink(int h) const {
+    return MODE == WINDOW ? 0.f : MODE == CHUNK || (MODE == CAUSAL && sinks) ? ld(sinks + h) : -INFINITY;
+  }
   // where the running maximum starts: finite, so that fully masked tiles are harmless
-  DEVINL float start(int h) const { return MODE == CAUSAL || MODE == KEPT ? -1e30f : sink(h); }
+  DEVINL float start(int h) const { return (MODE == CAUSAL && !sinks) || MODE == KEPT ? -1e30f : sink(h); }
   DEVINL float gate(const AttnArgs& a, size_t tok, int h) const {
     return MODE == WINDOW ? a.out_scale * sigmoidf(ld(proj + tok * a.N + a.g_at + h)) : a.out_scale;
+  }
+  // CAUSAL: columns of a token's gates, one per value channel of a head
+  DEVINL const T* gates(const AttnArgs& a, size_t tok, int h, int vdim) const {
+    return MODE == CAUSAL && proj ? proj + tok * a.N + a.g_at + h * vdim : nullptr;
   }
 };
 
@@ -230,6 +237,20 @@ __global__ __launch_bounds__(256) void attn_rows_prefill_kernel(
     const size_t tok = (size_t)b * a.S + s;
     if (s < len) f = side.gate(a, tok, h) * (MAPS == 2 ? f : 1.f / (sum + __expf(sink - m[t])));
     bf16_t* dst = out + tok * a.K + a.out_at + h * ws.vdim;
+    if (const bf16_t* gate = side.gates(a, tok, h, ws.vdim)) {
+      const bool vec = ((a.N | a.g_at | ws.vdim) & 3) == 0;
+#pragma unroll
+      for (int i = 0; i < VG; ++i) {
+        const int c = i * 16 + quad * 4;
+        float g[4];
+        if (vec && c < ws.vdim) ld4(gate + c, g);
+        else
+#pragma unroll
+          for (int r = 0; r < 4; ++r) g[r] = c + r < ws.vdim ? ld(gate + c + r) : 0.f;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[t][i][r] *= sigmoidf(g[r]);
+      }
+    }
 #pragma unroll
     for (int i = 0; i < VG; ++i) {
       const int c = i * 16 + quad * 4;
@@ -576,9 +597,10 @@ __global__ __launch_bounds__(64) void attn_rows_f32_kernel(
 #pragma unroll
     for (int i = 0; i < NC; ++i) sum[i] *= f;
   }
+  const float* gate = side.gates(a, (size_t)b * a.S + s, h, kv.vdim);
 #pragma unroll
   for (int i = 0; i < NC; ++i)
-    if (lane + i * 64 < kv.vdim) dst[lane + i * 64] = sum[i];
+    if (lane + i * 64 < kv.vdim) dst[lane + i * 64] = gate ? sum[i] / (1.f + expf(-gate[lane + i * 64])) : sum[i];
 }
 
 // ===========================================================================

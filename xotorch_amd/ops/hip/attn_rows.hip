@@ -330,8 +330,10 @@ void chunk_attn(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t H
 
 // Causal attention of prompt rows over workspaces in this file's layouts: q
 // [B,S,H,qd], k and v of every head for positions [0, rows), rows >= start+S.
+// sinks [H]; gates [B,S,N], of which columns g_at.. multiply the outputs.
 void causal_attn(Tensor q, Tensor k, Tensor v, int64_t dim, int64_t vdim, int64_t rows, double scale, OptT slots,
-                 OptT lens, int64_t start, Tensor out, int64_t out_at, double out_scale) {
+                 OptT lens, int64_t start, Tensor out, int64_t out_at, double out_scale, OptT sinks, OptT gates,
+                 int64_t g_at) {
   const auto dt = io_type(q);
   const bool bf = dt == torch::kBFloat16;
   for (const Tensor& t : {k, v, out}) check_io(t, dt);
@@ -343,15 +345,24 @@ void causal_attn(Tensor q, Tensor k, Tensor v, int64_t dim, int64_t vdim, int64_
   CHK(k.numel() == (int64_t)B * H * rows * (bf ? ws.kc * 32 : dim));
   CHK(v.numel() == (int64_t)B * H * rows * (bf ? ws.vg * 16 : vdim));
   CHK(out_at + H * vdim <= out.size(2) && out_at % 4 == 0 && out.size(2) % 4 == 0);
+  if (sinks) { check_io(*sinks, dt); CHK(sinks->numel() == H); }
+  if (gates) {
+    check_io(*gates, dt);
+    CHK(gates->dim() == 3 && gates->size(0) == B && gates->size(1) == S && g_at >= 0 && g_at + H * vdim <= gates->size(2));
+  }
   if (B == 0 || S == 0) return;
   const Step step = make_step(slots, c10::nullopt, lens, start, false, B);
-  const AttnArgs a{S, H, H, 0, (int)out.size(2), 0, 0, 0, 0, (int)out_at, (int)q.size(3), (float)scale, 0.f,
-                   (float)out_scale, 0, 0};
-  prefill_rows<CAUSAL>(bf, B, q, k, v, nullptr, nullptr, nullptr, nullptr, out, ws, (int)start, 0, a, step);
+  const AttnArgs a{S, H, H, gates ? (int)gates->size(2) : 0, (int)out.size(2), 0, 0, 0, (int)g_at, (int)out_at,
+                   (int)q.size(3), (float)scale, 0.f, (float)out_scale, 0, 0};
+  prefill_rows<CAUSAL>(bf, B, q, k, v, gates ? gates->data_ptr() : nullptr, sinks ? sinks->data_ptr() : nullptr, nullptr,
+                       nullptr, out, ws, (int)start, 0, a, step);
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("window_attn", &window_attn, "sliding-window attention with distance bias, sink and head gates");
   m.def("chunk_attn", &chunk_attn, "attention within chunks of the sequence: linear distance bias, learned sinks, mixed values");
-  m.def("causal_attn", &causal_attn, "causal attention of prompt rows over packed workspaces");
+  m.def("causal_attn", &causal_attn, "causal attention of prompt rows over packed workspaces, sinks, gates",
+        py::arg("q"), py::arg("k"), py::arg("v"), py::arg("dim"), py::arg("vdim"), py::arg("rows"), py::arg("scale"),
+        py::arg("slots"), py::arg("lens"), py::arg("start"), py::arg("out"), py::arg("out_at"), py::arg("out_scale"),
+        py::arg("sinks") = py::none(), py::arg("gates") = py::none(), py::arg("g_at") = 0);
 }

@@ -96,6 +96,8 @@ DEVINL void stv(T* p, const float* o) {
 // hardware exp2/log2/rcp (about one ulp each)
 DEVINL float sigmoidf(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 DEVINL float siluf(float x) { return x * sigmoidf(x); }
+// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) as z sigmoid(2 sqrt(2/pi) (..))
+DEVINL float gelu_tanh(float z) { return z * sigmoidf(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
 // log1p(e) = log(u) e / (u - 1) with u = 1 + e as rounded: exact where e is tiny
 DEVINL float softplusf(float x) {
   const float e = __expf(-fabsf(x)), u = 1.f + e;

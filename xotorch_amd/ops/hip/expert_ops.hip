@@ -2,12 +2,13 @@
 // routed and computed without the host seeing a count.
 //   - router: logits on matrix cores (fp32 accumulation), sigmoid scores, a
 //     correction that only chooses, group-limited top-k, or a softmax over the
-//     chosen logits; experts that every token uses; counts per block
+//     chosen logits; experts that every token uses, gated or not; counts per block
 //   - place: every (token, expert) pair gets a row; rows of an expert lie
 //     together, in token order
 //   - grouped products: gate and up of a pair's token with the gated activation
-//     in the epilogue, then down; a weight-streaming form for few tokens per
-//     expert and a tiled form for many
+//     in the epilogue, or up alone, squared where it is positive, then down; a
+//     weight-streaming form for few tokens per expert and a tiled form for many.
+//     A weight that multiplies a pair's input scales the product's rows
 //   - add_norm: stream += mult * (a sublayer's output, or the weighted sum of a
 //     token's expert rows), then the stream's norm for the next sublayer
 //
@@ -24,7 +25,8 @@ constexpr int MAX_EXPERTS = 512, MAX_PICK = 16;  // shared ones among the expert
 
 // pick of E experts are chosen, then come top - pick that every token uses, all
 // in all; tile: rows of a tile
-struct RouteArgs { int T, D, E, top, groups, keep, nblk, tile; float scale; int pick, all, softmax; };
+// gate: the weight of these is the sigmoid of one more row of w, else one
+struct RouteArgs { int T, D, E, top, groups, keep, nblk, tile; float scale; int pick, all, softmax, gate; };
 
 // RW waves share k. Sixteen lanes choose for a token, J experts each.
 template <typename T, bool WHOLE, int J, int RW>
@@ -38,7 +40,7 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
   float* part = score + RT * a.E;
   int* chosen = (int*)(part + RW * RT * 65);
   float* open = (float*)(chosen + RT * a.top);  // [RT], the gate of the experts that every token uses
-  const int Z = a.E + (a.all > a.E);
+  const int Z = a.E + a.gate;
   const int t0 = blockIdx.x * RT, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
   const T* xr = x + (size_t)min(t0 + col, a.T - 1) * a.D;
   const int steps = (a.D + F::K - 1) / F::K;
@@ -149,7 +151,7 @@ __global__ __launch_bounds__(64 * RW) void route_kernel(
       chosen[t * a.top + k] = valid ? e : -1;
       if (valid) {
         idx[(size_t)(t0 + t) * a.top + k] = e;
-        weight[(size_t)(t0 + t) * a.top + k] = open[t];
+        weight[(size_t)(t0 + t) * a.top + k] = a.gate ? open[t] : 1.f;
       }
     }
   }
@@ -196,12 +198,13 @@ __global__ __launch_bounds__(256) void count_scan_kernel(int* __restrict__ count
   if (threadIdx.x == 255) total[blockIdx.x] = sums[255];
 }
 
-// Rows of all pairs: row[pair], token[row]; first row of every expert
-// [E + 1]; tiles (expert, first row), expert -1 past the last.
+// Rows of all pairs: row[pair], token[row] and, by_row given, the pair's weight;
+// first row of every expert [E + 1]; tiles (expert, first row), expert -1 past
+// the last.
 __global__ __launch_bounds__(256) void place_kernel(
     const int* __restrict__ idx, const int* __restrict__ rank, const int* __restrict__ before,
-    const int* __restrict__ total, int* __restrict__ row, int* __restrict__ token, int* __restrict__ first,
-    int2* __restrict__ tiles, int max_tiles, RouteArgs a) {
+    const int* __restrict__ total, const float* __restrict__ weight, int* __restrict__ row, int* __restrict__ token,
+    float* __restrict__ by_row, int* __restrict__ first, int2* __restrict__ tiles, int max_tiles, RouteArgs a) {
   __shared__ int at[MAX_EXPERTS], cnt[MAX_EXPERTS], tile_at[MAX_EXPERTS], ends[2];
   // a single block of the router needs no scan: its counts are the totals
   for (int e = threadIdx.x; e < a.all; e += 256) cnt[e] = a.nblk == 1 ? before[e] : total[e];
@@ -233,6 +236,7 @@ __global__ __launch_bounds__(256) void place_kernel(
     const int r = at[e] + (a.nblk == 1 ? 0 : before[(size_t)e * a.nblk + t / RT]) + rank[pair];
     row[pair] = r;
     token[r] = t;
+    if (by_row) by_row[r] = weight[pair];
   }
   if (blockIdx.x) return;
   for (int e = threadIdx.x; e < a.all; e += 256) {
@@ -255,20 +259,35 @@ DEVINL float gated(float g, float u, const Act& a) {
   return g * sigmoidf(a.alpha * g) * (u + a.plus);
 }
 
+// What a product is: of a pair's own row; of its token with gate and up weights
+// and the gated activation; of its token with one set of weights and the square
+// of what is positive.
+enum Product { PLAIN, GATED, RELU2 };
+
 struct GroupArgs {
   int K, kp, F, E;  // valid and stored length of a weight row, output features, experts
   int xs, ys;       // row strides of input and output
 };
 
+// A product's rows times what scales them, through its activation
+template <int KIND>
+DEVINL float activated(float by, float g, float u, const Act& a) {
+  if (KIND == GATED) return gated(by * g, by * u, a);
+  g = by * g;
+  if (KIND == RELU2) g = fmaxf(g, 0.f) * g;
+  return g;
+}
+
 // Few tokens per expert: a block owns 16 output features of one expert; its
 // four waves split k and walk the expert's rows 16 * MT at a time. GATED:
-// weights [E][2][F][kp], input rows gathered by token; else [E][F][kp].
-template <typename T, bool GATED, bool WHOLE, int MT>
+// weights [E][2][F][kp]; else [E][F][kp]. Input rows are gathered by token but
+// for PLAIN. by_row: what the rows of the product are scaled with.
+template <typename T, int KIND, bool WHOLE, int MT>
 __global__ __launch_bounds__(256) void expert_stream_kernel(
     const T* __restrict__ x, const T* __restrict__ w, const int* __restrict__ first, const int* __restrict__ token,
-    T* __restrict__ y, GroupArgs a, Act act) {
+    const float* __restrict__ by_row, T* __restrict__ y, GroupArgs a, Act act) {
   typedef Frag<T> F;
-  constexpr int NW = GATED ? 2 : 1, UN = 4;
+  constexpr int NW = KIND == GATED ? 2 : 1, UN = 4;
   __shared__ float part[4][NW][MT * 16][17];
   const int e = blockIdx.y, f0 = blockIdx.x * 16;
   const int lo = first[e], hi = first[e + 1];
@@ -284,7 +303,7 @@ __global__ __launch_bounds__(256) void expert_stream_kernel(
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
       const int r = min(r0 + m * 16 + col, hi - 1);
-      xr[m] = x + (size_t)(GATED ? token[r] : r) * a.xs;
+      xr[m] = x + (size_t)(KIND == PLAIN ? r : token[r]) * a.xs;
 #pragma unroll
       for (int i = 0; i < NW; ++i) acc[i][m] = (floatx4)(0.f);
     }
@@ -322,7 +341,8 @@ __global__ __launch_bounds__(256) void expert_stream_kernel(
 #pragma unroll
       for (int j = 0; j < NW; ++j)
         v[j] = part[0][j][t][f] + part[1][j][t][f] + part[2][j][t][f] + part[3][j][t][f];
-      st(y + (size_t)(r0 + t) * a.ys + f0 + f, GATED ? gated(v[0], v[NW - 1], act) : v[0]);
+      const float by = KIND != PLAIN && by_row ? by_row[r0 + t] : 1.f;
+      st(y + (size_t)(r0 + t) * a.ys + f0 + f, activated<KIND>(by, v[0], v[NW - 1], act));
     }
     __syncthreads();
   }
@@ -340,17 +360,18 @@ template <int TOK> struct TileShape {
   static constexpr int WAVES = TOK / 32, BUFS = TOK == 256 ? 2 : 3, BUF = (TILE_W + TOK) * 64;  // elements of a buffer
 };
 
-template <bool GATED, int TOK>
+template <int KIND, int TOK>
 __global__ __launch_bounds__(TOK * 2) void expert_tile_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, const int* __restrict__ first,
-    const int* __restrict__ token, const int2* __restrict__ tiles, bf16_t* __restrict__ y, int max_tiles,
-    int group, GroupArgs a, Act act) {
+    const int* __restrict__ token, const int2* __restrict__ tiles, const float* __restrict__ by_row,
+    bf16_t* __restrict__ y, int max_tiles, int group, GroupArgs a, Act act) {
   typedef TileShape<TOK> Sh;
+  constexpr bool TWO = KIND == GATED;  // weight rows are gate and up
   constexpr int WL = TILE_W / Sh::WAVES / 8, XL = 4, LOADS = WL + XL;  // loads of a stage and wave
   extern __shared__ __attribute__((aligned(16))) bf16_t buf[];  // [BUFS][weights [256][64], tokens [TOK][64]]
   // blocks go round the eight dies: give a die `group` neighbouring tiles and
   // all their features, so that its L2 serves both operands
-  const int nf = (a.F + (GATED ? 127 : 255)) / (GATED ? 128 : 256);
+  const int nf = (a.F + (TWO ? 127 : 255)) / (TWO ? 128 : 256);
   const int local = blockIdx.x >> 3, per = group * nf;
   const int m = (local / per * 8 + (blockIdx.x & 7)) * group + local % group, fb = local % per / group;
   if (m >= max_tiles) return;
@@ -360,7 +381,7 @@ __global__ __launch_bounds__(TOK * 2) void expert_tile_kernel(
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
   const int wf = wave & 1, wt = wave >> 1;  // which 128 weight rows, which 64 tokens
-  const int f0 = fb * (GATED ? 128 : 256);
+  const int f0 = fb * (TWO ? 128 : 256);
   // each wave stages its share of the weight rows and 32 tokens, 8 rows a load
   const bf16_t *wsrc[WL], *xsrc[XL];
   const int piece = ((lane & 7) ^ (lane >> 3)) * 8;
@@ -368,14 +389,14 @@ __global__ __launch_bounds__(TOK * 2) void expert_tile_kernel(
   for (int i = 0; i < WL; ++i) {
     const int r = (wave * WL + i) * 8 + (lane >> 3);
     // GATED rows: [64 gate, the same 64 up] for either half of the features
-    const int f = GATED ? f0 + (r >> 7) * 64 + (r & 63) : f0 + r;
-    const int part = GATED ? (r >> 6) & 1 : 0;
-    wsrc[i] = w + (((size_t)tile.x * (GATED ? 2 : 1) + part) * a.F + min(f, a.F - 1)) * a.kp + piece;
+    const int f = TWO ? f0 + (r >> 7) * 64 + (r & 63) : f0 + r;
+    const int part = TWO ? (r >> 6) & 1 : 0;
+    wsrc[i] = w + (((size_t)tile.x * (TWO ? 2 : 1) + part) * a.F + min(f, a.F - 1)) * a.kp + piece;
   }
 #pragma unroll
   for (int i = 0; i < XL; ++i) {
     const int t = min(r0 + wave * 32 + i * 8 + (lane >> 3), hi - 1);
-    xsrc[i] = x + (size_t)(GATED ? token[t] : t) * a.xs;
+    xsrc[i] = x + (size_t)(KIND == PLAIN ? t : token[t]) * a.xs;
   }
   auto stage = [&](int s) {
     const int k = s * 64;
@@ -447,13 +468,14 @@ __global__ __launch_bounds__(TOK * 2) void expert_tile_kernel(
     const int t = r0 + wt * 64 + j * 16 + col;
     if (t >= hi) continue;
     bf16_t* dst = y + (size_t)t * a.ys;
-    constexpr int N = GATED ? 4 : 8;
+    const float by = KIND != PLAIN && by_row ? by_row[t] : 1.f;
+    constexpr int N = TWO ? 4 : 8;
 #pragma unroll
     for (int i = 0; i < N; ++i) {
       const int f = f0 + wf * 16 * N + i * 16 + quad * 4;
       float v[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) v[r] = GATED ? gated(acc[i][j][r], acc[(i + 4) & 7][j][r], act) : acc[i][j][r];
+      for (int r = 0; r < 4; ++r) v[r] = activated<KIND>(by, acc[i][j][r], acc[(i + 4) & 7][j][r], act);
       if (f < a.F) st4(dst + f, v);
     }
   }
@@ -482,7 +504,7 @@ __global__ __launch_bounds__(256) void add_norm_kernel(
       ldv<V>(x + off + i, xv + c * V);
       if (top == 0) ldv<V>(y + (size_t)blockIdx.x * ys + i, sum);
       for (int k = 0; k < top; ++k) {
-        const float wk = weight[(size_t)blockIdx.x * top + k];
+        const float wk = weight ? weight[(size_t)blockIdx.x * top + k] : 1.f;
         float v[V];
         ldv<V>(y + (size_t)rows[(size_t)blockIdx.x * top + k] * ys + i, v);
 #pragma unroll
@@ -518,13 +540,16 @@ __global__ __launch_bounds__(256) void add_norm_kernel(
 // x [.., D] -> (weights [T, top] fp32, row of every pair [T, top], token of
 // every row, first row of every expert [E + 1], tiles [max, 2], rows of a tile).
 // `shared` experts follow the routed ones in every token's list (top counts
-// them then); their weight is the sigmoid of one more row of w.
+// them then); their weight is the sigmoid of one more row of w (gate) or one.
+// on_input: the weights by row [T * top].
 std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tensor w, OptT correction, int64_t pick,
                                                                   int64_t groups, int64_t keep, double scale,
-                                                                  bool softmax, int64_t shared) {
+                                                                  bool softmax, int64_t shared, bool gate,
+                                                                  bool on_input) {
   const auto dt = io_type(x);
   check_io(w, dt);
-  const int D = x.size(-1), T_ = x.numel() / D, E = w.size(0) - (shared > 0);
+  gate = gate && shared > 0;
+  const int D = x.size(-1), T_ = x.numel() / D, E = w.size(0) - gate;
   if (correction) { check_io(*correction, dt); CHK(correction->numel() == E); }
   CHK(w.dim() == 2 && w.size(1) == D && T_ > 0 && shared >= 0);
   const int64_t top = pick + shared, all = E + shared;
@@ -537,10 +562,12 @@ std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tens
   const int tile = pairs >= 320 * all ? 256 : 128, max_tiles = pairs / tile + std::min(pairs, (int)all);
   const auto ints = x.options().dtype(torch::kInt32);
   auto weight = f32(x, {T_, top});
+  Tensor by_row;
+  if (on_input) by_row = f32(x, {pairs});
   auto idx = torch::empty({T_, top}, ints), rank = torch::empty({T_, top}, ints), row = torch::empty({T_, top}, ints);
   auto counts = torch::empty({all, nblk}, ints), total = torch::empty({all}, ints), first = torch::empty({all + 1}, ints);
   auto token = torch::empty({pairs}, ints), tiles = torch::empty({max_tiles, 2}, ints);
-  const RouteArgs a{T_, D, E, (int)top, (int)groups, (int)keep, nblk, tile, (float)scale, (int)pick, (int)all, softmax};
+  const RouteArgs a{T_, D, E, (int)top, (int)groups, (int)keep, nblk, tile, (float)scale, (int)pick, (int)all, softmax, gate};
   const hipStream_t stream = cur_stream();
   CHK(groups <= 4 * 65);
   BY_TYPE(dt, {
@@ -562,22 +589,28 @@ std::tuple<Tensor, Tensor, Tensor, Tensor, Tensor, int64_t> route(Tensor x, Tens
   if (nblk > 1)
     hipLaunchKernelGGL(count_scan_kernel, dim3(all), dim3(256), 0, stream, counts.data_ptr<int>(), total.data_ptr<int>(), nblk);
   hipLaunchKernelGGL(place_kernel, dim3((pairs + 255) / 256), dim3(256), 0, stream, idx.data_ptr<int>(),
-                     rank.data_ptr<int>(), counts.data_ptr<int>(), total.data_ptr<int>(), row.data_ptr<int>(),
-                     token.data_ptr<int>(), first.data_ptr<int>(), (int2*)tiles.data_ptr<int>(), max_tiles, a);
-  return {weight, row, token, first, tiles, tile};
+                     rank.data_ptr<int>(), counts.data_ptr<int>(), total.data_ptr<int>(), P<float>(weight),
+                     row.data_ptr<int>(), token.data_ptr<int>(), on_input ? M<float>(by_row) : nullptr,
+                     first.data_ptr<int>(), (int2*)tiles.data_ptr<int>(), max_tiles, a);
+  return {on_input ? by_row : weight, row, token, first, tiles, tile};
 }
 
-// One grouped product over all pairs: gated (x by token, weights [E,2,F,kp]) or
-// plain (x by row, weights [E,F,kp]); kp: row length padded with zeros.
-Tensor expert_product(Tensor x, Tensor w, Tensor token, Tensor first, Tensor tiles, int64_t tile, bool gated_,
-                      double alpha, double limit, double plus) {
+// One grouped product over all pairs: GATED (x by token, weights [E,2,F,kp]),
+// RELU2 (x by token, weights [E,F,kp]) or PLAIN (x by row, weights [E,F,kp]); kp:
+// row length padded with zeros. by_row [pairs]: scales of the product's rows.
+Tensor expert_product(Tensor x, Tensor w, Tensor token, Tensor first, Tensor tiles, int64_t tile, int64_t kind,
+                      double alpha, double limit, double plus, OptT by_row) {
   const auto dt = io_type(x);
   check_io(w, dt);
+  CHK(kind == PLAIN || kind == GATED || kind == RELU2);
+  const bool gated_ = kind == GATED;
   CHK(w.dim() == (gated_ ? 4 : 3) && x.dim() == 2);
   for (const Tensor& t : {token, first, tiles}) check_io(t, torch::kInt32);
   const int E = w.size(0), F_ = w.size(-2), kp = w.size(-1), K = x.size(1), pairs = token.numel();
   CHK((!gated_ || w.size(1) == 2) && first.numel() == E + 1 && K <= kp && kp % 64 == 0 && F_ % 16 == 0 && kp - K < 64);
-  CHK(gated_ || x.size(0) == pairs);
+  CHK(kind != PLAIN || x.size(0) == pairs);
+  if (by_row) { check_io(*by_row, torch::kFloat32); CHK(kind != PLAIN && by_row->numel() == pairs); }
+  const float* bp = by_row ? P<float>(*by_row) : nullptr;
   auto y = torch::empty({pairs, F_}, x.options());
   const GroupArgs a{K, kp, F_, E, K, F_};
   const Act act{(float)alpha, (float)limit, (float)plus};
@@ -593,29 +626,33 @@ Tensor expert_product(Tensor x, Tensor w, Tensor token, Tensor first, Tensor til
     auto run = [&](auto kernel, int threads, int lds) {
       static const hipError_t err = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
       TORCH_CHECK(err == hipSuccess, "no LDS for expert tiles");
-      hipLaunchKernelGGL(kernel, grid, dim3(threads), lds, stream, P<bf16_t>(x), P<bf16_t>(w), fp, tp, tl, M<bf16_t>(y),
-                         max_tiles, group, a, act);
+      hipLaunchKernelGGL(kernel, grid, dim3(threads), lds, stream, P<bf16_t>(x), P<bf16_t>(w), fp, tp, tl, bp,
+                         M<bf16_t>(y), max_tiles, group, a, act);
     };
-#define TILES(GATED, TOK) \
-  run(expert_tile_kernel<GATED, TOK>, TOK * 2, TileShape<TOK>::BUFS * TileShape<TOK>::BUF * (int)sizeof(bf16_t))
-    if (gated_) { if (tile == 256) TILES(true, 256); else TILES(true, 128); }
-    else { if (tile == 256) TILES(false, 256); else TILES(false, 128); }
+#define TILES(KIND, TOK) \
+  run(expert_tile_kernel<KIND, TOK>, TOK * 2, TileShape<TOK>::BUFS * TileShape<TOK>::BUF * (int)sizeof(bf16_t))
+#define TILES_OF(KIND) if (tile == 256) TILES(KIND, 256); else TILES(KIND, 128)
+    if (kind == GATED) { TILES_OF(GATED); }
+    else if (kind == RELU2) { TILES_OF(RELU2); }
+    else { TILES_OF(PLAIN); }
+#undef TILES_OF
 #undef TILES
     return y;
   }
   const dim3 grid(F_ / 16, E);
-#define STREAM(GATED, WHOLE, MT)                                                                                \
-  hipLaunchKernelGGL((expert_stream_kernel<T, GATED, WHOLE, MT>), grid, dim3(256), 0, stream, P<T>(x), P<T>(w), fp, \
-                     tp, M<T>(y), a, act)
-#define STREAM_ROWS(GATED, WHOLE) \
-  if (pairs > 2 * E) STREAM(GATED, WHOLE, 2); else STREAM(GATED, WHOLE, 1)
+#define STREAM(KIND, WHOLE, MT)                                                                                 \
+  hipLaunchKernelGGL((expert_stream_kernel<T, KIND, WHOLE, MT>), grid, dim3(256), 0, stream, P<T>(x), P<T>(w), fp, \
+                     tp, bp, M<T>(y), a, act)
+#define STREAM_ROWS(KIND, WHOLE) \
+  if (pairs > 2 * E) STREAM(KIND, WHOLE, 2); else STREAM(KIND, WHOLE, 1)
+#define STREAM_OF(KIND) \
+  if (K % Frag<T>::K == 0) { STREAM_ROWS(KIND, true); } else { STREAM_ROWS(KIND, false); }
   BY_TYPE(dt, {
-    if (gated_) {
-      if (K % Frag<T>::K == 0) { STREAM_ROWS(true, true); } else { STREAM_ROWS(true, false); }
-    } else {
-      if (K % Frag<T>::K == 0) { STREAM_ROWS(false, true); } else { STREAM_ROWS(false, false); }
-    }
+    if (kind == GATED) { STREAM_OF(GATED) }
+    else if (kind == RELU2) { STREAM_OF(RELU2) }
+    else { STREAM_OF(PLAIN) }
   });
+#undef STREAM_OF
 #undef STREAM_ROWS
 #undef STREAM
   return y;
@@ -628,11 +665,10 @@ OptT add_norm(Tensor y, OptT rows, OptT weight, Tensor x, OptT w_next, double mu
   const int D = x.size(-1), n = x.numel() / D, ys = y.size(-1);
   int top = 0;
   if (rows) {
-    CHK(weight);
     check_io(*rows, torch::kInt32);
-    check_io(*weight, torch::kFloat32);
+    if (weight) { check_io(*weight, torch::kFloat32); CHK(weight->numel() == rows->numel()); }
     top = rows->size(-1);
-    CHK(rows->numel() == (int64_t)n * top && weight->numel() == rows->numel() && y.numel() == (int64_t)n * top * ys && ys >= D);
+    CHK(rows->numel() == (int64_t)n * top && y.numel() == (int64_t)n * top * ys && ys >= D);
   } else {
     CHK(y.numel() == x.numel() && ys == D);
   }
@@ -665,7 +701,13 @@ OptT add_norm(Tensor y, OptT rows, OptT weight, Tensor x, OptT w_next, double mu
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route", &route, "router: sigmoid scores or a softmax over the chosen, group-limited top-k, shared experts; rows of all pairs",
         py::arg("x"), py::arg("w"), py::arg("correction"), py::arg("top"), py::arg("groups"), py::arg("keep"),
-        py::arg("scale"), py::arg("softmax") = false, py::arg("shared") = 0);
-  m.def("expert_product", &expert_product, "grouped product of all (token, expert) pairs, gated or plain");
+        py::arg("scale"), py::arg("softmax") = false, py::arg("shared") = 0, py::arg("gate") = true,
+        py::arg("on_input") = false);
+  m.def("expert_product", &expert_product, "grouped product of all (token, expert) pairs, with an activation or plain",
+        py::arg("x"), py::arg("w"), py::arg("token"), py::arg("first"), py::arg("tiles"), py::arg("tile"), py::arg("kind"),
+        py::arg("alpha") = 0.0, py::arg("limit") = 0.0, py::arg("plus") = 0.0, py::arg("by_row") = py::none());
+  m.attr("PLAIN") = (int)PLAIN;
+  m.attr("GATED") = (int)GATED;
+  m.attr("RELU2") = (int)RELU2;
   m.def("add_norm", &add_norm, "stream += mult * (output or weighted expert rows); norm of the stream");
 }

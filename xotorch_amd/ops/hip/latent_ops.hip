@@ -6,7 +6,9 @@
 //   - prompts: latents of all earlier tokens are expanded by a GEMM;
 //     pack_heads lays its output out for causal_attn (attn_rows.hip)
 //   - decode: the expansion folds into query and output, so one pass over the
-//     latents serves all heads (latent_decode)
+//     latents serves all heads (latent_decode); gather_heads lays the expanded
+//     output out by token, times its gates
+// A head may have a sink, a learned score that joins the softmax's denominator.
 //
 // Cache, bf16: keys [slots][rows/16][KC][64][8] over R + r channels and values
 // [slots][VG][rows/32][64][8] over R channels, both in the fragment order of
@@ -180,8 +182,8 @@ __global__ __launch_bounds__(256) void pack_heads_kernel(
 template <int GW>
 __global__ __launch_bounds__(256) void latent_decode_kernel(
     const bf16_t* __restrict__ ql, const bf16_t* __restrict__ qr, const bf16_t* __restrict__ kc_,
-    const bf16_t* __restrict__ vc_, bf16_t* __restrict__ out, float* __restrict__ part, int splits, KVShape cache,
-    float scale, int H, int R, int r, Step step) {
+    const bf16_t* __restrict__ vc_, const bf16_t* __restrict__ sinks, bf16_t* __restrict__ out,
+    float* __restrict__ part, int splits, KVShape cache, float scale, int H, int R, int r, Step step) {
   extern __shared__ __attribute__((aligned(16))) bf16_t q[];  // [16][kc*32 + 8]
   __shared__ __attribute__((aligned(16))) bf16_t probs[16][128 + 8];
   __shared__ float tops[4][16], sums[4][16];
@@ -309,7 +311,7 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
           if (c < R) p[2 + c] = o[i][j];
         }
   } else {
-    const float f = 1.f / sum;
+    const float f = 1.f / (sum + (sinks ? __expf(ld(sinks + h) - m) : 0.f));
 #pragma unroll
     for (int i = 0; i < GW; ++i)
       if (i < ng)
@@ -321,7 +323,8 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
   }
 }
 
-__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part, bf16_t* __restrict__ out,
+__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part,
+                                                           const bf16_t* __restrict__ sinks, bf16_t* __restrict__ out,
                                                            int splits, int H, int R, Step step) {
   extern __shared__ float fac[];  // [splits]
   const int h = blockIdx.x, b = blockIdx.y, B = gridDim.y;
@@ -337,7 +340,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
       fac[s] = __expf(p0[s * stride] - M);
       L += fac[s] * p0[s * stride + 1];
     }
-    L = 1.f / wave_sum(L);
+    L = 1.f / (wave_sum(L) + (sinks ? __expf(ld(sinks + h) - M) : 0.f));
     for (int s = threadIdx.x; s < splits; s += 64) fac[s] *= L;
   }
   __syncthreads();
@@ -354,7 +357,8 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
 // of the cache through a running maximum; lanes over tokens, then over channels.
 __global__ __launch_bounds__(256) void latent_decode_f32_kernel(
     const float* __restrict__ ql, const float* __restrict__ qr, const float* __restrict__ kc,
-    const float* __restrict__ vc, float* __restrict__ out, KVShape cache, float scale, int H, int R, int r, Step step) {
+    const float* __restrict__ vc, const float* __restrict__ sinks, float* __restrict__ out, KVShape cache, float scale,
+    int H, int R, int r, Step step) {
   extern __shared__ float lds[];  // query [R + r], output [R]
   __shared__ float prob[256], red[8];
   const int h = blockIdx.x, b = blockIdx.y, B = gridDim.y, slot = step.slot(b), tid = threadIdx.x;
@@ -397,7 +401,24 @@ __global__ __launch_bounds__(256) void latent_decode_f32_kernel(
     }
     __syncthreads();
   }
+  if (sinks) l += expf(sinks[h] - m);
   for (int c = tid; c < R; c += 256) dst[c] = acc[c] / l;
+}
+
+// o [H,B,e] -> columns out_at.. of out [B,1,K], times the sigmoid of the
+// columns g_at.. of gates [B,1,N]
+template <typename T, int V>
+__global__ __launch_bounds__(256) void gather_heads_kernel(const T* __restrict__ o, const T* __restrict__ gates,
+                                                           T* __restrict__ out, int B, int HE, int e, int N, int g_at,
+                                                           int K, int out_at, float scale) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * V, b = blockIdx.y;
+  if (c >= HE) return;
+  float v[V], g[V];
+  ldv<V>(o + ((size_t)(c / e) * B + b) * e + c % e, v);
+  if (gates) ldv<V>(gates + (size_t)b * N + g_at + c, g);
+#pragma unroll
+  for (int i = 0; i < V; ++i) v[i] *= gates ? scale * sigmoidf(g[i]) : scale;
+  stv<V>(out + (size_t)b * K + out_at + c, v);
 }
 
 // ===========================================================================
@@ -499,7 +520,8 @@ std::tuple<Tensor, Tensor, int64_t> pack_heads(Tensor kv, Tensor rot, int64_t H,
 
 // Folded queries ql [H,B,R] and rotated ones qr [B,H,r] against the cache:
 // -> weighted latents [H,B,R]
-Tensor latent_decode(Tensor ql, Tensor qr, Tensor kc, Tensor vc, double scale, OptT slots, Tensor positions) {
+Tensor latent_decode(Tensor ql, Tensor qr, Tensor kc, Tensor vc, double scale, OptT slots, Tensor positions,
+                     OptT sinks) {
   const auto dt = io_type(ql);
   const bool bf = dt == torch::kBFloat16;
   for (const Tensor& t : {qr, kc, vc}) check_io(t, dt);
@@ -507,6 +529,7 @@ Tensor latent_decode(Tensor ql, Tensor qr, Tensor kc, Tensor vc, double scale, O
   const int H = ql.size(0), B = ql.size(1), R = ql.size(2), r = qr.size(2);
   const KVShape cache = cache_shape(bf, R, r, kc, vc);
   CHK((slots || B <= kc.size(0)) && B > 0 && B <= 65535);
+  if (sinks) { check_io(*sinks, dt); CHK(sinks->numel() == H); }
   const Step step = make_step(slots, positions, c10::nullopt, 0, true, B);
   auto out = torch::empty_like(ql);
   const hipStream_t stream = cur_stream();
@@ -514,7 +537,8 @@ Tensor latent_decode(Tensor ql, Tensor qr, Tensor kc, Tensor vc, double scale, O
     const size_t lds = (2 * R + r) * sizeof(float);
     TORCH_CHECK(lds <= 60000, "a latent of ", R, " channels does not fit LDS");
     hipLaunchKernelGGL(latent_decode_f32_kernel, dim3(H, B), dim3(256), lds, stream, P<float>(ql), P<float>(qr),
-                       P<float>(kc), P<float>(vc), M<float>(out), cache, (float)scale, H, R, r, step);
+                       P<float>(kc), P<float>(vc), sinks ? P<float>(*sinks) : nullptr, M<float>(out), cache,
+                       (float)scale, H, R, r, step);
     return out;
   }
   const size_t lds = 16 * (cache.kc * 32 + 8) * sizeof(bf16_t);
@@ -524,10 +548,11 @@ Tensor latent_decode(Tensor ql, Tensor qr, Tensor kc, Tensor vc, double scale, O
   Tensor part;
   if (splits > 1) part = f32(ql, {B, splits, H, R + 2});
   float* pp = splits > 1 ? M<float>(part) : nullptr;
+  const bf16_t* sp = sinks ? P<bf16_t>(*sinks) : nullptr;
   const dim3 grid(splits, hg, B);
 #define DECODE(GW)                                                                                                \
   hipLaunchKernelGGL((latent_decode_kernel<GW>), grid, dim3(256), lds, stream, P<bf16_t>(ql), P<bf16_t>(qr),      \
-                     P<bf16_t>(kc), P<bf16_t>(vc), M<bf16_t>(out), pp, splits, cache, (float)scale, H, R, r, step)
+                     P<bf16_t>(kc), P<bf16_t>(vc), sp, M<bf16_t>(out), pp, splits, cache, (float)scale, H, R, r, step)
   const int gw = (cache.vg + 3) / 4;
   if (gw <= 2) DECODE(2);
   else if (gw <= 4) DECODE(4);
@@ -535,13 +560,38 @@ Tensor latent_decode(Tensor ql, Tensor qr, Tensor kc, Tensor vc, double scale, O
   else DECODE(16);
 #undef DECODE
   if (splits > 1)
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(H, B), dim3(256), splits * sizeof(float), stream, pp, M<bf16_t>(out), splits, H, R, step);
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(H, B), dim3(256), splits * sizeof(float), stream, pp, sp, M<bf16_t>(out), splits, H, R, step);
   return out;
+}
+
+void gather_heads(Tensor o, OptT gates, int64_t g_at, Tensor out, int64_t out_at, double out_scale) {
+  const auto dt = io_type(o);
+  check_io(out, dt);
+  CHK(o.dim() == 3 && out.dim() == 3 && out.size(0) == o.size(1) && out.size(1) == 1);
+  const int H = o.size(0), B = o.size(1), e = o.size(2), K = out.size(2), N = gates ? gates->size(2) : 0;
+  CHK(out_at >= 0 && out_at + H * e <= K && B <= 65535);
+  if (gates) {
+    check_io(*gates, dt);
+    CHK(gates->dim() == 3 && gates->size(0) == B && gates->size(1) == 1 && g_at >= 0 && g_at + H * e <= N);
+  }
+  if (B == 0) return;
+#define GATHER(V)                                                                                                   \
+  hipLaunchKernelGGL((gather_heads_kernel<T, V>), dim3((H * e + 256 * V - 1) / (256 * V), B), dim3(256), 0,         \
+                     cur_stream(), P<T>(o), gates ? P<T>(*gates) : nullptr, M<T>(out), B, H * e, e, N, (int)g_at, K, \
+                     (int)out_at, (float)out_scale)
+  BY_TYPE(dt, {
+    if (((e | N | g_at | K | out_at) & 3) == 0) GATHER(4);
+    else GATHER(1);
+  });
+#undef GATHER
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_append", &latent_append, "latent norm, rotations, cache append and workspaces of a prompt chunk");
   m.def("latent_append_step", &latent_append_step, "the same for a decode step");
   m.def("pack_heads", &pack_heads, "expanded keys and values of all heads in attention order");
-  m.def("latent_decode", &latent_decode, "decode attention of all heads over cached latents");
+  m.def("latent_decode", &latent_decode, "decode attention of all heads over cached latents, with sinks",
+        py::arg("ql"), py::arg("qr"), py::arg("kc"), py::arg("vc"), py::arg("scale"), py::arg("slots"),
+        py::arg("positions"), py::arg("sinks") = py::none());
+  m.def("gather_heads", &gather_heads, "expanded outputs of a decode step by token, times their gates");
 }

@@ -17,9 +17,6 @@
 // width, channels of a part, input row and columns, taps, output row and column
 struct UnitArgs { int S, W, n, N, y_at, x_at, taps, K, out_at; float rate, out_scale; };
 
-// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) as z sigmoid(2 sqrt(2/pi) (..))
-DEVINL float gelu_tanh(float z) { return z * sigmoidf(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
-
 DEVINL float softplus_of(float lam) { return fmaxf(lam, 0.f) + log1pf(expf(-fabsf(lam))); }
 
 // 1 - exp(-x), x >= 0: the series where the difference would cancel

@@ -49,7 +49,7 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(
 #pragma unroll
           for (int j = 0; j < V; ++j) yv[c * V + j] = 0.f;
         for (int k = 0; rows && k < top; ++k) {
-          const float wk = weight[(size_t)blockIdx.x * top + k];
+          const float wk = weight ? weight[(size_t)blockIdx.x * top + k] : 1.f;
           float v[V];
           ldv<V>(y + (size_t)rows[(size_t)blockIdx.x * top + k] * ys + i, v);
 #pragma unroll
@@ -806,12 +806,12 @@ static OptT norm_host(const OptT& y, Tensor x, const OptT& w_post, const OptT& w
     CHK(w_post->numel() == D);
   }
   if (take) {
-    CHK(y && weight);
+    CHK(y);
     check_io(*take, torch::kInt32);
-    check_io(*weight, torch::kFloat32);
-    from = Gather{take->data_ptr<int>(), weight->data_ptr<float>(), (int)take->size(-1), (int)y->size(-1)};
-    CHK(take->numel() == (int64_t)rows * from.top && weight->numel() == take->numel() && from.ys >= D &&
-        y->numel() == take->numel() * from.ys);
+    if (weight) { check_io(*weight, torch::kFloat32); CHK(weight->numel() == take->numel()); }
+    from = Gather{take->data_ptr<int>(), weight ? weight->data_ptr<float>() : nullptr, (int)take->size(-1),
+                  (int)y->size(-1)};
+    CHK(take->numel() == (int64_t)rows * from.top && from.ys >= D && y->numel() == take->numel() * from.ys);
   } else if (y) {
     CHK(y->numel() == x.numel() && y->size(-1) == D);
   }
@@ -831,6 +831,7 @@ static OptT norm_host(const OptT& y, Tensor x, const OptT& w_post, const OptT& w
 }
 
 // take, weight [tokens, top]: y is not yet summed, row take[t, k] counts weight[t, k]
+// (no weight: one)
 OptT sandwich_norm(Tensor y, Tensor x, Tensor w_post, OptT w_next, double eps, bool copy, OptT take, OptT weight) {
   return norm_host(y, x, w_post, w_next, eps, copy, take, weight, io_type(y));
 }

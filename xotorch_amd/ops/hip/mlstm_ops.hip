@@ -1,0 +1,656 @@
+// CDNA4 (gfx950) kernels of matrix memories with exponential gates (the mLSTM
+// of xLSTM). Per head, with logs i and f of the input and forget gate,
+//   m_t = max(f_t + m_(t-1), i_t)                       m starts at 0
+//   S_t = e^{f_t + m_(t-1) - m_t} S_(t-1) + e^{i_t - m_t} k_t v_t^T
+//   o_t = S_t^T q_t / (max(|n_t q_t|, e^{-m_t}) + 1e-6)  n: S with v = 1
+// and o's RMS norm per head, a weight and a sigmoid gate. Gates, state, decays
+// and norms are fp32; q, k, v are bf16 or fp32.
+//
+// Prompts: gates_kernel makes the running maximum of a whole row, so that
+// chunks of tokens know theirs; memory_kernel walks the chunks. With F_t the log
+// forget gates of a chunk summed up to t, u_t = F_t - m_t and r_s = i_s - F_s:
+//   O_t = e^{u_t + m} q_t S + sum_{s<=t} e^{u_t + r_s} (q_t k_s) v_s
+//   S'  = e^{u_C + m} S + sum_s e^{u_C + r_s} k_s v_s^T
+// (m: the maximum before the chunk, C: its last token). No exponent is positive.
+// Decays scale whole tokens, so q, k and v enter the products as they are; what
+// is fp32 (S, decayed v, scores) enters bf16 products as a sum of two bf16
+// parts, which keeps 16 bits of mantissa.
+//
+// Rows of a step address state by slot (struct Step): slot -1 is a parked row,
+// which reads and writes no state and yields zeros. A row at position 0
+// ignores what its slot holds.
+
+#include "common.h"
+
+struct MemArgs {
+  int S, H, N, K;                            // tokens, heads, widths of input and output
+  int q_at, k_at, v_at, g_at, i_at, f_at, out_at;
+  int dim, vdim, dp;                         // dp: key channels of a state row
+  int P;                                     // tokens of a row in whole chunks
+  int seg, nseg;                             // chunks of a segment, segments
+  float cap, eps, scale, out_scale;
+};
+
+template <typename T> constexpr int chunk_of() { return sizeof(T) == 2 ? 64 : 32; }
+
+// log gates of a token: cap tanh((z + b) / cap), of the forget gate through logsigmoid
+DEVINL float log_gate(float z, float bias, float cap) { return cap * tanhf((z + bias) / cap); }
+DEVINL float log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
+
+// One block per (head, row): u, r [B][H][P] and m [B][H][P + 1], m[0] that before
+// the row. A thread has `per` tokens (a power of two, so that chunks begin at
+// threads or threads at chunks).
+template <typename T>
+__global__ __launch_bounds__(256) void gates_kernel(
+    const T* __restrict__ proj, const T* __restrict__ bias, float* __restrict__ state_m, float* __restrict__ u,
+    float* __restrict__ r, float* __restrict__ m, int per, MemArgs a, Step step) {
+  constexpr int C = chunk_of<T>();
+  const int h = blockIdx.x, b = blockIdx.y, slot = step.slot(b), len = step.len(b, a.S);
+  if (slot < 0 || len <= 0) return;
+  __shared__ float wf[4], wm[4];
+  const size_t row = (size_t)b * a.H + h;
+  u += row * a.P;
+  r += row * a.P;
+  m += row * (a.P + 1);
+  const float bi = ld(bias + h), bf = ld(bias + a.H + h);
+  const float m0 = step.first(b) ? state_m[(size_t)slot * a.H + h] : 0.f;
+  const int t0 = threadIdx.x * per, t1 = min(t0 + per, a.P), lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  float F = 0.f, M = -INFINITY;  // of the thread's tokens: summed log forget gates, maximum
+  for (int t = t0; t < t1; ++t) {
+    float li = -INFINITY, lf = 0.f;
+    if (t < len) {
+      const T* z = proj + ((size_t)b * a.S + t) * a.N;
+      li = log_gate(ld(z + a.i_at + h), bi, a.cap);
+      lf = log_sigmoid(log_gate(ld(z + a.f_at + h), bf, a.cap));
+    }
+    r[t] = li;  // read again below
+    u[t] = lf;
+    if (per > C && t % C == 0) F = 0.f;
+    F += lf;
+    M = fmaxf(M + lf, li);
+  }
+  // summed forget gates of the chunk before this thread (threads of a chunk are neighbours)
+  const int group = per >= C ? 1 : C / per;
+  float before = F;
+  for (int d = 1; d < group; d <<= 1) {
+    const float o = __shfl_up(before, d);
+    if ((lane & (group - 1)) >= d) before += o;
+  }
+  before = __shfl_up(before, 1);
+  if ((lane & (group - 1)) == 0) before = 0.f;
+  // maxima: (F, M) of a range followed by (F', M') is (F + F', max(M + F', M'))
+  float sf = 0.f, sm = M;
+  for (int t = t0; t < t1; ++t) sf += u[t];
+  for (int d = 1; d < 64; d <<= 1) {
+    const float of = __shfl_up(sf, d), om = __shfl_up(sm, d);
+    if (lane >= d) { sm = fmaxf(om + sf, sm); sf += of; }
+  }
+  if (lane == 63) { wf[wave] = sf; wm[wave] = sm; }
+  sf = __shfl_up(sf, 1);
+  sm = __shfl_up(sm, 1);
+  if (lane == 0) { sf = 0.f; sm = -INFINITY; }
+  __syncthreads();
+  float now = m0;
+  for (int w = 0; w < wave; ++w) now = fmaxf(now + wf[w], wm[w]);
+  now = fmaxf(now + sf, sm);
+  if (threadIdx.x == 0) m[0] = m0;
+  F = before;
+  for (int t = t0; t < t1; ++t) {
+    const float li = r[t], lf = u[t];
+    if (t % C == 0) F = 0.f;
+    F += lf;
+    now = fmaxf(now + lf, li);
+    m[t + 1] = now;
+    u[t] = F - now;
+    r[t] = li - F;
+    if (t == a.P - 1) state_m[(size_t)slot * a.H + h] = now;
+  }
+}
+
+// operand of a product whose k runs over tiles of 16: a lane holds 4 of each
+// tile at quad * 4, as it does of accumulators, so that these are operands too
+template <typename T> DEVINL typename Frag<T>::V ld_tiles(const T* p);
+template <> DEVINL bf16x8 ld_tiles<bf16_t>(const bf16_t* p) {
+  union { bf16x8 v; ushort4_t h[2]; } f;
+  f.h[0] = *(const ushort4_t*)p;
+  f.h[1] = *(const ushort4_t*)(p + 16);
+  return f.v;
+}
+template <> DEVINL floatx4 ld_tiles<float>(const float* p) { return *(const floatx4*)p; }
+
+// fp32 numbers of one k step as operands: bf16 in two parts, fp32 as it is
+template <typename T> struct Parts;
+template <> struct Parts<bf16_t> {
+  bf16x8 hi, lo;
+  DEVINL void set(const floatx4* v) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const float f = v[i >> 2][i & 3];
+      hi[i] = (__bf16)f;
+      lo[i] = (__bf16)(f - (float)hi[i]);
+    }
+  }
+  static DEVINL floatx4 times(const Parts& x, const bf16x8& y, floatx4 c) { return mma(x.lo, y, mma(x.hi, y, c)); }
+  static DEVINL floatx4 by(const bf16x8& y, const Parts& x, floatx4 c) { return mma(y, x.lo, mma(y, x.hi, c)); }
+};
+template <> struct Parts<float> {
+  floatx4 x;
+  DEVINL void set(const floatx4* v) { x = v[0]; }
+  static DEVINL floatx4 times(const Parts& x, const floatx4& y, floatx4 c) { return mma(x.x, y, c); }
+  static DEVINL floatx4 by(const floatx4& y, const Parts& x, floatx4 c) { return mma(y, x.x, c); }
+};
+DEVINL void to_floats(const bf16x8& f, floatx4* o) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) o[i >> 2][i & 3] = (float)f[i];
+}
+DEVINL void to_floats(const floatx4& f, floatx4* o) { o[0] = f; }
+
+// WHOLE walks a row from its state to its end. Where rows are few and long, they
+// are cut into segments: STATES walks each from zero and keeps its last state and
+// decay, segment_kernel makes the state every segment starts from, OUTPUTS walks
+// again from there.
+enum Pass { WHOLE, STATES, OUTPUTS };
+
+constexpr int ET = 2;  // tiles of 16 value channels that a wave owns
+
+template <typename T, int DT> struct MemShape {
+  static constexpr int C = chunk_of<T>(), DP = DT * 16;
+  static constexpr int QS = DP + (sizeof(T) == 2 ? 8 : 4), CS = C + 4;  // padded LDS rows
+  static size_t lds(int waves, bool outputs) {
+    size_t n = (size_t)(DP + waves * 32) * CS * sizeof(T) + (DP + 4 * C) * sizeof(float);
+    if (outputs) n += 2 * C * QS * sizeof(T) + (waves * 64 / C + waves + 1) * C * sizeof(float);
+    return n;
+  }
+};
+
+// One block per (segment, head, row), a wave per 32 value channels. A wave holds
+// its channels of the state as accumulators, DT tiles of 16 key channels.
+template <typename T, int DT, int PASS>
+__global__ __launch_bounds__(512) void memory_kernel(
+    const T* __restrict__ proj, const float* __restrict__ u, const float* __restrict__ r, const float* __restrict__ m,
+    const T* __restrict__ norm, float* __restrict__ state, float* __restrict__ part, float* __restrict__ decay,
+    T* __restrict__ out, MemArgs a, Step step) {
+  typedef MemShape<T, DT> Sh;
+  typedef typename Frag<T>::V V;
+  constexpr int C = Sh::C, DP = Sh::DP, QS = Sh::QS, CS = Sh::CS, KT = Frag<T>::K / 16;  // tiles of a k step
+  constexpr int TT = C / 16;
+  extern __shared__ __attribute__((aligned(16))) char mem[];
+  const int TH = blockDim.x, waves = TH >> 6, EP = waves * 32, parts = TH / C;
+  T* sKT = (T*)mem;             // [DP][CS] keys by channel
+  T* sVT = sKT + DP * CS;       // [EP][CS] values by channel
+  float* sn = (float*)(sVT + EP * CS);  // [DP] the sum of keys
+  float *su = sn + DP, *sr = su + C, *sw = sr + C, *sa = sw + C;
+  T* sQ = (T*)(sa + C);         // [C][QS]
+  T* sK = sQ + C * QS;          // [C][QS]
+  float* sdot = (float*)(sK + C * QS);  // [parts][C] queries with the sum of keys
+  float* ssq = sdot + parts * C;        // [waves][C] squares of outputs
+  float* srow = ssq + waves * C;        // [C] summed scores
+  const int seg = blockIdx.x, h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63, col = lane & 15, quad = lane >> 4;
+  const int slot = step.slot(b), len = slot < 0 ? 0 : step.len(b, a.S);
+  const int c_lo = seg * a.seg, c_hi = min(c_lo + a.seg, a.P / C), c_end = min(c_hi, (len + C - 1) / C);
+  const size_t head = (size_t)b * a.H + h;
+  const float *ur = u + head * a.P, *rr = r + head * a.P, *mr = m + head * (a.P + 1);
+  const T* rows = proj + (size_t)b * a.S * a.N;
+  const int e0 = wave * 32;  // first value channel of this wave
+  const size_t plane = (size_t)(a.vdim + 1) * a.dp;
+  float* own = slot < 0 ? nullptr : state + ((size_t)slot * a.H + h) * plane;
+  float* mine = PASS == WHOLE ? own : part + (((size_t)b * a.nseg + seg) * a.H + h) * plane;
+  floatx4 S[DT][ET];
+  const bool from_zero = PASS == STATES || (PASS == WHOLE && (slot < 0 || step.first(b) == 0)) || c_lo >= c_end;
+#pragma unroll
+  for (int i = 0; i < DT; ++i)
+#pragma unroll
+    for (int e = 0; e < ET; ++e) {
+      const int c = e0 + e * 16 + col;
+      S[i][e] = from_zero || c >= a.vdim || i * 16 >= a.dp ? (floatx4)(0.f)
+                                                           : *(const floatx4*)(mine + (size_t)c * a.dp + i * 16 + quad * 4);
+    }
+  for (int d = tid; d < DP; d += TH) sn[d] = from_zero || d >= a.dp ? 0.f : mine[(size_t)a.vdim * a.dp + d];
+  float log_decay = 0.f;
+  const bool vec = ((a.dim | a.vdim | a.N | a.q_at | a.k_at | a.v_at) & 3) == 0;
+  for (int ch = c_lo; ch < c_end; ++ch) {
+    const int t0 = ch * C;
+    __syncthreads();  // everyone is done with the previous chunk
+    // 4 channels of 4 tokens at a time: rows of q and k, columns of k and v
+    auto stage = [&](int at, int n, int wide, T* by_row, T* by_col) {
+      const int groups = wide >> 2, low = groups % 16 ? 8 : 16;  // (widths are multiples of 32)
+      for (int idx = tid; idx < groups * (C / 4); idx += TH) {
+        const int cg = idx % low + idx / (low * 4) % (groups / low) * low;
+        const int tg = idx / low % 4 + idx / (groups * 4) * 4;
+        T x[4][4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int t = t0 + tg * 4 + j;
+          const T* src = rows + (size_t)t * a.N + at + cg * 4;
+          if (vec && t < len && cg * 4 < n) {
+            typedef __attribute__((ext_vector_type(4))) T T4;
+            *(T4*)x[j] = *(const T4*)src;
+          } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) x[j][i] = t < len && cg * 4 + i < n ? src[i] : (T)0;
+          }
+        }
+        typedef __attribute__((ext_vector_type(4))) T T4;
+        if (by_row)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) *(T4*)(by_row + (tg * 4 + j) * QS + cg * 4) = T4{x[j][0], x[j][1], x[j][2], x[j][3]};
+        if (by_col)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) *(T4*)(by_col + (cg * 4 + i) * CS + tg * 4) = T4{x[0][i], x[1][i], x[2][i], x[3][i]};
+      }
+    };
+    if (PASS != STATES) stage(a.q_at + h * a.dim, a.dim, DP, sQ, (T*)nullptr);
+    stage(a.k_at + h * a.dim, a.dim, DP, PASS != STATES ? sK : (T*)nullptr, sKT);
+    stage(a.v_at + h * a.vdim, a.vdim, EP, (T*)nullptr, sVT);
+    const float m_prev = mr[t0], u_last = ur[t0 + C - 1], whole = expf(u_last + m_prev);
+    for (int t = tid; t < C; t += TH) {
+      const float ut = ur[t0 + t], rt = rr[t0 + t];
+      su[t] = ut;
+      sr[t] = rt;
+      sw[t] = expf(u_last + rt);
+      sa[t] = expf(ut + m_prev) * a.scale;
+    }
+    __syncthreads();
+    if (PASS != STATES) {
+      {
+        const int t = tid % C, p = tid / C;
+        float dot = 0.f;
+        for (int d = p * DP / parts; d < (p + 1) * DP / parts; ++d) dot += sn[d] * ld(sQ + t * QS + d);
+        sdot[p * C + t] = dot;
+      }
+      floatx4 O[TT][ET];
+#pragma unroll
+      for (int tt = 0; tt < TT; ++tt) {
+        const int t = tt * 16 + col;
+        V qf[DT / KT];
+#pragma unroll
+        for (int c = 0; c < DT / KT; ++c) qf[c] = ld_tiles<T>(sQ + t * QS + c * KT * 16 + quad * 4);
+        // what earlier chunks left
+#pragma unroll
+        for (int e = 0; e < ET; ++e) O[tt][e] = (floatx4)(0.f);
+#pragma unroll
+        for (int c = 0; c < DT / KT; ++c)
+#pragma unroll
+          for (int e = 0; e < ET; ++e) {
+            floatx4 s[KT];
+#pragma unroll
+            for (int k = 0; k < KT; ++k) s[k] = S[c * KT + k][e];
+            Parts<T> p;
+            p.set(s);
+            O[tt][e] = Parts<T>::times(p, qf[c], O[tt][e]);
+          }
+        const float at = sa[t], ut = su[t];
+#pragma unroll
+        for (int e = 0; e < ET; ++e) O[tt][e] *= at;
+        // this chunk's tokens up to t
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j * KT <= tt; ++j) {
+          floatx4 w[KT];
+#pragma unroll
+          for (int k = 0; k < KT; ++k) {
+            const int st = j * KT + k;
+            w[k] = (floatx4)(0.f);
+            if (st > tt) continue;
+#pragma unroll
+            for (int c = 0; c < DT / KT; ++c)
+              w[k] = mma(ld_tiles<T>(sK + (st * 16 + col) * QS + c * KT * 16 + quad * 4), qf[c], w[k]);
+            const floatx4 r4 = *(const floatx4*)(sr + st * 16 + quad * 4);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const int s = st * 16 + quad * 4 + i;
+              w[k][i] = s <= t ? w[k][i] * a.scale * expf(ut + r4[i]) : 0.f;
+              sum += w[k][i];
+            }
+          }
+          Parts<T> p;
+          p.set(w);
+#pragma unroll
+          for (int e = 0; e < ET; ++e)
+            O[tt][e] = Parts<T>::by(ld_tiles<T>(sVT + (e0 + e * 16 + col) * CS + j * KT * 16 + quad * 4), p, O[tt][e]);
+        }
+        float sq = 0.f;
+#pragma unroll
+        for (int e = 0; e < ET; ++e)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) sq += O[tt][e][i] * O[tt][e][i];
+        sq += __shfl_xor(sq, 16);
+        sq += __shfl_xor(sq, 32);
+        sum += __shfl_xor(sum, 16);
+        sum += __shfl_xor(sum, 32);
+        if (quad == 0) ssq[wave * C + t] = sq;
+        if (quad == 0 && wave == 0) srow[t] = sum;
+      }
+      __syncthreads();
+#pragma unroll
+      for (int tt = 0; tt < TT; ++tt) {
+        const int t = tt * 16 + col;
+        if (t0 + t >= a.S) continue;
+        float dot = 0.f, sq = 0.f;
+        for (int p = 0; p < parts; ++p) dot += sdot[p * C + t];
+        for (int w = 0; w < waves; ++w) sq += ssq[w * C + t];
+        const bool live = t0 + t < len;
+        const float found = fabsf(srow[t] + sa[t] * dot);
+        const float inv = 1.f / (fmaxf(found, expf(live ? -mr[t0 + t + 1] : 0.f)) + 1e-6f);
+        const float f = inv / sqrtf(sq * inv * inv / (float)a.vdim + a.eps) * a.out_scale;
+        const size_t tok = (size_t)b * a.S + t0 + t;
+        T* dst = out + tok * a.K + a.out_at + h * a.vdim;
+        const T *gate = proj + tok * a.N + a.g_at + h * a.vdim, *nw = norm + h * a.vdim;
+#pragma unroll
+        for (int e = 0; e < ET; ++e) {
+          const int c = e0 + e * 16 + quad * 4;
+          float g[4], w[4], o[4];
+          const bool four = ((a.vdim | a.N | a.g_at | a.K | a.out_at) & 3) == 0;
+          if (c >= a.vdim) continue;
+          if (four) {
+            ld4(gate + c, g);
+            ld4(nw + c, w);
+          } else
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              g[i] = c + i < a.vdim ? ld(gate + c + i) : 0.f;
+              w[i] = c + i < a.vdim ? ld(nw + c + i) : 0.f;
+            }
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o[i] = live ? O[tt][e][i] * f * w[i] * sigmoidf(g[i]) : 0.f;
+          if (four) st4(dst + c, o);
+          else
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+              if (c + i < a.vdim) st(dst + c + i, o[i]);
+        }
+      }
+    }
+    // the state after this chunk
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+#pragma unroll
+      for (int e = 0; e < ET; ++e) S[i][e] *= whole;
+#pragma unroll
+    for (int j = 0; j < TT / KT; ++j) {
+      Parts<T> p[ET];
+#pragma unroll
+      for (int e = 0; e < ET; ++e) {
+        floatx4 w[KT];
+        to_floats(ld_tiles<T>(sVT + (e0 + e * 16 + col) * CS + j * KT * 16 + quad * 4), w);
+#pragma unroll
+        for (int k = 0; k < KT; ++k) w[k] *= *(const floatx4*)(sw + (j * KT + k) * 16 + quad * 4);
+        p[e].set(w);
+      }
+#pragma unroll
+      for (int i = 0; i < DT; ++i) {
+        const V kf = ld_tiles<T>(sKT + (i * 16 + col) * CS + j * KT * 16 + quad * 4);
+#pragma unroll
+        for (int e = 0; e < ET; ++e) S[i][e] = Parts<T>::by(kf, p[e], S[i][e]);
+      }
+    }
+    for (int d = tid; d < DP; d += TH) {
+      float n = sn[d] * whole;
+      for (int s = 0; s < C; s += 4) {
+        float k[4], w[4];
+        ld4(sKT + d * CS + s, k);
+        ld4(sw + s, w);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) n += k[i] * w[i];
+      }
+      sn[d] = n;
+    }
+    log_decay += u_last + m_prev;
+  }
+  // tokens past a row's end, and parked rows
+  if (PASS != STATES)
+    for (int t = max(c_lo, c_end) * C + wave; t < min(c_hi * C, a.S); t += waves)
+      for (int c = lane; c < a.vdim; c += 64) st(out + ((size_t)b * a.S + t) * a.K + a.out_at + h * a.vdim + c, 0.f);
+  if (PASS == OUTPUTS || len <= 0) return;
+  if (PASS == STATES && tid == 0) decay[((size_t)b * a.nseg + seg) * a.H + h] = expf(log_decay);
+#pragma unroll
+  for (int i = 0; i < DT; ++i)
+#pragma unroll
+    for (int e = 0; e < ET; ++e) {
+      const int c = e0 + e * 16 + col;
+      if (c < a.vdim && i * 16 < a.dp) *(floatx4*)(mine + (size_t)c * a.dp + i * 16 + quad * 4) = S[i][e];
+    }
+  for (int d = tid; d < a.dp; d += TH) mine[(size_t)a.vdim * a.dp + d] = sn[d];
+}
+
+// part [B][nseg][H][..]: every segment's own last state -> the state it starts
+// from; state: that after the row
+__global__ __launch_bounds__(256) void segment_kernel(float* __restrict__ part, const float* __restrict__ decay,
+                                                      float* __restrict__ state, int plane, MemArgs a, Step step) {
+  const int i = (blockIdx.x * 256 + threadIdx.x) * 4, h = blockIdx.y, b = blockIdx.z, slot = step.slot(b);
+  if (i >= plane || slot < 0 || step.len(b, a.S) <= 0) return;
+  floatx4* own = (floatx4*)(state + ((size_t)slot * a.H + h) * plane + i);
+  floatx4 now = step.first(b) ? *own : (floatx4)(0.f);
+  const size_t stride = (size_t)a.H * plane;
+  float* p = part + ((size_t)b * a.nseg * a.H + h) * plane + i;
+  constexpr int AHEAD = 8;
+  for (int s0 = 0; s0 < a.nseg; s0 += AHEAD) {
+    floatx4 x[AHEAD];
+    float d[AHEAD];
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (s0 + j < a.nseg) {
+        x[j] = *(const floatx4*)(p + (s0 + j) * stride);
+        d[j] = decay[((size_t)b * a.nseg + s0 + j) * a.H + h];
+      }
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (s0 + j < a.nseg) {
+        *(floatx4*)(p + (s0 + j) * stride) = now;
+        now = now * d[j] + x[j];
+      }
+  }
+  *own = now;
+}
+
+// Decode: one block per (head, row); 16 lanes share a column of the state, RPL
+// key channels each.
+template <int RPL> struct Rows {
+  static constexpr int V = RPL % 4 == 0 ? 4 : RPL % 2 == 0 ? 2 : 1;
+  static DEVINL int at(int j, int r) { return j * 16 * V + V * r; }
+};
+template <int V>
+DEVINL void ld_any(const float* p, float* o) {
+  if (V == 4) ld4(p, o);
+  else if (V == 2) ld2(p, o);
+  else o[0] = *p;
+}
+template <int V>
+DEVINL void st_any(float* p, const float* o) {
+  if (V == 4) st4(p, o);
+  else if (V == 2) st2(p, o);
+  else *p = o[0];
+}
+
+template <typename T, int RPL>
+__global__ __launch_bounds__(256) void memory_step_kernel(const T* __restrict__ proj, const T* __restrict__ bias,
+                                                          const T* __restrict__ norm, float* __restrict__ state,
+                                                          float* __restrict__ state_m, T* __restrict__ out, MemArgs a,
+                                                          Step step) {
+  constexpr int DP = 16 * RPL, NB = RPL <= 8 ? 4 : 2, VW = Rows<RPL>::V;  // NB: columns in flight per 16 lanes
+  __shared__ __attribute__((aligned(16))) float sq[DP], sk[DP];
+  __shared__ float so[257], red[4];
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, slot = step.slot(b);
+  T* dst = out + (size_t)b * a.K + a.out_at + h * a.vdim;
+  if (slot < 0) {
+    if (tid < a.vdim) st(dst + tid, 0.f);
+    return;
+  }
+  const int pos = step.first(b), r = tid & 15, cl = tid >> 4, cols = a.vdim + 1;
+  const T* row = proj + (size_t)b * a.N;
+  float* base = state + ((size_t)slot * a.H + h) * (size_t)cols * DP;
+  float s[NB][RPL];
+  auto load = [&](int c0) {
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      const int c = c0 + i * 16 + cl;
+#pragma unroll
+      for (int j = 0; j < RPL / VW; ++j) {
+        if (c < cols && pos > 0) ld_any<VW>(base + (size_t)c * DP + Rows<RPL>::at(j, r), s[i] + j * VW);
+        else
+#pragma unroll
+          for (int x = 0; x < VW; ++x) s[i][j * VW + x] = 0.f;
+      }
+    }
+  };
+  load(0);  // in flight while the gates are made
+  float v[(256 + 16) / 16 / NB + 1][NB];  // this lane's columns' values
+  const int rounds = (cols + 16 * NB - 1) / (16 * NB);
+#pragma unroll
+  for (int k = 0; k < (256 + 16) / 16 / NB + 1; ++k)
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      const int c = (k * NB + i) * 16 + cl;
+      v[k][i] = c < a.vdim ? ld(row + a.v_at + h * a.vdim + c) : 1.f;
+    }
+  if (tid < DP) {
+    sq[tid] = tid < a.dim ? ld(row + a.q_at + h * a.dim + tid) * a.scale : 0.f;
+    sk[tid] = tid < a.dim ? ld(row + a.k_at + h * a.dim + tid) : 0.f;
+  }
+  float* mp = state_m + (size_t)slot * a.H + h;
+  const float li = log_gate(ld(row + a.i_at + h), ld(bias + h), a.cap);
+  const float lf = log_sigmoid(log_gate(ld(row + a.f_at + h), ld(bias + a.H + h), a.cap));
+  const float m0 = pos > 0 ? *mp : 0.f, top = fmaxf(lf + m0, li);
+  const float keep = expf(lf + m0 - top), take = expf(li - top);
+  float gate = 0.f, weight = 0.f;
+  if (tid < a.vdim) {
+    gate = ld(row + a.g_at + h * a.vdim + tid);
+    weight = ld(norm + h * a.vdim + tid);
+  }
+  __syncthreads();
+  if (tid == 0) *mp = top;  // everyone has read it
+  float q[RPL], k[RPL];
+#pragma unroll
+  for (int j = 0; j < RPL / VW; ++j) {
+    ld_any<VW>(sq + Rows<RPL>::at(j, r), q + j * VW);
+    ld_any<VW>(sk + Rows<RPL>::at(j, r), k + j * VW);
+  }
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) k[i] *= take;
+#pragma unroll
+  for (int rd = 0; rd < (256 + 16) / 16 / NB + 1; ++rd) {
+    if (rd >= rounds) break;
+    const int c0 = rd * 16 * NB;
+    if (rd) load(c0);
+#pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      const int c = c0 + i * 16 + cl;
+      float o = 0.f;
+#pragma unroll
+      for (int j = 0; j < RPL; ++j) {
+        s[i][j] = keep * s[i][j] + k[j] * v[rd][i];
+        o += s[i][j] * q[j];
+      }
+      o = row_sum(o);
+      if (c < cols) {
+        if (r == 0) so[c] = o;
+#pragma unroll
+        for (int j = 0; j < RPL / VW; ++j) st_any<VW>(base + (size_t)c * DP + Rows<RPL>::at(j, r), s[i] + j * VW);
+      }
+    }
+  }
+  __syncthreads();
+  const float inv = 1.f / (fmaxf(fabsf(so[a.vdim]), expf(-top)) + 1e-6f);
+  const float y = tid < a.vdim ? so[tid] * inv : 0.f;
+  const float f = 1.f / sqrtf(block_sum(y * y, red) / (float)a.vdim + a.eps) * a.out_scale;
+  if (tid < a.vdim) st(dst + tid, y * f * weight * sigmoidf(gate));
+}
+
+// ===========================================================================
+// host side
+// ===========================================================================
+
+static int row_pad(int dim) {
+  for (int p : {1, 2, 3, 4, 6, 8, 12, 16})
+    if (dim <= 16 * p) return 16 * p;
+  TORCH_CHECK(false, "a memory of ", dim, " key channels (at most 256)");
+}
+
+template <typename T, int DT>
+static void prompt(const Tensor& proj, const Tensor& u, const Tensor& r, const Tensor& m, const Tensor& norm,
+                   Tensor& state, Tensor& out, int B, MemArgs a, const Step& step) {
+  typedef MemShape<T, DT> Sh;
+  const int waves = (a.vdim + 31) / 32, chunks = a.P / Sh::C, plane = (a.vdim + 1) * a.dp;
+  // rows are cut while the chip's 256 units do not have two blocks each; a
+  // segment is worth its second walk from four chunks on
+  const int want = (512 + B * a.H - 1) / (B * a.H), most = std::max(1, chunks / 4);
+  a.seg = (chunks + std::min(want, most) - 1) / std::min(want, most);
+  a.nseg = (chunks + a.seg - 1) / a.seg;
+  TORCH_CHECK(B <= 65535 && a.H <= 65535, "a prefill step of ", B, " rows and ", a.H, " heads is too large");
+  const hipStream_t stream = cur_stream();
+  Tensor part, decay;
+  if (a.nseg > 1) {
+    part = f32(proj, {B, a.nseg, a.H, plane});
+    decay = f32(proj, {B, a.nseg, a.H});
+  }
+  float *pp = a.nseg > 1 ? M<float>(part) : nullptr, *dp = a.nseg > 1 ? M<float>(decay) : nullptr;
+  auto run = [&](auto kernel, bool outputs) {
+    static const hipError_t err = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    TORCH_CHECK(err == hipSuccess, "no LDS for the memory's chunks");
+    const size_t lds = Sh::lds(waves, outputs);
+    TORCH_CHECK(lds <= 160 * 1024, "a memory of ", a.dim, " by ", a.vdim, " channels does not fit LDS");
+    hipLaunchKernelGGL(kernel, dim3(a.nseg, a.H, B), dim3(64 * waves), lds, stream, P<T>(proj), P<float>(u), P<float>(r),
+                       P<float>(m), P<T>(norm), M<float>(state), pp, dp, M<T>(out), a, step);
+  };
+  if (a.nseg == 1) { run(memory_kernel<T, DT, WHOLE>, true); return; }
+  run(memory_kernel<T, DT, STATES>, false);
+  hipLaunchKernelGGL(segment_kernel, dim3((plane / 4 + 255) / 256, a.H, B), dim3(256), 0, stream, pp, dp, M<float>(state),
+                     plane, a, step);
+  run(memory_kernel<T, DT, OUTPUTS>, true);
+}
+
+// proj [B,S,N]; bias [2,H] of input and forget gate; state [slots,H,vdim+1,dp]
+// (the last row sums the keys), state_m [slots,H]
+void matrix_memory(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_t g_at, int64_t i_at, int64_t f_at,
+                   int64_t H, int64_t dim, int64_t vdim, Tensor bias, double cap, Tensor norm, double eps, Tensor state,
+                   Tensor state_m, OptT slots, OptT positions, OptT lens, int64_t start, bool decode, Tensor out,
+                   int64_t out_at, double out_scale) {
+  const auto dt = io_type(proj);
+  for (const Tensor& t : {bias, norm, out}) check_io(t, dt);
+  check_io(state, torch::kFloat32);
+  check_io(state_m, torch::kFloat32);
+  CHK(proj.dim() == 3 && out.dim() == 3 && out.size(0) == proj.size(0) && out.size(1) == proj.size(1));
+  const int B = proj.size(0), S = proj.size(1), N = proj.size(2), dp = row_pad(dim);
+  CHK(H > 0 && dim > 0 && vdim > 0 && cap > 0);
+  TORCH_CHECK(vdim <= 256, "a memory of ", vdim, " value channels (at most 256)");
+  for (int64_t at : {q_at, k_at}) CHK(at >= 0 && at + H * dim <= N);
+  for (int64_t at : {v_at, g_at}) CHK(at >= 0 && at + H * vdim <= N);
+  CHK(i_at >= 0 && i_at + H <= N && f_at >= 0 && f_at + H <= N && out_at >= 0 && out_at + H * vdim <= out.size(2));
+  CHK(bias.numel() == 2 * H && norm.numel() == H * vdim && (!decode || S == 1));
+  CHK(state.dim() == 4 && state.size(1) == H && state.size(2) == vdim + 1 && state.size(3) == dp);
+  CHK(state_m.dim() == 2 && state_m.size(0) == state.size(0) && state_m.size(1) == H && (slots || B <= state.size(0)));
+  if (B == 0 || S == 0) return;
+  const Step step = make_step(slots, positions, lens, start, decode, B);
+  MemArgs a{S, (int)H, N, (int)out.size(2), (int)q_at, (int)k_at, (int)v_at, (int)g_at, (int)i_at, (int)f_at, (int)out_at,
+            (int)dim, (int)vdim, dp, 0, 0, 0, (float)cap, (float)eps, 1.f / sqrtf((float)dim), (float)out_scale};
+  const hipStream_t stream = cur_stream();
+  if (decode) {
+#define STEP(R)                                                                                                    \
+  case R: hipLaunchKernelGGL((memory_step_kernel<T, R>), dim3(H, B), dim3(256), 0, stream, P<T>(proj), P<T>(bias), \
+                             P<T>(norm), M<float>(state), M<float>(state_m), M<T>(out), a, step);                  \
+    break
+    BY_TYPE(dt, {
+      switch (dp / 16) { STEP(1); STEP(2); STEP(3); STEP(4); STEP(6); STEP(8); STEP(12); STEP(16); }
+    });
+#undef STEP
+    return;
+  }
+  BY_TYPE(dt, {
+    constexpr int C = chunk_of<T>();
+    a.P = (S + C - 1) / C * C;
+    auto u = f32(proj, {B, H, a.P}), r = f32(proj, {B, H, a.P}), m = f32(proj, {B, H, a.P + 1});
+    int per = 1;
+    while (per * 256 < a.P) per *= 2;
+    hipLaunchKernelGGL((gates_kernel<T>), dim3(H, B), dim3(256), 0, stream, P<T>(proj), P<T>(bias), M<float>(state_m),
+                       M<float>(u), M<float>(r), M<float>(m), per, a, step);
+    if (dp <= 32) prompt<T, 2>(proj, u, r, m, norm, state, out, B, a, step);
+    else if (dp <= 64) prompt<T, 4>(proj, u, r, m, norm, state, out, B, a, step);
+    else if (dp <= 128) prompt<T, 8>(proj, u, r, m, norm, state, out, B, a, step);
+    else prompt<T, 16>(proj, u, r, m, norm, state, out, B, a, step);
+  });
+}
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("matrix_memory", &matrix_memory, "matrix memory with exponential gates, per-head norm and output gate");
+}

@@ -10,7 +10,8 @@
 
 #include "common.h"
 
-struct ConvArgs { int S, C, N, at, taps, silu; };  // tokens, channels, input row, first column
+// tokens, channels, input row, first column; add: the input joins its convolution
+struct ConvArgs { int S, C, N, at, taps, silu, add; };
 
 constexpr int RUN = 16;  // tokens a thread walks
 
@@ -45,7 +46,9 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
   };
   constexpr int NT = TAPS ? TAPS : 1;
   float tw[NT][V], in[NT][V], bs[V];
-  ldv<V>(bias + c, bs);
+#pragma unroll
+  for (int i = 0; i < V; ++i) bs[i] = 0.f;
+  if (bias) ldv<V>(bias + c, bs);
   if (TAPS && s0 < len) {
 #pragma unroll
     for (int j = 0; j < NT; ++j)
@@ -82,6 +85,12 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
       if (a.silu)
 #pragma unroll
         for (int i = 0; i < V; ++i) y[i] = siluf(y[i]);
+      if (a.add) {
+        float v[V];
+        input(s, v);
+#pragma unroll
+        for (int i = 0; i < V; ++i) y[i] += v[i];
+      }
       if (step.decode) {
         float v[V];
         ldv<V>(rows, v);
@@ -333,26 +342,27 @@ __global__ __launch_bounds__(256) void scan_step_kernel(
 // ===========================================================================
 
 // x: C columns of proj [B,S,N] from column `at` on
-Tensor short_conv(Tensor proj, int64_t at, Tensor w, Tensor bias, OptT in_bias, bool silu, Tensor ring, OptT slots,
-                  OptT positions, OptT lens, int64_t start, bool decode) {
+Tensor short_conv(Tensor proj, int64_t at, Tensor w, OptT bias, OptT in_bias, bool silu, Tensor ring, OptT slots,
+                  OptT positions, OptT lens, int64_t start, bool decode, bool add) {
   const auto dt = io_type(proj);
-  for (const Tensor& t : {w, bias, ring}) check_io(t, dt);
+  for (const Tensor& t : {w, ring}) check_io(t, dt);
+  if (bias) { check_io(*bias, dt); CHK(bias->numel() == w.size(0)); }
   CHK(proj.dim() == 3 && w.dim() == 2 && ring.dim() == 3);
   const int B = proj.size(0), S = proj.size(1), N = proj.size(2), C = w.size(0), taps = w.size(1);
-  CHK(at + C <= N && bias.numel() == C && taps >= 1 && ring.size(1) == taps && ring.size(2) == C);
+  CHK(at + C <= N && taps >= 1 && ring.size(1) == taps && ring.size(2) == C);
   CHK((slots || B <= ring.size(0)) && (!decode || S == 1) && B <= 65535);
   auto out = torch::empty({B, S, C}, proj.options());
   if (B == 0 || S == 0) return out;
   const Step step = make_step(slots, positions, lens, start, decode, B);
   if (in_bias) { check_io(*in_bias, dt); CHK(in_bias->numel() == C); }
-  const ConvArgs a{S, C, N, (int)at, taps, silu};
+  const ConvArgs a{S, C, N, (int)at, taps, silu, add};
   const hipStream_t stream = cur_stream();
   const bool vec = ((C | N | (int)at) & 3) == 0;
   CHK((S + RUN - 1) / RUN <= 65535);
   const dim3 grid((C + (vec ? 1023 : 255)) / (vec ? 1024 : 256), (S + RUN - 1) / RUN, B);
 #define CONV(V, TAPS)                                                                                            \
-  hipLaunchKernelGGL((short_conv_kernel<T, V, TAPS>), grid, dim3(256), 0, stream, P<T>(proj), P<T>(w), P<T>(bias), \
-                     in_bias ? P<T>(*in_bias) : nullptr, M<T>(ring), M<T>(out), a, step)
+  hipLaunchKernelGGL((short_conv_kernel<T, V, TAPS>), grid, dim3(256), 0, stream, P<T>(proj), P<T>(w),             \
+                     bias ? P<T>(*bias) : nullptr, in_bias ? P<T>(*in_bias) : nullptr, M<T>(ring), M<T>(out), a, step)
 #define CONV_TAPS(V)               \
   if (taps == 4) CONV(V, 4);       \
   else if (taps == 3) CONV(V, 3);  \
@@ -442,6 +452,9 @@ void selective_scan(Tensor x, Tensor pre, Tensor bc, int64_t b_at, int64_t c_at,
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
-  m.def("short_conv", &short_conv, "short causal convolution with bias, and silu");
+  m.def("short_conv", &short_conv, "short causal convolution with bias, and silu; added to its input",
+        py::arg("proj"), py::arg("at"), py::arg("w"), py::arg("bias"), py::arg("in_bias"), py::arg("silu"),
+        py::arg("ring"), py::arg("slots"), py::arg("positions"), py::arg("lens"), py::arg("start"), py::arg("decode"),
+        py::arg("add") = false);
   m.def("selective_scan", &selective_scan, "selective state space scan with skip and gate");
 }

@@ -1,8 +1,8 @@
 """Dispatch of the token mixers' ops and of the fp32-residual norms.
 
 CUDA tensors run the HIP kernels of `_hip_mixers`, `_hip_attn`, `_hip_latent`,
-`_hip_scan`, `_hip_rotary`, `_hip_lru` and `_hip_experts` (hip/*.hip) in
-bfloat16 or true 32-bit, CPU tensors and training run torch_ref_mixers. A CUDA
+`_hip_scan`, `_hip_rotary`, `_hip_lru`, `_hip_mlstm`, `_hip_stream` and
+`_hip_experts` (hip/*.hip) in bfloat16 or true 32-bit, CPU tensors and training run torch_ref_mixers. A CUDA
 tensor never falls back: without the extension the op raises.
 
 A mixer's state is one tuple of tensors per layer whose first dimension is
@@ -50,6 +50,8 @@ class StepRows:
   carried: Dict[str, torch.Tensor] = field(default_factory=dict)
   # (state, source, key norm) of layers whose keys and values others read
   kept: Dict[int, tuple] = field(default_factory=dict)
+  # the stream as it was after the embedding and after every layer so far
+  depth: Optional["Depth"] = None
 
 
 def row_pad(dim: int) -> int:
@@ -88,7 +90,7 @@ class Weighted(NamedTuple):
   """sum_k weight[t, k] y[row[t, k]] for every token t, not yet summed."""
   y: torch.Tensor
   row: torch.Tensor
-  weight: torch.Tensor
+  weight: Optional[torch.Tensor]  # None: all one
 
 
 def sandwich_norm(y: Union[torch.Tensor, Weighted], x, w_post, w_next,
@@ -113,6 +115,117 @@ def add_norm(y: Union[torch.Tensor, Weighted], x, mult: float, w_next, eps: floa
   if _on_hip(y):
     return x, load_hip("_hip_experts").add_norm(y, None, None, x, w_next, mult, eps)
   return ref.add_norm(y, x, mult, w_next, eps)
+
+
+# ------------------------------------- embedding of pairs, averages over depth
+
+class Depth:
+  """The streams that averages over depth read: `streams[j]` in fp32, as views of
+  one slab on the HIP path, whose kernels fill it."""
+
+  def __init__(self, like, tokens: tuple, count: int, width: Optional[int] = None):
+    self.slab = None
+    if _on_hip(like):
+      self.slab = torch.empty(count, *tokens, width or like.shape[-1], dtype=torch.float32, device=like.device)
+    self.streams = []
+
+  def place(self):
+    """The slab's next place, which counts as filled."""
+    self.streams.append(self.slab[len(self.streams)])
+    return self.streams[-1]
+
+  def add(self, x):
+    if self.slab is not None:
+      self.place().copy_(x)
+    else:
+      self.streams.append(x)
+
+
+class Reads(NamedTuple):
+  """What a layer reads of the stream: RMS norms with one number each, and a
+  causal convolution over time that is added to the first."""
+  norms: Tuple[torch.Tensor, ...]
+  taps: Optional[torch.Tensor] = None
+  ring: Optional[torch.Tensor] = None  # the convolution's last inputs
+
+
+def embed_pairs(tokens, table, scale: float, pairs, rule: dict, last, rows: StepRows):
+  """fp32 rows of `table` times scale plus rows (previous token * mul_prev + token
+  * mul_cur) mod buckets of `pairs`; row `buckets` for a sequence's first token.
+  last: int32 [slots, 1], the token before a row's step, updated. The result is
+  the first of rows.depth."""
+  if _on_hip(table):
+    x = rows.depth.place()
+    load_hip("_hip_stream").embed_pairs(tokens, table, scale, pairs, rule["buckets"], rule["mul_prev"], rule["mul_cur"],
+                                        last, rows.slots, rows.positions, rows.lens, rows.start, rows.decode, x)
+    return x
+  x = ref.embed_pairs(tokens, table, scale, pairs, rule, last, rows)
+  rows.depth.add(x)
+  return x
+
+
+def input_conv(h, taps, ring, rows: StepRows):
+  """h plus its causal convolution over time."""
+  if _on_hip(h):
+    return load_hip("_hip_scan").short_conv(h, 0, taps, None, None, False, ring, rows.slots, rows.positions, rows.lens,
+                                            rows.start, rows.decode, True)
+  return ref.with_conv(h, taps, ring, rows)
+
+
+def read_stream(x, reads: Reads, eps: float, dtype: torch.dtype, rows: StepRows):
+  """A tuple: what `reads` says of the fp32 stream, in `dtype`."""
+  if _on_hip(x):
+    return _depth_norm(None, None, x, None, None, reads, eps, dtype, rows)[1]
+  h = [ref.scalar_norm(x, g, eps, dtype) for g in reads.norms]
+  if reads.taps is not None:
+    h[0] = input_conv(h[0], reads.taps, reads.ring, rows)
+  return tuple(h)
+
+
+def depth_norm(y, z, x, weights, reads: Optional[Reads], eps: float, dtype: torch.dtype, rows: StepRows):
+  """One layer's end: x + y + z joins rows.depth, the sum of its streams times
+  `weights` is the new stream. Returns it and what is read of it next."""
+  if _on_hip(y):
+    return _depth_norm(y, z, x, rows.depth, weights, reads, eps, dtype, rows)
+  new = x + y.float() if z is None else x + y.float() + z.float()
+  rows.depth.add(new)
+  x = sum(c * t for c, t in zip(weights.float(), rows.depth.streams, strict=True))
+  return x, None if reads is None else read_stream(x, reads, eps, dtype, rows)
+
+
+def _depth_norm(y, z, x, depth, weights, reads, eps, dtype, rows):
+  take = weigh = None
+  if isinstance(z, Weighted):
+    z, take, weigh = z
+  norms, taps, ring = reads if reads is not None else ((), None, None)
+  fused = rows.decode and taps is not None  # one token a row: the convolution's other inputs are in its state
+  done = len(depth.streams) if depth is not None else 0
+  x, *h = load_hip("_hip_stream").depth_norm(
+    y, z, take, weigh, x, depth.slab if depth is not None else None, done, weights, norms[0] if norms else None,
+    norms[1] if len(norms) > 1 else None, taps if fused else None, ring if fused else None, rows.slots, rows.positions,
+    eps, dtype == torch.bfloat16)
+  if depth is not None:
+    depth.place()
+  h = h[:len(norms)]
+  if taps is not None and not fused:
+    h[0] = input_conv(h[0], taps, ring, rows)
+  return x, tuple(h)
+
+
+def soft_cap(x, cap: float):
+  """cap * tanh(x / cap) in fp32."""
+  if _on_hip(x):
+    return load_hip("_hip_stream").soft_cap(x, cap)
+  return cap * torch.tanh(x.float() / cap)
+
+
+def gated_packed(gu, act: str):
+  """gelu_tanh(gate) * up on a packed [.., 2I] projection of any width and dtype."""
+  if act != "gelu_tanh":
+    raise ValueError(f"unknown activation {act!r}")
+  if _on_hip(gu):
+    return load_hip("_hip_stream").geglu_packed(gu)
+  return ref.gated_packed(gu, act)
 
 
 def swiglu_packed(gu):
@@ -201,14 +314,17 @@ def chunk_attn(proj, at, H: int, G: int, dim: int, vdim: int, q_norm, k_norm, si
 
 
 def latent_attn(proj, q_at: int, c_at: int, H: int, dim: int, rot_dim: int, rank: int, vdim: int, norm, up, freq,
-                scale: float, eps: float, state, rows: StepRows, out=None, out_at: int = 0, out_scale: float = 1.0):
+                scale: float, eps: float, state, rows: StepRows, sink=None, g_at: Optional[int] = None, out=None,
+                out_at: int = 0, out_scale: float = 1.0):
   """Causal attention over normed latents (`rank` columns of proj from c_at on,
   then a rotated key part that all heads share). `up` expands a latent into the
-  keys, then the values of all heads. Prompts expand the latents of all earlier
-  tokens; decode steps fold the expansion into query and output."""
+  keys, then the values of all heads. sink: a score per head that joins the
+  denominator; g_at: columns whose sigmoid multiplies the result. Prompts expand
+  the latents of all earlier tokens; decode steps fold the expansion into query
+  and output."""
   if not _on_hip(proj):
     return ref.latent_attn(proj, q_at, c_at, H, dim, rot_dim, rank, vdim, norm, up.weight, freq, scale, eps, state,
-                           rows) * out_scale
+                           rows, sink, g_at) * out_scale
   hip = load_hip("_hip_latent")
   out = _out(out, proj, H * vdim)
   sizes = (q_at, c_at, H, dim, rot_dim, rank, norm, freq, eps, state[0], state[1], rows.slots)
@@ -216,15 +332,29 @@ def latent_attn(proj, q_at: int, c_at: int, H: int, dim: int, rot_dim: int, rank
     qn, qr = hip.latent_append_step(proj, *sizes, rows.positions)
     w = up.weight
     folded = torch.bmm(qn, w[:H * dim].view(H, dim, rank))
-    seen = hip.latent_decode(folded, qr, state[0], state[1], scale, rows.slots, rows.positions)
+    seen = hip.latent_decode(folded, qr, state[0], state[1], scale, rows.slots, rows.positions, sink)
     o = torch.bmm(seen, _value_weights(up, H, dim))  # [H, B, vdim]
-    o = o.transpose(0, 1)
-    out[:, 0, out_at:out_at + H * vdim].unflatten(-1, (H, vdim)).copy_(o if out_scale == 1.0 else o * out_scale)
+    hip.gather_heads(o, proj if g_at is not None else None, g_at or 0, out, out_at, out_scale)
     return out
   q, latents, turned = hip.latent_append(proj, *sizes, rows.lens, rows.start)
   k, v, n = hip.pack_heads(up(latents), turned, H, dim, rot_dim, vdim)
   load_hip("_hip_attn").causal_attn(q, k, v, dim + rot_dim, vdim, n, scale, rows.slots, rows.lens, rows.start, out,
-                                    out_at, out_scale)
+                                    out_at, out_scale, sink, proj if g_at is not None else None, g_at or 0)
+  return out
+
+
+def matrix_memory(proj, at, H: int, dim: int, vdim: int, gate_bias, cap: float, norm, eps: float, state, rows: StepRows,
+                  out=None, out_at: int = 0, out_scale: float = 1.0):
+  """S = e^f S + e^i k v^T, read with q and divided by max(|n q|, 1), n the same
+  sum of the keys alone; all relative to a running maximum of the exponents (from
+  0 on), which a small constant in the divisor sees. An RMS norm per head, `norm`
+  and a sigmoid gate follow. `at` gives the columns of q, k, v, the output gate
+  and the logs of input and forget gate before cap, bias and sigmoid."""
+  if not _on_hip(proj):
+    return ref.matrix_memory(proj, at, H, dim, vdim, gate_bias, cap, norm, eps, state, rows) * out_scale
+  out = _out(out, proj, H * vdim)
+  load_hip("_hip_mlstm").matrix_memory(proj, *at, H, dim, vdim, gate_bias, cap, norm, eps, state[0], state[1], rows.slots,
+                                       rows.positions, rows.lens, rows.start, rows.decode, out, out_at, out_scale)
   return out
 
 
@@ -329,18 +459,36 @@ class Routing(NamedTuple):
   scale: float
   softmax: bool = False   # weights are the softmax over the chosen logits
   shared: int = 0         # experts after the routed ones that every token uses
+  shared_gate: bool = True  # their weight is the sigmoid of the router's last row (else one)
+  on_input: bool = False  # weights multiply the experts' input, not their output
 
 
-def expert_mixture(h, router, correction, gate_up, down, ff: int, rule: Routing, act):
-  """Weighted sum of each token's best experts and, weighed with the sigmoid of
-  the router's last row, of the shared ones. act: (alpha, limit, plus), the gated activation
-  min(g, limit) sigmoid(alpha min(g, limit)) (clamp(u, +-limit) + plus).
-  gate_up [E, 2, F, K] and down [E, D, F] are padded with zeros past the model's
-  width and `ff`."""
+class GatedAct(NamedTuple):
+  """min(g, limit) sigmoid(alpha min(g, limit)) (clamp(u, +-limit) + plus)."""
+  alpha: float
+  limit: float
+  plus: float
+  gated: bool = True
+
+
+class _Relu2:
+  gated = False
+
+
+RELU2 = _Relu2()
+
+
+def expert_mixture(h, router, correction, first, down, ff: int, rule: Routing, act):
+  """Weighted sum of each token's best experts and of the shared ones. first
+  [E, 2, F, K] (gate and up of a gated activation) or [E, F, K] and down [E, D, F]
+  are padded with zeros past the model's width and `ff`."""
   if _on_hip(h):
     hip = load_hip("_hip_experts")
     flat = h.view(-1, h.shape[-1])
+    # weights are per token and choice, for the sum, or per row, for the first product
     weight, row, *places = hip.route(flat, router, correction, *rule)
-    g = hip.expert_product(flat, gate_up, *places, True, *act)
-    return Weighted(hip.expert_product(g, down, *places, False, *act), row, weight)
-  return ref.expert_mixture(h, router, correction, gate_up, down, ff, rule, act)
+    alpha, limit, plus = act[:3] if act.gated else (0.0, 0.0, 0.0)
+    g = hip.expert_product(flat, first, *places, hip.GATED if act.gated else hip.RELU2, alpha, limit, plus,
+                           weight if rule.on_input else None)
+    return Weighted(hip.expert_product(g, down, *places, hip.PLAIN), row, None if rule.on_input else weight)
+  return ref.expert_mixture(h, router, correction, first, down, ff, rule, act)

@@ -227,7 +227,8 @@ def _rotate_pairs(x, start, freq):
   return torch.stack([u * a.cos() - v * a.sin(), v * a.cos() + u * a.sin()], dim=-1).flatten(-2)
 
 
-def latent_attn(proj, q_at, c_at, H, dim, rot_dim, rank, vdim, norm, up, freq, scale, eps, state, rows):
+def latent_attn(proj, q_at, c_at, H, dim, rot_dim, rank, vdim, norm, up, freq, scale, eps, state, rows, sink=None,
+                g_at=None):
   B, S, _ = proj.shape
   parts = {}
   for b, slot, start, n in _each_row(rows, B, S):
@@ -247,9 +248,69 @@ def latent_attn(proj, q_at, c_at, H, dim, rot_dim, rank, vdim, norm, up, freq, s
     s = torch.einsum("nhd,thd->nth", q, k) * scale
     i = torch.arange(T - n, T, device=proj.device)[:, None]
     s = s.masked_fill((torch.arange(T, device=proj.device)[None] > i)[:, :, None], float("-inf"))
-    o = torch.einsum("nth,the->nhe", torch.softmax(s, dim=1), kv[:, H * dim:].reshape(T, H, vdim))
+    if sink is not None:
+      s = torch.cat([s, sink.float().expand(n, 1, H)], dim=1)
+    o = torch.einsum("nth,the->nhe", torch.softmax(s, dim=1)[:, :T], kv[:, H * dim:].reshape(T, H, vdim))
     parts[b] = o.reshape(n, H * vdim)
+    if g_at is not None:
+      parts[b] = parts[b] * torch.sigmoid(row[:, g_at:g_at + H * vdim])
   return _scatter(parts, proj, H * vdim)
+
+
+def matrix_memory(proj, at, H, dim, vdim, gate_bias, cap, norm, eps, state, rows):
+  B, S, _ = proj.shape
+  parts = {}
+  for b, slot, start, n in _each_row(rows, B, S):
+    q, k, v, g, i, f = (proj[b, :n, a:a + w].float() for a, w in
+                        zip(at, (H * dim, H * dim, H * vdim, H * vdim, H, H)))
+    q, k, v = (t.reshape(n, H, -1) for t in (q * dim ** -0.5, k, v))
+    v = torch.cat([v, torch.ones_like(v[..., :1])], dim=-1)
+    i, f = (cap * torch.tanh((t + c.float()) / cap) for t, c in zip((i, f), gate_bias))
+    f = F.logsigmoid(f)
+    if state is None or start == 0:
+      M, m = q.new_zeros(H, vdim + 1, dim), q.new_zeros(H)
+    else:
+      M, m = state[0][slot][:, :, :dim].clone(), state[1][slot].clone()
+    outs = []
+    for t in range(n):
+      top = torch.maximum(f[t] + m, i[t])
+      M = (M * torch.exp(f[t] + m - top)[:, None, None]
+           + torch.exp(i[t] - top)[:, None, None] * v[t][:, :, None] * k[t][:, None, :])
+      m = top
+      o = (M * q[t][:, None, :]).sum(-1)
+      outs.append(o[:, :-1] / (torch.maximum(o[:, -1].abs(), torch.exp(-m)) + 1e-6)[:, None])
+    o = _rms(torch.stack(outs), eps).reshape(n, H * vdim) * norm.float()
+    parts[b] = o * torch.sigmoid(g)
+    if state is not None:
+      state[0][slot][:, :, :dim] = M
+      state[1][slot] = m
+  return _scatter(parts, proj, H * vdim)
+
+
+def embed_pairs(tokens, table, scale, pairs, rule, last, rows):
+  B, S = tokens.shape
+  row = torch.full_like(tokens, rule["buckets"])
+  row[:, 1:] = (tokens[:, :-1] * rule["mul_prev"] + tokens[:, 1:] * rule["mul_cur"]) % rule["buckets"]
+  if last is not None:
+    for b, slot, start, n in _each_row(rows, B, S):
+      if start:
+        row[b, 0] = (last[slot, 0].long() * rule["mul_prev"] + tokens[b, 0] * rule["mul_cur"]) % rule["buckets"]
+      last[slot, 0] = tokens[b, n - 1]
+  return F.embedding(tokens, table).float() * scale + F.embedding(row, pairs).float()
+
+
+def scalar_norm(x, weight, eps, dtype):
+  return (_rms(x.float(), eps) * weight.float()).to(dtype)
+
+
+def with_conv(h, taps, ring, rows):
+  y = short_conv(h, 0, taps, taps.new_zeros(taps.shape[0]), ring, rows, None, False)
+  return (h.float() + y.float()).to(h.dtype)
+
+
+def gated_packed(gu, act):
+  g, u = gu.float().chunk(2, dim=-1)
+  return (F.gelu(g, approximate="tanh") * u).to(gu.dtype)
 
 
 def _rotate(x, start, freq, pairs):
@@ -387,10 +448,9 @@ def selective_scan(x, pre, bc, b_at, c_at, z, z_at, a_log, dt_bias, skip, state,
   return _scatter(parts, x, C)
 
 
-def expert_mixture(h, router, correction, gate_up, down, ff, rule, act):
-  top, groups, keep, scale, softmax, shared = rule
-  alpha, limit, plus = act
-  D, E = h.shape[-1], router.shape[0] - bool(shared)
+def expert_mixture(h, router, correction, first, down, ff, rule, act):
+  top, groups, keep, scale, softmax, shared, shared_gate, on_input = rule
+  D, E = h.shape[-1], router.shape[0] - bool(shared_gate)
   flat = h.reshape(-1, D)
   z = flat.float() @ router.float().t()
   z, open_ = z[:, :E], torch.sigmoid(z[:, E:])
@@ -406,15 +466,19 @@ def expert_mixture(h, router, correction, gate_up, down, ff, rule, act):
   weight = (torch.softmax(weight, dim=-1) if softmax else weight) * scale
   if shared:
     idx = torch.cat([idx, torch.arange(E, E + shared, device=h.device).expand(len(idx), -1)], dim=1)
-    weight = torch.cat([weight, open_.expand(-1, shared)], dim=1)
+    weight = torch.cat([weight, open_.expand(-1, shared) if shared_gate else weight.new_ones(len(idx), shared)], dim=1)
   out = torch.zeros(flat.shape[0], D, dtype=torch.float32, device=h.device)
   for e in range(E + shared):
     tok, k = torch.where(idx == e)
     if tok.numel() == 0:
       continue
-    x, F_ = flat[tok], ff if e < E else gate_up.shape[2]
-    g, u = (F.linear(x, gate_up[e, i, :F_, :D]).float() for i in (0, 1))
-    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
-    a = (g * torch.sigmoid(alpha * g) * (u + plus)).to(h.dtype)
-    out = out.index_add(0, tok, F.linear(a, down[e, :D, :F_]).float() * weight[tok, k, None])
+    x, F_, w = flat[tok], ff if e < E else first.shape[-2], weight[tok, k, None]
+    before, after = (w, 1.0) if on_input else (1.0, w)  # the products are linear in their input
+    if act.gated:
+      g, u = (F.linear(x, first[e, i, :F_, :D]).float() * before for i in (0, 1))
+      g, u = g.clamp(max=act.limit), u.clamp(-act.limit, act.limit)
+      a = g * torch.sigmoid(act.alpha * g) * (u + act.plus)
+    else:
+      a = (F.linear(x, first[e, :F_, :D]).float() * before).relu().square()
+    out = out.index_add(0, tok, F.linear(a.to(h.dtype), down[e, :D, :F_]).float() * after)
   return out.to(h.dtype).view(h.shape)

@@ -114,7 +114,26 @@ def _tapupel_pair(model_id):
     "layers": [{"type": like[e["type"]][0], "mixer": like[e["type"]][1], "mlp": mlp} for e in cfg["layers"]]})]
 
 
-DESIGNS = {"didipel": _didipel_pair, "lebotar": _lebotar_pair, "tapupel": _tapupel_pair}
+def _dupolorn_pair(model_id):
+  """The registry's Dupolorn of that size, and lebotar (latent attention,
+  selective scan, sigmoid routing) with the same width, depth, heads, latent,
+  experts, vocabulary. Its experts have two products before the activation and
+  two thirds of the width, and it chooses one more in place of the shared one."""
+  from xotorch_amd.models.registry import builtin_config
+  cfg = builtin_config(model_id)
+  width, moe = cfg["width"], cfg["layers"][0]["mlp"]
+  lat = next(e["mixer"] for e in cfg["layers"] if e["type"] == "latent_attention")
+  like = {"latent_attention": ("latent_attention", lat), "latent_attention_2": ("latent_attention", lat),
+          "mlstm": ("mamba1", {"inner": 2 * width, "state": 16, "conv": 4, "dt_rank": width // 16})}
+  mlp = {"kind": "moe", "expert": {"ff": moe["expert"]["ff"] * 2 // 3, "limit": 7.0},
+         "router": {"experts": moe["router"]["experts"], "top": moe["router"]["top"] + 1, "scale": 2.5,
+                    "groups": {"count": 8, "keep": 4}}}
+  return [(model_id, cfg), ("lebotar of that size", {
+    "architecture": "Lebotar", "vocab": cfg["vocab"], "width": width, "norm": cfg["norm"], "residual_mult": 0.5,
+    "layers": [{"type": like[e["type"]][0], "mixer": like[e["type"]][1], "mlp": mlp} for e in cfg["layers"]]})]
+
+
+DESIGNS = {"didipel": _didipel_pair, "lebotar": _lebotar_pair, "tapupel": _tapupel_pair, "dupolorn": _dupolorn_pair}
 
 
 def design_bench(args):

@@ -43,7 +43,7 @@ def random_weights(cfg, seed=0, settled=False):
     w[name] = torch.randn(*shape, generator=g) * (shape[-1] ** -0.5 if std is None else std)
 
   def uniform(name, lo, hi, *shape):
-    w[name] = torch.rand(*shape, generator=g) * (hi - lo) + lo
+    w[name] = torch.rand(shape, generator=g) * (hi - lo) + lo
 
   def out(name, *shape):
     normal(name, *shape)
@@ -76,7 +76,7 @@ def random_weights(cfg, seed=0, settled=False):
       normal(p + "uk", H * d, R)
       normal(p + "uv", H * e, R)
       if layer["type"] == "latent_attention_2":
-        normal(p + "sink", H, std=1.5)
+        uniform(p + "sink", 0.0, 5.0, H)
         normal(p + "g", H * e, D)
     out(p + "o", D, m["heads"] * m["vdim"])
     p, m = f"l{i}.mlp.", layer["mlp"]

@@ -92,8 +92,10 @@ class DupolornLayer(nn.Module):
     return mo.Reads((self.norm1,) if self.mlp is None else (self.norm1, self.norm2), self.taps, ring)
 
   def step(self, x, h, cache, rows, after):
-    y = self.mix(h[0], cache, rows)
-    z = self.mlp(h[1]) if self.mlp is not None else None
+    if self.mlp is None:
+      y, z = self.mix(h[0], cache, rows), None
+    else:
+      y, z = mo.side_by_side(lambda: self.mix(h[0], cache, rows), lambda: self.mlp(h[1]))
     head = isinstance(after, nn.Parameter)
     x, h = mo.depth_norm(y, z, x, self.average, mo.Reads((after,)) if head else after, self.eps, y.dtype, rows)
     return x, h[0] if head else h

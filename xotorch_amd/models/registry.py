@@ -198,6 +198,29 @@ def _tapupel_sized(width, order, experts, top, ff=1408, vocab=32000, dim=128, wi
     moe={"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff}})
 
 
+def _dupolorn_cfg(width, order, vocab, latent, gated, mlstm, moe, dense, buckets, taps=4, scale=1.0, cap=30.0, eps=1e-6):
+  """order: one letter a layer, l(atent attention), g(ated latent attention) or
+  m(atrix memory); capitals have the dense feed-forward."""
+  kinds = {"l": ("latent_attention", latent), "g": ("latent_attention_2", gated), "m": ("mlstm", mlstm)}
+  return {
+    "architecture": "Dupolorn", "vocab": vocab, "width": width, "norm": {"eps": eps}, "logit_softcap": cap,
+    "canon": {"taps": taps}, "embedding": {"scale": scale, "bigram": {"buckets": buckets, "mul_prev": 31, "mul_cur": 17}},
+    "layers": [{"type": kinds[c.lower()][0], "mixer": kinds[c.lower()][1], "mlp": dense if c.isupper() else moe}
+               for c in order],
+  }
+
+
+def _dupolorn_sized(width, order, experts, top, ff=2112, vocab=32000, dim=128):
+  """Real-model proportions: heads and memories span the width."""
+  heads = width // dim
+  latent = {"heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 4 * dim,
+            "rot": {"base": 10000.0, "dims": dim // 2}, "scale": (dim + dim // 2) ** -0.5}
+  return _dupolorn_cfg(
+    width, order, vocab, latent, latent, mlstm={"heads": heads, "dim": dim, "vdim": dim, "gate_cap": 15.0},
+    moe={"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff}},
+    dense={"kind": "dense", "ff": 4 * width}, buckets=65521)
+
+
 BUILTIN_CONFIGS: Dict[str, dict] = {
   # llama 3.x family
   "llama-3.2-1b": _llama_cfg(2048, 16, 32, 8, 8192, tie=True, llama3_scaling=True, head_dim=64),
@@ -304,6 +327,16 @@ BUILTIN_CONFIGS: Dict[str, dict] = {
     rglru={"width": 96, "blocks": 6, "conv": 4},
     moe={"kind": "moe", "expert": {"ff": 40}, "router": {"experts": 6, "top": 2}, "shared": {"ff": 72}},
     dense={"kind": "dense", "ff": 104}),
+  # dupolorn, likewise (3B: 32 experts, 9B: 64 experts a layer)
+  "dupolorn-3b": _dupolorn_sized(2048, "gmlmgmlm", 32, 3),
+  "dupolorn-9b": _dupolorn_sized(2048, "gmlmgmlm" * 2, 64, 5),
+  "dupolorn-dummy": _dupolorn_cfg(
+    80, "mGlm", 256, buckets=97, taps=3, scale=3.0, cap=20.0,
+    latent={"heads": 3, "dim": 20, "rot_dim": 8, "vdim": 28, "kv_rank": 36, "rot": {"base": 1000.0, "dims": 8}, "scale": 0.19},
+    gated={"heads": 5, "dim": 24, "rot_dim": 16, "vdim": 16, "kv_rank": 52, "rot": {"base": 300.0, "dims": 16}, "scale": 0.16},
+    mlstm={"heads": 3, "dim": 28, "vdim": 20, "gate_cap": 9.0},
+    moe={"kind": "moe", "expert": {"ff": 40}, "router": {"experts": 6, "top": 2}, "shared": {"ff": 72}},
+    dense={"kind": "dense", "ff": 104}),
   "dummy": _llama_cfg(64, 4, 4, 2, 128, vocab=256, theta=10000.0, max_pos=256, tie=True),
 }
 # DeepSeek-Coder-V2-Lite shares the V2-Lite architecture exactly
@@ -376,6 +409,9 @@ model_cards: Dict[str, dict] = {
   "tapupel-3b": {"layers": 8, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "tapupel-9b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "tapupel-dummy": {"layers": 5, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "dupolorn-3b": {"layers": 8, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "dupolorn-9b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "dupolorn-dummy": {"layers": 3, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "dummy": {"layers": 4, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy", "DummyEngine": "dummy"}},
 }
 
@@ -435,6 +471,9 @@ pretty_names = {
   "tapupel-3b": "Tapupel 3B (random weights)",
   "tapupel-9b": "Tapupel 9B (random weights)",
   "tapupel-dummy": "Tapupel dummy (test)",
+  "dupolorn-3b": "Dupolorn 3B (random weights)",
+  "dupolorn-9b": "Dupolorn 9B (random weights)",
+  "dupolorn-dummy": "Dupolorn dummy (test)",
   "dummy": "Dummy (test)",
 }
 

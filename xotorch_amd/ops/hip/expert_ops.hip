@@ -279,17 +279,18 @@ DEVINL float activated(float by, float g, float u, const Act& a) {
 }
 
 // Few tokens per expert: a block owns 16 output features of one expert; its
-// four waves split k and walk the expert's rows 16 * MT at a time. GATED:
+// four waves split k and walk the expert's rows up to 64 at a time. GATED:
 // weights [E][2][F][kp]; else [E][F][kp]. Input rows are gathered by token but
 // for PLAIN. by_row: what the rows of the product are scaled with.
-template <typename T, int KIND, bool WHOLE, int MT>
+template <typename T, int KIND, bool WHOLE>
 __global__ __launch_bounds__(256) void expert_stream_kernel(
     const T* __restrict__ x, const T* __restrict__ w, const int* __restrict__ first, const int* __restrict__ token,
     const float* __restrict__ by_row, T* __restrict__ y, GroupArgs a, Act act) {
   typedef Frag<T> F;
-  constexpr int NW = KIND == GATED ? 2 : 1, UN = 4;
-  __shared__ float part[4][NW][MT * 16][17];
-  const int e = blockIdx.y, f0 = blockIdx.x * 16;
+  constexpr int NW = KIND == GATED ? 2 : 1;
+  __shared__ float part[4][NW][64][17];
+  // the last experts are the ones that every token uses: the longest come first
+  const int e = gridDim.y - 1 - blockIdx.y, f0 = blockIdx.x * 16;
   const int lo = first[e], hi = first[e + 1];
   if (lo == hi) return;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
@@ -297,7 +298,8 @@ __global__ __launch_bounds__(256) void expert_stream_kernel(
 #pragma unroll
   for (int i = 0; i < NW; ++i) wr[i] = w + (((size_t)e * NW + i) * a.F + f0 + col) * a.kp + quad * F::PER;
   const int steps = (a.K + F::K - 1) / F::K;
-  for (int r0 = lo; r0 < hi; r0 += 16 * MT) {
+  auto round = [&](int r0, auto tiles) {  // 16 * MT rows
+    constexpr int MT = decltype(tiles)::value, UN = MT == 4 ? 4 : 8 / NW;
     floatx4 acc[NW][MT];
     const T* xr[MT];
 #pragma unroll
@@ -345,7 +347,11 @@ __global__ __launch_bounds__(256) void expert_stream_kernel(
       st(y + (size_t)(r0 + t) * a.ys + f0 + f, activated<KIND>(by, v[0], v[NW - 1], act));
     }
     __syncthreads();
-  }
+  };
+  int r0 = lo;
+  for (; hi - r0 > 32; r0 += 64) round(r0, std::integral_constant<int, 4>());
+  if (hi - r0 > 16) round(r0, std::integral_constant<int, 2>());
+  else if (hi > r0) round(r0, std::integral_constant<int, 1>());
 }
 
 // Many tokens per expert (bf16): TOK tokens x 256 weight rows (GATED: 128 gate
@@ -640,20 +646,16 @@ Tensor expert_product(Tensor x, Tensor w, Tensor token, Tensor first, Tensor til
     return y;
   }
   const dim3 grid(F_ / 16, E);
-#define STREAM(KIND, WHOLE, MT)                                                                                 \
-  hipLaunchKernelGGL((expert_stream_kernel<T, KIND, WHOLE, MT>), grid, dim3(256), 0, stream, P<T>(x), P<T>(w), fp, \
+#define STREAM(KIND, WHOLE)                                                                                     \
+  hipLaunchKernelGGL((expert_stream_kernel<T, KIND, WHOLE>), grid, dim3(256), 0, stream, P<T>(x), P<T>(w), fp,     \
                      tp, bp, M<T>(y), a, act)
-#define STREAM_ROWS(KIND, WHOLE) \
-  if (pairs > 2 * E) STREAM(KIND, WHOLE, 2); else STREAM(KIND, WHOLE, 1)
-#define STREAM_OF(KIND) \
-  if (K % Frag<T>::K == 0) { STREAM_ROWS(KIND, true); } else { STREAM_ROWS(KIND, false); }
+#define STREAM_OF(KIND) if (K % Frag<T>::K == 0) STREAM(KIND, true); else STREAM(KIND, false);
   BY_TYPE(dt, {
     if (kind == GATED) { STREAM_OF(GATED) }
     else if (kind == RELU2) { STREAM_OF(RELU2) }
     else { STREAM_OF(PLAIN) }
   });
 #undef STREAM_OF
-#undef STREAM_ROWS
 #undef STREAM
   return y;
 }

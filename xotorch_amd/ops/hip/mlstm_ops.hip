@@ -14,7 +14,8 @@
 // (m: the maximum before the chunk, C: its last token). No exponent is positive.
 // Decays scale whole tokens, so q, k and v enter the products as they are; what
 // is fp32 (S, decayed v, scores) enters bf16 products as a sum of two bf16
-// parts, which keeps 16 bits of mantissa.
+// parts, which keeps 16 bits of mantissa. i, f, m, u and r are kept as logarithms
+// to base 2.
 //
 // Rows of a step address state by slot (struct Step): slot -1 is a parked row,
 // which reads and writes no state and yields zeros. A row at position 0
@@ -31,11 +32,17 @@ struct MemArgs {
   float cap, eps, scale, out_scale;
 };
 
-template <typename T> constexpr int chunk_of() { return sizeof(T) == 2 ? 64 : 32; }
+constexpr int C = 32;  // tokens of a chunk
 
 // log gates of a token: cap tanh((z + b) / cap), of the forget gate through logsigmoid
-DEVINL float log_gate(float z, float bias, float cap) { return cap * tanhf((z + bias) / cap); }
-DEVINL float log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
+constexpr float LOG2E = 1.4426950408889634f;
+DEVINL float capped(float z, float bias, float cap) { return cap * tanhf((z + bias) / cap); }
+DEVINL float log_input(float z, float bias, float cap) { return LOG2E * capped(z, bias, cap); }
+DEVINL float log_forget(float z, float bias, float cap) {
+  const float x = capped(z, bias, cap);
+  return LOG2E * (fminf(x, 0.f) - log1pf(expf(-fabsf(x))));
+}
+DEVINL float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
 
 // One block per (head, row): u, r [B][H][P] and m [B][H][P + 1], m[0] that before
 // the row. A thread has `per` tokens (a power of two, so that chunks begin at
@@ -44,7 +51,6 @@ template <typename T>
 __global__ __launch_bounds__(256) void gates_kernel(
     const T* __restrict__ proj, const T* __restrict__ bias, float* __restrict__ state_m, float* __restrict__ u,
     float* __restrict__ r, float* __restrict__ m, int per, MemArgs a, Step step) {
-  constexpr int C = chunk_of<T>();
   const int h = blockIdx.x, b = blockIdx.y, slot = step.slot(b), len = step.len(b, a.S);
   if (slot < 0 || len <= 0) return;
   __shared__ float wf[4], wm[4];
@@ -56,12 +62,13 @@ __global__ __launch_bounds__(256) void gates_kernel(
   const float m0 = step.first(b) ? state_m[(size_t)slot * a.H + h] : 0.f;
   const int t0 = threadIdx.x * per, t1 = min(t0 + per, a.P), lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   float F = 0.f, M = -INFINITY;  // of the thread's tokens: summed log forget gates, maximum
+#pragma unroll 4
   for (int t = t0; t < t1; ++t) {
     float li = -INFINITY, lf = 0.f;
     if (t < len) {
       const T* z = proj + ((size_t)b * a.S + t) * a.N;
-      li = log_gate(ld(z + a.i_at + h), bi, a.cap);
-      lf = log_sigmoid(log_gate(ld(z + a.f_at + h), bf, a.cap));
+      li = log_input(ld(z + a.i_at + h), bi, a.cap);
+      lf = log_forget(ld(z + a.f_at + h), bf, a.cap);
     }
     r[t] = li;  // read again below
     u[t] = lf;
@@ -154,12 +161,41 @@ enum Pass { WHOLE, STATES, OUTPUTS };
 constexpr int ET = 2;  // tiles of 16 value channels that a wave owns
 
 template <typename T, int DT> struct MemShape {
-  static constexpr int C = chunk_of<T>(), DP = DT * 16;
-  static constexpr int QS = DP + (sizeof(T) == 2 ? 8 : 4), CS = C + 4;  // padded LDS rows
+  static constexpr int DP = DT * 16;
+  static constexpr int PAD = sizeof(T) == 2 ? 8 : 4, QS = DP + PAD, CS = C + PAD;  // padded LDS rows
   static size_t lds(int waves, bool outputs) {
     size_t n = (size_t)(DP + waves * 32) * CS * sizeof(T) + (DP + 4 * C) * sizeof(float);
     if (outputs) n += 2 * C * QS * sizeof(T) + (waves * 64 / C + waves + 1) * C * sizeof(float);
     return n;
+  }
+};
+
+// four channels of four tokens, and the same by channel
+template <typename T> struct Block4;
+template <> struct Block4<bf16_t> {
+  typedef ushort4_t Row;
+  Row row[4];
+  DEVINL void by_channel(Row* o) const {
+    typedef __attribute__((ext_vector_type(2))) unsigned int uint2_t;
+    uint2_t x[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) x[j] = __builtin_bit_cast(uint2_t, row[j]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const unsigned sel = i & 1 ? 0x07060302u : 0x05040100u;
+      uint2_t v;
+      v[0] = __builtin_amdgcn_perm(x[1][i >> 1], x[0][i >> 1], sel);
+      v[1] = __builtin_amdgcn_perm(x[3][i >> 1], x[2][i >> 1], sel);
+      o[i] = __builtin_bit_cast(Row, v);
+    }
+  }
+};
+template <> struct Block4<float> {
+  typedef floatx4 Row;
+  Row row[4];
+  DEVINL void by_channel(Row* o) const {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = Row{row[0][i], row[1][i], row[2][i], row[3][i]};
   }
 };
 
@@ -172,8 +208,9 @@ __global__ __launch_bounds__(512) void memory_kernel(
     T* __restrict__ out, MemArgs a, Step step) {
   typedef MemShape<T, DT> Sh;
   typedef typename Frag<T>::V V;
-  constexpr int C = Sh::C, DP = Sh::DP, QS = Sh::QS, CS = Sh::CS, KT = Frag<T>::K / 16;  // tiles of a k step
-  constexpr int TT = C / 16;
+  typedef typename Block4<T>::Row Row;
+  constexpr int DP = Sh::DP, QS = Sh::QS, CS = Sh::CS, KT = Frag<T>::K / 16;  // tiles of a k step
+  constexpr int TT = C / 16, TG = C / 4;
   extern __shared__ __attribute__((aligned(16))) char mem[];
   const int TH = blockDim.x, waves = TH >> 6, EP = waves * 32, parts = TH / C;
   T* sKT = (T*)mem;             // [DP][CS] keys by channel
@@ -209,77 +246,123 @@ __global__ __launch_bounds__(512) void memory_kernel(
   for (int d = tid; d < DP; d += TH) sn[d] = from_zero || d >= a.dp ? 0.f : mine[(size_t)a.vdim * a.dp + d];
   float log_decay = 0.f;
   const bool vec = ((a.dim | a.vdim | a.N | a.q_at | a.k_at | a.v_at) & 3) == 0;
+  const bool vec_io = ((a.vdim | a.N | a.g_at | a.K | a.out_at) & 3) == 0;
+  float nw[ET][4];  // the norm's weights of this lane's outputs
+#pragma unroll
+  for (int e = 0; e < ET; ++e)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = e0 + e * 16 + quad * 4 + i;
+      nw[e][i] = PASS != STATES && c < a.vdim ? ld(norm + h * a.vdim + c) * a.out_scale : 0.f;
+    }
   for (int ch = c_lo; ch < c_end; ++ch) {
     const int t0 = ch * C;
-    __syncthreads();  // everyone is done with the previous chunk
-    // 4 channels of 4 tokens at a time: rows of q and k, columns of k and v
-    auto stage = [&](int at, int n, int wide, T* by_row, T* by_col) {
-      const int groups = wide >> 2, low = groups % 16 ? 8 : 16;  // (widths are multiples of 32)
-      for (int idx = tid; idx < groups * (C / 4); idx += TH) {
-        const int cg = idx % low + idx / (low * 4) % (groups / low) * low;
-        const int tg = idx / low % 4 + idx / (groups * 4) * 4;
-        T x[4][4];
+    // channels c.. of token t0 + t, zeros past n and past the row's end
+    auto fetch = [&](int at, int t, int c, int n) {
+      const T* src = rows + (size_t)(t0 + t) * a.N + at + c;
+      if (vec) return t0 + t < len && c < n ? *(const Row*)src : (Row)(0);
+      Row x;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int t = t0 + tg * 4 + j;
-          const T* src = rows + (size_t)t * a.N + at + cg * 4;
-          if (vec && t < len && cg * 4 < n) {
-            typedef __attribute__((ext_vector_type(4))) T T4;
-            *(T4*)x[j] = *(const T4*)src;
-          } else {
-#pragma unroll
-            for (int i = 0; i < 4; ++i) x[j][i] = t < len && cg * 4 + i < n ? src[i] : (T)0;
-          }
-        }
-        typedef __attribute__((ext_vector_type(4))) T T4;
-        if (by_row)
-#pragma unroll
-          for (int j = 0; j < 4; ++j) *(T4*)(by_row + (tg * 4 + j) * QS + cg * 4) = T4{x[j][0], x[j][1], x[j][2], x[j][3]};
-        if (by_col)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) *(T4*)(by_col + (cg * 4 + i) * CS + tg * 4) = T4{x[0][i], x[1][i], x[2][i], x[3][i]};
-      }
+      for (int i = 0; i < 4; ++i) x[i] = t0 + t < len && c + i < n ? src[i] : (T)0;
+      return x;
     };
-    if (PASS != STATES) stage(a.q_at + h * a.dim, a.dim, DP, sQ, (T*)nullptr);
-    stage(a.k_at + h * a.dim, a.dim, DP, PASS != STATES ? sK : (T*)nullptr, sKT);
-    stage(a.v_at + h * a.vdim, a.vdim, EP, (T*)nullptr, sVT);
-    const float m_prev = mr[t0], u_last = ur[t0 + C - 1], whole = expf(u_last + m_prev);
-    for (int t = tid; t < C; t += TH) {
-      const float ut = ur[t0 + t], rt = rr[t0 + t];
-      su[t] = ut;
-      sr[t] = rt;
-      sw[t] = expf(u_last + rt);
-      sa[t] = expf(ut + m_prev) * a.scale;
+    // a block of four channels by four tokens: neighbouring lanes take 16
+    // channels, then 8 tokens' blocks, which spreads LDS writes over all banks
+    auto put = [&](const Block4<T>& x, int c, int t, T* by_col, T* by_row) {
+      Row col4[4];
+      x.by_channel(col4);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) *(Row*)(by_col + (c + i) * CS + t) = col4[i];
+      if (by_row)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) *(Row*)(by_row + (t + j) * QS + c) = x.row[j];
+    };
+    __syncthreads();  // everyone is done with the previous chunk
+    for (int idx = tid, first = 1; first || idx < (PASS != STATES ? 2 : 1) * DT * C; idx += TH, first = 0) {
+      // keys: DT * C blocks; queries: twice as many halves of them; values: a wave's own
+      const int kc = (idx & 3) * 4 + idx / C * 16, kt = (idx >> 2) % TG * 4;
+      const bool key = idx < DT * C, query = PASS != STATES && idx < 2 * DT * C;
+      Block4<T> k, v;
+      Row q[2];
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (key) k.row[j] = fetch(a.k_at + h * a.dim, kt + j, kc, a.dim);
+      const int vc = e0 + ((lane & 3) + (lane >> 5) * 4) * 4, vt = ((lane >> 2) & 7) * 4;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (first) v.row[j] = fetch(a.v_at + h * a.vdim, vt + j, vc, a.vdim);
+      const int qc = idx % (DP / 8) * 8, qt = idx / (DP / 8);
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+        if (query) q[j] = fetch(a.q_at + h * a.dim, qt, qc + j * 4, a.dim);
+      if (key) put(k, kc, kt, sKT, PASS != STATES ? sK : (T*)nullptr);
+      if (first) put(v, vc, vt, sVT, (T*)nullptr);
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+        if (query) *(Row*)(sQ + qt * QS + qc + j * 4) = q[j];
+    }
+    const float m_prev = mr[t0], u_last = ur[t0 + C - 1], whole = pow2(u_last + m_prev);
+    if (tid < C) {
+      const float ut = ur[t0 + tid], rt = rr[t0 + tid];
+      su[tid] = ut;
+      sr[tid] = rt;
+      sw[tid] = pow2(u_last + rt);
+      sa[tid] = pow2(ut + m_prev) * a.scale;
     }
     __syncthreads();
     if (PASS != STATES) {
+      Row gate[TT][ET];
+#pragma unroll
+      for (int tt = 0; tt < TT; ++tt)
+#pragma unroll
+        for (int e = 0; e < ET; ++e) {
+          const int t = t0 + tt * 16 + col, c = e0 + e * 16 + quad * 4;
+          const T* g = rows + (size_t)t * a.N + a.g_at + h * a.vdim + c;
+          if (vec_io) gate[tt][e] = t < len && c < a.vdim ? *(const Row*)g : (Row)(0);
+          else
+#pragma unroll
+            for (int i = 0; i < 4; ++i) gate[tt][e][i] = t < len && c + i < a.vdim ? g[i] : (T)0;
+        }
       {
-        const int t = tid % C, p = tid / C;
+        const int t = tid % C;
         float dot = 0.f;
-        for (int d = p * DP / parts; d < (p + 1) * DP / parts; ++d) dot += sn[d] * ld(sQ + t * QS + d);
-        sdot[p * C + t] = dot;
+        for (int d = tid / C * 4; d < DP; d += parts * 4) {
+          float n[4], q[4];
+          ld4(sn + d, n);
+          ld4(sQ + t * QS + d, q);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) dot += n[i] * q[i];
+        }
+        sdot[tid] = dot;
       }
+      // what earlier chunks left
       floatx4 O[TT][ET];
+#pragma unroll
+      for (int tt = 0; tt < TT; ++tt)
+#pragma unroll
+        for (int e = 0; e < ET; ++e) O[tt][e] = (floatx4)(0.f);
+#pragma unroll
+      for (int c = 0; c < DT / KT; ++c) {
+        V qf[TT];
+#pragma unroll
+        for (int tt = 0; tt < TT; ++tt) qf[tt] = ld_tiles<T>(sQ + (tt * 16 + col) * QS + c * KT * 16 + quad * 4);
+#pragma unroll
+        for (int e = 0; e < ET; ++e) {
+          floatx4 s[KT];
+#pragma unroll
+          for (int k = 0; k < KT; ++k) s[k] = S[c * KT + k][e];
+          Parts<T> p;
+          p.set(s);
+#pragma unroll
+          for (int tt = 0; tt < TT; ++tt) O[tt][e] = Parts<T>::times(p, qf[tt], O[tt][e]);
+        }
+      }
 #pragma unroll
       for (int tt = 0; tt < TT; ++tt) {
         const int t = tt * 16 + col;
         V qf[DT / KT];
 #pragma unroll
         for (int c = 0; c < DT / KT; ++c) qf[c] = ld_tiles<T>(sQ + t * QS + c * KT * 16 + quad * 4);
-        // what earlier chunks left
-#pragma unroll
-        for (int e = 0; e < ET; ++e) O[tt][e] = (floatx4)(0.f);
-#pragma unroll
-        for (int c = 0; c < DT / KT; ++c)
-#pragma unroll
-          for (int e = 0; e < ET; ++e) {
-            floatx4 s[KT];
-#pragma unroll
-            for (int k = 0; k < KT; ++k) s[k] = S[c * KT + k][e];
-            Parts<T> p;
-            p.set(s);
-            O[tt][e] = Parts<T>::times(p, qf[c], O[tt][e]);
-          }
         const float at = sa[t], ut = su[t];
 #pragma unroll
         for (int e = 0; e < ET; ++e) O[tt][e] *= at;
@@ -299,8 +382,8 @@ __global__ __launch_bounds__(512) void memory_kernel(
             const floatx4 r4 = *(const floatx4*)(sr + st * 16 + quad * 4);
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-              const int s = st * 16 + quad * 4 + i;
-              w[k][i] = s <= t ? w[k][i] * a.scale * expf(ut + r4[i]) : 0.f;
+              const float x = w[k][i] * (a.scale * pow2(ut + r4[i]));
+              w[k][i] = st < tt || quad * 4 + i <= col ? x : 0.f;
               sum += w[k][i];
             }
           }
@@ -332,29 +415,20 @@ __global__ __launch_bounds__(512) void memory_kernel(
         for (int w = 0; w < waves; ++w) sq += ssq[w * C + t];
         const bool live = t0 + t < len;
         const float found = fabsf(srow[t] + sa[t] * dot);
-        const float inv = 1.f / (fmaxf(found, expf(live ? -mr[t0 + t + 1] : 0.f)) + 1e-6f);
-        const float f = inv / sqrtf(sq * inv * inv / (float)a.vdim + a.eps) * a.out_scale;
-        const size_t tok = (size_t)b * a.S + t0 + t;
-        T* dst = out + tok * a.K + a.out_at + h * a.vdim;
-        const T *gate = proj + tok * a.N + a.g_at + h * a.vdim, *nw = norm + h * a.vdim;
+        const float inv = 1.f / (fmaxf(found, pow2(live ? -mr[t0 + t + 1] : 0.f)) + 1e-6f);
+        const float f = live ? inv / sqrtf(sq * inv * inv / (float)a.vdim + a.eps) : 0.f;
+        T* dst = out + ((size_t)b * a.S + t0 + t) * a.K + a.out_at + h * a.vdim;
 #pragma unroll
         for (int e = 0; e < ET; ++e) {
           const int c = e0 + e * 16 + quad * 4;
-          float g[4], w[4], o[4];
-          const bool four = ((a.vdim | a.N | a.g_at | a.K | a.out_at) & 3) == 0;
           if (c >= a.vdim) continue;
-          if (four) {
-            ld4(gate + c, g);
-            ld4(nw + c, w);
-          } else
+          float o[4];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              g[i] = c + i < a.vdim ? ld(gate + c + i) : 0.f;
-              w[i] = c + i < a.vdim ? ld(nw + c + i) : 0.f;
-            }
-#pragma unroll
-          for (int i = 0; i < 4; ++i) o[i] = live ? O[tt][e][i] * f * w[i] * sigmoidf(g[i]) : 0.f;
-          if (four) st4(dst + c, o);
+          for (int i = 0; i < 4; ++i) {
+            T g = gate[tt][e][i];
+            o[i] = O[tt][e][i] * f * nw[e][i] * sigmoidf(ld(&g));
+          }
+          if (vec_io) st4(dst + c, o);
           else
 #pragma unroll
             for (int i = 0; i < 4; ++i)
@@ -387,6 +461,7 @@ __global__ __launch_bounds__(512) void memory_kernel(
     }
     for (int d = tid; d < DP; d += TH) {
       float n = sn[d] * whole;
+#pragma unroll
       for (int s = 0; s < C; s += 4) {
         float k[4], w[4];
         ld4(sKT + d * CS + s, k);
@@ -403,7 +478,7 @@ __global__ __launch_bounds__(512) void memory_kernel(
     for (int t = max(c_lo, c_end) * C + wave; t < min(c_hi * C, a.S); t += waves)
       for (int c = lane; c < a.vdim; c += 64) st(out + ((size_t)b * a.S + t) * a.K + a.out_at + h * a.vdim + c, 0.f);
   if (PASS == OUTPUTS || len <= 0) return;
-  if (PASS == STATES && tid == 0) decay[((size_t)b * a.nseg + seg) * a.H + h] = expf(log_decay);
+  if (PASS == STATES && tid == 0) decay[((size_t)b * a.nseg + seg) * a.H + h] = pow2(log_decay);
 #pragma unroll
   for (int i = 0; i < DT; ++i)
 #pragma unroll
@@ -509,10 +584,10 @@ __global__ __launch_bounds__(256) void memory_step_kernel(const T* __restrict__ 
     sk[tid] = tid < a.dim ? ld(row + a.k_at + h * a.dim + tid) : 0.f;
   }
   float* mp = state_m + (size_t)slot * a.H + h;
-  const float li = log_gate(ld(row + a.i_at + h), ld(bias + h), a.cap);
-  const float lf = log_sigmoid(log_gate(ld(row + a.f_at + h), ld(bias + a.H + h), a.cap));
+  const float li = log_input(ld(row + a.i_at + h), ld(bias + h), a.cap);
+  const float lf = log_forget(ld(row + a.f_at + h), ld(bias + a.H + h), a.cap);
   const float m0 = pos > 0 ? *mp : 0.f, top = fmaxf(lf + m0, li);
-  const float keep = expf(lf + m0 - top), take = expf(li - top);
+  const float keep = pow2(lf + m0 - top), take = pow2(li - top);
   float gate = 0.f, weight = 0.f;
   if (tid < a.vdim) {
     gate = ld(row + a.g_at + h * a.vdim + tid);
@@ -551,7 +626,7 @@ __global__ __launch_bounds__(256) void memory_step_kernel(const T* __restrict__ 
     }
   }
   __syncthreads();
-  const float inv = 1.f / (fmaxf(fabsf(so[a.vdim]), expf(-top)) + 1e-6f);
+  const float inv = 1.f / (fmaxf(fabsf(so[a.vdim]), pow2(-top)) + 1e-6f);
   const float y = tid < a.vdim ? so[tid] * inv : 0.f;
   const float f = 1.f / sqrtf(block_sum(y * y, red) / (float)a.vdim + a.eps) * a.out_scale;
   if (tid < a.vdim) st(dst + tid, y * f * weight * sigmoidf(gate));
@@ -571,10 +646,10 @@ template <typename T, int DT>
 static void prompt(const Tensor& proj, const Tensor& u, const Tensor& r, const Tensor& m, const Tensor& norm,
                    Tensor& state, Tensor& out, int B, MemArgs a, const Step& step) {
   typedef MemShape<T, DT> Sh;
-  const int waves = (a.vdim + 31) / 32, chunks = a.P / Sh::C, plane = (a.vdim + 1) * a.dp;
+  const int waves = (a.vdim + 31) / 32, chunks = a.P / C, plane = (a.vdim + 1) * a.dp;
   // rows are cut while the chip's 256 units do not have two blocks each; a
-  // segment is worth its second walk from four chunks on
-  const int want = (512 + B * a.H - 1) / (B * a.H), most = std::max(1, chunks / 4);
+  // segment is worth its second walk from eight chunks on
+  const int want = (512 + B * a.H - 1) / (B * a.H), most = std::max(1, chunks / 8);
   a.seg = (chunks + std::min(want, most) - 1) / std::min(want, most);
   a.nseg = (chunks + a.seg - 1) / a.seg;
   TORCH_CHECK(B <= 65535 && a.H <= 65535, "a prefill step of ", B, " rows and ", a.H, " heads is too large");
@@ -637,7 +712,6 @@ void matrix_memory(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_
     return;
   }
   BY_TYPE(dt, {
-    constexpr int C = chunk_of<T>();
     a.P = (S + C - 1) / C * C;
     auto u = f32(proj, {B, H, a.P}), r = f32(proj, {B, H, a.P}), m = f32(proj, {B, H, a.P + 1});
     int per = 1;

@@ -69,7 +69,8 @@ template <> DEVINL float rounded<bf16_t>(float f) { bf16_t u = f2b(f); return ld
 // One block per token; its row stays in registers (NC pieces of 256 V). y null:
 // x is read as it is. streams [done + 1][tokens][D]: the last one is written
 // here. h1 = norm(x) g1, h2 = norm(x) g2, the first plus its convolution if
-// there are taps.
+// there are taps. Loads that hang on nothing come first: one token's blocks are
+// all that a decode step of few rows has.
 template <typename T, int V, int NC>
 __global__ __launch_bounds__(256) void depth_norm_kernel(
     const T* __restrict__ y, const T* __restrict__ z, const int* __restrict__ rows, const float* __restrict__ weight,
@@ -78,6 +79,21 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
     T* __restrict__ h1, T* __restrict__ h2, DepthArgs a, Step step) {
   const size_t tok = blockIdx.x, off = tok * a.D;
   __shared__ float red[4];
+  constexpr int BACK = NC <= 2 ? 3 : 0;  // inputs of the convolution in registers
+  const int slot = taps ? step.slot((int)tok) : -1, pos = slot >= 0 ? step.first((int)tok) : 0;
+  T* hist = ring + (size_t)max(slot, 0) * a.taps * a.D;
+  float old[BACK + 1][NC * V];
+#pragma unroll
+  for (int k = 0; k < BACK; ++k)
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int i = (c * 256 + threadIdx.x) * V;
+#pragma unroll
+      for (int j = 0; j < V; ++j) old[k][c * V + j] = 0.f;
+      if (slot >= 0 && k + 1 < a.taps && k + 1 <= pos && i < a.D)
+        ldv<V>(hist + (size_t)((pos - 1 - k) % a.taps) * a.D + i, old[k] + c * V);
+    }
+  const float n1 = g1 ? ld(g1) : 0.f, n2 = g2 ? ld(g2) : 0.f;
   float xv[NC * V], ss = 0.f;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
@@ -88,7 +104,23 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
     if (i < a.D) {
       ldv<V>(x + off + i, v);
       if (y) {
-        float t[V];
+        float sum[V], t[V];
+#pragma unroll
+        for (int j = 0; j < V; ++j) sum[j] = 0.f;
+        const float* s = streams + off + i;
+        auto add = [&](int n, auto count) {  // `count` streams from n on, loads first
+          constexpr int N = decltype(count)::value;
+          float u[N][V], w[N];
+#pragma unroll
+          for (int k = 0; k < N; ++k) {
+            ldv<V>(s + (n + k) * a.plane, u[k]);
+            w[k] = ld(average + n + k);
+          }
+#pragma unroll
+          for (int k = 0; k < N; ++k)
+#pragma unroll
+            for (int j = 0; j < V; ++j) sum[j] += w[k] * u[k][j];
+        };
         ldv<V>(y + off + i, t);
 #pragma unroll
         for (int j = 0; j < V; ++j) v[j] += t[j];
@@ -97,36 +129,22 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
 #pragma unroll
           for (int j = 0; j < V; ++j) v[j] += t[j];
         }
+#pragma unroll 4
         for (int k = 0; k < a.top; ++k) {
           const float w = weight ? weight[tok * a.top + k] : 1.f;
           ldv<V>(z + (size_t)rows[tok * a.top + k] * a.zs + i, t);
 #pragma unroll
           for (int j = 0; j < V; ++j) v[j] += w * t[j];
         }
+        int n = 0;
+        for (; n + 8 <= a.done; n += 8) add(n, std::integral_constant<int, 8>());
+        if (n + 4 <= a.done) { add(n, std::integral_constant<int, 4>()); n += 4; }
+        if (n + 2 <= a.done) { add(n, std::integral_constant<int, 2>()); n += 2; }
+        if (n < a.done) add(n, std::integral_constant<int, 1>());
         stv<V>(streams + a.done * a.plane + off + i, v);
         const float last = ld(average + a.done);
 #pragma unroll
-        for (int j = 0; j < V; ++j) v[j] *= last;
-        const float* s = streams + off + i;
-        int n = 0;
-        for (; n + 4 <= a.done; n += 4) {  // loads first
-          float u[4][V], w[4];
-#pragma unroll
-          for (int k = 0; k < 4; ++k) {
-            ldv<V>(s + (n + k) * a.plane, u[k]);
-            w[k] = ld(average + n + k);
-          }
-#pragma unroll
-          for (int k = 0; k < 4; ++k)
-#pragma unroll
-            for (int j = 0; j < V; ++j) v[j] += w[k] * u[k][j];
-        }
-        for (; n < a.done; ++n) {
-          const float w = ld(average + n);
-          ldv<V>(s + n * a.plane, t);
-#pragma unroll
-          for (int j = 0; j < V; ++j) v[j] += w * t[j];
-        }
+        for (int j = 0; j < V; ++j) v[j] = sum[j] + last * v[j];
         stv<V>(out + off + i, v);
       }
 #pragma unroll
@@ -135,8 +153,7 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
   }
   if (!g1) return;
   const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
-  const float f1 = inv * ld(g1), f2 = g2 ? inv * ld(g2) : 0.f;
-  const int slot = taps ? step.slot((int)tok) : -1, pos = slot >= 0 ? step.first((int)tok) : 0;
+  const float f1 = inv * n1, f2 = inv * n2;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
     const int i = (c * 256 + threadIdx.x) * V;
@@ -145,16 +162,21 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
 #pragma unroll
     for (int j = 0; j < V; ++j) o[j] = rounded<T>(xv[c * V + j] * f1);
     if (slot >= 0) {
-      T* hist = ring + (size_t)slot * a.taps * a.D + i;
-      stv<V>(hist + (size_t)(pos % a.taps) * a.D, o);  // the oldest input: no tap reaches it any more
+      stv<V>(hist + (size_t)(pos % a.taps) * a.D + i, o);  // the oldest input: no tap reaches it any more
+      const T* w = taps + (size_t)i * a.taps + a.taps - 1;
       float sum[V];
 #pragma unroll
-      for (int j = 0; j < V; ++j) sum[j] = o[j] + o[j] * ld(taps + (size_t)(i + j) * a.taps + a.taps - 1);
-      for (int back = min(a.taps - 1, pos); back > 0; --back) {
-        float t[V];
-        ldv<V>(hist + (size_t)((pos - back) % a.taps) * a.D, t);
+      for (int j = 0; j < V; ++j) sum[j] = o[j] + o[j] * ld(w + j * a.taps);
 #pragma unroll
-        for (int j = 0; j < V; ++j) sum[j] += t[j] * ld(taps + (size_t)(i + j) * a.taps + a.taps - 1 - back);
+      for (int k = 0; k < BACK; ++k)
+        if (k + 1 < a.taps)
+#pragma unroll
+          for (int j = 0; j < V; ++j) sum[j] += old[k][c * V + j] * ld(w + j * a.taps - 1 - k);
+      for (int back = min(a.taps - 1, pos); back > BACK; --back) {
+        float t[V];
+        ldv<V>(hist + (size_t)((pos - back) % a.taps) * a.D + i, t);
+#pragma unroll
+        for (int j = 0; j < V; ++j) sum[j] += t[j] * ld(w + j * a.taps - back);
       }
 #pragma unroll
       for (int j = 0; j < V; ++j) o[j] = sum[j];

@@ -67,6 +67,25 @@ def packed_kv(dtype: torch.dtype, device) -> bool:
   return dtype == torch.bfloat16 and str(device).startswith("cuda")
 
 
+_side: Dict[int, "torch.cuda.Stream"] = {}
+
+
+def side_by_side(first, second):
+  """Results of two functions that do not depend on each other. In a captured step
+  they are branches of the graph, so that what is bound by latency overlaps.
+  Whatever the second allocates is used up before the current stream forks again."""
+  if not (torch.cuda.is_available() and torch.cuda.is_current_stream_capturing()):
+    return first(), second()
+  main = torch.cuda.current_stream()
+  side = _side.setdefault(main.device_index, torch.cuda.Stream(main.device_index))
+  side.wait_stream(main)
+  with torch.cuda.stream(side):
+    b = second()
+  a = first()
+  main.wait_stream(side)
+  return a, b
+
+
 # ---------------------------------------------------------------- norms
 
 class _Stream:

@@ -140,14 +140,15 @@ class DupolornModel(LayeredModel):
 
   def embed(self, tokens, caches, rows):
     last = caches[0][-1][0] if caches is not None else None
-    rows.depth = mo.Depth(self.embed_tokens.weight, tokens.shape, 1 + len(self.local_layer_ids))
+    rows.depth = mo.Depth(self.embed_tokens.weight, tokens.shape, 1 + len(self.local_layer_ids),
+                          keep=rows.streamed)
     return mo.embed_pairs(tokens, self.embed_tokens.weight, self.cfg.embed_scale, self.embed_pairs.weight,
                           self.cfg.bigram, last, rows)
 
   def receive(self, x, rows, dtype):
     D = self.cfg.dim
     now, *streams = x.float().split(D, dim=-1)
-    rows.depth = mo.Depth(x, x.shape[:-1], self.shard.end_layer + 2, D)
+    rows.depth = mo.Depth(x, x.shape[:-1], self.shard.end_layer + 2, D, keep=rows.streamed)
     for t in streams[:self.shard.start_layer + 1]:
       rows.depth.add(t)
     return now.contiguous()

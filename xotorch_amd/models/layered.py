@@ -125,7 +125,7 @@ class LayeredModel(nn.Module):
     dtype = self.layers[str(self.shard.start_layer)].norm1.dtype
     B, S = x.shape[0], x.shape[1]
     rows = mo.StepRows(is_decode, 0 if is_decode else int(start_pos),
-                       positions.reshape(-1) if is_decode else None, slots, lens)
+                       positions.reshape(-1) if is_decode else None, slots, lens, streamed=layers_out is not None)
     if x.dtype in (torch.int32, torch.int64):
       x = self.embed(x, caches, rows)
     else:

@@ -279,7 +279,7 @@ DEVINL float activated(float by, float g, float u, const Act& a) {
 }
 
 // Few tokens per expert: a block owns 16 output features of one expert; its
-// four waves split k and walk the expert's rows up to 64 at a time. GATED:
+// four waves split k and walk the expert's rows up to 64 (GATED: 32) at a time. GATED:
 // weights [E][2][F][kp]; else [E][F][kp]. Input rows are gathered by token but
 // for PLAIN. by_row: what the rows of the product are scaled with.
 template <typename T, int KIND, bool WHOLE>
@@ -287,8 +287,8 @@ __global__ __launch_bounds__(256) void expert_stream_kernel(
     const T* __restrict__ x, const T* __restrict__ w, const int* __restrict__ first, const int* __restrict__ token,
     const float* __restrict__ by_row, T* __restrict__ y, GroupArgs a, Act act) {
   typedef Frag<T> F;
-  constexpr int NW = KIND == GATED ? 2 : 1;
-  __shared__ float part[4][NW][64][17];
+  constexpr int NW = KIND == GATED ? 2 : 1, MOST = 4 / NW;
+  __shared__ float part[4][NW][MOST * 16][17];
   // the last experts are the ones that every token uses: the longest come first
   const int e = gridDim.y - 1 - blockIdx.y, f0 = blockIdx.x * 16;
   const int lo = first[e], hi = first[e + 1];
@@ -349,7 +349,7 @@ __global__ __launch_bounds__(256) void expert_stream_kernel(
     __syncthreads();
   };
   int r0 = lo;
-  for (; hi - r0 > 32; r0 += 64) round(r0, std::integral_constant<int, 4>());
+  for (; hi - r0 > 32; r0 += MOST * 16) round(r0, std::integral_constant<int, MOST>());
   if (hi - r0 > 16) round(r0, std::integral_constant<int, 2>());
   else if (hi > r0) round(r0, std::integral_constant<int, 1>());
 }

@@ -224,6 +224,14 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
   for (int i = 0; i < GW; ++i) o[i] = (floatx4)(0.f);
   for (int t4 = begin; t4 < end; t4 += 4) {
     const int tile = t4 + wave;
+    // values of two tiles are on their way before the scores are needed; groups
+    // past the wave's own are read again and dropped
+    bf16x8 vf[2][GW];
+    auto load_values = [&](int w) {
+      const bf16_t* v0 = vb + (size_t)min(t4 + w, end - 1) * 512 + lane * 8;
+#pragma unroll
+      for (int i = 0; i < GW; ++i) vf[w & 1][i] = *(const bf16x8*)(v0 + min(g0 + i, cache.vg - 1) * vstride);
+    };
     floatx4 sc[2] = {(floatx4)(0.f), (floatx4)(0.f)};
     if (tile < end) {
       const bf16_t* k0 = kb + (size_t)tile * 2 * cache.kc * 512 + lane * 8;
@@ -247,6 +255,8 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
       for (; c + 9 <= cache.kc; c += 9) run(c, std::integral_constant<int, 9>());
       for (; c < cache.kc; ++c) run(c, std::integral_constant<int, 1>());
     }
+    load_values(0);
+    load_values(1);
     float top = -1e30f;
 #pragma unroll
     for (int hf = 0; hf < 2; ++hf)
@@ -279,15 +289,14 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < GW; ++i) o[i] *= al;
-    const int n = min(4, end - t4);
-    for (int w = 0; w < n; ++w) {
+    // all four: tiles past the end weigh nothing, and without branches between
+    // them the products follow each other
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
       const bf16x8 pf = *(const bf16x8*)&probs[col][w * 32 + quad * 8];
-      const bf16_t* v0 = vb + (size_t)(t4 + w) * 512 + lane * 8;
-      bf16x8 vf[GW];  // groups past the wave's own are read again and dropped
 #pragma unroll
-      for (int i = 0; i < GW; ++i) vf[i] = *(const bf16x8*)(v0 + min(g0 + i, cache.vg - 1) * vstride);
-#pragma unroll
-      for (int i = 0; i < GW; ++i) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[i], pf, o[i], 0, 0, 0);
+      for (int i = 0; i < GW; ++i) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[w & 1][i], pf, o[i], 0, 0, 0);
+      if (w < 2) load_values(w + 2);
     }
     // the next round's writes to `tops` are two barriers behind these reads;
     // those to `probs` are one behind

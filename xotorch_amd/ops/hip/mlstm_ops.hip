@@ -131,10 +131,11 @@ template <> struct Parts<bf16_t> {
   bf16x8 hi, lo;
   DEVINL void set(const floatx4* v) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float f = v[i >> 2][i & 3];
-      hi[i] = (__bf16)f;
-      lo[i] = (__bf16)(f - (float)hi[i]);
+    for (int i = 0; i < 8; i += 2) {  // the upper halves as they are, and what they leave
+      const unsigned x = __float_as_uint(v[i >> 2][i & 3]), y = __float_as_uint(v[i >> 2][(i & 3) + 1]);
+      ((unsigned*)&hi)[i >> 1] = __builtin_amdgcn_perm(y, x, 0x07060302u);
+      lo[i] = (__bf16)(__uint_as_float(x) - __uint_as_float(x & 0xffff0000u));
+      lo[i + 1] = (__bf16)(__uint_as_float(y) - __uint_as_float(y & 0xffff0000u));
     }
   }
   static DEVINL floatx4 times(const Parts& x, const bf16x8& y, floatx4 c) { return mma(x.lo, y, mma(x.hi, y, c)); }
@@ -162,9 +163,10 @@ constexpr int ET = 2;  // tiles of 16 value channels that a wave owns
 
 template <typename T, int DT> struct MemShape {
   static constexpr int DP = DT * 16;
+  static constexpr int NP = 4;  // parts of the sum of keys, each of a share of the tokens
   static constexpr int PAD = sizeof(T) == 2 ? 8 : 4, QS = DP + PAD, CS = C + PAD;  // padded LDS rows
   static size_t lds(int waves, bool outputs) {
-    size_t n = (size_t)(DP + waves * 32) * CS * sizeof(T) + (DP + 4 * C) * sizeof(float);
+    size_t n = (size_t)(DP + waves * 32) * CS * sizeof(T) + (NP * DP + 4 * C) * sizeof(float);
     if (outputs) n += 2 * C * QS * sizeof(T) + (waves * 64 / C + waves + 1) * C * sizeof(float);
     return n;
   }
@@ -200,8 +202,9 @@ template <> struct Block4<float> {
 };
 
 // One block per (segment, head, row), a wave per 32 value channels. A wave holds
-// its channels of the state as accumulators, DT tiles of 16 key channels.
-template <typename T, int DT, int PASS>
+// its channels of the state as accumulators, DT tiles of 16 key channels. VEC:
+// addresses and widths allow loads and stores of four.
+template <typename T, int DT, int PASS, bool VEC>
 __global__ __launch_bounds__(512) void memory_kernel(
     const T* __restrict__ proj, const float* __restrict__ u, const float* __restrict__ r, const float* __restrict__ m,
     const T* __restrict__ norm, float* __restrict__ state, float* __restrict__ part, float* __restrict__ decay,
@@ -215,8 +218,8 @@ __global__ __launch_bounds__(512) void memory_kernel(
   const int TH = blockDim.x, waves = TH >> 6, EP = waves * 32, parts = TH / C;
   T* sKT = (T*)mem;             // [DP][CS] keys by channel
   T* sVT = sKT + DP * CS;       // [EP][CS] values by channel
-  float* sn = (float*)(sVT + EP * CS);  // [DP] the sum of keys
-  float *su = sn + DP, *sr = su + C, *sw = sr + C, *sa = sw + C;
+  float* sn = (float*)(sVT + EP * CS);  // [NP][DP] the sum of keys
+  float *su = sn + Sh::NP * DP, *sr = su + C, *sw = sr + C, *sa = sw + C;
   T* sQ = (T*)(sa + C);         // [C][QS]
   T* sK = sQ + C * QS;          // [C][QS]
   float* sdot = (float*)(sK + C * QS);  // [parts][C] queries with the sum of keys
@@ -243,10 +246,13 @@ __global__ __launch_bounds__(512) void memory_kernel(
       S[i][e] = from_zero || c >= a.vdim || i * 16 >= a.dp ? (floatx4)(0.f)
                                                            : *(const floatx4*)(mine + (size_t)c * a.dp + i * 16 + quad * 4);
     }
-  for (int d = tid; d < DP; d += TH) sn[d] = from_zero || d >= a.dp ? 0.f : mine[(size_t)a.vdim * a.dp + d];
-  float log_decay = 0.f;
-  const bool vec = ((a.dim | a.vdim | a.N | a.q_at | a.k_at | a.v_at) & 3) == 0;
-  const bool vec_io = ((a.vdim | a.N | a.g_at | a.K | a.out_at) & 3) == 0;
+  int np = 1;
+  while (np < Sh::NP && np * 2 * DP <= TH) np *= 2;
+  for (int d = tid; d < np * DP; d += TH) sn[d] = from_zero || d >= a.dp ? 0.f : mine[(size_t)a.vdim * a.dp + d];
+  // the state is 2^held times the accumulators (and `sn`): while that does not get
+  // too small, a chunk's decay goes there alone
+  float log_decay = 0.f, held = 0.f;
+  const float per_channel = 1.f / (float)a.vdim;
   float nw[ET][4];  // the norm's weights of this lane's outputs
 #pragma unroll
   for (int e = 0; e < ET; ++e)
@@ -255,86 +261,163 @@ __global__ __launch_bounds__(512) void memory_kernel(
       const int c = e0 + e * 16 + quad * 4 + i;
       nw[e][i] = PASS != STATES && c < a.vdim ? ld(norm + h * a.vdim + c) * a.out_scale : 0.f;
     }
+  // Channels c.. of token t0 + t + j; those past n hold others' numbers until
+  // `within` clears them, which waits for the load. Tokens past the row's end are
+  // read as its last: their weights are zero. In whole chunks a thread's places are
+  // the same every time, apart from what is uniform.
+  typedef __attribute__((ext_vector_type(sizeof(Row) / 4))) unsigned Bits;
+  auto within = [](Row x, int c, int n) {
+    if (VEC) return __builtin_bit_cast(Row, __builtin_bit_cast(Bits, x) & (c < n ? ~0u : 0u));
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (c + i >= n) x[i] = (T)0;
+    return x;
+  };
+  auto fetch = [&](int t0, bool tail, int at, int t, int j, int c, int n) {
+    Row x;
+    if (VEC) {
+      if (!tail) x = *(const Row*)((rows + (size_t)(t0 + j) * a.N + at) + (unsigned)(t * a.N + min(c, n - 4)));
+      else x = *(const Row*)(rows + (size_t)min(t0 + t + j, len - 1) * a.N + at + min(c, n - 4));
+    } else {
+      const T* src = rows + (size_t)min(t0 + t + j, len - 1) * a.N + at;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[i] = src[min(c + i, n - 1)];
+    }
+    return x;
+  };
+  // a block of four channels by four tokens: neighbouring lanes take 16
+  // channels, then 8 tokens' blocks, which spreads LDS writes over all banks
+  auto put = [&](const Block4<T>& x, int c, int t, T* by_col, T* by_row) {
+    Row col4[4];
+    x.by_channel(col4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) *(Row*)(by_col + (c + i) * CS + t) = col4[i];
+    if (by_row)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) *(Row*)(by_row + (t + j) * QS + c) = x.row[j];
+  };
+  // keys: DT * C blocks; queries: twice as many halves of them; values: a wave's own
+  auto key_at = [&](int idx, int& c, int& t) {
+    c = (idx & 3) * 4 + idx / C * 16;
+    t = (idx >> 2) % TG * 4;
+  };
+  auto fetch_key = [&](int t0, bool tail, int idx, Block4<T>& k) {
+    int c, t;
+    key_at(idx, c, t);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) k.row[j] = fetch(t0, tail, a.k_at + h * a.dim, t, j, c, a.dim);
+  };
+  auto put_key = [&](int idx, const Block4<T>& k) {
+    int c, t;
+    key_at(idx, c, t);
+    if (idx < DT * C) put(k, c, t, sKT, PASS != STATES ? sK : (T*)nullptr);
+  };
+  auto fetch_query = [&](int t0, bool tail, int idx, Row* q) {
+    const int t = min(idx / (DP / 8), C - 1);
+#pragma unroll
+    for (int j = 0; j < 2; ++j) q[j] = fetch(t0, tail, a.q_at + h * a.dim, t, 0, idx % (DP / 8) * 8 + j * 4, a.dim);
+  };
+  auto put_query = [&](int idx, const Row* q) {
+    const int c = idx % (DP / 8) * 8;
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+      if (idx < 2 * DT * C) *(Row*)(sQ + idx / (DP / 8) * QS + c + j * 4) = within(q[j], c + j * 4, a.dim);
+  };
+  const int vc = e0 + ((lane & 3) + (lane >> 5) * 4) * 4, vt = ((lane >> 2) & 7) * 4;
+  // what a thread's first blocks of the next chunk hold, on its way while this one is computed
+  constexpr int R = C / 32;
+  Block4<T> k0[R], v0[R];
+  Row q0[2 * R][2];
+  float ut, rt, m_prev, u_last;
+  auto ahead_of = [&](int t0, bool tail) {
+#pragma unroll
+    for (int i = 0; i < R; ++i) fetch_key(t0, tail, tid + i * TH, k0[i]);
+#pragma unroll
+    for (int i = 0; i < R; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v0[i].row[j] = fetch(t0, tail, a.v_at + h * a.vdim, i * 32 + vt, j, vc, a.vdim);
+    if (PASS != STATES)
+#pragma unroll
+      for (int i = 0; i < 2 * R; ++i) fetch_query(t0, tail, tid + i * TH, q0[i]);
+  };
+  auto ahead = [&](int t0) {
+    if (t0 + C > len) ahead_of(t0, true);
+    else ahead_of(t0, false);
+    ut = ur[t0 + tid % C];
+    rt = rr[t0 + tid % C];
+    m_prev = mr[t0];
+    u_last = ur[t0 + C - 1];
+  };
+  if (c_lo < c_end) ahead(c_lo * C);
   for (int ch = c_lo; ch < c_end; ++ch) {
     const int t0 = ch * C;
-    // channels c.. of token t0 + t, zeros past n and past the row's end
-    auto fetch = [&](int at, int t, int c, int n) {
-      const T* src = rows + (size_t)(t0 + t) * a.N + at + c;
-      if (vec) return t0 + t < len && c < n ? *(const Row*)src : (Row)(0);
-      Row x;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) x[i] = t0 + t < len && c + i < n ? src[i] : (T)0;
-      return x;
-    };
-    // a block of four channels by four tokens: neighbouring lanes take 16
-    // channels, then 8 tokens' blocks, which spreads LDS writes over all banks
-    auto put = [&](const Block4<T>& x, int c, int t, T* by_col, T* by_row) {
-      Row col4[4];
-      x.by_channel(col4);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) *(Row*)(by_col + (c + i) * CS + t) = col4[i];
-      if (by_row)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) *(Row*)(by_row + (t + j) * QS + c) = x.row[j];
-    };
+    const bool tail = t0 + C > len;
     __syncthreads();  // everyone is done with the previous chunk
-    for (int idx = tid, first = 1; first || idx < (PASS != STATES ? 2 : 1) * DT * C; idx += TH, first = 0) {
-      // keys: DT * C blocks; queries: twice as many halves of them; values: a wave's own
-      const int kc = (idx & 3) * 4 + idx / C * 16, kt = (idx >> 2) % TG * 4;
-      const bool key = idx < DT * C, query = PASS != STATES && idx < 2 * DT * C;
-      Block4<T> k, v;
-      Row q[2];
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (key) k.row[j] = fetch(a.k_at + h * a.dim, kt + j, kc, a.dim);
-      const int vc = e0 + ((lane & 3) + (lane >> 5) * 4) * 4, vt = ((lane >> 2) & 7) * 4;
+    for (int i = 0; i < R; ++i) {
+      put_key(tid + i * TH, k0[i]);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (first) v.row[j] = fetch(a.v_at + h * a.vdim, vt + j, vc, a.vdim);
-      const int qc = idx % (DP / 8) * 8, qt = idx / (DP / 8);
-#pragma unroll
-      for (int j = 0; j < 2; ++j)
-        if (query) q[j] = fetch(a.q_at + h * a.dim, qt, qc + j * 4, a.dim);
-      if (key) put(k, kc, kt, sKT, PASS != STATES ? sK : (T*)nullptr);
-      if (first) put(v, vc, vt, sVT, (T*)nullptr);
-#pragma unroll
-      for (int j = 0; j < 2; ++j)
-        if (query) *(Row*)(sQ + qt * QS + qc + j * 4) = q[j];
+      for (int j = 0; j < 4; ++j) v0[i].row[j] = within(v0[i].row[j], vc, a.vdim);
+      put(v0[i], vc, i * 32 + vt, sVT, (T*)nullptr);
     }
-    const float m_prev = mr[t0], u_last = ur[t0 + C - 1], whole = pow2(u_last + m_prev);
+    for (int idx = tid + R * TH; idx < DT * C; idx += TH) {
+      Block4<T> k;
+      fetch_key(t0, tail, idx, k);
+      put_key(idx, k);
+    }
+    if (PASS != STATES) {
+#pragma unroll
+      for (int i = 0; i < 2 * R; ++i) put_query(tid + i * TH, q0[i]);
+      for (int idx = tid + 2 * R * TH; idx < 2 * DT * C; idx += TH) {
+        Row q[2];
+        fetch_query(t0, tail, idx, q);
+        put_query(idx, q);
+      }
+    }
+    const float before = held;
+    held += u_last + m_prev;
+    log_decay += u_last + m_prev;
+    const bool rescale = held < -20.f;
+    const float whole = rescale ? pow2(held) : 1.f;
+    if (rescale) held = 0.f;
     if (tid < C) {
-      const float ut = ur[t0 + tid], rt = rr[t0 + tid];
       su[tid] = ut;
       sr[tid] = rt;
-      sw[tid] = pow2(u_last + rt);
-      sa[tid] = pow2(ut + m_prev) * a.scale;
+      sw[tid] = pow2(u_last + rt - held);
+      sa[tid] = pow2(ut + m_prev + before) * a.scale;
     }
     __syncthreads();
+    if (ch + 1 < c_end) ahead(t0 + C);
     if (PASS != STATES) {
       Row gate[TT][ET];
 #pragma unroll
       for (int tt = 0; tt < TT; ++tt)
 #pragma unroll
         for (int e = 0; e < ET; ++e) {
-          const int t = t0 + tt * 16 + col, c = e0 + e * 16 + quad * 4;
-          const T* g = rows + (size_t)t * a.N + a.g_at + h * a.vdim + c;
-          if (vec_io) gate[tt][e] = t < len && c < a.vdim ? *(const Row*)g : (Row)(0);
-          else
-#pragma unroll
-            for (int i = 0; i < 4; ++i) gate[tt][e][i] = t < len && c + i < a.vdim ? g[i] : (T)0;
+          gate[tt][e] = fetch(t0, tail, a.g_at + h * a.vdim, tt * 16 + col, 0, e0 + e * 16 + quad * 4, a.vdim);
         }
       {
         const int t = tid % C;
         float dot = 0.f;
         for (int d = tid / C * 4; d < DP; d += parts * 4) {
-          float n[4], q[4];
-          ld4(sn + d, n);
+          floatx4 n = *(const floatx4*)(sn + d);
+          for (int p = 1; p < np; ++p) n += *(const floatx4*)(sn + p * DP + d);
+          float q[4];
           ld4(sQ + t * QS + d, q);
 #pragma unroll
           for (int i = 0; i < 4; ++i) dot += n[i] * q[i];
         }
         sdot[tid] = dot;
       }
+      constexpr bool HOLD = DT <= 8;  // queries' operands stay in registers
+      V qf[HOLD ? TT : 1][HOLD ? DT / KT : 1];
+      auto load_q = [&](int tt, int c) { return ld_tiles<T>(sQ + (tt * 16 + col) * QS + c * KT * 16 + quad * 4); };
+      auto q_of = [&](int tt, int c) { return HOLD ? qf[HOLD ? tt : 0][HOLD ? c : 0] : load_q(tt, c); };
+      if (HOLD)
+#pragma unroll
+        for (int tt = 0; tt < TT; ++tt)
+#pragma unroll
+          for (int c = 0; c < DT / KT; ++c) qf[HOLD ? tt : 0][HOLD ? c : 0] = load_q(tt, c);
       // what earlier chunks left
       floatx4 O[TT][ET];
 #pragma unroll
@@ -342,10 +425,7 @@ __global__ __launch_bounds__(512) void memory_kernel(
 #pragma unroll
         for (int e = 0; e < ET; ++e) O[tt][e] = (floatx4)(0.f);
 #pragma unroll
-      for (int c = 0; c < DT / KT; ++c) {
-        V qf[TT];
-#pragma unroll
-        for (int tt = 0; tt < TT; ++tt) qf[tt] = ld_tiles<T>(sQ + (tt * 16 + col) * QS + c * KT * 16 + quad * 4);
+      for (int c = 0; c < DT / KT; ++c)
 #pragma unroll
         for (int e = 0; e < ET; ++e) {
           floatx4 s[KT];
@@ -354,45 +434,55 @@ __global__ __launch_bounds__(512) void memory_kernel(
           Parts<T> p;
           p.set(s);
 #pragma unroll
-          for (int tt = 0; tt < TT; ++tt) O[tt][e] = Parts<T>::times(p, qf[tt], O[tt][e]);
+          for (int tt = 0; tt < TT; ++tt) O[tt][e] = Parts<T>::times(p, q_of(tt, c), O[tt][e]);
         }
-      }
+      // scores of this chunk's tokens, keys by queries
+      floatx4 w[TT][TT];
+#pragma unroll
+      for (int st = 0; st < TT; ++st)
+#pragma unroll
+        for (int tt = 0; tt < TT; ++tt) w[tt][st] = (floatx4)(0.f);
+#pragma unroll
+      for (int st = 0; st < TT; ++st)
+#pragma unroll
+        for (int c = 0; c < DT / KT; ++c) {
+          const V kf = ld_tiles<T>(sK + (st * 16 + col) * QS + c * KT * 16 + quad * 4);
+#pragma unroll
+          for (int tt = st; tt < TT; ++tt) w[tt][st] = mma(kf, q_of(tt, c), w[tt][st]);
+        }
+      Parts<T> p[TT][TT / KT];
+      float sum[TT];
 #pragma unroll
       for (int tt = 0; tt < TT; ++tt) {
         const int t = tt * 16 + col;
-        V qf[DT / KT];
-#pragma unroll
-        for (int c = 0; c < DT / KT; ++c) qf[c] = ld_tiles<T>(sQ + t * QS + c * KT * 16 + quad * 4);
-        const float at = sa[t], ut = su[t];
+        const float at = sa[t], here = su[t];
+        sum[tt] = 0.f;
 #pragma unroll
         for (int e = 0; e < ET; ++e) O[tt][e] *= at;
-        // this chunk's tokens up to t
-        float sum = 0.f;
 #pragma unroll
-        for (int j = 0; j * KT <= tt; ++j) {
-          floatx4 w[KT];
+        for (int st = 0; st <= tt; ++st) {
+          const floatx4 r4 = *(const floatx4*)(sr + st * 16 + quad * 4);
 #pragma unroll
-          for (int k = 0; k < KT; ++k) {
-            const int st = j * KT + k;
-            w[k] = (floatx4)(0.f);
-            if (st > tt) continue;
-#pragma unroll
-            for (int c = 0; c < DT / KT; ++c)
-              w[k] = mma(ld_tiles<T>(sK + (st * 16 + col) * QS + c * KT * 16 + quad * 4), qf[c], w[k]);
-            const floatx4 r4 = *(const floatx4*)(sr + st * 16 + quad * 4);
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              const float x = w[k][i] * (a.scale * pow2(ut + r4[i]));
-              w[k][i] = st < tt || quad * 4 + i <= col ? x : 0.f;
-              sum += w[k][i];
-            }
+          for (int i = 0; i < 4; ++i) {
+            const float x = w[tt][st][i] * (a.scale * pow2(here + r4[i]));
+            w[tt][st][i] = st < tt || quad * 4 + i <= col ? x : 0.f;
+            sum[tt] += w[tt][st][i];
           }
-          Parts<T> p;
-          p.set(w);
-#pragma unroll
-          for (int e = 0; e < ET; ++e)
-            O[tt][e] = Parts<T>::by(ld_tiles<T>(sVT + (e0 + e * 16 + col) * CS + j * KT * 16 + quad * 4), p, O[tt][e]);
         }
+#pragma unroll
+        for (int j = 0; j * KT <= tt; ++j) p[tt][j].set(&w[tt][j * KT]);
+      }
+#pragma unroll
+      for (int j = 0; j < TT / KT; ++j)
+#pragma unroll
+        for (int e = 0; e < ET; ++e) {
+          const V vf = ld_tiles<T>(sVT + (e0 + e * 16 + col) * CS + j * KT * 16 + quad * 4);
+#pragma unroll
+          for (int tt = j * KT; tt < TT; ++tt) O[tt][e] = Parts<T>::by(vf, p[tt][j], O[tt][e]);
+        }
+#pragma unroll
+      for (int tt = 0; tt < TT; ++tt) {
+        const int t = tt * 16 + col;
         float sq = 0.f;
 #pragma unroll
         for (int e = 0; e < ET; ++e)
@@ -400,10 +490,10 @@ __global__ __launch_bounds__(512) void memory_kernel(
           for (int i = 0; i < 4; ++i) sq += O[tt][e][i] * O[tt][e][i];
         sq += __shfl_xor(sq, 16);
         sq += __shfl_xor(sq, 32);
-        sum += __shfl_xor(sum, 16);
-        sum += __shfl_xor(sum, 32);
+        sum[tt] += __shfl_xor(sum[tt], 16);
+        sum[tt] += __shfl_xor(sum[tt], 32);
         if (quad == 0) ssq[wave * C + t] = sq;
-        if (quad == 0 && wave == 0) srow[t] = sum;
+        if (quad == 0 && wave == 0) srow[t] = sum[tt];
       }
       __syncthreads();
 #pragma unroll
@@ -415,8 +505,8 @@ __global__ __launch_bounds__(512) void memory_kernel(
         for (int w = 0; w < waves; ++w) sq += ssq[w * C + t];
         const bool live = t0 + t < len;
         const float found = fabsf(srow[t] + sa[t] * dot);
-        const float inv = 1.f / (fmaxf(found, pow2(live ? -mr[t0 + t + 1] : 0.f)) + 1e-6f);
-        const float f = live ? inv / sqrtf(sq * inv * inv / (float)a.vdim + a.eps) : 0.f;
+        const float inv = __builtin_amdgcn_rcpf(fmaxf(found, pow2(live ? -mr[t0 + t + 1] : 0.f)) + 1e-6f);
+        const float f = live ? inv * __builtin_amdgcn_rsqf(sq * inv * inv * per_channel + a.eps) : 0.f;
         T* dst = out + ((size_t)b * a.S + t0 + t) * a.K + a.out_at + h * a.vdim;
 #pragma unroll
         for (int e = 0; e < ET; ++e) {
@@ -428,7 +518,7 @@ __global__ __launch_bounds__(512) void memory_kernel(
             T g = gate[tt][e][i];
             o[i] = O[tt][e][i] * f * nw[e][i] * sigmoidf(ld(&g));
           }
-          if (vec_io) st4(dst + c, o);
+          if (VEC) st4(dst + c, o);
           else
 #pragma unroll
             for (int i = 0; i < 4; ++i)
@@ -437,10 +527,11 @@ __global__ __launch_bounds__(512) void memory_kernel(
       }
     }
     // the state after this chunk
+    if (rescale)
 #pragma unroll
-    for (int i = 0; i < DT; ++i)
+      for (int i = 0; i < DT; ++i)
 #pragma unroll
-      for (int e = 0; e < ET; ++e) S[i][e] *= whole;
+        for (int e = 0; e < ET; ++e) S[i][e] *= whole;
 #pragma unroll
     for (int j = 0; j < TT / KT; ++j) {
       Parts<T> p[ET];
@@ -459,34 +550,39 @@ __global__ __launch_bounds__(512) void memory_kernel(
         for (int e = 0; e < ET; ++e) S[i][e] = Parts<T>::by(kf, p[e], S[i][e]);
       }
     }
-    for (int d = tid; d < DP; d += TH) {
-      float n = sn[d] * whole;
-#pragma unroll
-      for (int s = 0; s < C; s += 4) {
+    for (int i = tid; i < np * DP; i += TH) {
+      const int d = i % DP, share = C / np, s0 = i / DP * share;
+      float n = sn[i] * whole;
+      for (int s = s0; s < s0 + share; s += 4) {
         float k[4], w[4];
         ld4(sKT + d * CS + s, k);
         ld4(sw + s, w);
 #pragma unroll
         for (int i = 0; i < 4; ++i) n += k[i] * w[i];
       }
-      sn[d] = n;
+      sn[i] = n;
     }
-    log_decay += u_last + m_prev;
   }
   // tokens past a row's end, and parked rows
   if (PASS != STATES)
     for (int t = max(c_lo, c_end) * C + wave; t < min(c_hi * C, a.S); t += waves)
       for (int c = lane; c < a.vdim; c += 64) st(out + ((size_t)b * a.S + t) * a.K + a.out_at + h * a.vdim + c, 0.f);
   if (PASS == OUTPUTS || len <= 0) return;
+  const float scale = pow2(held);
   if (PASS == STATES && tid == 0) decay[((size_t)b * a.nseg + seg) * a.H + h] = pow2(log_decay);
 #pragma unroll
   for (int i = 0; i < DT; ++i)
 #pragma unroll
     for (int e = 0; e < ET; ++e) {
       const int c = e0 + e * 16 + col;
-      if (c < a.vdim && i * 16 < a.dp) *(floatx4*)(mine + (size_t)c * a.dp + i * 16 + quad * 4) = S[i][e];
+      if (c < a.vdim && i * 16 < a.dp) *(floatx4*)(mine + (size_t)c * a.dp + i * 16 + quad * 4) = S[i][e] * scale;
     }
-  for (int d = tid; d < a.dp; d += TH) mine[(size_t)a.vdim * a.dp + d] = sn[d];
+  __syncthreads();
+  for (int d = tid; d < a.dp; d += TH) {
+    float n = sn[d];
+    for (int p = 1; p < np; ++p) n += sn[p * DP + d];
+    mine[(size_t)a.vdim * a.dp + d] = n * scale;
+  }
 }
 
 // part [B][nseg][H][..]: every segment's own last state -> the state it starts
@@ -543,42 +639,31 @@ __global__ __launch_bounds__(256) void memory_step_kernel(const T* __restrict__ 
                                                           const T* __restrict__ norm, float* __restrict__ state,
                                                           float* __restrict__ state_m, T* __restrict__ out, MemArgs a,
                                                           Step step) {
-  constexpr int DP = 16 * RPL, NB = RPL <= 8 ? 4 : 2, VW = Rows<RPL>::V;  // NB: columns in flight per 16 lanes
+  constexpr int DP = 16 * RPL, NB = RPL <= 8 ? 8 : 4, VW = Rows<RPL>::V;  // NB: columns in flight per 16 lanes
   __shared__ __attribute__((aligned(16))) float sq[DP], sk[DP];
-  __shared__ float so[257], red[4];
+  __shared__ float so[256], red[4], sfound;
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, slot = step.slot(b);
   T* dst = out + (size_t)b * a.K + a.out_at + h * a.vdim;
   if (slot < 0) {
     if (tid < a.vdim) st(dst + tid, 0.f);
     return;
   }
-  const int pos = step.first(b), r = tid & 15, cl = tid >> 4, cols = a.vdim + 1;
+  const int pos = step.first(b), r = tid & 15, cl = tid >> 4;
   const T* row = proj + (size_t)b * a.N;
-  float* base = state + ((size_t)slot * a.H + h) * (size_t)cols * DP;
-  float s[NB][RPL];
+  float* base = state + ((size_t)slot * a.H + h) * (size_t)(a.vdim + 1) * DP;
+  float s[NB][RPL], v[NB], n[RPL];
   auto load = [&](int c0) {
 #pragma unroll
     for (int i = 0; i < NB; ++i) {
-      const int c = c0 + i * 16 + cl;
+      const int c = min(c0 + i * 16 + cl, a.vdim - 1);
+      v[i] = ld(row + a.v_at + h * a.vdim + c);
 #pragma unroll
-      for (int j = 0; j < RPL / VW; ++j) {
-        if (c < cols && pos > 0) ld_any<VW>(base + (size_t)c * DP + Rows<RPL>::at(j, r), s[i] + j * VW);
-        else
-#pragma unroll
-          for (int x = 0; x < VW; ++x) s[i][j * VW + x] = 0.f;
-      }
+      for (int j = 0; j < RPL / VW; ++j) ld_any<VW>(base + (size_t)c * DP + Rows<RPL>::at(j, r), s[i] + j * VW);
     }
   };
   load(0);  // in flight while the gates are made
-  float v[(256 + 16) / 16 / NB + 1][NB];  // this lane's columns' values
-  const int rounds = (cols + 16 * NB - 1) / (16 * NB);
 #pragma unroll
-  for (int k = 0; k < (256 + 16) / 16 / NB + 1; ++k)
-#pragma unroll
-    for (int i = 0; i < NB; ++i) {
-      const int c = (k * NB + i) * 16 + cl;
-      v[k][i] = c < a.vdim ? ld(row + a.v_at + h * a.vdim + c) : 1.f;
-    }
+  for (int j = 0; j < RPL / VW; ++j) ld_any<VW>(base + (size_t)a.vdim * DP + Rows<RPL>::at(j, r), n + j * VW);
   if (tid < DP) {
     sq[tid] = tid < a.dim ? ld(row + a.q_at + h * a.dim + tid) * a.scale : 0.f;
     sk[tid] = tid < a.dim ? ld(row + a.k_at + h * a.dim + tid) : 0.f;
@@ -603,30 +688,33 @@ __global__ __launch_bounds__(256) void memory_step_kernel(const T* __restrict__ 
   }
 #pragma unroll
   for (int i = 0; i < RPL; ++i) k[i] *= take;
+  // a row of 16 channels of one column; what a new sequence's slot held does not count
+  auto advance = [&](float* x, float value, float* to) {
+    float o = 0.f;
 #pragma unroll
-  for (int rd = 0; rd < (256 + 16) / 16 / NB + 1; ++rd) {
-    if (rd >= rounds) break;
-    const int c0 = rd * 16 * NB;
-    if (rd) load(c0);
+    for (int j = 0; j < RPL; ++j) {
+      x[j] = (pos > 0 ? keep * x[j] : 0.f) + k[j] * value;
+      o += x[j] * q[j];
+    }
+    if (to)
+#pragma unroll
+      for (int j = 0; j < RPL / VW; ++j) st_any<VW>(to + Rows<RPL>::at(j, r), x + j * VW);
+    return row_sum(o);
+  };
+  for (int c0 = 0; c0 < a.vdim; c0 += 16 * NB) {
+    if (c0) load(c0);
 #pragma unroll
     for (int i = 0; i < NB; ++i) {
       const int c = c0 + i * 16 + cl;
-      float o = 0.f;
-#pragma unroll
-      for (int j = 0; j < RPL; ++j) {
-        s[i][j] = keep * s[i][j] + k[j] * v[rd][i];
-        o += s[i][j] * q[j];
-      }
-      o = row_sum(o);
-      if (c < cols) {
-        if (r == 0) so[c] = o;
-#pragma unroll
-        for (int j = 0; j < RPL / VW; ++j) st_any<VW>(base + (size_t)c * DP + Rows<RPL>::at(j, r), s[i] + j * VW);
-      }
+      const float o = advance(s[i], v[i], c < a.vdim ? base + (size_t)c * DP : nullptr);
+      if (r == 0 && c < a.vdim) so[c] = o;
     }
   }
+  __syncthreads();  // every wave has read the sum of keys
+  const float found = advance(n, 1.f, cl == 0 ? base + (size_t)a.vdim * DP : nullptr);
+  if (tid == 0) sfound = fabsf(found);
   __syncthreads();
-  const float inv = 1.f / (fmaxf(fabsf(so[a.vdim]), pow2(-top)) + 1e-6f);
+  const float inv = 1.f / (fmaxf(sfound, pow2(-top)) + 1e-6f);
   const float y = tid < a.vdim ? so[tid] * inv : 0.f;
   const float f = 1.f / sqrtf(block_sum(y * y, red) / (float)a.vdim + a.eps) * a.out_scale;
   if (tid < a.vdim) st(dst + tid, y * f * weight * sigmoidf(gate));
@@ -660,6 +748,8 @@ static void prompt(const Tensor& proj, const Tensor& u, const Tensor& r, const T
     decay = f32(proj, {B, a.nseg, a.H});
   }
   float *pp = a.nseg > 1 ? M<float>(part) : nullptr, *dp = a.nseg > 1 ? M<float>(decay) : nullptr;
+  const bool vec = ((a.dim | a.vdim | a.N | a.q_at | a.k_at | a.v_at | a.g_at | a.K | a.out_at) & 3) == 0;
+  if (!vec) { a.seg = chunks; a.nseg = 1; }
   auto run = [&](auto kernel, bool outputs) {
     static const hipError_t err = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     TORCH_CHECK(err == hipSuccess, "no LDS for the memory's chunks");
@@ -668,11 +758,12 @@ static void prompt(const Tensor& proj, const Tensor& u, const Tensor& r, const T
     hipLaunchKernelGGL(kernel, dim3(a.nseg, a.H, B), dim3(64 * waves), lds, stream, P<T>(proj), P<float>(u), P<float>(r),
                        P<float>(m), P<T>(norm), M<float>(state), pp, dp, M<T>(out), a, step);
   };
-  if (a.nseg == 1) { run(memory_kernel<T, DT, WHOLE>, true); return; }
-  run(memory_kernel<T, DT, STATES>, false);
+  if (!vec) { run(memory_kernel<T, DT, WHOLE, false>, true); return; }
+  if (a.nseg == 1) { run(memory_kernel<T, DT, WHOLE, true>, true); return; }
+  run(memory_kernel<T, DT, STATES, true>, false);
   hipLaunchKernelGGL(segment_kernel, dim3((plane / 4 + 255) / 256, a.H, B), dim3(256), 0, stream, pp, dp, M<float>(state),
                      plane, a, step);
-  run(memory_kernel<T, DT, OUTPUTS>, true);
+  run(memory_kernel<T, DT, OUTPUTS, true>, true);
 }
 
 // proj [B,S,N]; bias [2,H] of input and forget gate; state [slots,H,vdim+1,dp]

@@ -67,16 +67,16 @@ template <typename T> DEVINL float rounded(float f) { return f; }
 template <> DEVINL float rounded<bf16_t>(float f) { bf16_t u = f2b(f); return ld(&u); }
 
 // One block per token; its row stays in registers (NC pieces of 256 V). y null:
-// x is read as it is. streams [done + 1][tokens][D]: the last one is written
-// here. h1 = norm(x) g1, h2 = norm(x) g2, the first plus its convolution if
+// x is read as it is; x null: it is the average with `before`. streams [done +
+// 1][tokens][D]: the last one is written here. out null: nobody reads it. h1 = norm(x) g1, h2 = norm(x) g2, the first plus its convolution if
 // there are taps. Loads that hang on nothing come first: one token's blocks are
 // all that a decode step of few rows has.
 template <typename T, int V, int NC>
 __global__ __launch_bounds__(256) void depth_norm_kernel(
     const T* __restrict__ y, const T* __restrict__ z, const int* __restrict__ rows, const float* __restrict__ weight,
-    const float* __restrict__ x, float* __restrict__ streams, const T* __restrict__ average, float* __restrict__ out,
-    const T* __restrict__ g1, const T* __restrict__ g2, const T* __restrict__ taps, T* __restrict__ ring,
-    T* __restrict__ h1, T* __restrict__ h2, DepthArgs a, Step step) {
+    const float* __restrict__ x, float* __restrict__ streams, const T* __restrict__ before,
+    const T* __restrict__ average, float* __restrict__ out, const T* __restrict__ g1, const T* __restrict__ g2,
+    const T* __restrict__ taps, T* __restrict__ ring, T* __restrict__ h1, T* __restrict__ h2, DepthArgs a, Step step) {
   const size_t tok = blockIdx.x, off = tok * a.D;
   __shared__ float red[4];
   constexpr int BACK = NC <= 2 ? 3 : 0;  // inputs of the convolution in registers
@@ -102,7 +102,7 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
 #pragma unroll
     for (int j = 0; j < V; ++j) v[j] = 0.f;
     if (i < a.D) {
-      ldv<V>(x + off + i, v);
+      if (x) ldv<V>(x + off + i, v);
       if (y) {
         float sum[V], t[V];
 #pragma unroll
@@ -110,16 +110,20 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
         const float* s = streams + off + i;
         auto add = [&](int n, auto count) {  // `count` streams from n on, loads first
           constexpr int N = decltype(count)::value;
-          float u[N][V], w[N];
+          float u[N][V], w[N], p[N];
 #pragma unroll
           for (int k = 0; k < N; ++k) {
             ldv<V>(s + (n + k) * a.plane, u[k]);
             w[k] = ld(average + n + k);
+            p[k] = before ? ld(before + n + k) : 0.f;
           }
 #pragma unroll
           for (int k = 0; k < N; ++k)
 #pragma unroll
-            for (int j = 0; j < V; ++j) sum[j] += w[k] * u[k][j];
+            for (int j = 0; j < V; ++j) {
+              sum[j] += w[k] * u[k][j];
+              v[j] += p[k] * u[k][j];
+            }
         };
         ldv<V>(y + off + i, t);
 #pragma unroll
@@ -145,7 +149,7 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
         const float last = ld(average + a.done);
 #pragma unroll
         for (int j = 0; j < V; ++j) v[j] = sum[j] + last * v[j];
-        stv<V>(out + off + i, v);
+        if (out) stv<V>(out + off + i, v);
       }
 #pragma unroll
       for (int j = 0; j < V; ++j) ss += v[j] * v[j];
@@ -251,23 +255,27 @@ void embed_pairs(Tensor tokens, Tensor table, double scale, Tensor pairs, int64_
 }
 
 // y [tokens,D] (none: x is read as it is), z the same, or with rows (and weight)
-// [tokens,top] rows that a token sums; x [..,D]; streams [n,..,D], of which
-// `done` are filled; average [done + 1]. -> (new stream, h1, h2)
-std::vector<OptT> depth_norm(OptT y, OptT z, OptT rows, OptT weight, Tensor x, OptT streams, int64_t done, OptT average,
-                             OptT g1, OptT g2, OptT taps, OptT ring, OptT slots, OptT positions, double eps, bool bf16) {
+// [tokens,top] rows that a token sums; streams [n,..,D], of which `done` are
+// filled; x [..,D], or before [done]: it is their average with these weights;
+// average [done + 1]. -> (new stream if `keep`, h1, h2)
+std::vector<OptT> depth_norm(OptT y, OptT z, OptT rows, OptT weight, OptT x, OptT before, OptT streams, int64_t done,
+                             OptT average, bool keep, OptT g1, OptT g2, OptT taps, OptT ring, OptT slots, OptT positions,
+                             double eps, bool bf16) {
   const auto dt = bf16 ? torch::kBFloat16 : torch::kFloat32;
-  check_io(x, torch::kFloat32);
-  const int D = x.size(-1), n = x.numel() / D;
-  DepthArgs a{D, 0, D, (int)done, 0, (size_t)x.numel(), (float)eps};
-  CHK(y || (!z && !streams));
+  CHK(y ? (bool)streams : x && !z && !streams);
+  if (x) check_io(*x, torch::kFloat32);
+  if (streams) check_io(*streams, torch::kFloat32);
+  const Tensor like = x ? *x : (*streams)[0];
+  const int D = like.size(-1), n = like.numel() / D;
+  DepthArgs a{D, 0, D, (int)done, 0, (size_t)like.numel(), (float)eps};
   if (y) {
     check_io(*y, dt);
-    CHK(y->numel() == x.numel() && streams && average);
-    check_io(*streams, torch::kFloat32);
+    CHK(y->numel() == like.numel() && average && (bool)x != (bool)before);
     check_io(*average, dt);
-    CHK(done >= 0 && streams->size(0) > done && streams->numel() == streams->size(0) * x.numel());
+    CHK(done >= 0 && streams->size(0) > done && streams->numel() == streams->size(0) * like.numel());
     CHK(average->numel() == done + 1);
   }
+  if (before) { check_io(*before, dt); CHK(y && before->numel() == done); }
   if (z) {
     check_io(*z, dt);
     a.zs = z->size(-1);
@@ -275,7 +283,7 @@ std::vector<OptT> depth_norm(OptT y, OptT z, OptT rows, OptT weight, Tensor x, O
       check_io(*rows, torch::kInt32);
       a.top = rows->size(-1);
       CHK(rows->numel() == (int64_t)n * a.top && z->numel() == rows->numel() * a.zs && a.zs >= D);
-    } else CHK(z->numel() == x.numel() && a.zs == D);
+    } else CHK(z->numel() == like.numel() && a.zs == D);
   } else CHK(!rows && !weight);
   if (weight) { check_io(*weight, torch::kFloat32); CHK(rows && weight->numel() == rows->numel()); }
   CHK((g1 || !g2) && (g1 || !taps));
@@ -290,19 +298,18 @@ std::vector<OptT> depth_norm(OptT y, OptT z, OptT rows, OptT weight, Tensor x, O
     CHK(ring->dim() == 3 && ring->size(1) == a.taps && ring->size(2) == D && (slots || n <= ring->size(0)));
     step = make_step(slots, positions, c10::nullopt, 0, true, n);
   }
-  const auto io = x.options().dtype(dt);
+  const auto io = like.options().dtype(dt);
   OptT out, h1, h2;
-  if (y) out = torch::empty_like(x);
-  else out = x;
-  if (g1) h1 = torch::empty(x.sizes(), io);
-  if (g2) h2 = torch::empty(x.sizes(), io);
+  if (y && keep) out = torch::empty_like(like);
+  if (g1) h1 = torch::empty(like.sizes(), io);
+  if (g2) h2 = torch::empty(like.sizes(), io);
   if (n == 0) return {out, h1, h2};
 #define AT(TYPE, t) (t ? (TYPE*)t->data_ptr() : nullptr)
 #define NORM(V, NC)                                                                                                   \
   if (nc <= NC) {                                                                                                     \
     hipLaunchKernelGGL((depth_norm_kernel<T, V, NC>), dim3(n), dim3(256), 0, cur_stream(), AT(const T, y), AT(const T, z), \
-                       AT(const int, rows), AT(const float, weight), P<float>(x), AT(float, streams),                 \
-                       AT(const T, average), AT(float, out), AT(const T, g1), AT(const T, g2), AT(const T, taps),     \
+                       AT(const int, rows), AT(const float, weight), AT(const float, x), AT(float, streams),          \
+                       AT(const T, before), AT(const T, average), AT(float, out), AT(const T, g1), AT(const T, g2), AT(const T, taps),     \
                        AT(T, ring), AT(T, h1), AT(T, h2), a, step);                                                   \
     return {out, h1, h2};                                                                                             \
   }

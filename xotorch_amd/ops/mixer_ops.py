@@ -50,6 +50,7 @@ class StepRows:
   carried: Dict[str, torch.Tensor] = field(default_factory=dict)
   # (state, source, key norm) of layers whose keys and values others read
   kept: Dict[int, tuple] = field(default_factory=dict)
+  streamed: bool = False  # whether the stream between layers is read by others than layers
   # the stream as it was after the embedding and after every layer so far
   depth: Optional["Depth"] = None
 
@@ -140,10 +141,12 @@ def add_norm(y: Union[torch.Tensor, Weighted], x, mult: float, w_next, eps: floa
 
 class Depth:
   """The streams that averages over depth read: `streams[j]` in fp32, as views of
-  one slab on the HIP path, whose kernels fill it."""
+  one slab on the HIP path, whose kernels fill it. before: weights of the last
+  average, where that itself was not written."""
 
-  def __init__(self, like, tokens: tuple, count: int, width: Optional[int] = None):
-    self.slab = None
+  def __init__(self, like, tokens: tuple, count: int, width: Optional[int] = None, keep: bool = True):
+    self.slab = self.before = None
+    self.keep = keep  # whether averages between layers are read by others
     if _on_hip(like):
       self.slab = torch.empty(count, *tokens, width or like.shape[-1], dtype=torch.float32, device=like.device)
     self.streams = []
@@ -203,7 +206,9 @@ def read_stream(x, reads: Reads, eps: float, dtype: torch.dtype, rows: StepRows)
 
 def depth_norm(y, z, x, weights, reads: Optional[Reads], eps: float, dtype: torch.dtype, rows: StepRows):
   """One layer's end: x + y + z joins rows.depth, the sum of its streams times
-  `weights` is the new stream. Returns it and what is read of it next."""
+  `weights` is the new stream. Returns it and what is read of it next. On the HIP
+  path a stream between two layers is None, unless it is asked for: the next
+  layer's end makes it again of what it reads anyway."""
   if _on_hip(y):
     return _depth_norm(y, z, x, rows.depth, weights, reads, eps, dtype, rows)
   new = x + y.float() if z is None else x + y.float() + z.float()
@@ -219,12 +224,14 @@ def _depth_norm(y, z, x, depth, weights, reads, eps, dtype, rows):
   norms, taps, ring = reads if reads is not None else ((), None, None)
   fused = rows.decode and taps is not None  # one token a row: the convolution's other inputs are in its state
   done = len(depth.streams) if depth is not None else 0
+  slab, before, keep = (depth.slab, depth.before, depth.keep or taps is None) if depth is not None else (None, None, False)
   x, *h = load_hip("_hip_stream").depth_norm(
-    y, z, take, weigh, x, depth.slab if depth is not None else None, done, weights, norms[0] if norms else None,
+    y, z, take, weigh, x, None if x is not None else before, slab, done, weights, keep, norms[0] if norms else None,
     norms[1] if len(norms) > 1 else None, taps if fused else None, ring if fused else None, rows.slots, rows.positions,
     eps, dtype == torch.bfloat16)
   if depth is not None:
     depth.place()
+    depth.before = weights
   h = h[:len(norms)]
   if taps is not None and not fused:
     h[0] = input_conv(h[0], taps, ring, rows)

@@ -144,7 +144,8 @@ class Ending:
 
 
 @on
-@pytest.mark.parametrize("D,done,taps", [(72, 1, 3), (50, 3, 4), (257, 4, 1), (1024, 9, 2), (3000, 6, 6), (36, 17, 4)])
+@pytest.mark.parametrize("D,done,taps", [(72, 1, 3), (50, 3, 4), (257, 4, 1), (1024, 9, 2), (3000, 6, 6), (36, 17, 4),
+                                          (40, 64, 2), (2048, 150, 4), (5000, 3, 2)])
 def test_layer_end(kind, D, done, taps):
   op = Ending(kind, 24, D, done, taps)
   want = op.expected()

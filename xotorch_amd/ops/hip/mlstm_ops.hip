@@ -46,11 +46,12 @@ DEVINL float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
 
 // One block per (head, row): u, r [B][H][P] and m [B][H][P + 1], m[0] that before
 // the row. A thread has `per` tokens (a power of two, so that chunks begin at
-// threads or threads at chunks).
-template <typename T>
+// threads or threads at chunks), PER of them in registers; PER 0: any number, kept
+// in u and r between the two walks.
+template <typename T, int PER>
 __global__ __launch_bounds__(256) void gates_kernel(
-    const T* __restrict__ proj, const T* __restrict__ bias, float* __restrict__ state_m, float* __restrict__ u,
-    float* __restrict__ r, float* __restrict__ m, int per, MemArgs a, Step step) {
+    const T* __restrict__ proj, const T* __restrict__ bias, float* __restrict__ state_m, float* u, float* r,
+    float* __restrict__ m, int per, MemArgs a, Step step) {
   const int h = blockIdx.x, b = blockIdx.y, slot = step.slot(b), len = step.len(b, a.S);
   if (slot < 0 || len <= 0) return;
   __shared__ float wf[4], wm[4];
@@ -58,24 +59,44 @@ __global__ __launch_bounds__(256) void gates_kernel(
   u += row * a.P;
   r += row * a.P;
   m += row * (a.P + 1);
+  if (PER) per = PER;
   const float bi = ld(bias + h), bf = ld(bias + a.H + h);
   const float m0 = step.first(b) ? state_m[(size_t)slot * a.H + h] : 0.f;
   const int t0 = threadIdx.x * per, t1 = min(t0 + per, a.P), lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  float F = 0.f, M = -INFINITY;  // of the thread's tokens: summed log forget gates, maximum
-#pragma unroll 4
-  for (int t = t0; t < t1; ++t) {
-    float li = -INFINITY, lf = 0.f;
-    if (t < len) {
-      const T* z = proj + ((size_t)b * a.S + t) * a.N;
-      li = log_input(ld(z + a.i_at + h), bi, a.cap);
-      lf = log_forget(ld(z + a.f_at + h), bf, a.cap);
+  constexpr int NR = PER ? PER : 1;
+  float i_of[NR], f_of[NR];
+  auto gates = [&](int t, float zi, float zf, float& li, float& lf) {
+    li = t < len ? log_input(zi, bi, a.cap) : -INFINITY;
+    lf = t < len ? log_forget(zf, bf, a.cap) : 0.f;
+  };
+  auto inputs = [&](int t) { return proj + ((size_t)b * a.S + min(t, len - 1)) * a.N + h; };
+  if (PER) {
+#pragma unroll
+    for (int k = 0; k < NR; ++k) {
+      i_of[k] = ld(inputs(t0 + k) + a.i_at);
+      f_of[k] = ld(inputs(t0 + k) + a.f_at);
     }
-    r[t] = li;  // read again below
-    u[t] = lf;
-    if (per > C && t % C == 0) F = 0.f;
-    F += lf;
-    M = fmaxf(M + lf, li);
+#pragma unroll
+    for (int k = 0; k < NR; ++k) gates(t0 + k, i_of[k], f_of[k], i_of[k], f_of[k]);
+  } else {
+    for (int t = t0; t < t1; ++t) gates(t, ld(inputs(t) + a.i_at), ld(inputs(t) + a.f_at), r[t], u[t]);
   }
+  // f(token, log input gate, log forget gate) for the thread's tokens
+  auto walk = [&](auto f) {
+    if (PER) {
+#pragma unroll
+      for (int k = 0; k < NR; ++k)
+        if (t0 + k < t1) f(t0 + k, i_of[k], f_of[k]);
+    } else
+      for (int t = t0; t < t1; ++t) f(t, r[t], u[t]);
+  };
+  float F = 0.f, sf = 0.f, sm = -INFINITY;  // summed log forget gates, of the last chunk and in all; maximum
+  walk([&](int t, float li, float lf) {
+    if (t % C == 0) F = 0.f;
+    F += lf;
+    sf += lf;
+    sm = fmaxf(sm + lf, li);
+  });
   // summed forget gates of the chunk before this thread (threads of a chunk are neighbours)
   const int group = per >= C ? 1 : C / per;
   float before = F;
@@ -86,8 +107,6 @@ __global__ __launch_bounds__(256) void gates_kernel(
   before = __shfl_up(before, 1);
   if ((lane & (group - 1)) == 0) before = 0.f;
   // maxima: (F, M) of a range followed by (F', M') is (F + F', max(M + F', M'))
-  float sf = 0.f, sm = M;
-  for (int t = t0; t < t1; ++t) sf += u[t];
   for (int d = 1; d < 64; d <<= 1) {
     const float of = __shfl_up(sf, d), om = __shfl_up(sm, d);
     if (lane >= d) { sm = fmaxf(om + sf, sm); sf += of; }
@@ -102,8 +121,7 @@ __global__ __launch_bounds__(256) void gates_kernel(
   now = fmaxf(now + sf, sm);
   if (threadIdx.x == 0) m[0] = m0;
   F = before;
-  for (int t = t0; t < t1; ++t) {
-    const float li = r[t], lf = u[t];
+  walk([&](int t, float li, float lf) {
     if (t % C == 0) F = 0.f;
     F += lf;
     now = fmaxf(now + lf, li);
@@ -111,7 +129,7 @@ __global__ __launch_bounds__(256) void gates_kernel(
     u[t] = F - now;
     r[t] = li - F;
     if (t == a.P - 1) state_m[(size_t)slot * a.H + h] = now;
-  }
+  });
 }
 
 // operand of a product whose k runs over tiles of 16: a lane holds 4 of each
@@ -807,8 +825,14 @@ void matrix_memory(Tensor proj, int64_t q_at, int64_t k_at, int64_t v_at, int64_
     auto u = f32(proj, {B, H, a.P}), r = f32(proj, {B, H, a.P}), m = f32(proj, {B, H, a.P + 1});
     int per = 1;
     while (per * 256 < a.P) per *= 2;
-    hipLaunchKernelGGL((gates_kernel<T>), dim3(H, B), dim3(256), 0, stream, P<T>(proj), P<T>(bias), M<float>(state_m),
-                       M<float>(u), M<float>(r), M<float>(m), per, a, step);
+    auto gates = [&](auto kernel) {
+      hipLaunchKernelGGL(kernel, dim3(H, B), dim3(256), 0, stream, P<T>(proj), P<T>(bias), M<float>(state_m), M<float>(u),
+                         M<float>(r), M<float>(m), per, a, step);
+    };
+    if (per == 1) gates(gates_kernel<T, 1>);
+    else if (per <= 4) { per = 4; gates(gates_kernel<T, 4>); }
+    else if (per <= 16) { per = 16; gates(gates_kernel<T, 16>); }
+    else gates(gates_kernel<T, 0>);
     if (dp <= 32) prompt<T, 2>(proj, u, r, m, norm, state, out, B, a, step);
     else if (dp <= 64) prompt<T, 4>(proj, u, r, m, norm, state, out, B, a, step);
     else if (dp <= 128) prompt<T, 8>(proj, u, r, m, norm, state, out, B, a, step);

@@ -66,19 +66,19 @@ struct DepthArgs {
 template <typename T> DEVINL float rounded(float f) { return f; }
 template <> DEVINL float rounded<bf16_t>(float f) { bf16_t u = f2b(f); return ld(&u); }
 
-// One block per token; its row stays in registers (NC pieces of 256 V). y null:
+// One block per token; its row stays in registers (NC pieces of TB V). y null:
 // x is read as it is; x null: it is the average with `before`. streams [done +
 // 1][tokens][D]: the last one is written here. out null: nobody reads it. h1 = norm(x) g1, h2 = norm(x) g2, the first plus its convolution if
 // there are taps. Loads that hang on nothing come first: one token's blocks are
 // all that a decode step of few rows has.
-template <typename T, int V, int NC>
-__global__ __launch_bounds__(256) void depth_norm_kernel(
+template <typename T, int V, int NC, int TB>
+__global__ __launch_bounds__(TB) void depth_norm_kernel(
     const T* __restrict__ y, const T* __restrict__ z, const int* __restrict__ rows, const float* __restrict__ weight,
     const float* __restrict__ x, float* __restrict__ streams, const T* __restrict__ before,
     const T* __restrict__ average, float* __restrict__ out, const T* __restrict__ g1, const T* __restrict__ g2,
     const T* __restrict__ taps, T* __restrict__ ring, T* __restrict__ h1, T* __restrict__ h2, DepthArgs a, Step step) {
   const size_t tok = blockIdx.x, off = tok * a.D;
-  __shared__ float red[4];
+  __shared__ float red[TB / 64];
   constexpr int BACK = NC <= 2 ? 3 : 0;  // inputs of the convolution in registers
   const int slot = taps ? step.slot((int)tok) : -1, pos = slot >= 0 ? step.first((int)tok) : 0;
   T* hist = ring + (size_t)max(slot, 0) * a.taps * a.D;
@@ -87,80 +87,92 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(
   for (int k = 0; k < BACK; ++k)
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
-      const int i = (c * 256 + threadIdx.x) * V;
+      const int i = (c * TB + threadIdx.x) * V;
 #pragma unroll
       for (int j = 0; j < V; ++j) old[k][c * V + j] = 0.f;
       if (slot >= 0 && k + 1 < a.taps && k + 1 <= pos && i < a.D)
         ldv<V>(hist + (size_t)((pos - 1 - k) % a.taps) * a.D + i, old[k] + c * V);
     }
   const float n1 = g1 ? ld(g1) : 0.f, n2 = g2 ? ld(g2) : 0.f;
+  // a lane has the weights of one stream of 64
+  const int lane = threadIdx.x & 63;
+  auto lane_weight = [&](const T* w, int n0, int count) { return w && n0 + lane < count ? ld(w + n0 + lane) : 0.f; };
+  auto of_lane = [](float w, int n) { return __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(w), n & 63)); };
+  const float first_now = lane_weight(average, 0, a.done), first_before = lane_weight(before, 0, a.done);
+  const float last = average ? ld(average + a.done) : 0.f;
   float xv[NC * V], ss = 0.f;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
-    const int i = (c * 256 + threadIdx.x) * V;
+    const int at = (c * TB + threadIdx.x) * V, i = min(at, a.D - V);  // all lanes go along: weights are theirs
     float* v = xv + c * V;
 #pragma unroll
     for (int j = 0; j < V; ++j) v[j] = 0.f;
-    if (i < a.D) {
-      if (x) ldv<V>(x + off + i, v);
-      if (y) {
-        float sum[V], t[V];
+    if (x) ldv<V>(x + off + i, v);
+    if (y) {
+      float sum[V], t[V];
 #pragma unroll
-        for (int j = 0; j < V; ++j) sum[j] = 0.f;
-        const float* s = streams + off + i;
-        auto add = [&](int n, auto count) {  // `count` streams from n on, loads first
-          constexpr int N = decltype(count)::value;
-          float u[N][V], w[N], p[N];
+      for (int j = 0; j < V; ++j) sum[j] = 0.f;
+      const float* s = streams + off + i;
+      float now = first_now, then = first_before;
+      auto add = [&](int n, auto count) {  // `count` streams from n on, loads first
+        constexpr int N = decltype(count)::value;
+        float u[N][V];
 #pragma unroll
-          for (int k = 0; k < N; ++k) {
-            ldv<V>(s + (n + k) * a.plane, u[k]);
-            w[k] = ld(average + n + k);
-            p[k] = before ? ld(before + n + k) : 0.f;
+        for (int k = 0; k < N; ++k) ldv<V>(s + (n + k) * a.plane, u[k]);
+        if (n && (n & 63) == 0) {
+          now = lane_weight(average, n, a.done);
+          then = lane_weight(before, n, a.done);
+        }
+#pragma unroll
+        for (int k = 0; k < N; ++k) {
+          const float w = of_lane(now, n + k), p = of_lane(then, n + k);
+#pragma unroll
+          for (int j = 0; j < V; ++j) {
+            sum[j] += w * u[k][j];
+            v[j] += p * u[k][j];
           }
+        }
+      };
+      ldv<V>(y + off + i, t);
 #pragma unroll
-          for (int k = 0; k < N; ++k)
-#pragma unroll
-            for (int j = 0; j < V; ++j) {
-              sum[j] += w[k] * u[k][j];
-              v[j] += p[k] * u[k][j];
-            }
-        };
-        ldv<V>(y + off + i, t);
+      for (int j = 0; j < V; ++j) v[j] += t[j];
+      if (z && !rows) {
+        ldv<V>(z + tok * a.zs + i, t);
 #pragma unroll
         for (int j = 0; j < V; ++j) v[j] += t[j];
-        if (z && !rows) {
-          ldv<V>(z + tok * a.zs + i, t);
-#pragma unroll
-          for (int j = 0; j < V; ++j) v[j] += t[j];
-        }
-#pragma unroll 4
-        for (int k = 0; k < a.top; ++k) {
-          const float w = weight ? weight[tok * a.top + k] : 1.f;
-          ldv<V>(z + (size_t)rows[tok * a.top + k] * a.zs + i, t);
-#pragma unroll
-          for (int j = 0; j < V; ++j) v[j] += w * t[j];
-        }
-        int n = 0;
-        for (; n + 8 <= a.done; n += 8) add(n, std::integral_constant<int, 8>());
-        if (n + 4 <= a.done) { add(n, std::integral_constant<int, 4>()); n += 4; }
-        if (n + 2 <= a.done) { add(n, std::integral_constant<int, 2>()); n += 2; }
-        if (n < a.done) add(n, std::integral_constant<int, 1>());
-        stv<V>(streams + a.done * a.plane + off + i, v);
-        const float last = ld(average + a.done);
-#pragma unroll
-        for (int j = 0; j < V; ++j) v[j] = sum[j] + last * v[j];
-        if (out) stv<V>(out + off + i, v);
       }
+#pragma unroll 4
+      for (int k = 0; k < a.top; ++k) {
+        const float w = weight ? weight[tok * a.top + k] : 1.f;
+        ldv<V>(z + (size_t)rows[tok * a.top + k] * a.zs + i, t);
 #pragma unroll
-      for (int j = 0; j < V; ++j) ss += v[j] * v[j];
+        for (int j = 0; j < V; ++j) v[j] += w * t[j];
+      }
+      int n = 0;
+      for (; n + 8 <= a.done; n += 8) add(n, std::integral_constant<int, 8>());
+      if (n + 4 <= a.done) { add(n, std::integral_constant<int, 4>()); n += 4; }
+      if (n + 2 <= a.done) { add(n, std::integral_constant<int, 2>()); n += 2; }
+      if (n < a.done) add(n, std::integral_constant<int, 1>());
+      if (at < a.D) stv<V>(streams + a.done * a.plane + off + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] = sum[j] + last * v[j];
+      if (out && at < a.D) stv<V>(out + off + i, v);
     }
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss += at < a.D ? v[j] * v[j] : 0.f;
   }
   if (!g1) return;
-  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  ss = wave_sum(ss);
+  if (lane == 0) red[threadIdx.x >> 6] = ss;
+  __syncthreads();
+  ss = 0.f;
+#pragma unroll
+  for (int w = 0; w < TB / 64; ++w) ss += red[w];
+  const float inv = 1.f / sqrtf(ss / (float)a.D + a.eps);
   const float f1 = inv * n1, f2 = inv * n2;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
-    const int i = (c * 256 + threadIdx.x) * V;
+    const int i = (c * TB + threadIdx.x) * V;
     if (i >= a.D) continue;
     float o[V];
 #pragma unroll
@@ -305,9 +317,9 @@ std::vector<OptT> depth_norm(OptT y, OptT z, OptT rows, OptT weight, OptT x, Opt
   if (g2) h2 = torch::empty(like.sizes(), io);
   if (n == 0) return {out, h1, h2};
 #define AT(TYPE, t) (t ? (TYPE*)t->data_ptr() : nullptr)
-#define NORM(V, NC)                                                                                                   \
+#define NORM(V, NC, TB)                                                                                               \
   if (nc <= NC) {                                                                                                     \
-    hipLaunchKernelGGL((depth_norm_kernel<T, V, NC>), dim3(n), dim3(256), 0, cur_stream(), AT(const T, y), AT(const T, z), \
+    hipLaunchKernelGGL((depth_norm_kernel<T, V, NC, TB>), dim3(n), dim3(TB), 0, cur_stream(), AT(const T, y), AT(const T, z), \
                        AT(const int, rows), AT(const float, weight), AT(const float, x), AT(float, streams),          \
                        AT(const T, before), AT(const T, average), AT(float, out), AT(const T, g1), AT(const T, g2), AT(const T, taps),     \
                        AT(T, ring), AT(T, h1), AT(T, h2), a, step);                                                   \
@@ -315,11 +327,16 @@ std::vector<OptT> depth_norm(OptT y, OptT z, OptT rows, OptT weight, OptT x, Opt
   }
   BY_TYPE(dt, {
     if (((D | a.zs) & 3) == 0) {
+      if (n <= 256 && D > 1024) {  // few tokens: a row over more waves
+        const int nc = (D + 4095) / 4096;
+        if (D <= 2048) NORM(4, 1, 512)
+        NORM(4, 1, 1024) NORM(4, 2, 1024) NORM(4, 4, 1024)
+      }
       const int nc = (D + 1023) / 1024;
-      NORM(4, 1) NORM(4, 2) NORM(4, 4) NORM(4, 8) NORM(4, 16)
+      NORM(4, 1, 256) NORM(4, 2, 256) NORM(4, 4, 256) NORM(4, 8, 256) NORM(4, 16, 256)
     } else {
       const int nc = (D + 255) / 256;
-      NORM(1, 1) NORM(1, 4) NORM(1, 16)
+      NORM(1, 1, 256) NORM(1, 4, 256) NORM(1, 16, 256)
     }
   });
 #undef NORM

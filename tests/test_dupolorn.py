@@ -923,6 +923,16 @@ def test_cacheless_forward_trains(checkpoints, references):
   assert not dead
 
 
+@on
+def test_cacheless_forward_without_gradients(kind, checkpoints, references):
+  name = case(kind, "base")
+  model = load_model(checkpoints[name][0], *kind)
+  with torch.no_grad():
+    out = model(torch.stack([TOKENS[:20], TOKENS[30:50]]).to(kind[0]), None, torch.arange(20), 0, last_only=False)
+  near(out[0], references(name, TOKENS[:20]), kind[1])
+  near(out[1], references(name, TOKENS[30:50]), kind[1])
+
+
 # ---------------------------------------------------------------- loading
 
 def test_config(checkpoints):

@@ -64,7 +64,7 @@ def dupolorn_config(raw: dict, model_id: str, shapes: Dict[str, tuple]) -> Model
   return ModelConfig(
     model_id=model_id, model_type="dupolorn", vocab_size=raw["vocab"], dim=raw["width"], n_layers=len(specs),
     norm_eps=float(raw["norm"]["eps"]), max_seq_len=max_positions(raw), layer_specs=specs,
-    embed_scale=float(raw["embedding"]["scale"]), bigram=bigram, final_logit_softcapping=float(raw["logit_softcap"]),
+    embed_scale=float(raw["embedding"]["scale"]), bigram=bigram, final_logit_softcapping=float(raw.get("logit_softcap") or 0.0),
     carried={"streams": len(specs) * raw["width"]},
     n_experts=max((m["router"]["experts"] for m in moes), default=0), moe_intermediate_dim=experts,
     intermediate_dim=max([experts, *(s.ff for s in specs)]),

@@ -124,6 +124,9 @@ class LayeredModel(nn.Module):
     every local layer."""
     dtype = self.layers[str(self.shard.start_layer)].norm1.dtype
     B, S = x.shape[0], x.shape[1]
+    if caches is None and x.is_cuda and not torch.is_grad_enabled():  # the kernels keep state somewhere
+      from xotorch_amd.engine.kvcache import make_cache
+      caches = make_cache(self.cfg, self.shard, B, S, dtype, x.device).caches
     rows = mo.StepRows(is_decode, 0 if is_decode else int(start_pos),
                        positions.reshape(-1) if is_decode else None, slots, lens, streamed=layers_out is not None)
     if x.dtype in (torch.int32, torch.int64):

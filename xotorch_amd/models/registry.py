@@ -411,7 +411,7 @@ model_cards: Dict[str, dict] = {
   "tapupel-dummy": {"layers": 5, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "dupolorn-3b": {"layers": 8, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "dupolorn-9b": {"layers": 16, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
-  "dupolorn-dummy": {"layers": 3, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
+  "dupolorn-dummy": {"layers": 4, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy"}},
   "dummy": {"layers": 4, "repo": {"TorchEngine": "dummy", "HIPEngine": "dummy", "DummyEngine": "dummy"}},
 }
 
